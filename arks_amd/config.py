@@ -140,7 +140,7 @@ class ModelConfig:
         with open(os.path.join(model_path, "config.json")) as f:
             cfg = json.load(f)
         if HybridModelConfig.matches(cfg):
-            return HybridModelConfig.from_dict(cfg)
+            return HybridModelConfig.from_dict(cfg, model_path)
         return cls.from_hf_config(cfg)
 
     @property
@@ -152,12 +152,17 @@ class ModelConfig:
 class HybridModelConfig:
     """Layer-list decoders: config.json names one architecture and lists the
     layers, each with its mixer type ("attention", "lightning", "mamba1",
-    "parallel", "latent_attention", "mamba2", "attention_2": what a type
-    means is the architecture's), the mixer's sizes and an optional
-    feed-forward (dense, or "moe" where the architecture has one). Every size and every
-    per-model constant comes from that file; what the architecture itself
-    fixes (block arrangement, activation, rotary pairing) lives with the
-    model code (arks_amd/models/hybrid.py)."""
+    "parallel", "latent_attention", "mamba2", "attention_2",
+    "channel_delta": what a type means is the architecture's), the mixer's
+    sizes and an optional feed-forward (dense, or "moe" where the
+    architecture has one). Every per-model constant and every size comes from
+    that file, except sizes that only the checkpoint's tensor shapes give
+    (SHAPE_SIZES); what the architecture itself fixes (block arrangement,
+    activation, rotary pairing) lives with the model code
+    (arks_amd/models/hybrid.py).
+
+    A layer with "weights_of": j runs layer j's weights with a cache and
+    state of its own (weight_owner)."""
 
     architecture: str = "Gagorax"
     vocab_size: int = 512
@@ -178,14 +183,18 @@ class HybridModelConfig:
     # a row with the same weights ({"start", "stop", "times"} or None)
     residual_mult: float = 1.0
     loop: dict = None
+    # cap c on the logits, c tanh(z / c) (0: none)
+    logit_softcap: float = 0.0
 
     # what the engine asks of any model config
     sliding_window = None
 
-    ARCHITECTURES = ("Gagorax", "Fusolix", "Legalix", "Rivolix")
-    MOE_ARCHITECTURES = ("Fusolix", "Rivolix")
+    ARCHITECTURES = ("Gagorax", "Fusolix", "Legalix", "Rivolix", "Pazilorn")
+    MOE_ARCHITECTURES = ("Fusolix", "Rivolix", "Pazilorn")
     # the logits are taken with the embedding table (no "head" tensor)
-    TIED_HEAD_ARCHITECTURES = ("Rivolix",)
+    TIED_HEAD_ARCHITECTURES = ("Rivolix", "Pazilorn")
+    # mixer type -> {size: tensor whose row count it is}
+    SHAPE_SIZES = {"channel_delta": {"decay_rank": "a1", "gate_rank": "g1"}}
 
     @property
     def tied_head(self) -> bool:
@@ -201,9 +210,14 @@ class HybridModelConfig:
         return cfg.get("architecture") in cls.ARCHITECTURES
 
     @classmethod
-    def from_dict(cls, cfg: dict) -> "HybridModelConfig":
+    def from_dict(cls, cfg: dict, model_path: str | None = None) -> "HybridModelConfig":
+        """model_path: the checkpoint folder, for sizes that only its tensor
+        shapes give."""
         layers = []
         for entry in cfg["layers"]:
+            owner = entry.get("weights_of")
+            if owner is not None:  # what it does not repeat is the owner's
+                entry = {**cfg["layers"][int(owner)], **entry}
             mlp = entry.get("mlp")
             kind = mlp.get("kind", "dense") if mlp is not None else "dense"
             if kind != "dense" and not (
@@ -211,6 +225,10 @@ class HybridModelConfig:
                 raise ValueError(f"unknown feed-forward kind {kind!r}")
             layers.append({"type": entry["type"], "mixer": dict(entry["mixer"]),
                            "mlp": dict(mlp) if mlp is not None else None})
+            if entry.get("weights_of") is not None:
+                layers[-1]["weights_of"] = int(entry["weights_of"])
+        cls._check_weight_owners(layers)
+        cls._read_shape_sizes(layers, model_path)
         for i, entry in enumerate(layers):
             src = entry["mixer"].get("kv_from")
             if src is not None and not (
@@ -234,7 +252,48 @@ class HybridModelConfig:
             embed_scale=float((cfg.get("embedding") or {}).get("scale", 1.0)),
             residual_mult=float(cfg.get("residual_mult", 1.0)),
             loop=cls._read_loop(cfg.get("loop"), len(layers)),
+            logit_softcap=float(cfg.get("logit_softcap") or 0.0),
         )
+
+    @staticmethod
+    def _check_weight_owners(layers: list) -> None:
+        for i, entry in enumerate(layers):
+            j = entry.get("weights_of")
+            if j is None:
+                continue
+            if not (0 <= j < len(layers)
+                    and layers[j].get("weights_of") is None
+                    and layers[j]["type"] == entry["type"]):
+                raise ValueError(
+                    f"layer {i}: weights_of {j!r} must name a layer of the "
+                    "same type with weights of its own")
+            if entry["mixer"] != layers[j]["mixer"] or entry["mlp"] != layers[j]["mlp"]:
+                raise ValueError(f"layer {i} differs from layer {j}, whose "
+                                 "weights it uses")
+
+    def weight_owner(self, i: int) -> int:
+        """The layer whose weights layer i runs."""
+        j = self.layers[i].get("weights_of")
+        return i if j is None else j
+
+    @classmethod
+    def _read_shape_sizes(cls, layers: list, model_path: str | None) -> None:
+        shapes = None
+        for i, entry in enumerate(layers):
+            for key, tensor in cls.SHAPE_SIZES.get(entry["type"], {}).items():
+                if key in entry["mixer"]:
+                    continue
+                if model_path is None:
+                    raise ValueError(f"layer {i}: the mixer lacks {key!r}")
+                if shapes is None:
+                    from .loader.safetensors_loader import tensor_shapes
+
+                    shapes = tensor_shapes(model_path)
+                j = entry.get("weights_of")
+                name = f"l{i if j is None else j}.mix.{tensor}"
+                if name not in shapes:
+                    raise ValueError(f"checkpoint lacks tensors: ['{name}']")
+                entry["mixer"][key] = int(shapes[name][0])
 
     @staticmethod
     def _read_loop(loop, n_layers: int):
@@ -275,6 +334,11 @@ class HybridModelConfig:
                 out["loop"] = dict(self.loop)
         if self.architecture == "Rivolix":
             out.pop("logit_scale")
+        if self.architecture == "Pazilorn":
+            out.pop("logit_scale")
+            out.update({"embedding": {"scale": self.embed_scale},
+                        "residual_mult": self.residual_mult,
+                        "logit_softcap": self.logit_softcap})
         return out
 
     @property
@@ -402,6 +466,39 @@ def _rivolix_preset(width, vocab, pattern, heads, kv_heads, dim, vdim, taps,
     return HybridModelConfig(
         architecture="Rivolix", vocab_size=vocab, hidden_size=width,
         layers=layers, rms_norm_eps=1e-6)
+
+
+def _pazilorn_preset(width, vocab, pattern, heads, kv_heads, dim, vdim, taps,
+                     low_rank, l_heads, l_dim, l_rot, l_vdim, kv_rank, q_rank,
+                     window, experts, top, expert_ff,
+                     shared=None) -> HybridModelConfig:
+    """pattern: one letter per layer, c (channel-decay delta rule) or l
+    (windowed latent attention); every layer has the routed feed-forward.
+    shared: {layer: layer whose weights it runs}."""
+    layers = []
+    for i, ch in enumerate(pattern):
+        if ch == "c":
+            spec = {"type": "channel_delta", "mixer": {
+                "heads": heads, "kv_heads": kv_heads, "dim": dim,
+                "vdim": vdim, "conv": taps, "decay_rank": low_rank,
+                "gate_rank": low_rank}}
+        else:
+            spec = {"type": "latent_attention", "mixer": {
+                "heads": l_heads, "dim": l_dim, "rot_dim": l_rot,
+                "vdim": l_vdim, "kv_rank": kv_rank, "q_rank": q_rank,
+                "mask": {"size": window}, "scale": (l_dim + l_rot) ** -0.5,
+                "rot": {"base": 1000000.0, "dims": l_rot,
+                        "scaling": {"factor": 4.0, "original": 4096,
+                                    "fast": 16.0, "slow": 2.0}}}}
+        spec["mlp"] = {"kind": "moe", "expert": {"ff": expert_ff},
+                       "router": {"experts": experts, "top": top}}
+        if shared and i in shared:
+            spec["weights_of"] = shared[i]
+        layers.append(spec)
+    return HybridModelConfig(
+        architecture="Pazilorn", vocab_size=vocab, hidden_size=width,
+        layers=layers, rms_norm_eps=1e-6, embed_scale=1.0,
+        residual_mult=0.5, logit_softcap=30.0)
 
 
 # Named synthetic configs for benchmarks / tests (random-init weights; no
@@ -708,6 +805,16 @@ PRESET_CONFIGS: dict[str, ModelConfig] = {
         3584),
     "tiny-rivolix": _rivolix_preset(
         128, 512, "dsk", 6, 2, 16, 24, 4, 4, 2, 32, 8, 2, 48, 80),
+    # Pazilorn at the layer sizes of an ~8B model: channel-decay delta rule
+    # with 32 heads x 128/128, 4 taps, low-rank projections of 128; latent
+    # attention with 32 heads x (128 + 64 rotated), values 128, latents 512
+    # and 1536, window 1024; 16 experts of ff 3584, 4 per row
+    "pazilorn-8b-slice": _pazilorn_preset(
+        4096, 32000, "cclccclc", 32, 32, 128, 128, 4, 128, 32, 128, 64, 128,
+        512, 1536, 1024, 16, 4, 3584),
+    "tiny-pazilorn": _pazilorn_preset(
+        128, 512, "clcl", 4, 2, 16, 24, 4, 12, 4, 16, 8, 24, 32, 40, 24, 8, 2,
+        48, shared={2: 0, 3: 1}),
     "tiny-gpu": ModelConfig(  # GPU-test-sized (head_dim 128 kernels)
         architecture="Qwen2ForCausalLM",
         vocab_size=2048,

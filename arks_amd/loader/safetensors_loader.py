@@ -71,6 +71,15 @@ def _parse_header(path: str):
     return data_start, ts
 
 
+def tensor_shapes(model_path: str) -> dict:
+    """{tensor name: shape} of a checkpoint folder, from the headers alone."""
+    files = sorted(glob.glob(os.path.join(model_path, "*.safetensors")))
+    if not files:
+        raise FileNotFoundError(f"no *.safetensors under {model_path}")
+    return {name: shape for path in files
+            for name, _, shape, _, _ in _parse_header(path)[1]}
+
+
 def load_model_weights(model, model_path: str, device: torch.device,
                        chunk_bytes: int = 1 << 30) -> None:
     """Stream HF-layout safetensors into the (possibly TP-sharded) model.

@@ -37,6 +37,11 @@ _REGISTRY = {
     # keys; logits through the embedding table (models/hybrid.py
     # DualNormBlock)
     "Rivolix": HybridForCausalLM,
+    # layer-list decoder: RMS norms before and after every sublayer;
+    # channel-decay delta rule and windowed latent attention, routed experts
+    # in every layer, layers on other layers' weights; capped logits through
+    # the embedding table (models/hybrid.py SandwichBlock)
+    "Pazilorn": HybridForCausalLM,
 }
 
 

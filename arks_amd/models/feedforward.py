@@ -20,12 +20,16 @@ constants as constructor parameters:
   captured; above it the (row, expert) pairs are sorted by expert and every
   expert runs plain GEMMs on its own segment (its row block of the stacked
   matrix).
-- InputScaledMoE: `experts` small silu-GLU feed-forwards of which every row
-  uses the `top` with the highest sigmoid (or softmax) score; the score
-  multiplies the expert's INPUT, expert(s h), and the results are summed as
-  they are; a shared expert of its own size runs on every row. Since
-  W (s h) = s (W h), the factor is applied to the gate and up projections
-  of h in the activation kernel, in fp32. One matrix holds every gate|up
+- RoutedMoE: `experts` small silu-GLU feed-forwards of which every row
+  uses the `top` with the highest sigmoid or softmax score, optionally
+  renormalised over the chosen ones (for a softmax: the softmax over the
+  chosen logits only); the router may have a bias; a shared expert of its
+  own size may run on every row. weigh="input": the score multiplies the
+  expert's INPUT, expert(s h), and the results are summed as they are;
+  weigh="output": the sum of s expert(h). Since W (s h) = s (W h), the
+  factor is applied in the activation kernel, in fp32, to the gate and up
+  projections of h (input) or to their activated product (output: the down
+  projection is linear). One matrix holds every gate|up
   projection, per expert and then the shared one, one matrix [width,
   experts * ff + shared_ff] every down projection. Up to DENSE_TOKENS rows
   the step is three GEMMs with data-independent shapes: all gate|up
@@ -151,22 +155,29 @@ class GroupedMoE(nn.Module):
         return ops.moe_mix_rows_seq(y, weights, inv.view(T, k).to(torch.int32))
 
 
-class InputScaledMoE(nn.Module):
+class RoutedMoE(nn.Module):
     DENSE_TOKENS = 256  # see models/llama_family.py MoEMLP.DENSE_TOKENS
 
     def __init__(self, width: int, experts: int, ff: int, top: int, dtype,
                  shared_ff: int = 0, score: str = "sigmoid",
-                 renorm: bool = False):
+                 renorm: bool = False, weigh: str = "input",
+                 router_bias: bool = False):
         super().__init__()
         assert 1 <= top <= experts and score in ("sigmoid", "softmax")
+        assert weigh in ("input", "output")
+        self.weigh_input = weigh == "input"
         self.E, self.ff, self.top, self.sff = experts, ff, top, int(shared_ff)
         self.width, self.score, self.renorm = width, score, renorm
         self.router = _param(experts, width, dtype=dtype)
+        self.router_b = (_param(experts, dtype=torch.float32) if router_bias
+                         else None)
         self.w_gu = _param(experts * 2 * ff + 2 * self.sff, width, dtype=dtype)
         self.w_down = _param(width, experts * ff + self.sff, dtype=dtype)
 
     def weight_map(self) -> dict:
         m = {"router": (self.router, 0)}
+        if self.router_b is not None:
+            m["router.b"] = (self.router_b, 0)
         W, ff, E, sff = self.width, self.ff, self.E, self.sff
         for e in range(E):
             m[f"e{e}.gate"] = (self.w_gu, e * 2 * ff)
@@ -184,12 +195,13 @@ class InputScaledMoE(nn.Module):
         z = linear_f32(h, self.router)  # fp32 logits
         if T <= self.DENSE_TOKENS:
             _, _, scale = ops.moe_route_grouped(
-                z, k, 1, 1, self.score, self.renorm, matrix=True)
+                z, k, 1, 1, self.score, self.renorm, matrix=True,
+                bias=self.router_b)
             gu = linear(h, self.w_gu)
-            return linear(ops.moe_glu_scaled(gu, scale, E, ff, sff),
-                          self.w_down)
+            return linear(ops.moe_glu_scaled(gu, scale, E, ff, sff,
+                                             self.weigh_input), self.w_down)
         weights, ids = ops.moe_route_grouped(z, k, 1, 1, self.score,
-                                             self.renorm)
+                                             self.renorm, bias=self.router_b)
         # (row, expert) pairs sorted by expert: every expert runs two plain
         # GEMMs on its own contiguous segment (one host read of the sizes)
         flat = ids.reshape(-1).long()
@@ -205,7 +217,8 @@ class InputScaledMoE(nn.Module):
                          self.w_gu[e * 2 * ff:(e + 1) * 2 * ff].t(),
                          out=gu[at:at + n])
             at += n
-        a = ops.glu_act(gu, "swiglu", row_scale=weights.reshape(-1)[order])
+        a = ops.glu_act(gu, "swiglu", row_scale=weights.reshape(-1)[order]
+                        if self.weigh_input else None)
         y = torch.empty((T * k, self.width), dtype=h.dtype, device=h.device)
         at = 0
         for e, n in enumerate(counts):
@@ -220,7 +233,8 @@ class InputScaledMoE(nn.Module):
         if sff:
             sa = ops.glu_act(linear(h, self.w_gu[E * 2 * ff:]), "swiglu")
             shared = linear(sa, self.w_down[:, E * ff:])
-        return ops.moe_mix_rows_seq(y, torch.ones_like(weights),
+        return ops.moe_mix_rows_seq(y, torch.ones_like(weights)
+                                    if self.weigh_input else weights,
                                     inv.view(T, k).to(torch.int32), shared)
 
 
@@ -230,9 +244,16 @@ def build_feedforward(mlp: dict, width: int, dtype, arch: str = "") -> nn.Module
         if kind != "moe":
             raise ValueError(f"unknown feed-forward kind {kind!r}")
         r = mlp["router"]
-        return InputScaledMoE(width, r["experts"], mlp["expert"]["ff"],
-                              r["top"], dtype,
-                              shared_ff=(mlp.get("shared") or {}).get("ff", 0))
+        return RoutedMoE(width, r["experts"], mlp["expert"]["ff"],
+                         r["top"], dtype,
+                         shared_ff=(mlp.get("shared") or {}).get("ff", 0))
+    if arch == "Pazilorn":
+        if kind != "moe":
+            raise ValueError(f"unknown feed-forward kind {kind!r}")
+        r = mlp["router"]
+        return RoutedMoE(width, r["experts"], mlp["expert"]["ff"], r["top"],
+                         dtype, score="softmax", renorm=True, weigh="output",
+                         router_bias=True)
     if kind == "dense":
         return ClampedGLU(width, mlp["ff"], mlp["limit"], dtype)
     if kind == "moe":

@@ -56,12 +56,26 @@ Rivolix's is:
   - mixers "attention" (two-map difference attention behind short
     convolutions; a layer may read an earlier layer's key/value pages) and
     "attention_2" (values are the keys; rotary with ramp-scaled
-    frequencies, then unit RMS of q and k); feed-forward InputScaledMoE;
+    frequencies, then unit RMS of q and k); feed-forward RoutedMoE;
     the logits are taken with the embedding table
   Kernel plan per layer: residual_pair_norm (adds the previous layer's two
   results, scaled, to the fp32 residual and writes both normed rows, one
   pass) -> mixer and feed-forward, each with GEMMs of its own (their
   inputs differ).
+
+Pazilorn's is:
+  - RMS norms in FRONT of and BEHIND every sublayer, one sublayer after the
+    other: x += mult * post(sub(pre(x))) (SandwichBlock); x starts as the
+    scaled embedding
+  - mixers "channel_delta" (delta rule with a decay per key channel) and
+    "latent_attention" (windowed, ramp-scaled rotary, a gate per head);
+    feed-forward RoutedMoE weighing the experts' outputs
+  - a layer may run another layer's weights (weights_of) with a cache and
+    state of its own; the logits are taken with the embedding table and
+    capped, c tanh(z / c)
+  Kernel plan per sublayer: residual_sandwich_norm (norms the previous
+  sublayer's result, adds it to the fp32 residual and norms the new row for
+  the next sublayer, one pass) -> sublayer.
 
 The per-layer cache is a dict of tensors (paged KV for attention, slot
 state for the recurrent mixers and the token shift), allocated by
@@ -97,7 +111,9 @@ class BlockArrangement:
     # side (SharedNormBlock);
     # "dual": two RMS norms of the same rows, one per sublayer, the
     # sublayers side by side, a per-channel scale on each result
-    # (DualNormBlock)
+    # (DualNormBlock);
+    # "sandwich": an RMS norm in front of and one behind each sublayer
+    # (SandwichBlock)
     norm_place: str = "output"
 
 
@@ -109,6 +125,8 @@ ARRANGEMENTS = {
                                 norm_place="shared"),
     "Rivolix": BlockArrangement(token_shift=False, gated_residual=False,
                                 norm_place="dual"),
+    "Pazilorn": BlockArrangement(token_shift=False, gated_residual=False,
+                                 norm_place="sandwich"),
 }
 
 
@@ -325,6 +343,42 @@ class DualNormBlock(nn.Module):
         return dict(self.mixer.cache_layout(block_size, dtype))
 
 
+class SandwichBlock(nn.Module):
+    """x += mult * norm1b(mixer(norm1(x))), then
+    x += mult * norm2b(ff(norm2(x))), all four RMS norms with a plain
+    weight. The norms and the sum are the kernels between the sublayers
+    (ops.residual_sandwich_norm, called by the model's forward); this module
+    holds the weights and the two sublayers."""
+
+    def __init__(self, width: int, spec: dict, eps: float, dtype, arch: str):
+        super().__init__()
+        f32 = torch.float32
+        self.mixer = build_mixer(spec["type"], spec["mixer"], width, eps, dtype,
+                                 arch=arch)
+        self.ffn = (build_feedforward(spec["mlp"], width, dtype, arch)
+                    if spec.get("mlp") is not None else None)
+        for q in (1, 2) if self.ffn is not None else (1,):
+            setattr(self, f"norm{q}", _param(width, dtype=f32))
+            setattr(self, f"norm{q}b", _param(width, dtype=f32))
+
+    def weight_map(self) -> dict:
+        m = {"mix." + k: v for k, v in self.mixer.weight_map().items()}
+        m["norm1"], m["norm1b"] = (self.norm1, 0), (self.norm1b, 0)
+        if self.ffn is not None:
+            m.update({"mlp." + k: v for k, v in self.ffn.weight_map().items()})
+            m["norm2"], m["norm2b"] = (self.norm2, 0), (self.norm2b, 0)
+        return m
+
+    def cache_layout(self, block_size: int, dtype) -> dict:
+        return dict(self.mixer.cache_layout(block_size, dtype))
+
+    def sublayers(self):
+        """(norm in front, sublayer, norm behind) in order."""
+        yield self.norm1, self.mixer, self.norm1b
+        if self.ffn is not None:
+            yield self.norm2, self.ffn, self.norm2b
+
+
 class HybridForCausalLM(nn.Module):
     supports_float32 = True
     has_sequence_state = True  # engine: state slots, no prefix reuse
@@ -354,6 +408,13 @@ class HybridForCausalLM(nn.Module):
                 DualNormBlock(W, spec, cfg.rms_norm_eps, dtype,
                               cfg.architecture)
                 for spec in cfg.layers)
+        elif arr.norm_place == "sandwich":
+            own = {i: SandwichBlock(W, spec, cfg.rms_norm_eps, dtype,
+                                    cfg.architecture)
+                   for i, spec in enumerate(cfg.layers)
+                   if cfg.weight_owner(i) == i}
+            self.layers = nn.ModuleList(own[cfg.weight_owner(i)]
+                                        for i in range(len(cfg.layers)))
         else:
             self.layers = nn.ModuleList(
                 HybridBlock(W, spec, cfg.rms_norm_eps, dtype, arr)
@@ -387,6 +448,8 @@ class HybridForCausalLM(nn.Module):
                 self.loop_in = _param(W, 2 * W, dtype=dtype)
                 self._wmap["loop.in"] = (self.loop_in, 0)
         for i, layer in enumerate(self.layers):
+            if cfg.weight_owner(i) != i:
+                continue  # layer weight_owner(i)'s module and tensors
             for k, v in layer.weight_map().items():
                 self._wmap[f"l{i}.{k}"] = v
         self._loaded: set = set()
@@ -435,6 +498,8 @@ class HybridForCausalLM(nn.Module):
             return self._forward_shared(batch, caches)
         if self.arr.norm_place == "dual":
             return self._forward_dual(batch, caches)
+        if self.arr.norm_place == "sandwich":
+            return self._forward_sandwich(batch, caches)
         x = self.embed[batch.input_ids].float()
         for i, layer in enumerate(self.layers):
             layer(x, batch, caches[i], self.dtype)
@@ -551,6 +616,37 @@ class HybridForCausalLM(nn.Module):
                                       dtype)
         return linear_f32(n, self.head) * cfg.logit_scale
 
+    def _forward_sandwich(self, batch: ForwardBatch, caches: list) -> torch.Tensor:
+        """Sandwich-norm arrangement: a sublayer's result waits until the
+        kernel that norms the next sublayer's input; that kernel norms the
+        result, adds it to the residual and norms the new row, so each
+        sublayer costs one pass over the fp32 rows."""
+        cfg, dtype = self.cfg, self.dtype
+        eps, mult = cfg.rms_norm_eps, cfg.residual_mult
+        x = self.embed[batch.input_ids].float()
+        if cfg.embed_scale != 1.0:
+            x *= cfg.embed_scale
+        y = post = None
+        for i, layer in enumerate(self.layers):
+            for pre, sub, after in layer.sublayers():
+                h = ops.residual_sandwich_norm(x, y, post, mult, pre, eps, dtype)
+                y, post = sub(h, batch, caches[i]), after
+            if self.residual_tap is not None:
+                ops.residual_sandwich_norm(x, y, post, mult, None, eps, dtype)
+                y = None
+                self.residual_tap(i, x)
+        if batch.logits_indices is not None:
+            x = x[batch.logits_indices]
+            y = y[batch.logits_indices] if y is not None else None
+        n = ops.residual_sandwich_norm(x, y, post, mult, self.final_norm, eps,
+                                       dtype)
+        logits = linear_f32(n, self.head)
+        if cfg.logit_scale != 1.0:
+            logits = logits * cfg.logit_scale
+        if cfg.logit_softcap > 0:
+            ops.softcap_(logits, cfg.logit_softcap)
+        return logits
+
     # ------------------------------------------------------------ weights
     @staticmethod
     def _span(entry, w):
@@ -630,7 +726,8 @@ class HybridForCausalLM(nn.Module):
                 w = rn(0.3)
             elif leaf in ("mix.q.conv", "mix.k.conv", "mix.v.conv"):
                 w = rn(0.5)
-            elif leaf.endswith("norm") or leaf in ("norm1", "norm2"):
+            elif leaf.endswith("norm") or leaf in ("norm1", "norm2", "norm1b",
+                                                   "norm2b"):
                 w = 1.0 + rn(0.1)
             elif leaf == "mix.dt_bias":
                 w = rn(0.5) - 1.0

@@ -41,8 +41,15 @@ constructor parameters so that more than one design can use it:
   position, a sigmoid output gate; optionally on the pages of an earlier
   layer's keys and values.
 
-WindowPoolAttention, RetentionMixer, LatentAttention and Mamba2Mixer are
-"split" mixers: they name the rows of their
+- LatentAttention also takes half-split pairs, ramp-scaled rotary
+  frequencies, a sliding window, no sink and a sigmoid gate per head.
+- ChannelDeltaMixer: delta rule (every token corrects what the state holds
+  for its key) with one decay per head and key channel from a low-rank
+  projection, unit queries and keys behind short convolutions, a
+  [dim x vdim] fp32 state per head and sequence, gated unit-RMS read-out.
+
+WindowPoolAttention, RetentionMixer, LatentAttention, Mamba2Mixer,
+DiffAttention and ChannelDeltaMixer are "split" mixers: they name the rows of their
 in-projection (in_spans) and the columns of their out-projection
 (out_cols) and do everything between in core(), so that a parent can fuse
 the projections of several of them; alone, SplitMixer.forward runs the
@@ -403,6 +410,9 @@ class SplitMixer(nn.Module):
     fused ones and calls core() on its slice."""
 
     out_has_bias = False
+    # rows of an own in-projection are padded with zero rows to a multiple
+    # of this, which keeps the rows of its result on 16-byte borders
+    pad_rows = 1
 
     def in_spans(self) -> list:
         raise NotImplementedError
@@ -410,6 +420,7 @@ class SplitMixer(nn.Module):
     def _make_projections(self, width: int, dtype) -> None:
         spans = self.in_spans()
         rows = sum(n for _, n, _ in spans)
+        rows += -rows % self.pad_rows
         self.w_in = _param(rows, width, dtype=dtype)
         self.b_in = (_param(rows, dtype=dtype)
                      if any(b for _, _, b in spans) else None)
@@ -419,7 +430,7 @@ class SplitMixer(nn.Module):
     def weight_map(self) -> dict:
         m, row = {}, 0
         for name, n, has_b in self.in_spans():
-            m[name] = (self.w_in, row)
+            m[name] = (self.w_in, row, 0, (n, self.w_in.shape[1]))
             if has_b:
                 m[name + ".b"] = (self.b_in, row)
             row += n
@@ -541,9 +552,12 @@ class LatentAttention(SplitMixer):
     """Attention through low-rank latents. Per row: c_q = rmsnorm(W_dq h),
     q = W_uq c_q, laid out per head as [dim plain | rot_dim rotated];
     W_dkv h = [kv_rank | rot_dim]: the first part RMS-normed is the latent c,
-    the second, rotated (interleaved pairs), is one key part shared by all
-    heads. Keys are [W_uk c | shared part], values W_uv c, causal softmax
-    with a learned per-head sink in the denominator.
+    the second, rotated (interleaved pairs unless interleaved is off;
+    frequencies scaled along rot_scaling's ramp if given), is one key part
+    shared by all heads. Keys are [W_uk c | shared part], values W_uv c,
+    causal softmax with a learned per-head sink in the denominator (sink);
+    window w > 0: row i sees key j only if i - j < w. head_gate: head h's
+    output is multiplied by sigmoid(W_g h)_h.
 
     Only [c | rotated part] is cached, one row per token ("ckv", one
     key/value head). The up-projections move to the other side of the
@@ -557,19 +571,26 @@ class LatentAttention(SplitMixer):
     head, key), against dim + rot_dim + vdim for per-head keys and values,
     and pays for a step of few rows over a long context. A step with a long
     portion (EXPAND_ROWS rows or more of one sequence) therefore takes the
-    other form: the latents of every sequence's context are gathered from
+    other form: the latents of every sequence's context (with a window: of
+    the pages its rows can reach) are gathered from
     the pages and up-projected once into per-head keys and values for the
     step (temporary pages of the usual layout with a block table of their
     own), and the same attention kernels run on H key/value heads."""
+
+    pad_rows = 64
 
     EXPAND_ROWS = 192
 
     def __init__(self, width: int, heads: int, dim: int, rot_dim: int,
                  vdim: int, kv_rank: int, q_rank: int, scale: float,
                  rot_base: float, eps: float, dtype,
-                 own_projections: bool = True):
+                 own_projections: bool = True, sink: bool = True,
+                 interleaved: bool = True, rot_scaling: dict | None = None,
+                 window: int = 0, head_gate: bool = False):
         super().__init__()
         assert rot_dim % 2 == 0
+        self.interleaved, self.window = interleaved, int(window)
+        self.head_gate = head_gate
         self.H, self.D, self.R, self.V = heads, dim, rot_dim, vdim
         self.rank, self.q_rank = kv_rank, q_rank
         self.scale, self.eps = float(scale), eps
@@ -581,19 +602,31 @@ class LatentAttention(SplitMixer):
         # per head [dim, kv_rank] and [vdim, kv_rank], heads stacked by rows
         self.uk = _param(heads * dim, kv_rank, dtype=dtype)
         self.uv = _param(heads * vdim, kv_rank, dtype=dtype)
-        self.sink = _param(heads, dtype=f32)
-        self.register_buffer("inv_freq", rotary_inv_freq(rot_base, rot_dim),
+        # per head [kv_rank, vdim]: uv as the right operand of a batched product
+        self.register_buffer("uv_t", torch.zeros(heads, kv_rank, vdim, dtype=dtype),
                              persistent=False)
+        self.sink = _param(heads, dtype=f32) if sink else None
+        freqs, self.rot_mag = ramp_scaled_inv_freq(rot_base, rot_dim, rot_scaling)
+        self.register_buffer("inv_freq", freqs, persistent=False)
         if own_projections:
             self._make_projections(width, dtype)
 
     def in_spans(self) -> list:
-        return [("dq", self.q_rank, False), ("dkv", self.rank + self.R, False)]
+        spans = [("dq", self.q_rank, False), ("dkv", self.rank + self.R, False)]
+        if self.head_gate:
+            spans.append(("g", self.H, False))
+        return spans
 
     def extra_weights(self) -> dict:
-        return {"dq.norm": (self.dq_norm, 0), "dkv.norm": (self.dkv_norm, 0),
-                "uq": (self.uq, 0), "sink": (self.sink, 0),
-                "uk": (self.uk, 0), "uv": (self.uv, 0)}
+        m = {"dq.norm": (self.dq_norm, 0), "dkv.norm": (self.dkv_norm, 0),
+             "uq": (self.uq, 0), "uk": (self.uk, 0), "uv": (self.uv, 0)}
+        if self.sink is not None:
+            m["sink"] = (self.sink, 0)
+        return m
+
+    def finish_loading(self) -> None:
+        self.uv_t.copy_(self.uv.data.view(self.H, self.V, self.rank)
+                        .transpose(1, 2))
 
     def cache_layout(self, block_size: int, dtype) -> dict:
         return {"ckv": ("paged", (1, block_size, self.rank + self.R), dtype)}
@@ -605,48 +638,67 @@ class LatentAttention(SplitMixer):
         cq = ops.latent_prepare(
             p[:, :self.q_rank], p[:, self.q_rank:self.q_rank + rank + R],
             self.dq_norm, self.dkv_norm, self.eps, batch.positions,
-            self.inv_freq, ckv, batch.slot_mapping)
+            self.inv_freq, ckv, batch.slot_mapping, self.interleaved,
+            self.rot_mag)
         q = linear(cq, self.uq).view(T, H, D + R)
+        gate = None
+        if self.head_gate:
+            at = self.q_rank + rank + R
+            gate = p[:, at:at + H]
         if (batch.max_q_len >= self.EXPAND_ROWS
                 and batch.kv_lens_list is not None):
-            self._expanded(q, batch, ckv, out, out_scale)
+            self._expanded(q, batch, ckv, gate, out, out_scale)
             return
         # [H, T, D] x [H, D, rank]: the key up-projection applied to q
         q_abs = torch.bmm(q[..., :D].transpose(0, 1),
                           self.uk.view(H, D, rank))
         qf = torch.empty((T, H, rank + R), dtype=p.dtype, device=p.device)
-        ops.latent_query(q, q_abs, batch.positions, self.inv_freq, qf)
+        ops.latent_query(q, q_abs, batch.positions, self.inv_freq, qf,
+                         self.interleaved, self.rot_mag)
         o_lat = ops.attention_sink_paged(
             qf, ckv, ckv[..., :rank], batch.block_tables, batch.seq_lens,
             batch.cu_seqlens, batch.token_seq, self.scale, False, None, True,
-            batch.max_q_len, batch.positions, sink_w=self.sink)
+            batch.max_q_len, batch.positions, sink_w=self.sink,
+            window=self.window)
         # [H, T, rank] x [H, rank, V]: the value up-projection
-        o = torch.bmm(o_lat.transpose(0, 1),
-                      self.uv.view(H, V, rank).transpose(1, 2))
-        if out_scale != 1.0:
-            o = o * out_scale
-        out.unflatten(-1, (H, V)).copy_(o.transpose(0, 1))
+        o = torch.bmm(o_lat.transpose(0, 1), self.uv_t)
+        ops.head_gate(o.transpose(0, 1), gate, out.unflatten(-1, (H, V)),
+                      out_scale)
 
+    def _reachable_pages(self, batch: ForwardBatch, bs: int):
+        """(page ids of every sequence's reachable context in sequence
+        order, block table of the temporary pages (consecutive), lengths
+        less the positions of the skipped leading pages), once per step and
+        window."""
+        key = ("latent_pages", bs, self.window)
+        if key not in batch.tile_cache:
+            dev = batch.block_tables.device
+            ids, spans, at = [], [], 0
+            lens = []
+            for s, (n, rows) in enumerate(zip(batch.kv_lens_list,
+                                              batch.seq_lens_list)):
+                first = (max(0, n - rows - self.window + 1) // bs
+                         if self.window else 0)
+                last = -(-n // bs)
+                ids.append(batch.block_tables[s, first:last].long())
+                spans.append((at, last - first))
+                lens.append(n - first * bs)
+                at += last - first
+            table = torch.zeros((len(spans), max(n for _, n in spans)),
+                                dtype=torch.int32)
+            for s, (a, n) in enumerate(spans):
+                table[s, :n] = torch.arange(a, a + n, dtype=torch.int32)
+            batch.tile_cache[key] = (
+                torch.cat(ids), table.to(dev),
+                torch.tensor(lens, dtype=torch.int32, device=dev))
+        return batch.tile_cache[key]
 
-    def _expanded(self, q, batch: ForwardBatch, ckv, out, out_scale) -> None:
+    def _expanded(self, q, batch: ForwardBatch, ckv, gate, out,
+                  out_scale) -> None:
         T = q.shape[0]
         H, D, R, V, rank = self.H, self.D, self.R, self.V, self.rank
         bs = ckv.shape[2]
-        nb = [-(-n // bs) for n in batch.kv_lens_list]
-        key = ("latent_pages", bs)
-        if key not in batch.tile_cache:
-            # the context's pages in sequence order, and the block table
-            # of the temporary pages (consecutive), once per step
-            dev = q.device
-            idx = torch.cat([batch.block_tables[s, :n].long()
-                             for s, n in enumerate(nb)])
-            table = torch.zeros((len(nb), max(nb)), dtype=torch.int32)
-            at = 0
-            for s, n in enumerate(nb):
-                table[s, :n] = torch.arange(at, at + n, dtype=torch.int32)
-                at += n
-            batch.tile_cache[key] = (idx, table.to(dev))
-        idx, table = batch.tile_cache[key]
+        idx, table, lens = self._reachable_pages(batch, bs)
         NB = idx.shape[0]
         lat = ckv[idx]  # [NB, 1, bs, rank + R]
         c = lat[..., :rank].reshape(NB * bs, rank)
@@ -655,12 +707,18 @@ class LatentAttention(SplitMixer):
         kt[..., D:] = lat[..., rank:]
         vt = linear(c, self.uv).view(NB, bs, H, V).transpose(1, 2).contiguous()
         qf = torch.empty((T, H, D + R), dtype=q.dtype, device=q.device)
-        ops.latent_query(q, None, batch.positions, self.inv_freq, qf)
+        ops.latent_query(q, None, batch.positions, self.inv_freq, qf,
+                         self.interleaved, self.rot_mag)
+        heads = out.unflatten(-1, (H, V))
+        # only distances between rows and keys enter: lens without the
+        # skipped pages on both sides keeps them
         ops.attention_sink_paged(
-            qf, kt, vt, table, batch.seq_lens, batch.cu_seqlens,
-            batch.token_seq, self.scale, False, None, True, batch.max_q_len,
-            batch.positions, sink_w=self.sink, out=out.unflatten(-1, (H, V)),
+            qf, kt, vt, table, lens, batch.cu_seqlens, batch.token_seq,
+            self.scale, False, None, True, batch.max_q_len, batch.positions,
+            sink_w=self.sink, window=self.window, out=heads,
             out_scale=out_scale)
+        if gate is not None:
+            ops.head_gate(heads, gate, heads, 1.0)
 
 
 class Mamba2Mixer(SplitMixer):
@@ -853,6 +911,95 @@ class DiffAttention(SplitMixer):
                                 self.eps, 1.0 - self.diff, H, G, out)
 
 
+class ChannelDeltaMixer(SplitMixer):
+    """Delta rule with a decay per key channel. In-projection rows
+    [q: G*D | k: G*D | v: H*V | a1 | g1 | b: H]; head h uses q/k head
+    h // (H/G). q, k and v pass a causal depthwise convolution over time
+    (taps per channel, no bias) and silu; q and k are brought to unit length
+    per head (x / sqrt(sum x^2 + 1e-6)), q times D^-1/2. Per head, with
+    beta = sigmoid(b), the decays g = exp(-exp(A_log) softplus(W_a2 a1 +
+    dt_bias)) per key channel and S [D x V] fp32:
+    S <- g S (rows), u = beta (v - S^T k), S <- S + k u^T, o = S^T q.
+    Each head's o at unit RMS (eps), times the weight `norm` [V], times
+    sigmoid(W_g2 g1). The last taps-1 projected q|k|v rows of a sequence are
+    slot state beside S.
+
+    The two low-rank up-projections are blocks of one matrix [a2 0; 0 g2]:
+    a short step takes both in one GEMM, a long one each on its own."""
+
+    pad_rows = 64
+    JOINT_LOW_RANK_ROWS = 64
+
+    def __init__(self, width: int, heads: int, kv_heads: int, dim: int,
+                 vdim: int, conv: int, decay_rank: int, gate_rank: int,
+                 eps: float, dtype, own_projections: bool = True):
+        super().__init__()
+        assert heads % kv_heads == 0 and conv >= 1
+        self.H, self.G, self.D, self.V = heads, kv_heads, dim, vdim
+        self.taps, self.eps = int(conv), eps
+        self.ra, self.rg = int(decay_rank), int(gate_rank)
+        self.n_qk = kv_heads * dim
+        self.ch = 2 * self.n_qk + heads * vdim  # convolved channels
+        self.out_cols = heads * vdim
+        f32 = torch.float32
+        self.conv_w = _param(self.ch, self.taps, dtype=f32)
+        self.low = _param(heads * (dim + vdim), self.ra + self.rg, dtype=dtype)
+        self.dt_bias = _param(heads * dim, dtype=f32)
+        self.A_log = _param(heads, dtype=f32)
+        self.norm = _param(vdim, dtype=f32)
+        self.register_buffer("rate", torch.zeros(heads, dtype=f32),
+                             persistent=False)
+        self.register_buffer("conv_w_t", torch.zeros(self.taps, self.ch, dtype=f32),
+                             persistent=False)
+        if own_projections:
+            self._make_projections(width, dtype)
+
+    def in_spans(self) -> list:
+        return [("q", self.n_qk, False), ("k", self.n_qk, False),
+                ("v", self.H * self.V, False), ("a1", self.ra, False),
+                ("g1", self.rg, False), ("b", self.H, False)]
+
+    def extra_weights(self) -> dict:
+        HD, HV = self.H * self.D, self.H * self.V
+        return {"q.conv": (self.conv_w, 0, 0, (self.n_qk, self.taps)),
+                "k.conv": (self.conv_w, self.n_qk, 0, (self.n_qk, self.taps)),
+                "v.conv": (self.conv_w, 2 * self.n_qk, 0, (HV, self.taps)),
+                "a2": (self.low, 0, 0, (HD, self.ra)),
+                "g2": (self.low, HD, self.ra, (HV, self.rg)),
+                "dt_bias": (self.dt_bias, 0), "A_log": (self.A_log, 0),
+                "norm": (self.norm, 0)}
+
+    def finish_loading(self) -> None:
+        self.rate.copy_(torch.exp(self.A_log.data.float()))
+        self.conv_w_t.copy_(self.conv_w.data.t())
+
+    def cache_layout(self, block_size: int, dtype) -> dict:
+        out = {"S": ("slot", (self.H, self.D, self.V), torch.float32)}
+        if self.taps > 1:
+            out["conv"] = ("slot", (self.taps - 1, self.ch), torch.float32)
+        return out
+
+    def core(self, p, batch: ForwardBatch, cache: dict, out, out_scale) -> None:
+        assert out_scale == 1.0
+        H, D, ch, ra, rg = self.H, self.D, self.ch, self.ra, self.rg
+        u = ops.causal_conv_silu(
+            p[:, :ch], self.conv_w, None, cache.get("conv"), batch.cu_seqlens,
+            batch.seq_lens, batch.state_slots, batch.token_seq, self.conv_w_t,
+            batch.max_q_len)
+        at = ch + ra + rg
+        if p.shape[0] <= self.JOINT_LOW_RANK_ROWS:
+            low = linear_f32(p[:, ch:at], self.low)
+            decay, gate = low[:, :H * D], low[:, H * D:]
+        else:
+            decay = linear_f32(p[:, ch:ch + ra], self.low[:H * D, :ra])
+            gate = linear(p[:, ch + ra:at], self.low[H * D:, ra:])
+        ops.channel_delta(
+            u, decay, p[:, at:at + H], gate, self.rate, self.dt_bias,
+            self.norm, self.eps, cache["S"], batch.cu_seqlens, batch.seq_lens,
+            batch.state_slots, H, self.G, D, self.V, out, batch.max_q_len,
+            step_chunks(batch, p.device, ops.DELTA_CHUNK))
+
+
 class ParallelMixer(nn.Module):
     """left_scale * left(h) + right_scale * right(h) for two split mixers:
     one GEMM projects h for both, each core() writes its head outputs,
@@ -969,6 +1116,23 @@ def build_mixer(kind: str, m: dict, width: int, eps: float, dtype,
                 interleaved=False, own_projections=own_projections,
                 rot_scaling=rot.get("scaling"), unit_norm_after=True,
                 value_is_key=True)
+        raise ValueError(f"unknown mixer type {kind!r}")
+    if arch == "Pazilorn":
+        if kind == "channel_delta":
+            return ChannelDeltaMixer(
+                width, m["heads"], m["kv_heads"], m["dim"], m["vdim"],
+                m["conv"], m["decay_rank"], m["gate_rank"], eps, dtype,
+                own_projections=own_projections)
+        if kind == "latent_attention":
+            rot = m["rot"]
+            if rot["dims"] != m["rot_dim"]:
+                raise ValueError("latent_attention: rot.dims must equal rot_dim")
+            return LatentAttention(
+                width, m["heads"], m["dim"], m["rot_dim"], m["vdim"],
+                m["kv_rank"], m["q_rank"], m["scale"], rot["base"], eps, dtype,
+                own_projections=own_projections, sink=False,
+                interleaved=False, rot_scaling=rot.get("scaling"),
+                window=(m.get("mask") or {}).get("size") or 0, head_gate=True)
         raise ValueError(f"unknown mixer type {kind!r}")
     if kind == "attention":
         return SinkRotaryAttention(

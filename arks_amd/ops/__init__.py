@@ -844,13 +844,15 @@ def gated_rmsnorm(o, weight, gate, eps, out_dtype):
 
 
 def causal_conv_silu(x, weight, bias, state, cu_seqlens, seq_lens,
-                     state_slots, token_seq, weight_t=None):
-    """weight_t: [taps, C] copy of the taps for the vectorised bf16 kernel."""
+                     state_slots, token_seq, weight_t=None, max_q_len=0):
+    """weight_t: [taps, C] copy of the taps for the vectorised bf16 kernel;
+    bias may be None; max_q_len 1 (every sequence brings one row) lets the
+    kernel replace the history in the same launch."""
     if x.is_cuda:
         out = torch.empty(x.shape, dtype=x.dtype, device=x.device)
         _native_seq().causal_conv_silu(out, x, weight, weight_t, bias, state,
                                        cu_seqlens, seq_lens, state_slots,
-                                       token_seq)
+                                       token_seq, max_q_len == 1)
         return out
     return ref.causal_conv_silu(x, weight, bias, state, cu_seqlens, seq_lens,
                                 state_slots)
@@ -1046,10 +1048,10 @@ def glu_act(gu, kind, limit=0.0, alpha=1.0, out=None, row_scale=None):
 
 
 def moe_route_grouped(logits, top, groups=1, keep=1, score="softmax",
-                      renorm=True, matrix=False):
+                      renorm=True, matrix=False, bias=None):
     """Group-limited routing: (weights [T, top] fp32, ids [T, top] int32);
-    score "softmax" or "sigmoid", renorm: the chosen scores divided by their
-    sum. matrix: also a [T, E] fp32 tensor holding each row's weights at
+    score "softmax" or "sigmoid" of the logits (+ bias [E] fp32), renorm: the
+    chosen scores divided by their sum. matrix: also a [T, E] fp32 tensor holding each row's weights at
     the experts it uses and 0 elsewhere."""
     if logits.is_cuda:
         T, E = logits.shape
@@ -1059,9 +1061,10 @@ def moe_route_grouped(logits, top, groups=1, keep=1, score="softmax",
                if matrix else None)
         _native_seq().moe_route_grouped(w, ids, logits.contiguous(), top,
                                         groups, keep, score == "sigmoid",
-                                        bool(renorm), mat)
+                                        bool(renorm), mat, bias)
         return (w, ids, mat) if matrix else (w, ids)
-    w, ids = ref.moe_route_grouped(logits, top, groups, keep, score, renorm)
+    w, ids = ref.moe_route_grouped(logits, top, groups, keep, score, renorm,
+                                   bias)
     if matrix:
         return w, ids, ref.route_scale_matrix(w, ids, logits.shape[1])
     return w, ids
@@ -1107,25 +1110,30 @@ def residual_tanh_norm(x, y, mult, alpha, weight, bias, out_dtype, xa=None):
 
 
 def latent_prepare(cq, ckv, q_norm_w, kv_norm_w, eps, positions, inv_freq,
-                   cache, slot_mapping):
+                   cache, slot_mapping, interleaved=True, rot_mag=1.0):
     """Latent attention's row work before the up-projections
     (ref.latent_prepare): returns the normed query latent and writes the
     normed key/value latent with the turned shared key part to its page."""
     if cq.is_cuda:
         out = torch.empty(cq.shape, dtype=cq.dtype, device=cq.device)
         _native_seq().latent_prepare(out, cq, ckv, q_norm_w, kv_norm_w, eps,
-                                     positions, inv_freq, cache, slot_mapping)
+                                     positions, inv_freq, cache, slot_mapping,
+                                     bool(interleaved), float(rot_mag))
         return out
     return ref.latent_prepare(cq, ckv, q_norm_w, kv_norm_w, eps, positions,
-                              inv_freq, cache, slot_mapping)
+                              inv_freq, cache, slot_mapping, interleaved,
+                              rot_mag)
 
 
-def latent_query(q, q_abs, positions, inv_freq, out):
+def latent_query(q, q_abs, positions, inv_freq, out, interleaved=True,
+                 rot_mag=1.0):
     """out [T, H, Rk + 2P] = [q_abs ([H, T, Rk]) | turned last 2P dims of q]."""
     if q.is_cuda:
-        _native_seq().latent_query(out, q, q_abs, positions, inv_freq)
+        _native_seq().latent_query(out, q, q_abs, positions, inv_freq,
+                                   bool(interleaved), float(rot_mag))
         return out
-    return ref.latent_query(q, q_abs, positions, inv_freq, out)
+    return ref.latent_query(q, q_abs, positions, inv_freq, out, interleaved,
+                            rot_mag)
 
 
 # rows per chunk of mamba2's chunk-parallel prefill: a chunk's state
@@ -1234,13 +1242,69 @@ def diff_head_norm_gate(a, gate, lam, eps, mult, heads, kv_heads, out):
                                    out)
 
 
-def moe_glu_scaled(gu, scale, experts, ff, shared_ff):
+def moe_glu_scaled(gu, scale, experts, ff, shared_ff, scale_input=True):
     """Activated rows of all experts side by side, each expert's gate and
-    up scaled by the row's weight for it, plus the shared expert's
-    (ref.moe_glu_scaled)."""
+    up (or, without scale_input, their activated product) scaled by the
+    row's weight for it, plus the shared expert's (ref.moe_glu_scaled)."""
     if gu.is_cuda:
         out = torch.empty((gu.shape[0], experts * ff + shared_ff),
                           dtype=gu.dtype, device=gu.device)
-        _native_seq().moe_glu_scaled(out, gu, scale, experts, ff, shared_ff)
+        _native_seq().moe_glu_scaled(out, gu, scale, experts, ff, shared_ff,
+                                     bool(scale_input))
         return out
-    return ref.moe_glu_scaled(gu, scale, experts, ff, shared_ff)
+    return ref.moe_glu_scaled(gu, scale, experts, ff, shared_ff, scale_input)
+
+
+# ----------------------------------------------------------------------
+# Sandwich-norm blocks, per-head output gate, capped logits, channel-decay
+# delta rule (same extension, same rule).
+# ----------------------------------------------------------------------
+def residual_sandwich_norm(x, y, w_post, mult, w_pre, eps, out_dtype):
+    """x (fp32 residual, in place) += mult * rms_norm(y) * w_post when y is
+    given; returns rms_norm(x) * w_pre in out_dtype (None without w_pre):
+    the norm behind one sublayer, the sum and the norm in front of the next
+    from one pass."""
+    if x.is_cuda:
+        h = (torch.empty(x.shape, dtype=out_dtype, device=x.device)
+             if w_pre is not None else None)
+        _native_seq().residual_sandwich_norm(x, h, y, w_post, float(mult),
+                                             w_pre, float(eps))
+        return h
+    return ref.residual_sandwich_norm(x, y, w_post, mult, w_pre, eps, out_dtype)
+
+
+def softcap_(x, cap):
+    """x (fp32, in place) = cap * tanh(x / cap)."""
+    if x.is_cuda:
+        _native_seq().softcap(x, float(cap))
+        return x
+    return ref.softcap_(x, cap)
+
+
+def head_gate(o, gate, out, out_scale=1.0):
+    """out[t, h] = o[t, h] * sigmoid(gate[t, h]) * out_scale
+    (ref.head_gate); o and out [T, H, V] views with dense last dims."""
+    if o.is_cuda:
+        _native_seq().head_gate(out, o, gate, float(out_scale))
+        return out
+    return ref.head_gate(o, gate, out, out_scale)
+
+
+DELTA_CHUNK = 64  # rows per chunk of the matrix-core delta rule
+use_delta_mfma = True  # tests switch it off to compare both paths
+
+
+def channel_delta(u, decay, beta, gate, rate, dt_bias, norm_w, eps, state,
+                  cu_seqlens, seq_lens, state_slots, heads, kv_heads, dim,
+                  vdim, out, max_q_len=0, chunks=None):
+    """Delta rule with a decay per key channel and its gated unit-RMS
+    read-out (ref.channel_delta) into out [T, H*V] (rows may be strided)."""
+    if u.is_cuda:
+        _native_seq().channel_delta_scan(
+            out, u, decay, beta, gate, rate, dt_bias, norm_w, float(eps),
+            ref.DELTA_UNIT_EPS, state, cu_seqlens, seq_lens, state_slots,
+            heads, kv_heads, dim, vdim)
+        return out
+    return ref.channel_delta(u, decay, beta, gate, rate, dt_bias, norm_w, eps,
+                             state, cu_seqlens, seq_lens, state_slots, heads,
+                             kv_heads, dim, vdim, out)

@@ -56,6 +56,8 @@ SEQ_SOURCES = [
     os.path.join(CSRC, "seq_mamba2.hip"),
     os.path.join(CSRC, "seq_masked_mfma.hip"),
     os.path.join(CSRC, "seq_dual.hip"),
+    os.path.join(CSRC, "seq_sandwich.hip"),
+    os.path.join(CSRC, "seq_delta.hip"),
 ]
 
 EXTENSIONS = {EXT_NAME: SOURCES, SEQ_EXT_NAME: SEQ_SOURCES}

@@ -52,7 +52,7 @@ int arks_seq_causal_conv_silu(void* out, const void* x, int64_t ldx,
                               void* state,
                               const void* cu, const void* seq_lens,
                               const void* slots, const void* token_seq, int T,
-                              int S, int C, int taps, int act_f32,
+                              int S, int C, int taps, int single, int act_f32,
                               hipStream_t stream);
 int arks_seq_selective_scan(void* out, const void* u, const void* dbc,
                             int64_t ldd, const void* z, int64_t ldz,
@@ -128,11 +128,12 @@ void arks_seq_latent_prepare(void* cqn, const void* cq, int64_t ldq,
                              const void* kw, float eps, const void* positions,
                              const void* freq, void* cache,
                              const void* slot_mapping, int T, int Rq, int Rk,
-                             int P, int act_f32, hipStream_t stream);
+                             int P, int half_split, float mag, int act_f32,
+                             hipStream_t stream);
 void arks_seq_latent_query(void* out, const void* q, const void* q_abs,
                            const void* positions, const void* freq, int T,
-                           int H, int D, int Rk, int P, int act_f32,
-                           hipStream_t stream);
+                           int H, int D, int Rk, int P, int half_split,
+                           float mag, int act_f32, hipStream_t stream);
 int arks_seq_mamba2_scan(void* out, const void* xbc, int64_t ldx,
                          const void* dt_raw, int64_t ldd, const void* dt_bias,
                          const void* rate, const void* Dp, void* state,
@@ -164,7 +165,7 @@ int arks_seq_attn_masked_ksplit(int T, int H, int G, int max_blocks);
 int arks_seq_moe_route_grouped(void* weights, void* ids, const void* logits,
                                int T, int E, int top, int groups, int keep,
                                int sigmoid, int renorm, void* matrix,
-                               hipStream_t stream);
+                               const void* bias, hipStream_t stream);
 void arks_seq_moe_mix_rows(void* out, const void* y, const void* weights,
                            const void* rows, int T, int H, int k, int dense,
                            const void* add, int act_f32, hipStream_t stream);
@@ -189,7 +190,24 @@ int arks_seq_diff_head_norm_gate(void* out, int64_t ldo, const void* a,
                                  int V, int act_f32, hipStream_t stream);
 void arks_seq_moe_glu_scaled(void* out, const void* gu, int64_t ldg,
                              const void* scale, int64_t T, int E, int ff,
-                             int sff, int act_f32, hipStream_t stream);
+                             int sff, int scale_in, int act_f32,
+                             hipStream_t stream);
+void arks_seq_residual_sandwich_norm(void* x, void* h, const void* y,
+                                     const void* w_post, float mult,
+                                     const void* w_pre, float eps, int64_t T,
+                                     int C, int act_f32, hipStream_t stream);
+void arks_seq_softcap(void* x, int64_t n, float cap, hipStream_t stream);
+void arks_seq_head_gate(void* out, int64_t lot, int64_t loh, const void* o,
+                        int64_t lit, int64_t lih, const void* gate,
+                        int64_t ldg, float out_scale, int64_t T, int H, int V,
+                        int act_f32, hipStream_t stream);
+int arks_seq_channel_delta_scan(
+    void* out, int64_t ldo, const void* u, int64_t ldu, const void* decay,
+    int64_t lda, const void* beta, int64_t ldb, const void* gate, int64_t ldg,
+    int gate_f32, const void* rate, const void* dt_bias, const void* norm_w,
+    float eps, float unit_eps, void* state, const void* cu,
+    const void* seq_lens, const void* slots, int S, int H, int G, int D, int V,
+    int act_f32, hipStream_t stream);
 void arks_seq_lightning_combine(void* part, const void* decay, void* state,
                                 const void* chunk_off, const void* chunk_rows,
                                 const void* cu, const void* seq_lens,
@@ -543,15 +561,19 @@ void lightning_scan(Tensor out, Tensor q, Tensor k, Tensor v, Tensor decay,
 }
 
 void causal_conv_silu(Tensor out, Tensor x, Tensor w, OptTensor w_t,
-                      Tensor bias, OptTensor state, Tensor cu, Tensor seq_lens,
-                      Tensor slots, Tensor token_seq) {
+                      OptTensor bias, OptTensor state, Tensor cu,
+                      Tensor seq_lens, Tensor slots, Tensor token_seq,
+                      bool single) {
   const int f32 = act_flag(x, "x");
   const int T = x.size(0), C = x.size(1);
   TORCH_CHECK(out.scalar_type() == x.scalar_type() && out.is_contiguous() &&
               out.sizes() == x.sizes());
   check_f32(w, "conv weight");
-  check_f32(bias, "conv bias");
-  TORCH_CHECK(w.dim() == 2 && w.size(0) == C && bias.numel() == C);
+  TORCH_CHECK(w.dim() == 2 && w.size(0) == C);
+  if (bias.has_value()) {
+    check_f32(*bias, "conv bias");
+    TORCH_CHECK(bias->numel() == C);
+  }
   const int taps = w.size(1);
   const void* wt_p = nullptr;
   if (w_t.has_value()) {  // [taps, C] copy for the vectorised kernel
@@ -570,9 +592,9 @@ void causal_conv_silu(Tensor out, Tensor x, Tensor w, OptTensor w_t,
   const SeqMeta m = check_meta(cu, seq_lens, &slots, &token_seq, T);
   const int rc = arks_seq_causal_conv_silu(
       out.data_ptr(), x.data_ptr(), row_stride(x, "x"), w.data_ptr(), wt_p,
-      bias.data_ptr(), st_p, cu.data_ptr(), seq_lens.data_ptr(),
-      slots.data_ptr(), token_seq.data_ptr(), T, m.S, C, taps, f32,
-      current_stream());
+      bias.has_value() ? bias->data_ptr() : nullptr, st_p, cu.data_ptr(),
+      seq_lens.data_ptr(), slots.data_ptr(), token_seq.data_ptr(), T, m.S, C,
+      taps, single && T == m.S ? 1 : 0, f32, current_stream());
   TORCH_CHECK(rc == 0, "conv taps beyond the kernel's limit (", taps, ")");
 }
 
@@ -923,7 +945,7 @@ bool attention_window_pool_mfma(Tensor out, Tensor q, Tensor k_cache,
 
 void moe_route_grouped(Tensor weights, Tensor ids, Tensor logits, int64_t top,
                        int64_t groups, int64_t keep, bool sigmoid, bool renorm,
-                       OptTensor matrix) {
+                       OptTensor matrix, OptTensor bias) {
   check_f32(logits, "router logits");
   check_f32(weights, "weights");
   check_i32(ids, "ids");
@@ -937,10 +959,14 @@ void moe_route_grouped(Tensor weights, Tensor ids, Tensor logits, int64_t top,
                 matrix->size(1) == E);
     mat_p = matrix->data_ptr();
   }
+  if (bias.has_value()) {
+    check_f32(*bias, "router bias");
+    TORCH_CHECK(bias->numel() == E);
+  }
   const int rc = arks_seq_moe_route_grouped(
       weights.data_ptr(), ids.data_ptr(), logits.data_ptr(), T, E, (int)top,
       (int)groups, (int)keep, sigmoid ? 1 : 0, renorm ? 1 : 0, mat_p,
-      current_stream());
+      bias.has_value() ? bias->data_ptr() : nullptr, current_stream());
   TORCH_CHECK(rc == 0, "routing sizes the kernel does not hold");
 }
 
@@ -1097,7 +1123,7 @@ void diff_head_norm_gate(Tensor out, Tensor a, Tensor gate, double lam,
 }
 
 void moe_glu_scaled(Tensor out, Tensor gu, Tensor scale, int64_t experts,
-                    int64_t ff, int64_t shared_ff) {
+                    int64_t ff, int64_t shared_ff, bool scale_input) {
   const int f32 = act_flag(gu, "gate|up");
   check_f32(scale, "scale");
   const int64_t T = gu.size(0);
@@ -1110,8 +1136,8 @@ void moe_glu_scaled(Tensor out, Tensor gu, Tensor scale, int64_t experts,
               out.size(1) == experts * ff + shared_ff);
   arks_seq_moe_glu_scaled(out.data_ptr(), gu.data_ptr(),
                           row_stride(gu, "gate|up"), scale.data_ptr(), T,
-                          (int)experts, (int)ff, (int)shared_ff, f32,
-                          current_stream());
+                          (int)experts, (int)ff, (int)shared_ff,
+                          scale_input ? 1 : 0, f32, current_stream());
 }
 
 }  // namespace
@@ -1165,7 +1191,7 @@ void residual_tanh_norm(Tensor x, OptTensor h, OptTensor xa, OptTensor y,
 
 void latent_prepare(Tensor cqn, Tensor cq, Tensor ckv, Tensor qw, Tensor kw,
                     double eps, Tensor positions, Tensor freq, Tensor cache,
-                    Tensor slot_mapping) {
+                    Tensor slot_mapping, bool interleaved, double rot_mag) {
   const int f32 = act_flag(cq, "cq");
   const int T = cq.size(0), Rq = cq.size(1);
   check_f32(qw, "q norm");
@@ -1186,12 +1212,13 @@ void latent_prepare(Tensor cqn, Tensor cq, Tensor ckv, Tensor qw, Tensor kw,
                           ckv.data_ptr(), row_stride(ckv, "ckv"), qw.data_ptr(),
                           kw.data_ptr(), (float)eps, positions.data_ptr(),
                           freq.data_ptr(), cache.data_ptr(),
-                          slot_mapping.data_ptr(), T, Rq, Rk, P, f32,
+                          slot_mapping.data_ptr(), T, Rq, Rk, P,
+                          interleaved ? 0 : 1, (float)rot_mag, f32,
                           current_stream());
 }
 
 void latent_query(Tensor out, Tensor q, OptTensor q_abs, Tensor positions,
-                  Tensor freq) {
+                  Tensor freq, bool interleaved, double rot_mag) {
   const int f32 = act_flag(q, "q");
   check_f32(freq, "inv_freq");
   check_i64(positions, "positions");
@@ -1210,7 +1237,8 @@ void latent_query(Tensor out, Tensor q, OptTensor q_abs, Tensor positions,
   arks_seq_latent_query(out.data_ptr(), q.data_ptr(),
                         q_abs.has_value() ? q_abs->data_ptr() : nullptr,
                         positions.data_ptr(), freq.data_ptr(), T, H, D, Rk, P,
-                        f32, current_stream());
+                        interleaved ? 0 : 1, (float)rot_mag, f32,
+                        current_stream());
 }
 
 void mamba2_scan(OptTensor out, Tensor xbc, Tensor dt_raw, Tensor dt_bias,
@@ -1345,8 +1373,133 @@ bool attention_masked_mfma(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache,
              ksplit, (int)maps, current_stream()) == 0;
 }
 
+void residual_sandwich_norm(Tensor x, OptTensor h, OptTensor y,
+                            OptTensor w_post, double mult, OptTensor w_pre,
+                            double eps) {
+  check_f32(x, "x");
+  TORCH_CHECK(x.dim() == 2);
+  const int64_t T = x.size(0);
+  const int C = x.size(1);
+  int f32 = -1;
+  auto row_tensor = [&](const OptTensor& t, const char* name) -> void* {
+    if (!t.has_value()) return nullptr;
+    const int f = act_flag(*t, name);
+    TORCH_CHECK(f32 < 0 || f == f32, "activation dtypes differ");
+    f32 = f;
+    TORCH_CHECK(t->is_contiguous() && t->sizes() == x.sizes(), name,
+                " must be a contiguous [T, C] tensor");
+    return t->data_ptr();
+  };
+  auto weight = [&](const OptTensor& t, const char* name) -> const void* {
+    if (!t.has_value()) return nullptr;
+    check_f32(*t, name);
+    TORCH_CHECK(t->numel() == C);
+    return t->data_ptr();
+  };
+  void* h_p = row_tensor(h, "h");
+  const void* y_p = row_tensor(y, "y");
+  const void* wpo = weight(w_post, "w_post");
+  const void* wpr = weight(w_pre, "w_pre");
+  TORCH_CHECK((y_p != nullptr) <= (wpo != nullptr) &&
+              (h_p != nullptr) == (wpr != nullptr));
+  arks_seq_residual_sandwich_norm(x.data_ptr(), h_p, y_p, wpo, (float)mult,
+                                  wpr, (float)eps, T, C, f32 == 1 ? 1 : 0,
+                                  current_stream());
+}
+
+void softcap(Tensor x, double cap) {
+  check_f32(x, "x");
+  TORCH_CHECK(cap > 0);
+  arks_seq_softcap(x.data_ptr(), x.numel(), (float)cap, current_stream());
+}
+
+void head_gate(Tensor out, Tensor o, OptTensor gate, double out_scale) {
+  const int f32 = act_flag(o, "o");
+  TORCH_CHECK(o.dim() == 3 && out.dim() == 3 && o.sizes() == out.sizes() &&
+              o.stride(2) == 1 && out.stride(2) == 1 &&
+              out.scalar_type() == o.scalar_type(),
+              "head_gate takes [T, H, V] views with dense last dims");
+  const int64_t T = o.size(0);
+  const int H = o.size(1), V = o.size(2);
+  const void* g_p = nullptr;
+  int64_t ldg = 0;
+  if (gate.has_value()) {
+    TORCH_CHECK(gate->scalar_type() == o.scalar_type() && gate->size(0) == T &&
+                gate->size(1) == H);
+    g_p = gate->data_ptr();
+    ldg = row_stride(*gate, "gate");
+  }
+  arks_seq_head_gate(out.data_ptr(), out.stride(0), out.stride(1), o.data_ptr(),
+                     o.stride(0), o.stride(1), g_p, ldg, (float)out_scale, T,
+                     H, V, f32, current_stream());
+}
+
+// The operands every form of the channel-decay delta rule takes, checked.
+struct DeltaArgs {
+  int f32, gate_f32;
+  int64_t ldo, ldu, lda, ldb, ldg;
+};
+
+DeltaArgs check_delta(const Tensor& out, const Tensor& u, const Tensor& decay,
+                      const Tensor& beta, const Tensor& gate,
+                      const Tensor& rate, const Tensor& dt_bias,
+                      const Tensor& norm_w, const Tensor& state, int64_t H,
+                      int64_t G, int64_t D, int64_t V) {
+  DeltaArgs a;
+  a.f32 = act_flag(u, "u");
+  const int64_t T = u.size(0);
+  TORCH_CHECK(G >= 1 && H % G == 0 && D >= 1 && V >= 1);
+  TORCH_CHECK(u.dim() == 2 && u.size(1) == 2 * G * D + H * V);
+  TORCH_CHECK(decay.is_cuda() && decay.scalar_type() == torch::kFloat32 &&
+              decay.dim() == 2 && decay.size(0) == T && decay.size(1) == H * D);
+  TORCH_CHECK(beta.scalar_type() == u.scalar_type() && beta.dim() == 2 &&
+              beta.size(0) == T && beta.size(1) == H);
+  a.gate_f32 = act_flag(gate, "gate");
+  TORCH_CHECK((a.gate_f32 || !a.f32) && gate.dim() == 2 && gate.size(0) == T &&
+              gate.size(1) == H * V);
+  TORCH_CHECK(out.scalar_type() == u.scalar_type() && out.dim() == 2 &&
+              out.size(0) == T && out.size(1) == H * V);
+  check_f32(rate, "rate");
+  check_f32(dt_bias, "dt_bias");
+  check_f32(norm_w, "norm weight");
+  check_f32(state, "state");
+  TORCH_CHECK(rate.numel() == H && dt_bias.numel() == H * D &&
+              norm_w.numel() == V);
+  TORCH_CHECK(state.dim() == 4 && state.size(1) == H && state.size(2) == D &&
+              state.size(3) == V);
+  a.ldo = row_stride(out, "out");
+  a.ldu = row_stride(u, "u");
+  a.lda = row_stride(decay, "decay");
+  a.ldb = row_stride(beta, "beta");
+  a.ldg = row_stride(gate, "gate");
+  return a;
+}
+
+void channel_delta_scan(Tensor out, Tensor u, Tensor decay, Tensor beta,
+                        Tensor gate, Tensor rate, Tensor dt_bias,
+                        Tensor norm_w, double eps, double unit_eps,
+                        Tensor state, Tensor cu, Tensor seq_lens, Tensor slots,
+                        int64_t H, int64_t G, int64_t D, int64_t V) {
+  const DeltaArgs a = check_delta(out, u, decay, beta, gate, rate, dt_bias,
+                                  norm_w, state, H, G, D, V);
+  const SeqMeta m = check_meta(cu, seq_lens, &slots, nullptr, 0);
+  const int rc = arks_seq_channel_delta_scan(
+      out.data_ptr(), a.ldo, u.data_ptr(), a.ldu, decay.data_ptr(), a.lda,
+      beta.data_ptr(), a.ldb, gate.data_ptr(), a.ldg, a.gate_f32,
+      rate.data_ptr(), dt_bias.data_ptr(), norm_w.data_ptr(), (float)eps,
+      (float)unit_eps, state.data_ptr(), cu.data_ptr(), seq_lens.data_ptr(),
+      slots.data_ptr(), m.S, (int)H, (int)G, (int)D, (int)V, a.f32,
+      current_stream());
+  TORCH_CHECK(rc == 0, "delta-rule head sizes the kernel does not hold (", D,
+              ", ", V, ")");
+}
+
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("residual_tanh_norm", &residual_tanh_norm);
+  m.def("residual_sandwich_norm", &residual_sandwich_norm);
+  m.def("softcap", &softcap);
+  m.def("head_gate", &head_gate);
+  m.def("channel_delta_scan", &channel_delta_scan);
   m.def("latent_prepare", &latent_prepare);
   m.def("latent_query", &latent_query);
   m.def("mamba2_scan", &mamba2_scan);

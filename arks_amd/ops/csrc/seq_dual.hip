@@ -1,6 +1,6 @@
 // Row kernels of the two-norm parallel block and of difference attention
 // (arks_amd/models/hybrid.py DualNormBlock, models/mixers.py DiffAttention,
-// models/feedforward.py InputScaledMoE), bf16 or float rows, fp32
+// models/feedforward.py RoutedMoE), bf16 or float rows, fp32
 // arithmetic:
 //
 //   residual_pair_norm   x += s1 * y1 + s2 * y2 (per-channel s, each branch
@@ -16,9 +16,9 @@
 //       reader of the first sees the old ones)
 //   diff_head_norm_gate  (a1 - lambda a2) / rms * mult * sigmoid(gate) per
 //       head from the two maps' attention outputs
-//   moe_glu_scaled       silu(s g) * (s u) for every expert's [gate | up]
-//       columns with the row's factor for that expert, silu(g) * u for the
-//       shared expert's
+//   moe_glu_scaled       silu(s g) * (s u), or s * silu(g) * u, for every
+//       expert's [gate | up] columns with the row's factor for that expert,
+//       silu(g) * u for the shared expert's
 #include "seq_common.h"
 
 namespace arks {
@@ -441,7 +441,8 @@ __global__ __launch_bounds__(256) void diff_head_norm_gate_vec8_kernel(
 template <typename AT>
 __global__ __launch_bounds__(256) void moe_glu_scaled_kernel(
     AT* __restrict__ out, const AT* __restrict__ gu, int64_t ldg,
-    const float* __restrict__ scale, int64_t total, int E, int ff, int sff) {
+    const float* __restrict__ scale, int64_t total, int E, int ff, int sff,
+    int scale_in) {
   const int64_t idx = (int64_t)blockIdx.x * 256 + threadIdx.x;
   if (idx >= total) return;
   const int F = E * ff + sff;
@@ -456,7 +457,8 @@ __global__ __launch_bounds__(256) void moe_glu_scaled_kernel(
       Act<AT>::st(out + idx, 0.f);
       return;
     }
-    g = s * Act<AT>::ld(row + (int64_t)e * 2 * ff + i);
+    g = Act<AT>::ld(row + (int64_t)e * 2 * ff + i);
+    if (scale_in) g *= s;
     u = s * Act<AT>::ld(row + (int64_t)e * 2 * ff + ff + i);
   } else {
     const int i = c - E * ff;
@@ -469,7 +471,8 @@ __global__ __launch_bounds__(256) void moe_glu_scaled_kernel(
 // bf16, 8 columns per thread (ff and sff multiples of 8)
 __global__ __launch_bounds__(256) void moe_glu_scaled_vec8_kernel(
     bf16* __restrict__ out, const bf16* __restrict__ gu, int64_t ldg,
-    const float* __restrict__ scale, int64_t total8, int E, int ff, int sff) {
+    const float* __restrict__ scale, int64_t total8, int E, int ff, int sff,
+    int scale_in) {
   const int64_t idx = (int64_t)blockIdx.x * 256 + threadIdx.x;
   if (idx >= total8) return;
   const int F = E * ff + sff;
@@ -496,9 +499,10 @@ __global__ __launch_bounds__(256) void moe_glu_scaled_vec8_kernel(
   } else {
     const ushort8 gv = *reinterpret_cast<const ushort8*>(gp);
     const ushort8 uv = *reinterpret_cast<const ushort8*>(up);
+    const float sg = scale_in ? s : 1.f;
 #pragma unroll
     for (int e = 0; e < 8; ++e) {
-      const float g = s * bf16_bits_to_float(gv[e]);
+      const float g = sg * bf16_bits_to_float(gv[e]);
       const float u = s * bf16_bits_to_float(uv[e]);
       o[e] = float_to_bf16_bits(g / (1.f + __expf(-g)) * u);
     }
@@ -611,8 +615,8 @@ extern "C" int arks_seq_diff_head_norm_gate(
 
 extern "C" void arks_seq_moe_glu_scaled(void* out, const void* gu, int64_t ldg,
                                         const void* scale, int64_t T, int E,
-                                        int ff, int sff, int act_f32,
-                                        hipStream_t stream) {
+                                        int ff, int sff, int scale_in,
+                                        int act_f32, hipStream_t stream) {
   if (T == 0) return;
   const int64_t total = T * ((int64_t)E * ff + sff);
   if (!act_f32 && ff % 8 == 0 && sff % 8 == 0 && ldg % 8 == 0 &&
@@ -621,11 +625,11 @@ extern "C" void arks_seq_moe_glu_scaled(void* out, const void* gu, int64_t ldg,
     hipLaunchKernelGGL(moe_glu_scaled_vec8_kernel,
                        dim3((unsigned)((total8 + 255) / 256)), dim3(256), 0,
                        stream, (bf16*)out, (const bf16*)gu, ldg,
-                       (const float*)scale, total8, E, ff, sff);
+                       (const float*)scale, total8, E, ff, sff, scale_in);
     return;
   }
   SEQ_DISPATCH_ACT(act_f32, hipLaunchKernelGGL(
       (moe_glu_scaled_kernel<AT>), dim3((unsigned)((total + 255) / 256)),
       dim3(256), 0, stream, (AT*)out, (const AT*)gu, ldg, (const float*)scale,
-      total, E, ff, sff));
+      total, E, ff, sff, scale_in));
 }

@@ -8,26 +8,29 @@
 
 namespace arks {
 
-constexpr int CONV_MAX_HIST = 8;  // taps - 1
+constexpr int CONV_MAX_HIST = 31;     // taps - 1, general kernels
+constexpr int CONV_VEC_MAX_TAPS = 9;  // taps the vectorised kernel holds
 
 // One block per row, threads over channels. Inputs before the step's first
-// row come from the sequence's stored history (zeros at position 0). The
-// history is replaced by conv_state_update_kernel in a later launch, so
-// every reader here sees the old one.
+// row come from the sequence's stored history (zeros at position 0). bias
+// may be null. The history is replaced by conv_state_update_kernel in a
+// later launch, so every reader here sees the old one; in a step that brings
+// one row per sequence (single) the thread that reads a channel's history is
+// its only reader, and replaces it itself.
 template <typename AT>
 __global__ __launch_bounds__(256) void causal_conv_silu_kernel(
     AT* __restrict__ out, const AT* __restrict__ x, int64_t ldx,
     const float* __restrict__ w, const float* __restrict__ bias,
-    const float* __restrict__ state, const int* __restrict__ cu,
+    float* __restrict__ state, const int* __restrict__ cu,
     const int* __restrict__ seq_lens, const int* __restrict__ slots,
-    const int* __restrict__ token_seq, int C, int taps) {
+    const int* __restrict__ token_seq, int C, int taps, int single) {
   const int t = blockIdx.x;
   const SeqRow r = seq_row(t, token_seq, cu, seq_lens, slots);
   const int i = t - r.first_row;
   const bool has_state = r.start > 0 && r.slot >= 0;
-  const float* hist = state + (int64_t)(r.slot < 0 ? 0 : r.slot) * (taps - 1) * C;
+  float* hist = state + (int64_t)(r.slot < 0 ? 0 : r.slot) * (taps - 1) * C;
   for (int c = blockIdx.y * 256 + threadIdx.x; c < C; c += gridDim.y * 256) {
-    float acc = bias[c];
+    float acc = bias ? bias[c] : 0.f;
     for (int j = 0; j < taps; ++j) {
       const int src = i - (taps - 1 - j);
       float xv;
@@ -36,28 +39,35 @@ __global__ __launch_bounds__(256) void causal_conv_silu_kernel(
       else
         xv = has_state ? hist[(int64_t)(src + taps - 1) * C + c] : 0.f;
       acc += w[(int64_t)c * taps + j] * xv;
+      // one row a sequence: entry j of the history has been used, and its
+      // successor becomes the new entry j - 1
+      if (single && r.slot >= 0 && j > 0) hist[(int64_t)(j - 1) * C + c] = xv;
     }
     Act<AT>::st(out + (int64_t)t * C + c, silu_f(acc));
   }
 }
 
-// bf16 rows, 8 channels per thread and CONV_RPT consecutive rows per block:
-// 16-byte loads of each tap's row, the conv taps of the thread's channels
+// bf16 rows, 8 channels per thread and rpt consecutive rows per block
+// (CONV_RPT in long steps, fewer in short ones so that the launch still fills
+// the chip): 16-byte loads of each tap's row, the conv taps of the thread's channels
 // held in registers across the rows (w_t [taps, C] is a transposed copy of
 // the weights so that they load as two float4 per tap).
 constexpr int CONV_RPT = 8;
-constexpr int CONV_MAX_TAPS = CONV_MAX_HIST + 1;
+constexpr int CONV_MAX_TAPS = CONV_VEC_MAX_TAPS;
 
 __global__ __launch_bounds__(256) void causal_conv_silu_vec8_kernel(
     bf16* __restrict__ out, const bf16* __restrict__ x, int64_t ldx,
     const float* __restrict__ w_t, const float* __restrict__ bias,
-    const float* __restrict__ state, const int* __restrict__ cu,
+    float* __restrict__ state, const int* __restrict__ cu,
     const int* __restrict__ seq_lens, const int* __restrict__ slots,
-    const int* __restrict__ token_seq, int T, int C, int taps) {
+    const int* __restrict__ token_seq, int T, int C, int taps, int rpt,
+    int single) {
   const int c = (blockIdx.y * 256 + threadIdx.x) * 8;
   if (c >= C) return;
   float wv[CONV_MAX_TAPS][8], bv[8];
-  {
+#pragma unroll
+  for (int e = 0; e < 8; ++e) bv[e] = 0.f;
+  if (bias) {
     const float4v b0 = *reinterpret_cast<const float4v*>(bias + c);
     const float4v b1 = *reinterpret_cast<const float4v*>(bias + c + 4);
 #pragma unroll
@@ -72,12 +82,12 @@ __global__ __launch_bounds__(256) void causal_conv_silu_vec8_kernel(
       for (int e = 0; e < 4; ++e) { wv[j][e] = w0[e]; wv[j][4 + e] = w1[e]; }
     }
   }
-  const int t_end = min(T, (int)(blockIdx.x + 1) * CONV_RPT);
-  for (int t = blockIdx.x * CONV_RPT; t < t_end; ++t) {
+  const int t_end = min(T, (int)(blockIdx.x + 1) * rpt);
+  for (int t = blockIdx.x * rpt; t < t_end; ++t) {
     const SeqRow r = seq_row(t, token_seq, cu, seq_lens, slots);
     const int i = t - r.first_row;
     const bool has_state = r.start > 0 && r.slot >= 0;
-    const float* hist =
+    float* hist =
         state + (int64_t)(r.slot < 0 ? 0 : r.slot) * (taps - 1) * C;
     float acc[8];
 #pragma unroll
@@ -105,6 +115,16 @@ __global__ __launch_bounds__(256) void causal_conv_silu_vec8_kernel(
         if (have) {
 #pragma unroll
           for (int e = 0; e < 8; ++e) acc[e] += wv[j][e] * xv[e];
+        }
+        if (single && r.slot >= 0 && j > 0) {
+          float4v h0 = {0.f, 0.f, 0.f, 0.f}, h1 = {0.f, 0.f, 0.f, 0.f};
+          if (have) {
+#pragma unroll
+            for (int e = 0; e < 4; ++e) { h0[e] = xv[e]; h1[e] = xv[4 + e]; }
+          }
+          float* hp = hist + (int64_t)(j - 1) * C + c;
+          *reinterpret_cast<float4v*>(hp) = h0;
+          *reinterpret_cast<float4v*>(hp + 4) = h1;
         }
       }
     }
@@ -346,29 +366,30 @@ extern "C" int arks_seq_causal_conv_silu(
     void* out, const void* x, int64_t ldx, const void* w, const void* w_t,
     const void* bias, void* state, const void* cu, const void* seq_lens,
     const void* slots, const void* token_seq, int T, int S, int C, int taps,
-    int act_f32, hipStream_t stream) {
+    int single, int act_f32, hipStream_t stream) {
   if (taps - 1 > CONV_MAX_HIST || taps < 1) return 1;
   if (T == 0) return 0;
   const int cb = (C + 255) / 256;
   const bool vec8 = !act_f32 && w_t && C % 8 == 0 && ldx % 8 == 0 &&
-                    ((uintptr_t)x % 16) == 0;
+                    taps <= CONV_VEC_MAX_TAPS && ((uintptr_t)x % 16) == 0;
+  const int vb = (C / 8 + 255) / 256;
+  int rpt = CONV_RPT;
+  while (rpt > 1 && (int64_t)((T + rpt - 1) / rpt) * vb < 1024) rpt /= 2;
   SEQ_DISPATCH_ACT(act_f32, {
     if (vec8)
       hipLaunchKernelGGL(causal_conv_silu_vec8_kernel,
-                         dim3((T + CONV_RPT - 1) / CONV_RPT,
-                              (C / 8 + 255) / 256),
-                         dim3(256), 0, stream, (bf16*)out, (const bf16*)x, ldx,
-                         (const float*)w_t, (const float*)bias,
-                         (const float*)state, (const int*)cu,
+                         dim3((T + rpt - 1) / rpt, vb), dim3(256), 0, stream,
+                         (bf16*)out, (const bf16*)x, ldx, (const float*)w_t,
+                         (const float*)bias, (float*)state, (const int*)cu,
                          (const int*)seq_lens, (const int*)slots,
-                         (const int*)token_seq, T, C, taps);
+                         (const int*)token_seq, T, C, taps, rpt, single);
     else
     hipLaunchKernelGGL((causal_conv_silu_kernel<AT>), dim3(T, cb), dim3(256), 0,
                        stream, (AT*)out, (const AT*)x, ldx, (const float*)w,
-                       (const float*)bias, (const float*)state, (const int*)cu,
+                       (const float*)bias, (float*)state, (const int*)cu,
                        (const int*)seq_lens, (const int*)slots,
-                       (const int*)token_seq, C, taps);
-    if (taps > 1)
+                       (const int*)token_seq, C, taps, single);
+    if (taps > 1 && !single)
       hipLaunchKernelGGL((conv_state_update_kernel<AT>), dim3(S, cb), dim3(256),
                          0, stream, (float*)state, (const AT*)x, ldx,
                          (const int*)cu, (const int*)seq_lens,

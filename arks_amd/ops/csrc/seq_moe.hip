@@ -2,7 +2,7 @@
 // feed-forward (arks_amd/models/feedforward.py GroupedMoE), bf16 or float
 // rows.
 //
-//   moe_route_grouped  scores over all E experts in fp32, their softmax or
+//   moe_route_grouped  scores over all E experts (logits + bias) in fp32, their softmax or
 //       (sigmoid) each logit's own sigmoid; experts are cut into
 //       `groups` contiguous runs of E/groups, a run's score is its highest
 //       expert score and only the `keep` highest-scoring runs stay eligible; the `top`
@@ -25,20 +25,23 @@ constexpr int ROUTE_MAX_K = 32;
 __global__ __launch_bounds__(64) void moe_route_grouped_kernel(
     float* __restrict__ weights, int* __restrict__ ids,
     const float* __restrict__ logits, int E, int top, int groups, int keep,
-    int sigmoid, int renorm, float* __restrict__ matrix) {
+    int sigmoid, int renorm, float* __restrict__ matrix,
+    const float* __restrict__ bias) {
   __shared__ float s_s[ROUTE_MAX_E];
   __shared__ float g_s[ROUTE_MAX_E];  // group scores (groups <= E)
   const int t = blockIdx.x, lane = threadIdx.x;
   const float* row = logits + (int64_t)t * E;
   if (sigmoid) {
-    for (int e = lane; e < E; e += 64) s_s[e] = sigmoid_f(row[e]);
+    for (int e = lane; e < E; e += 64)
+      s_s[e] = sigmoid_f(row[e] + (bias ? bias[e] : 0.f));
   } else {
     float m = -FLT_MAX;
-    for (int e = lane; e < E; e += 64) m = fmaxf(m, row[e]);
+    for (int e = lane; e < E; e += 64)
+      m = fmaxf(m, row[e] + (bias ? bias[e] : 0.f));
     m = wave_reduce_max(m);
     float sum = 0.f;
     for (int e = lane; e < E; e += 64) {
-      const float p = expf(row[e] - m);
+      const float p = expf(row[e] + (bias ? bias[e] : 0.f) - m);
       s_s[e] = p;
       sum += p;
     }
@@ -171,14 +174,16 @@ extern "C" int arks_seq_moe_route_grouped(void* weights, void* ids,
                                           const void* logits, int T, int E,
                                           int top, int groups, int keep,
                                           int sigmoid, int renorm,
-                                          void* matrix, hipStream_t stream) {
+                                          void* matrix, const void* bias,
+                                          hipStream_t stream) {
   if (E > ROUTE_MAX_E || top > ROUTE_MAX_K || groups < 1 || E % groups ||
       keep > groups || top > keep * (E / groups))
     return 1;
   if (T == 0) return 0;
   hipLaunchKernelGGL(moe_route_grouped_kernel, dim3(T), dim3(64), 0, stream,
                      (float*)weights, (int*)ids, (const float*)logits, E, top,
-                     groups, keep, sigmoid, renorm, (float*)matrix);
+                     groups, keep, sigmoid, renorm, (float*)matrix,
+                     (const float*)bias);
   return 0;
 }
 

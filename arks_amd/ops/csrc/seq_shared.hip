@@ -92,6 +92,22 @@ __global__ __launch_bounds__(256) void residual_tanh_norm_vec8_kernel(
   }
 }
 
+// Pair i of a rotated part of 2P dims: (2i, 2i + 1), or (i, i + P) half-split;
+// cos and sin times mag.
+template <typename AT>
+__device__ __forceinline__ void turn_pair(AT* dst, const AT* src, int i, int P,
+                                          float angle, int half_split,
+                                          float mag) {
+  float sn, cs;
+  sincosf(angle, &sn, &cs);
+  sn *= mag;
+  cs *= mag;
+  const int i0 = half_split ? i : 2 * i, i1 = half_split ? i + P : 2 * i + 1;
+  const float a = Act<AT>::ld(src + i0), b = Act<AT>::ld(src + i1);
+  Act<AT>::st(dst + i0, a * cs - b * sn);
+  Act<AT>::st(dst + i1, b * cs + a * sn);
+}
+
 // One block per row. cq [T, Rq] (row stride ldq) -> cqn [T, Rq] dense;
 // ckv [T, Rk + 2P] (row stride ldk) -> its cache row.
 template <typename AT>
@@ -101,7 +117,7 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(
     const float* __restrict__ kw, float eps,
     const int64_t* __restrict__ positions, const float* __restrict__ freq,
     AT* __restrict__ cache, const int64_t* __restrict__ slot_mapping, int Rq,
-    int Rk, int P) {
+    int Rk, int P, int half_split, float mag) {
   __shared__ float scratch[4];
   __shared__ float scratch2[4];
   const int t = blockIdx.x;
@@ -129,14 +145,8 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(
   for (int i = threadIdx.x; i < Rk; i += 256)
     Act<AT>::st(dst + i, Act<AT>::ld(kr + i) * rk * kw[i]);
   const float pos = (float)positions[t];
-  for (int i = threadIdx.x; i < P; i += 256) {
-    float sn, cs;
-    sincosf(pos * freq[i], &sn, &cs);
-    const float a = Act<AT>::ld(kr + Rk + 2 * i);
-    const float b = Act<AT>::ld(kr + Rk + 2 * i + 1);
-    Act<AT>::st(dst + Rk + 2 * i, a * cs - b * sn);
-    Act<AT>::st(dst + Rk + 2 * i + 1, b * cs + a * sn);
-  }
+  for (int i = threadIdx.x; i < P; i += 256)
+    turn_pair<AT>(dst + Rk, kr + Rk, i, P, pos * freq[i], half_split, mag);
 }
 
 // out [T, H, Rk + 2P] = [q_abs[h, t, :] | rotated q[t, h, D:]]; one block
@@ -145,7 +155,8 @@ template <typename AT>
 __global__ __launch_bounds__(256) void latent_query_kernel(
     AT* __restrict__ out, const AT* __restrict__ q,
     const AT* __restrict__ q_abs, const int64_t* __restrict__ positions,
-    const float* __restrict__ freq, int T, int H, int D, int Rk, int P) {
+    const float* __restrict__ freq, int T, int H, int D, int Rk, int P,
+    int half_split, float mag) {
   const int t = blockIdx.x;
   const int wave = threadIdx.x / 64, lane = threadIdx.x % 64;
   const float pos = (float)positions[t];
@@ -156,14 +167,8 @@ __global__ __launch_bounds__(256) void latent_query_kernel(
                           : q + ((int64_t)t * H + hh) * (D + 2 * P);
     for (int i = lane; i < Rk; i += 64) dst[i] = src[i];
     const AT* qr = q + ((int64_t)t * H + hh) * (D + 2 * P) + D;
-    for (int i = lane; i < P; i += 64) {
-      float sn, cs;
-      sincosf(pos * freq[i], &sn, &cs);
-      const float a = Act<AT>::ld(qr + 2 * i);
-      const float b = Act<AT>::ld(qr + 2 * i + 1);
-      Act<AT>::st(dst + Rk + 2 * i, a * cs - b * sn);
-      Act<AT>::st(dst + Rk + 2 * i + 1, b * cs + a * sn);
-    }
+    for (int i = lane; i < P; i += 64)
+      turn_pair<AT>(dst + Rk, qr, i, P, pos * freq[i], half_split, mag);
   }
 }
 
@@ -197,23 +202,24 @@ extern "C" void arks_seq_latent_prepare(
     void* cqn, const void* cq, int64_t ldq, const void* ckv, int64_t ldk,
     const void* qw, const void* kw, float eps, const void* positions,
     const void* freq, void* cache, const void* slot_mapping, int T, int Rq,
-    int Rk, int P, int act_f32, hipStream_t stream) {
+    int Rk, int P, int half_split, float mag, int act_f32,
+    hipStream_t stream) {
   if (T == 0) return;
   SEQ_DISPATCH_ACT(act_f32, hipLaunchKernelGGL(
       (latent_prepare_kernel<AT>), dim3(T), dim3(256), 0, stream, (AT*)cqn,
       (const AT*)cq, ldq, (const AT*)ckv, ldk, (const float*)qw,
       (const float*)kw, eps, (const int64_t*)positions, (const float*)freq,
-      (AT*)cache, (const int64_t*)slot_mapping, Rq, Rk, P));
+      (AT*)cache, (const int64_t*)slot_mapping, Rq, Rk, P, half_split, mag));
 }
 
 extern "C" void arks_seq_latent_query(void* out, const void* q,
                                       const void* q_abs, const void* positions,
                                       const void* freq, int T, int H, int D,
-                                      int Rk, int P, int act_f32,
-                                      hipStream_t stream) {
+                                      int Rk, int P, int half_split, float mag,
+                                      int act_f32, hipStream_t stream) {
   if (T == 0) return;
   SEQ_DISPATCH_ACT(act_f32, hipLaunchKernelGGL(
       (latent_query_kernel<AT>), dim3(T), dim3(256), 0, stream, (AT*)out,
       (const AT*)q, (const AT*)q_abs, (const int64_t*)positions,
-      (const float*)freq, T, H, D, Rk, P));
+      (const float*)freq, T, H, D, Rk, P, half_split, mag));
 }

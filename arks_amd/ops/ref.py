@@ -545,7 +545,8 @@ def causal_conv_silu(x, weight, bias, state, cu_seqlens, seq_lens,
                 else torch.zeros(taps - 1, C))
         full = torch.cat([hist, xf[a:b]], 0)  # [taps-1+n, C]
         n = b - a
-        acc = bias.float()[None, :].expand(n, C).clone()
+        acc = (bias.float()[None, :].expand(n, C).clone() if bias is not None
+               else torch.zeros(n, C))
         for j in range(taps):
             acc += full[j:j + n] * weight.float()[:, j][None, :]
         out[a:b] = acc
@@ -782,14 +783,16 @@ def glu_act(gu, kind, limit=0.0, alpha=1.0, row_scale=None):
 
 
 def moe_route_grouped(logits, top, groups, keep, score="softmax",
-                      renorm=True):
-    """Scores over all experts: their softmax, or (score="sigmoid") each
+                      renorm=True, bias=None):
+    """Scores of logits (+ bias [E]) over all experts: their softmax, or (score="sigmoid") each
     logit's own sigmoid; without renorm the chosen scores are the weights as
     they are. Experts are cut into `groups`
     contiguous runs of E/groups, a run's score is its highest expert score
     and only the `keep` highest-scoring runs stay eligible; the `top` largest scores among those, their
     scores divided by their sum (+1e-20). Ties go to the lower index.
     logits [T, E] fp32 -> (weights [T, top] fp32, ids [T, top] int32)."""
+    if bias is not None:
+        logits = logits.float() + bias.float()
     s = (torch.sigmoid(logits.float()) if score == "sigmoid"
          else torch.softmax(logits.float(), -1))
     T, E = s.shape
@@ -825,12 +828,12 @@ def residual_tanh_norm(x, y, mult, alpha, weight, bias, out_dtype, xa=None):
 
 
 def latent_prepare(cq, ckv, q_norm_w, kv_norm_w, eps, positions, inv_freq,
-                   cache, slot_mapping):
+                   cache, slot_mapping, interleaved=True, rot_mag=1.0):
     """Row work of latent attention before its up-projections. cq [T, Rq]:
     RMS norm times q_norm_w, returned in cq.dtype. ckv [T, Rk + 2P]: the
     first Rk columns RMS-normed times kv_norm_w, the last 2P (P =
-    len(inv_freq)) turned by the row's position in interleaved pairs; the
-    row goes to its place in cache [blocks, 1, bs, Rk + 2P]."""
+    len(inv_freq)) turned by the row's position in interleaved or half-split
+    pairs with cos and sin times rot_mag; the row goes to its place in cache [blocks, 1, bs, Rk + 2P]."""
     def unit(t):
         return t * torch.rsqrt(t.pow(2).mean(-1, keepdim=True) + eps)
 
@@ -839,7 +842,7 @@ def latent_prepare(cq, ckv, q_norm_w, kv_norm_w, eps, positions, inv_freq,
     f = ckv.float()
     c = unit(f[:, :rank]) * kv_norm_w.float()
     ang = positions.float()[:, None] * inv_freq.float()[None, :]
-    kr = _rotate_pairs(f[:, rank:], ang, True)
+    kr = _rotate_pairs(f[:, rank:], ang, interleaved) * rot_mag
     row = torch.cat([c, kr], -1).to(cache.dtype)
     bs = cache.shape[2]
     ok = slot_mapping >= 0
@@ -847,15 +850,17 @@ def latent_prepare(cq, ckv, q_norm_w, kv_norm_w, eps, positions, inv_freq,
     return cqn
 
 
-def latent_query(q, q_abs, positions, inv_freq, out):
+def latent_query(q, q_abs, positions, inv_freq, out, interleaved=True,
+                 rot_mag=1.0):
     """out [T, H, Rk + 2P] = [q_abs (given as [H, T, Rk]) | the last 2P
-    dims of q [T, H, D + 2P] turned by the row's position, interleaved].
+    dims of q [T, H, D + 2P] turned by the row's position as latent_prepare].
     q_abs None: the first part is q's own first D dims."""
     D = q.shape[2] - 2 * inv_freq.numel()
     rank = q_abs.shape[2] if q_abs is not None else D
     ang = positions.float()[:, None, None] * inv_freq.float()[None, None, :]
     out[..., :rank] = q_abs.transpose(0, 1) if q_abs is not None else q[..., :D]
-    out[..., rank:] = _rotate_pairs(q[..., D:].float(), ang, True).to(out.dtype)
+    out[..., rank:] = (_rotate_pairs(q[..., D:].float(), ang, interleaved)
+                       * rot_mag).to(out.dtype)
     return out
 
 
@@ -994,16 +999,18 @@ def diff_head_norm_gate(a, gate, lam, eps, mult, heads, kv_heads, out):
     return out
 
 
-def moe_glu_scaled(gu, scale, experts, ff, shared_ff):
+def moe_glu_scaled(gu, scale, experts, ff, shared_ff, scale_input=True):
     """gu [T, experts * 2 ff + 2 shared_ff]: per expert [gate | up], then
     the shared expert's [gate | up]. Column c of expert e becomes
     silu(s g) * (s u) with s = scale[t, e] (fp32; 0 for an expert the row
-    does not use), the shared columns silu(g) * u. -> [T, experts * ff +
-    shared_ff]."""
+    does not use), or s * silu(g) * u without scale_input; the shared columns
+    silu(g) * u. -> [T, experts * ff + shared_ff]."""
     T = gu.shape[0]
     ex = gu[:, :experts * 2 * ff].float().view(T, experts, 2, ff)
     s = scale.float()[:, :, None]
-    g, u = ex[:, :, 0] * s, ex[:, :, 1] * s
+    g, u = ex[:, :, 0], ex[:, :, 1] * s
+    if scale_input:
+        g = g * s
     parts = [(g * torch.sigmoid(g) * u).reshape(T, experts * ff)]
     if shared_ff:
         sh = gu[:, experts * 2 * ff:].float()
@@ -1016,4 +1023,78 @@ def route_scale_matrix(weights, ids, experts):
     """[T, experts] fp32: a row's weight at each expert it uses, 0 elsewhere."""
     out = torch.zeros(weights.shape[0], experts, dtype=torch.float32)
     out.scatter_(1, ids.long(), weights.float())
+    return out
+
+
+# ----------------------------------------------------------------------
+# Sandwich-norm blocks, per-head output gate, channel-decay delta rule.
+# ----------------------------------------------------------------------
+def residual_sandwich_norm(x, y, w_post, mult, w_pre, eps, out_dtype):
+    """x (fp32, in place) += mult * rms_norm(y) * w_post when y is given;
+    returns rms_norm(x) * w_pre in out_dtype (None without w_pre)."""
+    def unit(t):
+        return t * torch.rsqrt(t.pow(2).mean(-1, keepdim=True) + eps)
+
+    if y is not None:
+        x += mult * (unit(y.float()) * w_post.float())
+    if w_pre is None:
+        return None
+    return (unit(x) * w_pre.float()).to(out_dtype)
+
+
+def softcap_(x, cap):
+    """x = cap * tanh(x / cap), in place."""
+    return x.copy_(cap * torch.tanh(x / cap))
+
+
+def head_gate(o, gate, out, out_scale=1.0):
+    """out[t, h] = o[t, h] * sigmoid(gate[t, h]) * out_scale; o [T, H, V]
+    (any strides), gate [T, H] or None (no gate); out may be o."""
+    f = o.float() * out_scale
+    if gate is not None:
+        f = f * torch.sigmoid(gate.float())[:, :, None]
+    out.copy_(f.to(out.dtype))
+    return out
+
+
+DELTA_UNIT_EPS = 1e-6  # under the root of q's and k's unit length
+
+
+def channel_delta(u, decay, beta, gate, rate, dt_bias, norm_w, eps, state,
+                  cu_seqlens, seq_lens, state_slots, heads, kv_heads, dim,
+                  vdim, out):
+    """Delta rule with a decay per head and key channel. u [T, 2*G*D + H*V] =
+    [q | k | v] (after conv and silu), decay [T, H*D] and beta [T, H] raw
+    projections, gate [T, H*V] raw. Per head h with q/k head h // (H/G):
+    q, k to unit length, q times D^-1/2; g = exp(-rate_h softplus(decay +
+    dt_bias)); S <- g S, w = sigmoid(beta) (v - S^T k), S <- S + k w^T,
+    o = S^T q; out = rms_norm(o) norm_w sigmoid(gate). state [slots, H, D, V]
+    fp32 (updated)."""
+    T, H, G, D, V = u.shape[0], heads, kv_heads, dim, vdim
+    f = u.float()
+
+    def unit(t):
+        return t * torch.rsqrt(t.pow(2).sum(-1, keepdim=True) + DELTA_UNIT_EPS)
+
+    q = unit(f[:, :G * D].reshape(T, G, D)) * D ** -0.5
+    k = unit(f[:, G * D:2 * G * D].reshape(T, G, D))
+    q, k = (t.repeat_interleave(H // G, 1) for t in (q, k))
+    v = f[:, 2 * G * D:].reshape(T, H, V)
+    g = torch.exp(-rate.float()[None, :, None] * torch.nn.functional.softplus(
+        decay.float() + dt_bias.float(), threshold=20.0).reshape(T, H, D))
+    b = torch.sigmoid(beta.float())
+    o = torch.empty(T, H, V, dtype=torch.float32)
+    for lo, hi, start, slot in _seq_spans(cu_seqlens, seq_lens, state_slots):
+        S = (state[slot].clone() if start > 0 and slot >= 0
+             else torch.zeros(H, D, V))
+        for t in range(lo, hi):
+            S = g[t][:, :, None] * S
+            w = b[t][:, None] * (v[t] - torch.einsum("hdv,hd->hv", S, k[t]))
+            S = S + k[t][:, :, None] * w[:, None, :]
+            o[t] = torch.einsum("hdv,hd->hv", S, q[t])
+        if slot >= 0:
+            state[slot] = S
+    o = o * torch.rsqrt(o.pow(2).mean(-1, keepdim=True) + eps) * norm_w.float()
+    o = o * torch.sigmoid(gate.float()).reshape(T, H, V)
+    out.copy_(o.reshape(T, H * V).to(out.dtype))
     return out

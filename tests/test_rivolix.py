@@ -380,9 +380,9 @@ def test_key_valued_head_sizes(tmp_path, device, dtype):
 def test_sorted_expert_segments(tmp_path, device, dtype, monkeypatch):
     """Steps above DENSE_TOKENS rows sort (row, expert) pairs by expert;
     below they run every expert with factor 0 where unused: same logits."""
-    from arks_amd.models.feedforward import InputScaledMoE
+    from arks_amd.models.feedforward import RoutedMoE
 
-    monkeypatch.setattr(InputScaledMoE, "DENSE_TOKENS", 6)
+    monkeypatch.setattr(RoutedMoE, "DENSE_TOKENS", 6)
     cfg = O.make_config([D(mlp=MOE(experts=5, top=3)),
                          K(mlp=MOE(experts=4, top=1, shared_ff=0))])
     w = write_checkpoint(tmp_path / "m", cfg)
