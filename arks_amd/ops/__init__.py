@@ -1298,8 +1298,18 @@ def channel_delta(u, decay, beta, gate, rate, dt_bias, norm_w, eps, state,
                   cu_seqlens, seq_lens, state_slots, heads, kv_heads, dim,
                   vdim, out, max_q_len=0, chunks=None):
     """Delta rule with a decay per key channel and its gated unit-RMS
-    read-out (ref.channel_delta) into out [T, H*V] (rows may be strided)."""
+    read-out (ref.channel_delta) into out [T, H*V] (rows may be strided).
+    chunks (scan_chunks of this step, DELTA_CHUNK rows each): bf16 rows with
+    head sizes the matrix-core kernels are built for run those; anything
+    else runs row by row."""
     if u.is_cuda:
+        if (chunks is not None and use_delta_mfma and u.dtype == torch.bfloat16
+                and _native_seq().channel_delta_chunks(
+                    out, u, decay, beta, gate, rate, dt_bias, norm_w,
+                    float(eps), ref.DELTA_UNIT_EPS, state, chunks["off"],
+                    chunks["cu"], cu_seqlens, seq_lens, state_slots, heads,
+                    kv_heads, dim, vdim)):
+            return out
         _native_seq().channel_delta_scan(
             out, u, decay, beta, gate, rate, dt_bias, norm_w, float(eps),
             ref.DELTA_UNIT_EPS, state, cu_seqlens, seq_lens, state_slots,

@@ -58,6 +58,7 @@ SEQ_SOURCES = [
     os.path.join(CSRC, "seq_dual.hip"),
     os.path.join(CSRC, "seq_sandwich.hip"),
     os.path.join(CSRC, "seq_delta.hip"),
+    os.path.join(CSRC, "seq_delta_mfma.hip"),
 ]
 
 EXTENSIONS = {EXT_NAME: SOURCES, SEQ_EXT_NAME: SEQ_SOURCES}

@@ -208,6 +208,18 @@ int arks_seq_channel_delta_scan(
     float eps, float unit_eps, void* state, const void* cu,
     const void* seq_lens, const void* slots, int S, int H, int G, int D, int V,
     int act_f32, hipStream_t stream);
+int64_t arks_seq_delta_chunk_floats(int D, int V);
+int arks_seq_delta_chunks_fit(int64_t ldo, int64_t ldu, int64_t ldg,
+                              const void* out, const void* u, const void* gate,
+                              int D, int V);
+int arks_seq_delta_chunks(
+    void* out, int64_t ldo, void* o, void* scratch, const void* u, int64_t ldu,
+    const void* decay, int64_t lda, const void* beta, int64_t ldb,
+    const void* gate, int64_t ldg, int gate_f32, const void* rate,
+    const void* dt_bias, const void* norm_w, float eps, float unit_eps,
+    void* state, const void* chunk_off, const void* chunk_cu, const void* cu,
+    const void* seq_lens, const void* slots, int64_t T, int chunks, int S,
+    int H, int G, int D, int V, hipStream_t stream);
 void arks_seq_lightning_combine(void* part, const void* decay, void* state,
                                 const void* chunk_off, const void* chunk_rows,
                                 const void* cu, const void* seq_lens,
@@ -1494,12 +1506,48 @@ void channel_delta_scan(Tensor out, Tensor u, Tensor decay, Tensor beta,
               ", ", V, ")");
 }
 
+// False: sizes the matrix-core kernels are not built for. chunk_cu: first row
+// of every chunk of at most 64 rows (and the end), chunk_off: first chunk of
+// every sequence (and the end).
+bool channel_delta_chunks(Tensor out, Tensor u, Tensor decay, Tensor beta,
+                          Tensor gate, Tensor rate, Tensor dt_bias,
+                          Tensor norm_w, double eps, double unit_eps,
+                          Tensor state, Tensor chunk_off, Tensor chunk_cu,
+                          Tensor cu, Tensor seq_lens, Tensor slots, int64_t H,
+                          int64_t G, int64_t D, int64_t V) {
+  const DeltaArgs a = check_delta(out, u, decay, beta, gate, rate, dt_bias,
+                                  norm_w, state, H, G, D, V);
+  const SeqMeta m = check_meta(cu, seq_lens, &slots, nullptr, 0);
+  check_i32(chunk_off, "chunk_off");
+  check_i32(chunk_cu, "chunk_cu");
+  TORCH_CHECK(chunk_off.numel() == m.S + 1 && chunk_cu.numel() >= 1);
+  if (a.f32 ||
+      !arks_seq_delta_chunks_fit(a.ldo, a.ldu, a.ldg, out.data_ptr(),
+                                 u.data_ptr(), gate.data_ptr(), (int)D, (int)V))
+    return false;
+  const int64_t T = u.size(0), chunks = chunk_cu.numel() - 1;
+  const auto f32 = u.options().dtype(torch::kFloat32);
+  Tensor o = torch::empty({T, H, V}, f32);
+  Tensor scratch = torch::empty(
+      {chunks * H * arks_seq_delta_chunk_floats((int)D, (int)V)}, f32);
+  return arks_seq_delta_chunks(
+             out.data_ptr(), a.ldo, o.data_ptr(), scratch.data_ptr(),
+             u.data_ptr(), a.ldu, decay.data_ptr(), a.lda, beta.data_ptr(),
+             a.ldb, gate.data_ptr(), a.ldg, a.gate_f32, rate.data_ptr(),
+             dt_bias.data_ptr(), norm_w.data_ptr(), (float)eps,
+             (float)unit_eps, state.data_ptr(), chunk_off.data_ptr(),
+             chunk_cu.data_ptr(), cu.data_ptr(), seq_lens.data_ptr(),
+             slots.data_ptr(), T, (int)chunks, m.S, (int)H, (int)G, (int)D,
+             (int)V, current_stream()) == 0;
+}
+
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("residual_tanh_norm", &residual_tanh_norm);
   m.def("residual_sandwich_norm", &residual_sandwich_norm);
   m.def("softcap", &softcap);
   m.def("head_gate", &head_gate);
   m.def("channel_delta_scan", &channel_delta_scan);
+  m.def("channel_delta_chunks", &channel_delta_chunks);
   m.def("latent_prepare", &latent_prepare);
   m.def("latent_query", &latent_query);
   m.def("mamba2_scan", &mamba2_scan);

@@ -1,0 +1,615 @@
+// Channel-decay delta rule of long portions on the fp32 matrix cores
+// (v_mfma_f32_16x16x4_f32): the recurrence of seq_delta.hip over chunks of
+// up to 64 rows. With G_i the running sum of log decays inside a chunk
+// (per key channel), S0 the state in front of it, and unit rows q_i, k_i:
+//
+//   (I + L) U = beta V - (beta K~) S0,   K~_i = k_i exp(G_i),
+//   L_ij = beta_i sum_d k_id k_jd exp(G_id - G_jd)   (j < i)
+//   O  = Q~ S0 + A U,   A_ij = sum_d q_id k_jd exp(G_id - G_jd)  (j <= i)
+//   S1 = exp(G_last) S0 + K^ U^,   K^_j = k_j exp(G_last - G_j) as columns
+//
+//   prepare  one block per (chunk, head), all chunks at once: A, and
+//       U0 = (I + L)^-1 beta V, W = (I + L)^-1 beta K~ by forward
+//       substitution over 16-row blocks, Q~, K^
+//   scan     one block per (sequence, head, 16 value columns), chunk by
+//       chunk: U = U0 - W S0, O, S1; the state stays in registers
+//   read-out unit RMS, weight and gate of O
+//
+// Exponents: exp(G_i - G_j) is split at the borders of the 16-row blocks
+// into factors whose exponents are sums of log decays, all <= 0, so nothing
+// overflows and no sums longer than a block are subtracted. Inside a 16-row block
+// exp(c_i) exp(-c_j) is used while the block's total log decay is above
+// MIN_BLOCK_LOG (both factors finite in fp32), else exp(c_i - c_j) per
+// channel, element by element.
+//
+// Fragments: with k = 4 g + e (g = lane / 16) the operand A of four
+// consecutive MFMAs is row lane % 16, columns 4 g .. 4 g + 3 of a 16x16 tile
+// (one float4 per lane), and the result's layout (rows 4 g + r, column
+// lane % 16) is itself the operand B of a following product. The state, U
+// and the substitution's columns are therefore never rearranged. Operands
+// that another kernel reads are stored tile by tile in lane order.
+#include "seq_common.h"
+
+namespace arks {
+
+constexpr int DC = 64;                  // rows per chunk
+constexpr float MIN_BLOCK_LOG = -80.f;  // exp(80) * exp(-80) stay finite
+
+__device__ __forceinline__ float4v mm16(float4v acc, float4v a, float4v b) {
+#pragma unroll
+  for (int e = 0; e < 4; ++e)
+    acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a[e], b[e], acc, 0, 0, 0);
+  return acc;
+}
+
+// log1p(exp(x)) with the hardware exponential and logarithm; log(1 + z) is
+// corrected by z / ((1 + z) - 1), which restores the digits 1 + z drops
+__device__ __forceinline__ float softplus_fast(float x) {
+  const float z = __expf(-fabsf(x));
+  const float w = 1.f + z;
+  const float d = w - 1.f;
+  const float l = d > 0.f ? __logf(w) * (z / d) : z;
+  return fmaxf(x, 0.f) + l;
+}
+
+struct DeltaChunk {  // float offsets inside the scratch of one (chunk, head)
+  int W, Q, K, U, A, E, total;
+};
+__host__ __device__ inline DeltaChunk delta_chunk_layout(int D, int V) {
+  DeltaChunk c;
+  c.W = 0;
+  c.Q = c.W + DC * D;
+  c.K = c.Q + DC * D;
+  c.U = c.K + DC * D;
+  c.A = c.U + DC * V;
+  c.E = c.A + DC * DC;
+  c.total = c.E + D;
+  return c;
+}
+
+__host__ __device__ constexpr int delta_prepare_lds(int D) {
+  return 2 * DC * (D + 8) * 2 + DC * (D + 4) * 4 + 14 * 64 * 16 + 4 * D * 4 +
+         (3 * DC + 4) * 4;
+}
+
+template <int KT>
+__global__ __launch_bounds__(256) void delta_chunk_prepare_kernel(
+    float* __restrict__ scratch, const bf16* __restrict__ u, int64_t ldu,
+    const float* __restrict__ decay, int64_t lda,
+    const bf16* __restrict__ beta, int64_t ldb, const float* __restrict__ rate,
+    const float* __restrict__ dt_bias, const int* __restrict__ cu, int H,
+    int G, int V, float unit_eps) {
+  constexpr int D = 16 * KT;
+  constexpr int LK = D + 8;  // bf16 row stride
+  constexpr int LC = D + 4;  // float row stride
+  extern __shared__ __align__(16) char smem[];
+  bf16* k_s = reinterpret_cast<bf16*>(smem);           // [DC][LK]
+  bf16* q_s = k_s + DC * LK;                           // [DC][LK]
+  float* c_s = reinterpret_cast<float*>(q_s + DC * LK);  // [DC][LC]
+  float4v* l_s = reinterpret_cast<float4v*>(c_s + DC * LC);  // [10][64]
+  float4v* inv_s = l_s + 10 * 64;                      // [4][64]
+  float* tot_s = reinterpret_cast<float*>(inv_s + 4 * 64);  // [4][D]
+  float* rk_s = tot_s + 4 * D;                         // [DC]
+  float* rq_s = rk_s + DC;                             // [DC]
+  float* b_s = rq_s + DC;                              // [DC]
+  float* min_s = b_s + DC;                             // [4]
+  const int h = blockIdx.x, chunk = blockIdx.y;
+  const int t0 = cu[chunk], n = min(cu[chunk + 1] - t0, DC);
+  const int I = threadIdx.x / 64, lane = threadIdx.x % 64;
+  const int g = lane / 16, m = lane % 16;
+  const int gk = h / (H / G);
+  const DeltaChunk lay = delta_chunk_layout(D, V);
+  float* base = scratch + ((int64_t)chunk * H + h) * lay.total;
+
+  // ---- rows of block I: raw q, k, their unit factors, log decays
+#pragma unroll
+  for (int it = 0; it < 4; ++it) {
+    const int row = 16 * I + 4 * it + g;  // 16 lanes per row
+    ushort8 qv, kv;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) { qv[e] = 0; kv[e] = 0; }
+    const bool live = m * 8 < D;
+    if (live && row < n) {
+      const bf16* qr = u + (int64_t)(t0 + row) * ldu + (int64_t)gk * D + m * 8;
+      qv = *reinterpret_cast<const ushort8*>(qr);
+      kv = *reinterpret_cast<const ushort8*>(qr + (int64_t)G * D);
+    }
+    float qq = 0.f, kk = 0.f;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      const float a = bf16_bits_to_float(qv[e]), b = bf16_bits_to_float(kv[e]);
+      qq += a * a;
+      kk += b * b;
+    }
+    qq = group16_reduce_sum(qq);
+    kk = group16_reduce_sum(kk);
+    if (live) {
+      *reinterpret_cast<ushort8*>(q_s + row * LK + m * 8) = qv;
+      *reinterpret_cast<ushort8*>(k_s + row * LK + m * 8) = kv;
+    }
+    if (m == 0) {
+      rq_s[row] = 1.f / sqrtf((qq + unit_eps) * (float)D);
+      rk_s[row] = 1.f / sqrtf(kk + unit_eps);
+    }
+  }
+  if (lane < 16) {
+    const int row = 16 * I + lane;
+    b_s[row] = row < n
+                   ? sigmoid_f(bf16_bits_to_float(beta[(int64_t)(t0 + row) * ldb + h]))
+                   : 0.f;
+  }
+  {
+    const float rt = rate[h];
+    float lowest = 0.f;
+    for (int d = lane; d < D; d += 64) {
+      const float db = dt_bias[(int64_t)h * D + d];
+      float c = 0.f;
+#pragma unroll
+      for (int r = 0; r < 16; ++r) {
+        const int row = 16 * I + r;
+        if (row < n)
+          c -= rt * softplus_fast(
+                        decay[(int64_t)(t0 + row) * lda + (int64_t)h * D + d] + db);
+        c_s[row * LC + d] = c;
+      }
+      tot_s[I * D + d] = c;
+      lowest = fminf(lowest, c);
+    }
+    lowest = -wave_reduce_max(-lowest);
+    if (lane == 0) min_s[I] = lowest;
+  }
+  __syncthreads();
+
+  // ---- scores of block row I against every block J <= I
+  {
+    float4v kI[KT], qI[KT];  // k_i exp(c_i), q_i exp(c_i): row m, 4 channels
+    const int row = 16 * I + m;
+    const float rk = rk_s[row], rq = rq_s[row];
+#pragma unroll
+    for (int kt = 0; kt < KT; ++kt) {
+      const int d = 16 * kt + 4 * g;
+      const ushort4v kr = *reinterpret_cast<const ushort4v*>(k_s + row * LK + d);
+      const ushort4v qr = *reinterpret_cast<const ushort4v*>(q_s + row * LK + d);
+      const float4v c = *reinterpret_cast<const float4v*>(c_s + row * LC + d);
+      float4v qg;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const float x = __expf(c[e]);
+        kI[kt][e] = bf16_bits_to_float(kr[e]) * rk * x;
+        qI[kt][e] = bf16_bits_to_float(qr[e]) * rq * x;
+        float pre = 0.f;
+        for (int M = 0; M < I; ++M) pre += tot_s[M * D + d + e];
+        qg[e] = qI[kt][e] * __expf(pre);
+      }
+      *reinterpret_cast<float4v*>(base + lay.Q + ((I * KT + kt) * 64 + lane) * 4) = qg;
+    }
+    const float bI = b_s[row];
+    for (int J = 0; J <= I; ++J) {
+      float4v kk = {0.f, 0.f, 0.f, 0.f}, qk = {0.f, 0.f, 0.f, 0.f};
+      const int rj = 16 * J + m;
+      const float rkj = rk_s[rj];
+      if (J < I || min_s[I] > MIN_BLOCK_LOG) {
+#pragma unroll
+        for (int kt = 0; kt < KT; ++kt) {
+          const int d = 16 * kt + 4 * g;
+          const ushort4v kr = *reinterpret_cast<const ushort4v*>(k_s + rj * LK + d);
+          const float4v c = *reinterpret_cast<const float4v*>(c_s + rj * LC + d);
+          float4v a;
+#pragma unroll
+          for (int e = 0; e < 4; ++e) {
+            float x = -c[e];
+            if (J < I) {
+              for (int M = J; M < I; ++M) x += tot_s[M * D + d + e];
+              x = fminf(x, 0.f);
+            }
+            a[e] = bf16_bits_to_float(kr[e]) * rkj * __expf(x);
+          }
+          kk = mm16(kk, a, kI[kt]);
+          qk = mm16(qk, a, qI[kt]);
+        }
+      } else {
+        // strong decays: element (i = m, j = 4 g + r) channel by channel
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int j = 16 * I + 4 * g + r;
+          float sk = 0.f, sq = 0.f;
+          if (j <= row) {
+            for (int d = 0; d < D; ++d) {
+              const float x = __expf(fminf(c_s[row * LC + d] - c_s[j * LC + d], 0.f)) *
+                              bf16_bits_to_float(k_s[j * LK + d]);
+              sk += x * bf16_bits_to_float(k_s[row * LK + d]);
+              sq += x * bf16_bits_to_float(q_s[row * LK + d]);
+            }
+          }
+          kk[r] = sk * rk * rk_s[j];
+          qk[r] = sq * rq * rk_s[j];
+        }
+      }
+      // lane holds (row i = m of block I, columns j = 4 g + r of block J)
+      if (J == I) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int j = 4 * g + r;
+          if (j >= m) kk[r] = 0.f;
+          if (j > m) qk[r] = 0.f;
+        }
+      }
+#pragma unroll
+      for (int r = 0; r < 4; ++r) kk[r] *= bI;
+      l_s[(J == I ? 6 + I : I * (I - 1) / 2 + J) * 64 + lane] = kk;
+      *reinterpret_cast<float4v*>(base + lay.A + ((I * 4 + J) * 64 + lane) * 4) = qk;
+    }
+  }
+  __syncthreads();
+
+  // ---- (I + L_II)^-1 of block I, a column per lane (column m)
+  {
+    float x[16];
+#pragma unroll
+    for (int i = 0; i < 16; ++i) {
+      float s = i == m ? 1.f : 0.f;
+#pragma unroll
+      for (int jb = 0; jb < 4; ++jb) {
+        if (4 * jb < i) {
+          const float4v l = l_s[(6 + I) * 64 + i + 16 * jb];
+#pragma unroll
+          for (int e = 0; e < 4; ++e)
+            if (4 * jb + e < i) s -= l[e] * x[4 * jb + e];
+        }
+      }
+      x[i] = s;
+    }
+    if (g == 0) {
+      float* dst = reinterpret_cast<float*>(inv_s + I * 64);
+#pragma unroll
+      for (int i = 0; i < 16; ++i) dst[(i + 16 * (m / 4)) * 4 + m % 4] = x[i];
+    }
+  }
+  __syncthreads();
+
+  // ---- columns of [K~ | V] through the substitution, 16 at a time
+  const int VT = V / 16;
+  for (int tile = I; tile < KT + VT; tile += 4) {
+    const bool is_k = tile < KT;
+    const int ct = is_k ? tile : tile - KT;
+    const int d = 16 * ct + m;
+    float4v X[4];
+    float pre = 0.f;
+#pragma unroll
+    for (int B = 0; B < 4; ++B) {
+      float4v rhs;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int row = 16 * B + 4 * g + r;
+        float x = 0.f;
+        if (is_k) {
+          x = bf16_bits_to_float(k_s[row * LK + d]) * rk_s[row] *
+              __expf(pre + c_s[row * LC + d]);
+        } else if (row < n) {
+          x = bf16_bits_to_float(
+              u[(int64_t)(t0 + row) * ldu + 2 * (int64_t)G * D + (int64_t)h * V + d]);
+        }
+        rhs[r] = x * b_s[row];
+      }
+      if (is_k) pre += tot_s[B * D + d];
+      float4v acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int J = 0; J < 4; ++J)
+        if (J < B) acc = mm16(acc, l_s[(B * (B - 1) / 2 + J) * 64 + lane], X[J]);
+      rhs -= acc;
+      const float4v zero = {0.f, 0.f, 0.f, 0.f};
+      X[B] = mm16(zero, inv_s[B * 64 + lane], rhs);
+      if (is_k) {
+        // -W as an operand A: element (row, column d) in its lane's place
+        float* dst = base + lay.W + (B * KT + ct) * 256;
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          dst[(4 * g + r + 16 * (m / 4)) * 4 + m % 4] = -X[B][r];
+      } else {
+        *reinterpret_cast<float4v*>(base + lay.U + ((ct * 4 + B) * 64 + lane) * 4) = X[B];
+      }
+    }
+  }
+
+  // ---- K^ transposed (rows = channels) and the chunk's decay
+  for (int tile = I; tile < KT * 4; tile += 4) {
+    const int rt = tile / 4, kt = tile % 4;
+    const int d = 16 * rt + m;
+    float post = 0.f;
+    for (int M = kt; M < 4; ++M) post += tot_s[M * D + d];
+    float4v o;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      const int j = 16 * kt + 4 * g + e;
+      o[e] = bf16_bits_to_float(k_s[j * LK + d]) * rk_s[j] *
+             __expf(fminf(post - c_s[j * LC + d], 0.f));
+    }
+    *reinterpret_cast<float4v*>(base + lay.K + ((rt * 4 + kt) * 64 + lane) * 4) = o;
+  }
+  for (int d = threadIdx.x; d < D; d += 256)
+    base[lay.E + d] = __expf(tot_s[d] + tot_s[D + d] + tot_s[2 * D + d] +
+                             tot_s[3 * D + d]);
+}
+
+// One block per (sequence, head, 16 value columns). Wave w owns the state's
+// 16-row tiles w, w + 4, ... (operands B as they are), sums its part of
+// [-W; Q~] S0 and rows 16 w .. 16 w + 15 of U and O.
+template <int KT>
+__global__ __launch_bounds__(256) void delta_chunk_scan_kernel(
+    float* __restrict__ o, const float* __restrict__ scratch,
+    float* __restrict__ state, const int* __restrict__ chunk_off,
+    const int* __restrict__ chunk_cu, const int* __restrict__ cu,
+    const int* __restrict__ seq_lens, const int* __restrict__ slots, int H,
+    int V, int groups) {
+  constexpr int D = 16 * KT;
+  constexpr int RT = (KT + 3) / 4;
+  __shared__ float4v part_s[4][8][64];
+  __shared__ float4v u_s[4][64];
+  // the column blocks of one (sequence, head) sit on one XCD, whose L2
+  // then reads the chunk operands once for all of them
+  const int VT = V / 16;
+  const int group = (blockIdx.x / 8 / VT) * 8 + blockIdx.x % 8;
+  const int ct = (blockIdx.x / 8) % VT;
+  if (group >= groups) return;
+  const int s = group / H, h = group % H;
+  const int c_begin = chunk_off[s], c_end = chunk_off[s + 1];
+  if (c_begin == c_end) return;
+  const int w = threadIdx.x / 64, lane = threadIdx.x % 64;
+  const int g = lane / 16, m = lane % 16;
+  const int start = seq_lens[s] - (cu[s + 1] - cu[s]);
+  const int slot = slots[s];
+  float* sp = state + ((int64_t)(slot < 0 ? 0 : slot) * H + h) * D * V + 16 * ct + m;
+  const DeltaChunk lay = delta_chunk_layout(D, V);
+  const int64_t step = (int64_t)H * lay.total;
+  const float* base = scratch + ((int64_t)c_begin * H + h) * lay.total;
+  float4v S[RT];
+#pragma unroll
+  for (int i = 0; i < RT; ++i) {
+    const int rt = w + 4 * i;
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+      S[i][r] = rt < KT && start > 0 && slot >= 0
+                    ? sp[(int64_t)(16 * rt + 4 * g + r) * V] : 0.f;
+  }
+  const float4v zero = {0.f, 0.f, 0.f, 0.f};
+  float4v wf[RT][4], qf[RT][4];
+  auto load_wq = [&](const float* b) {
+#pragma unroll
+    for (int i = 0; i < RT; ++i) {
+      const int kt = w + 4 * i;
+      if (kt < KT) {
+#pragma unroll
+        for (int t = 0; t < 4; ++t) {
+          wf[i][t] = *reinterpret_cast<const float4v*>(b + lay.W + ((t * KT + kt) * 64 + lane) * 4);
+          qf[i][t] = *reinterpret_cast<const float4v*>(b + lay.Q + ((t * KT + kt) * 64 + lane) * 4);
+        }
+      }
+    }
+  };
+  load_wq(base);
+  for (int c = c_begin; c < c_end; ++c, base += step) {
+    // this chunk's remaining operands, used after the first barrier
+    float4v kf[RT][4], eg[RT], af[4], u0;
+#pragma unroll
+    for (int i = 0; i < RT; ++i) {
+      const int rt = w + 4 * i;
+      if (rt < KT) {
+#pragma unroll
+        for (int t = 0; t < 4; ++t)
+          kf[i][t] = *reinterpret_cast<const float4v*>(base + lay.K + ((rt * 4 + t) * 64 + lane) * 4);
+        eg[i] = *reinterpret_cast<const float4v*>(base + lay.E + 16 * rt + 4 * g);
+      }
+    }
+#pragma unroll
+    for (int J = 0; J < 4; ++J)
+      af[J] = J <= w ? *reinterpret_cast<const float4v*>(base + lay.A + ((w * 4 + J) * 64 + lane) * 4)
+                     : zero;
+    u0 = *reinterpret_cast<const float4v*>(base + lay.U + ((ct * 4 + w) * 64 + lane) * 4);
+    const int t0 = chunk_cu[c];
+    const int n = chunk_cu[c + 1] - t0;
+
+    float4v aw[4], aq[4];
+#pragma unroll
+    for (int t = 0; t < 4; ++t) { aw[t] = zero; aq[t] = zero; }
+#pragma unroll
+    for (int i = 0; i < RT; ++i) {
+      if (w + 4 * i < KT) {
+        // independent accumulators take turns, so that no MFMA waits for
+        // the one before it
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+#pragma unroll
+          for (int t = 0; t < 4; ++t) {
+            aw[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(wf[i][t][e], S[i][e], aw[t], 0, 0, 0);
+            aq[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(qf[i][t][e], S[i][e], aq[t], 0, 0, 0);
+          }
+      }
+    }
+#pragma unroll
+    for (int t = 0; t < 4; ++t) {
+      part_s[w][t][lane] = aw[t];
+      part_s[w][4 + t][lane] = aq[t];
+    }
+    if (c + 1 < c_end) load_wq(base + step);
+    __syncthreads();
+    float4v uw = u0, ow = zero;
+#pragma unroll
+    for (int p = 0; p < 4; ++p) {
+      uw += part_s[p][w][lane];
+      ow += part_s[p][4 + w][lane];
+    }
+    u_s[w][lane] = uw;
+    __syncthreads();
+    float4v ub[4];
+#pragma unroll
+    for (int t = 0; t < 4; ++t) ub[t] = u_s[t][lane];
+#pragma unroll
+    for (int i = 0; i < RT; ++i)
+      if (w + 4 * i < KT) S[i] *= eg[i];
+#pragma unroll
+    for (int t = 0; t < 4; ++t) {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+#pragma unroll
+        for (int i = 0; i < RT; ++i)
+          if (w + 4 * i < KT)
+            S[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(kf[i][t][e], ub[t][e], S[i], 0, 0, 0);
+        if (t <= w)
+          ow = __builtin_amdgcn_mfma_f32_16x16x4f32(af[t][e], ub[t][e], ow, 0, 0, 0);
+      }
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int row = 16 * w + 4 * g + r;
+      if (row < n)
+        o[((int64_t)(t0 + row) * H + h) * V + 16 * ct + m] = ow[r];
+    }
+  }
+  if (slot >= 0) {
+#pragma unroll
+    for (int i = 0; i < RT; ++i) {
+      const int rt = w + 4 * i;
+      if (rt < KT) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          sp[(int64_t)(16 * rt + 4 * g + r) * V] = S[i][r];
+      }
+    }
+  }
+}
+
+// out = o / rms(o) * w * sigmoid(gate) per head: 16 lanes per (row, head),
+// VPL consecutive values per lane and turn (V a multiple of 16 * VPL).
+template <int VPL>
+__global__ __launch_bounds__(256) void delta_read_out_kernel(
+    bf16* __restrict__ out, int64_t ldo, const float* __restrict__ o,
+    const void* __restrict__ gate, int64_t ldg, int gate_f32,
+    const float* __restrict__ norm_w, float eps, int64_t heads_total, int H,
+    int V) {
+  const int64_t i = (int64_t)blockIdx.x * 16 + threadIdx.x / 16;
+  const int m = threadIdx.x % 16;
+  const bool live = i < heads_total;
+  const int64_t t = live ? i / H : 0;
+  const int h = live ? (int)(i % H) : 0;
+  const float* orow = o + (t * H + h) * V;
+  float ss = 0.f;
+  for (int v0 = m * VPL; v0 < V; v0 += 16 * VPL) {
+#pragma unroll
+    for (int e = 0; e < VPL; e += 4) {
+      const float4v x = *reinterpret_cast<const float4v*>(orow + v0 + e);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) ss += x[j] * x[j];
+    }
+  }
+  ss = group16_reduce_sum(ss);
+  if (!live) return;
+  const float r = 1.f / sqrtf(ss / (float)V + eps);
+  const int64_t gat = t * ldg + (int64_t)h * V;
+  bf16* dst = out + t * ldo + (int64_t)h * V;
+  for (int v0 = m * VPL; v0 < V; v0 += 16 * VPL) {
+#pragma unroll
+    for (int e = 0; e < VPL; e += 4) {
+      const int v = v0 + e;
+      const float4v x = *reinterpret_cast<const float4v*>(orow + v);
+      const float4v w = *reinterpret_cast<const float4v*>(norm_w + v);
+      float gv[4];
+      if (gate_f32) {
+        const float4v y = *reinterpret_cast<const float4v*>((const float*)gate + gat + v);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) gv[j] = y[j];
+      } else {
+        const ushort4v y = *reinterpret_cast<const ushort4v*>((const bf16*)gate + gat + v);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) gv[j] = bf16_bits_to_float(y[j]);
+      }
+      ushort4v z;
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        z[j] = float_to_bf16_bits(x[j] * r * w[j] / (1.f + __expf(-gv[j])));
+      *reinterpret_cast<ushort4v*>(dst + v) = z;
+    }
+  }
+}
+
+template <int KT>
+static void launch_delta_chunks(float* o, float* scratch, const void* u,
+                                int64_t ldu, const void* decay, int64_t lda,
+                                const void* beta, int64_t ldb, const void* rate,
+                                const void* dt_bias, float unit_eps,
+                                void* state, const int* chunk_off,
+                                const int* chunk_cu, const int* cu,
+                                const int* seq_lens, const int* slots,
+                                int chunks, int S, int H, int G, int V,
+                                hipStream_t stream) {
+  constexpr int lds = delta_prepare_lds(16 * KT);
+  static bool set = false;
+  if (!set) {
+    (void)hipFuncSetAttribute(
+        reinterpret_cast<const void*>(delta_chunk_prepare_kernel<KT>),
+        hipFuncAttributeMaxDynamicSharedMemorySize, lds);
+    set = true;
+  }
+  hipLaunchKernelGGL((delta_chunk_prepare_kernel<KT>), dim3(H, chunks),
+                     dim3(256), lds, stream, scratch, (const bf16*)u, ldu,
+                     (const float*)decay, lda, (const bf16*)beta, ldb,
+                     (const float*)rate, (const float*)dt_bias, chunk_cu, H, G,
+                     V, unit_eps);
+  const int groups = S * H;
+  hipLaunchKernelGGL((delta_chunk_scan_kernel<KT>),
+                     dim3((groups + 7) / 8 * 8 * (V / 16)), dim3(256), 0,
+                     stream, o, scratch, (float*)state, chunk_off, chunk_cu, cu,
+                     seq_lens, slots, H, V, groups);
+}
+
+}  // namespace arks
+
+using namespace arks;
+
+extern "C" int64_t arks_seq_delta_chunk_floats(int D, int V) {
+  return delta_chunk_layout(D, V).total;
+}
+
+// 1: sizes, strides or alignment the kernels are not built for.
+extern "C" int arks_seq_delta_chunks(
+    void* out, int64_t ldo, void* o, void* scratch, const void* u, int64_t ldu,
+    const void* decay, int64_t lda, const void* beta, int64_t ldb,
+    const void* gate, int64_t ldg, int gate_f32, const void* rate,
+    const void* dt_bias, const void* norm_w, float eps, float unit_eps,
+    void* state, const void* chunk_off, const void* chunk_cu, const void* cu,
+    const void* seq_lens, const void* slots, int64_t T, int chunks, int S,
+    int H, int G, int D, int V, hipStream_t stream) {
+  if (T == 0 || chunks == 0) return 0;
+#define DK(KT)                                                               \
+  launch_delta_chunks<KT>((float*)o, (float*)scratch, u, ldu, decay, lda,    \
+                          beta, ldb, rate, dt_bias, unit_eps, state,         \
+                          (const int*)chunk_off, (const int*)chunk_cu,       \
+                          (const int*)cu, (const int*)seq_lens,              \
+                          (const int*)slots, chunks, S, H, G, V, stream)
+  if (D == 32) DK(2);
+  else if (D == 64) DK(4);
+  else if (D == 96) DK(6);
+  else if (D == 128) DK(8);
+  else return 1;
+#undef DK
+  const int64_t heads = T * H;
+  const unsigned blocks = (unsigned)((heads + 15) / 16);
+#define RO(VPL)                                                              \
+  hipLaunchKernelGGL((delta_read_out_kernel<VPL>), dim3(blocks), dim3(256),  \
+                     0, stream, (bf16*)out, ldo, (const float*)o, gate, ldg, \
+                     gate_f32, (const float*)norm_w, eps, heads, H, V)
+  if (V % 128 == 0) RO(8);
+  else RO(4);
+#undef RO
+  return 0;
+}
+
+extern "C" int arks_seq_delta_chunks_fit(int64_t ldo, int64_t ldu,
+                                         int64_t ldg, const void* out,
+                                         const void* u, const void* gate,
+                                         int D, int V) {
+  if (D != 32 && D != 64 && D != 96 && D != 128) return 0;
+  if (V % 16 || V > 512) return 0;
+  if (ldu % 8 || ldo % 4 || ldg % 4) return 0;
+  return (((uintptr_t)u | (uintptr_t)gate) & 15) == 0 &&
+         ((uintptr_t)out & 7) == 0;
+}

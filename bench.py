@@ -54,16 +54,18 @@ def parse_args():
     # design (--design) at real layer sizes beside the closest llama-family
     # model cut to the same width and depth (for rivolix, whose feed-forward
     # is routed experts beside a shared one: a Qwen2-MoE-shaped model of the
-    # same width, depth, head and expert sizes, "moe"), one JSON line per
+    # same width, depth, head and expert sizes, "moe"; for pazilorn, routed
+    # experts alone: a Mixtral-shaped one, "mixtral"), one JSON line per
     # model and phase. --design-only NAME runs one of the two (profiling).
     p.add_argument("--design-bench", action="store_true")
     p.add_argument("--design-only",
-                   choices=["gagorax", "fusolix", "legalix", "rivolix", "llama",
-                            "moe"],
+                   choices=["gagorax", "fusolix", "legalix", "rivolix",
+                            "pazilorn", "llama", "moe", "mixtral"],
                    default=None)
     # which layer-list design --design-bench measures beside llama
     p.add_argument("--design",
-                   choices=["gagorax", "fusolix", "legalix", "rivolix"],
+                   choices=["gagorax", "fusolix", "legalix", "rivolix",
+                            "pazilorn"],
                    default="gagorax")
     p.add_argument("--cold-start", action="store_true")
     p.add_argument("--ckpt-dir", default="/tmp/arks_ckpt")
@@ -135,9 +137,10 @@ def run_cold_start(args):
 
 
 def run_design_bench(args):
-    """A layer-list design (--design: Gagorax, Fusolix, Legalix or Rivolix, 8
-    blocks at the sizes of an 8B model) against llama-3-8b cut to 8 layers
-    (Rivolix: against a Qwen2-MoE-shaped model of equal sizes): prefill
+    """A layer-list design (--design: Gagorax, Fusolix, Legalix, Rivolix or
+    Pazilorn, 8 blocks at the sizes of an 8B model) against llama-3-8b cut to
+    8 layers (Rivolix: against a Qwen2-MoE-shaped, Pazilorn: against a
+    Mixtral-shaped model of equal sizes): prefill
     tokens/s for one long prompt and for a batch of prompts, decode tokens/s
     for a batch at a fixed context. Random weights, synthetic tokens, one
     GPU."""
@@ -160,6 +163,14 @@ def run_design_bench(args):
             shared_expert_intermediate_size=3584, norm_topk_prob=False,
             attention_bias=True, tie_word_embeddings=True)
         models = {"rivolix": "rivolix-8b-slice", "moe": "qwen2moe-8b-8l"}
+    if args.design == "pazilorn":
+        # the same routed experts: 16 of ff 3584, 4 per row, 32/8 heads x 128
+        PRESET_CONFIGS["mixtral-8b-8l"] = dataclasses.replace(
+            PRESET_CONFIGS["llama-3-8b"], architecture="MixtralForCausalLM",
+            num_hidden_layers=8, vocab_size=32000, num_local_experts=16,
+            num_experts_per_tok=4, intermediate_size=3584,
+            tie_word_embeddings=True)
+        models = {"pazilorn": "pazilorn-8b-slice", "mixtral": "mixtral-8b-8l"}
     prefills = [(1, 8192), (8, 2048), (32, 128)]  # (prompts, tokens each)
     dec_batch, dec_ctx = args.batch, args.input_len
     for key, preset in models.items():

@@ -206,3 +206,129 @@ def forward(cfg, weights, tokens, margins=None):
     z = rms_norm(x, weights["final.norm"], eps) @ weights["embed"].T
     cap = cfg["logit_softcap"]
     return cap * torch.tanh(z / cap), after
+
+
+def clear_rows(margins, least=0.06):
+    """How many rows from the start every router chooses by a margin of at
+    least `least` between logits (margins as forward() collects them)."""
+    close = torch.stack(margins).amin(0) < least
+    return int(close.nonzero()[0]) if bool(close.any()) else close.numel()
+
+
+# ------------------------------------------------------- configs and weights
+def moe_spec(experts=6, top=2, ff=24):
+    return {"kind": "moe", "expert": {"ff": ff},
+            "router": {"experts": experts, "top": top}}
+
+
+def delta_spec(heads=4, kv_heads=2, dim=8, vdim=12, conv=4, mlp="default",
+               weights_of=None):
+    spec = {"type": "channel_delta",
+            "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": dim,
+                      "vdim": vdim, "conv": conv},
+            "mlp": moe_spec() if mlp == "default" else mlp}
+    if weights_of is not None:
+        spec["weights_of"] = weights_of
+    return spec
+
+
+def latent_spec(heads=3, dim=8, rot_dim=6, vdim=10, kv_rank=20, q_rank=14,
+                window=11, base=500.0, scaling="default", scale=None,
+                mlp="default", weights_of=None):
+    if scaling == "default":
+        scaling = {"factor": 4.0, "original": 24, "fast": 6.0, "slow": 1.0}
+    rot = {"base": base, "dims": rot_dim}
+    if scaling:
+        rot["scaling"] = scaling
+    spec = {"type": "latent_attention", "mixer": {
+        "heads": heads, "dim": dim, "rot_dim": rot_dim, "vdim": vdim,
+        "kv_rank": kv_rank, "q_rank": q_rank, "rot": rot,
+        "mask": {"size": window},
+        "scale": (dim + rot_dim) ** -0.5 if scale is None else scale},
+        "mlp": moe_spec() if mlp == "default" else mlp}
+    if weights_of is not None:
+        spec["weights_of"] = weights_of
+    return spec
+
+
+def make_config(layers, width=40, vocab=96, eps=1e-5, mult=0.6, scale=3.0,
+                cap=6.0):
+    return {"architecture": "Pazilorn", "vocab": vocab, "width": width,
+            "norm": {"eps": eps}, "embedding": {"scale": scale},
+            "residual_mult": mult, "logit_softcap": cap,
+            "layers": list(layers)}
+
+
+def tensor_shapes(cfg, ranks=(5, 7)):
+    """ranks: rows of the low-rank decay and gate projections, which only
+    the tensors' shapes give."""
+    W, out = cfg["width"], {}
+    out["embed"], out["final.norm"] = (cfg["vocab"], W), (W,)
+    ra, rg = ranks
+    for i, spec in enumerate(cfg["layers"]):
+        if "weights_of" in spec:
+            continue
+        p, m = f"l{i}.", spec["mixer"]
+        x = p + "mix."
+        H, V = m["heads"], m["vdim"]
+        out[p + "norm1"] = out[p + "norm1b"] = (W,)
+        if spec["type"] == "channel_delta":
+            G, D, K = m["kv_heads"], m["dim"], m["conv"]
+            for leaf, rows in (("q", G * D), ("k", G * D), ("v", H * V)):
+                out[x + leaf], out[x + leaf + ".conv"] = (rows, W), (rows, K)
+            out[x + "b"], out[x + "A_log"], out[x + "norm"] = (H, W), (H,), (V,)
+            out[x + "a1"], out[x + "a2"] = (ra, W), (H * D, ra)
+            out[x + "g1"], out[x + "g2"] = (rg, W), (H * V, rg)
+            out[x + "dt_bias"] = (H * D,)
+        else:
+            D, R, rk, rq = m["dim"], m["rot_dim"], m["kv_rank"], m["q_rank"]
+            out[x + "dq"], out[x + "dq.norm"] = (rq, W), (rq,)
+            out[x + "uq"] = (H * (D + R), rq)
+            out[x + "dkv"], out[x + "dkv.norm"] = (rk + R, W), (rk,)
+            out[x + "uk"], out[x + "uv"] = (H * D, rk), (H * V, rk)
+            out[x + "g"] = (H, W)
+        out[x + "o"] = (W, H * V)
+        mlp = spec.get("mlp")
+        if mlp is not None:
+            out[p + "norm2"] = out[p + "norm2b"] = (W,)
+            E, ff = mlp["router"]["experts"], mlp["expert"]["ff"]
+            out[p + "mlp.router"], out[p + "mlp.router.b"] = (E, W), (E,)
+            for e in range(E):
+                out[p + f"mlp.e{e}.gate"] = out[p + f"mlp.e{e}.up"] = (ff, W)
+                out[p + f"mlp.e{e}.down"] = (W, ff)
+    return out
+
+
+def random_weights(cfg, seed=0, ranks=(5, 7)):
+    """Random weights, rounded to bfloat16 (what a checkpoint holds), as
+    float64. Norm weights, taps, router biases and gates are of order one,
+    and decays spread between nearly none and strong, so that leaving any of
+    them out shows."""
+    gen = torch.Generator().manual_seed(seed)
+    w = {}
+    for name, shape in tensor_shapes(cfg, ranks).items():
+        leaf = name.rsplit(".", 1)[-1]
+
+        def rn(std):
+            return torch.randn(shape, generator=gen, dtype=F64) * std
+
+        if leaf in ("norm1", "norm2", "norm1b", "norm2b", "norm"):
+            t = 1.0 + rn(0.3)
+        elif leaf == "conv":
+            t = rn(0.6)
+        elif leaf == "A_log":
+            t = rn(0.7)
+        elif leaf == "dt_bias":
+            t = rn(1.5) - 2.5
+        elif name.endswith("router"):
+            t = rn(2.0 * shape[-1] ** -0.5)
+        elif name.endswith("router.b"):
+            t = rn(0.7)
+        elif leaf == "embed":
+            t = rn(0.4)
+        elif leaf in ("b", "g", "g1"):
+            t = rn(1.5 * shape[-1] ** -0.5)
+        else:
+            t = rn(shape[-1] ** -0.5)
+        w[name] = t.to(torch.bfloat16).to(F64)
+    return w
