@@ -48,6 +48,38 @@ from .. import ops
 from .mixers import _param, linear, linear_f32
 
 
+# rows of one expert's product are rounded up to a multiple of this
+SEGMENT_ROWS = 64
+
+
+def sort_by_expert(h, ids, experts: int):
+    """The rows of h gathered in expert order, SEGMENT_ROWS - 1 more behind
+    them; every (row, choice) pair's place there [T, k]; how many rows each
+    expert has (the step's one host read)."""
+    rows, place, counts = ops.moe_sort_pairs(ids, experts, SEGMENT_ROWS - 1)
+    return h.index_select(0, rows), place, counts.tolist()
+
+
+def expert_products(x, counts: list, weight) -> torch.Tensor:
+    """x: rows in expert order and SEGMENT_ROWS - 1 spare ones; rows of
+    expert e times weight(e). A product's row count is rounded up, so that
+    the library meets few different shapes (it prepares each new one on the
+    host); the rows too many belong to the experts behind, whose products
+    come later and overwrite them, or are spare."""
+    out = None
+    at = 0
+    for e, n in enumerate(counts):
+        if n:
+            w = weight(e)
+            if out is None:
+                out = torch.empty((x.shape[0], w.shape[1]), dtype=x.dtype,
+                                  device=x.device)
+            m = -(-n // SEGMENT_ROWS) * SEGMENT_ROWS
+            torch.mm(x[at:at + m], w, out=out[at:at + m])
+        at += n
+    return out
+
+
 class GLU(nn.Module):
     """W_down act(W_gate x, W_up x); act is one of ops.glu_act's kinds
     ("gelu_tanh": gelu_tanh(gate) * up; "swiglu"; "clamped"). Gate and up
@@ -127,32 +159,12 @@ class GroupedMoE(nn.Module):
             a = ops.glu_act(gu.view(T * E, 2 * ff), "swiglu")
             y = torch.bmm(a.view(T, E, ff).transpose(0, 1), self.w2)
             return ops.moe_mix_seq(y, weights, ids)
-        # (row, expert) pairs sorted by expert: every expert runs two plain
-        # GEMMs on its own contiguous segment, nothing is padded (one host
-        # read of the segment sizes)
-        flat = ids.reshape(-1).long()
-        order = torch.argsort(flat, stable=True)
-        tok = torch.div(order, k, rounding_mode="floor")
-        counts = torch.bincount(flat, minlength=E).tolist()
-        xs = h[tok]
-        gu = torch.empty((T * k, 2 * ff), dtype=h.dtype, device=h.device)
-        at = 0
-        for e, n in enumerate(counts):
-            if n:
-                torch.mm(xs[at:at + n],
-                         self.w13[e * 2 * ff:(e + 1) * 2 * ff].t(),
-                         out=gu[at:at + n])
-            at += n
+        xs, place, counts = sort_by_expert(h, ids, E)
+        gu = expert_products(
+            xs, counts, lambda e: self.w13[e * 2 * ff:(e + 1) * 2 * ff].t())
         a = ops.glu_act(gu, "swiglu")
-        y = torch.empty((T * k, W), dtype=h.dtype, device=h.device)
-        at = 0
-        for e, n in enumerate(counts):
-            if n:
-                torch.mm(a[at:at + n], self.w2[e], out=y[at:at + n])
-            at += n
-        inv = torch.empty_like(order)
-        inv[order] = torch.arange(T * k, device=h.device)
-        return ops.moe_mix_rows_seq(y, weights, inv.view(T, k).to(torch.int32))
+        y = expert_products(a, counts, lambda e: self.w2[e])
+        return ops.moe_mix_rows_seq(y, weights, place)
 
 
 class RoutedMoE(nn.Module):
@@ -202,40 +214,24 @@ class RoutedMoE(nn.Module):
                                              self.weigh_input), self.w_down)
         weights, ids = ops.moe_route_grouped(z, k, 1, 1, self.score,
                                              self.renorm, bias=self.router_b)
-        # (row, expert) pairs sorted by expert: every expert runs two plain
-        # GEMMs on its own contiguous segment (one host read of the sizes)
-        flat = ids.reshape(-1).long()
-        order = torch.argsort(flat, stable=True)
-        tok = torch.div(order, k, rounding_mode="floor")
-        counts = torch.bincount(flat, minlength=E).tolist()
-        xs = h[tok]
-        gu = torch.empty((T * k, 2 * ff), dtype=h.dtype, device=h.device)
-        at = 0
-        for e, n in enumerate(counts):
-            if n:
-                torch.mm(xs[at:at + n],
-                         self.w_gu[e * 2 * ff:(e + 1) * 2 * ff].t(),
-                         out=gu[at:at + n])
-            at += n
-        a = ops.glu_act(gu, "swiglu", row_scale=weights.reshape(-1)[order]
-                        if self.weigh_input else None)
-        y = torch.empty((T * k, self.width), dtype=h.dtype, device=h.device)
-        at = 0
-        for e, n in enumerate(counts):
-            if n:
-                torch.mm(a[at:at + n],
-                         self.w_down[:, e * ff:(e + 1) * ff].t(),
-                         out=y[at:at + n])
-            at += n
-        inv = torch.empty_like(order)
-        inv[order] = torch.arange(T * k, device=h.device)
+        xs, place, counts = sort_by_expert(h, ids, E)
+        gu = expert_products(
+            xs, counts, lambda e: self.w_gu[e * 2 * ff:(e + 1) * 2 * ff].t())
+        row_scale = None
+        if self.weigh_input:
+            row_scale = torch.zeros(gu.shape[0], dtype=torch.float32,
+                                    device=h.device)
+            row_scale[place.reshape(-1).long()] = weights.reshape(-1)
+        a = ops.glu_act(gu, "swiglu", row_scale=row_scale)
+        y = expert_products(
+            a, counts, lambda e: self.w_down[:, e * ff:(e + 1) * ff].t())
         shared = None
         if sff:
             sa = ops.glu_act(linear(h, self.w_gu[E * 2 * ff:]), "swiglu")
             shared = linear(sa, self.w_down[:, E * ff:])
         return ops.moe_mix_rows_seq(y, torch.ones_like(weights)
                                     if self.weigh_input else weights,
-                                    inv.view(T, k).to(torch.int32), shared)
+                                    place, shared)
 
 
 def build_feedforward(mlp: dict, width: int, dtype, arch: str = "") -> nn.Module:

@@ -730,7 +730,9 @@ class HybridForCausalLM(nn.Module):
                                                    "norm2b"):
                 w = 1.0 + rn(0.1)
             elif leaf == "mix.dt_bias":
-                w = rn(0.5) - 1.0
+                # delta-rule channels remember for tens to hundreds of tokens
+                w = (rn(1.0) - 4.0 if self.arr.norm_place == "sandwich"
+                     else rn(0.5) - 1.0)
             elif leaf == "mix.sink":
                 w = rn(1.0)
             elif leaf.startswith("canon"):

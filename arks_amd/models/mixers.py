@@ -570,7 +570,8 @@ class LatentAttention(SplitMixer):
     That form costs kv_rank + rot_dim + kv_rank multiply-adds per (row,
     head, key), against dim + rot_dim + vdim for per-head keys and values,
     and pays for a step of few rows over a long context. A step with a long
-    portion (EXPAND_ROWS rows or more of one sequence) therefore takes the
+    portion (EXPAND_ROWS rows or more of one sequence), or one whose reachable
+    context is hardly longer than its rows (_expand), therefore takes the
     other form: the latents of every sequence's context (with a window: of
     the pages its rows can reach) are gathered from
     the pages and up-projected once into per-head keys and values for the
@@ -580,6 +581,7 @@ class LatentAttention(SplitMixer):
     pad_rows = 64
 
     EXPAND_ROWS = 192
+    EXPAND_MIN_ROWS = 8
 
     def __init__(self, width: int, heads: int, dim: int, rot_dim: int,
                  vdim: int, kv_rank: int, q_rank: int, scale: float,
@@ -645,8 +647,7 @@ class LatentAttention(SplitMixer):
         if self.head_gate:
             at = self.q_rank + rank + R
             gate = p[:, at:at + H]
-        if (batch.max_q_len >= self.EXPAND_ROWS
-                and batch.kv_lens_list is not None):
+        if self._expand(batch):
             self._expanded(q, batch, ckv, gate, out, out_scale)
             return
         # [H, T, D] x [H, D, rank]: the key up-projection applied to q
@@ -664,6 +665,27 @@ class LatentAttention(SplitMixer):
         o = torch.bmm(o_lat.transpose(0, 1), self.uv_t)
         ops.head_gate(o.transpose(0, 1), gate, out.unflatten(-1, (H, V)),
                       out_scale)
+
+    def _expand(self, batch: ForwardBatch) -> bool:
+        """Whether the step takes the per-head form: by the length of its
+        longest portion, or by counting multiply-adds per head — up-projecting
+        every reachable token once, against up-projecting every row's query
+        and result and scoring wider keys."""
+        if batch.kv_lens_list is None or batch.max_q_len < self.EXPAND_MIN_ROWS:
+            return False
+        if batch.max_q_len >= self.EXPAND_ROWS:
+            return True
+        key = ("latent_expand", self.window, self.rank, self.D, self.V)
+        if key not in batch.tile_cache:
+            up = self.rank * (self.D + self.V)
+            wider = 2 * self.rank - self.D - self.V
+            cost = 0
+            for n, rows in zip(batch.kv_lens_list, batch.seq_lens_list):
+                reach = min(n, self.window + rows) if self.window else n
+                seen = min(n - rows / 2, self.window or n)
+                cost += reach * up - rows * (up + seen * wider)
+            batch.tile_cache[key] = cost < 0
+        return batch.tile_cache[key]
 
     def _reachable_pages(self, batch: ForwardBatch, bs: int):
         """(page ids of every sequence's reachable context in sequence
@@ -705,7 +727,8 @@ class LatentAttention(SplitMixer):
         kt = torch.empty((NB, H, bs, D + R), dtype=q.dtype, device=q.device)
         kt[..., :D] = linear(c, self.uk).view(NB, bs, H, D).transpose(1, 2)
         kt[..., D:] = lat[..., rank:]
-        vt = linear(c, self.uv).view(NB, bs, H, V).transpose(1, 2).contiguous()
+        vt = torch.empty((NB, H, bs, V), dtype=q.dtype, device=q.device)
+        vt.copy_(linear(c, self.uv).view(NB, bs, H, V).transpose(1, 2))
         qf = torch.empty((T, H, D + R), dtype=q.dtype, device=q.device)
         ops.latent_query(q, None, batch.positions, self.inv_freq, qf,
                          self.interleaved, self.rot_mag)

@@ -1070,6 +1070,19 @@ def moe_route_grouped(logits, top, groups=1, keep=1, score="softmax",
     return w, ids
 
 
+def moe_sort_pairs(ids, experts, pad=0):
+    """(row, expert) pairs in expert order (ref.moe_sort_pairs) from one
+    launch."""
+    if ids.is_cuda:
+        rows = torch.empty(ids.numel() + pad, dtype=torch.int32,
+                           device=ids.device)
+        place = torch.empty_like(ids)
+        counts = torch.empty(experts, dtype=torch.int32, device=ids.device)
+        if _native_seq().moe_sort_pairs(rows, place, counts, ids):
+            return rows, place, counts
+    return ref.moe_sort_pairs(ids, experts, pad)
+
+
 def moe_mix_seq(y, weights, ids):
     """moe_mix for callers of the sequence-state extension (any float
     dtype of y)."""
@@ -1313,7 +1326,7 @@ def channel_delta(u, decay, beta, gate, rate, dt_bias, norm_w, eps, state,
         _native_seq().channel_delta_scan(
             out, u, decay, beta, gate, rate, dt_bias, norm_w, float(eps),
             ref.DELTA_UNIT_EPS, state, cu_seqlens, seq_lens, state_slots,
-            heads, kv_heads, dim, vdim)
+            heads, kv_heads, dim, vdim, max_q_len)
         return out
     return ref.channel_delta(u, decay, beta, gate, rate, dt_bias, norm_w, eps,
                              state, cu_seqlens, seq_lens, state_slots, heads,

@@ -166,6 +166,9 @@ int arks_seq_moe_route_grouped(void* weights, void* ids, const void* logits,
                                int T, int E, int top, int groups, int keep,
                                int sigmoid, int renorm, void* matrix,
                                const void* bias, hipStream_t stream);
+int arks_seq_moe_sort_pairs(void* row_of_place, void* place, void* counts,
+                            const void* ids, int n, int k, int E, int pad,
+                            hipStream_t stream);
 void arks_seq_moe_mix_rows(void* out, const void* y, const void* weights,
                            const void* rows, int T, int H, int k, int dense,
                            const void* add, int act_f32, hipStream_t stream);
@@ -207,7 +210,7 @@ int arks_seq_channel_delta_scan(
     int gate_f32, const void* rate, const void* dt_bias, const void* norm_w,
     float eps, float unit_eps, void* state, const void* cu,
     const void* seq_lens, const void* slots, int S, int H, int G, int D, int V,
-    int act_f32, hipStream_t stream);
+    int max_rows, int one_row, int act_f32, hipStream_t stream);
 int64_t arks_seq_delta_chunk_floats(int D, int V);
 int arks_seq_delta_chunks_fit(int64_t ldo, int64_t ldu, int64_t ldg,
                               const void* out, const void* u, const void* gate,
@@ -982,6 +985,22 @@ void moe_route_grouped(Tensor weights, Tensor ids, Tensor logits, int64_t top,
   TORCH_CHECK(rc == 0, "routing sizes the kernel does not hold");
 }
 
+// False: more experts than the kernel holds.
+bool moe_sort_pairs(Tensor row_of_place, Tensor place, Tensor counts,
+                    Tensor ids) {
+  check_i32(row_of_place, "row_of_place");
+  check_i32(place, "place");
+  check_i32(counts, "counts");
+  check_i32(ids, "ids");
+  TORCH_CHECK(ids.dim() == 2 && place.sizes() == ids.sizes() &&
+              row_of_place.numel() >= ids.numel());
+  return arks_seq_moe_sort_pairs(
+             row_of_place.data_ptr(), place.data_ptr(), counts.data_ptr(),
+             ids.data_ptr(), (int)ids.numel(), (int)ids.size(1),
+             (int)counts.numel(), (int)(row_of_place.numel() - ids.numel()),
+             current_stream()) == 0;
+}
+
 void moe_mix_common(Tensor out, Tensor y, Tensor weights, Tensor rows,
                     int dense, const OptTensor& add = c10::nullopt) {
   const int f32 = act_flag(y, "y");
@@ -1491,7 +1510,8 @@ void channel_delta_scan(Tensor out, Tensor u, Tensor decay, Tensor beta,
                         Tensor gate, Tensor rate, Tensor dt_bias,
                         Tensor norm_w, double eps, double unit_eps,
                         Tensor state, Tensor cu, Tensor seq_lens, Tensor slots,
-                        int64_t H, int64_t G, int64_t D, int64_t V) {
+                        int64_t H, int64_t G, int64_t D, int64_t V,
+                        int64_t max_rows) {
   const DeltaArgs a = check_delta(out, u, decay, beta, gate, rate, dt_bias,
                                   norm_w, state, H, G, D, V);
   const SeqMeta m = check_meta(cu, seq_lens, &slots, nullptr, 0);
@@ -1500,8 +1520,8 @@ void channel_delta_scan(Tensor out, Tensor u, Tensor decay, Tensor beta,
       beta.data_ptr(), a.ldb, gate.data_ptr(), a.ldg, a.gate_f32,
       rate.data_ptr(), dt_bias.data_ptr(), norm_w.data_ptr(), (float)eps,
       (float)unit_eps, state.data_ptr(), cu.data_ptr(), seq_lens.data_ptr(),
-      slots.data_ptr(), m.S, (int)H, (int)G, (int)D, (int)V, a.f32,
-      current_stream());
+      slots.data_ptr(), m.S, (int)H, (int)G, (int)D, (int)V, (int)max_rows,
+      u.size(0) == m.S ? 1 : 0, a.f32, current_stream());
   TORCH_CHECK(rc == 0, "delta-rule head sizes the kernel does not hold (", D,
               ", ", V, ")");
 }
@@ -1566,6 +1586,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("attention_window_pool", &attention_window_pool);
   m.def("attention_window_pool_mfma", &attention_window_pool_mfma);
   m.def("moe_route_grouped", &moe_route_grouped);
+  m.def("moe_sort_pairs", &moe_sort_pairs);
   m.def("moe_mix", &moe_mix);
   m.def("moe_mix_rows", &moe_mix_rows);
   def_paged_attention(m);

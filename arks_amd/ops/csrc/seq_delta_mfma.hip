@@ -18,9 +18,12 @@
 // Exponents: exp(G_i - G_j) is split at the borders of the 16-row blocks
 // into factors whose exponents are sums of log decays, all <= 0, so nothing
 // overflows and no sums longer than a block are subtracted. Inside a 16-row block
-// exp(c_i) exp(-c_j) is used while the block's total log decay is above
-// MIN_BLOCK_LOG (both factors finite in fp32), else exp(c_i - c_j) per
-// channel, element by element.
+// exp(c_i - c_7) exp(c_7 - c_j), about its middle row, is used while the
+// log decays of either half sum to more than MIN_HALF_LOG (both factors
+// finite in fp32). Stronger decays: pairs of different 4-row groups are split
+// at the last row of j's group (exponents <= 0 again, one pass per group),
+// pairs inside a group about its second row; and where even two rows decay
+// past MIN_HALF_LOG, exp(c_i - c_j) is taken per channel, element by element.
 //
 // Fragments: with k = 4 g + e (g = lane / 16) the operand A of four
 // consecutive MFMAs is row lane % 16, columns 4 g .. 4 g + 3 of a 16x16 tile
@@ -32,8 +35,9 @@
 
 namespace arks {
 
-constexpr int DC = 64;                  // rows per chunk
-constexpr float MIN_BLOCK_LOG = -80.f;  // exp(80) * exp(-80) stay finite
+constexpr int DC = 64;                 // rows per chunk
+constexpr int DELTA_CUS = 256;         // compute units of the chip
+constexpr float MIN_HALF_LOG = -80.f;  // exp(80) and exp(-80) are finite
 
 __device__ __forceinline__ float4v mm16(float4v acc, float4v a, float4v b) {
 #pragma unroll
@@ -68,12 +72,12 @@ __host__ __device__ inline DeltaChunk delta_chunk_layout(int D, int V) {
 }
 
 __host__ __device__ constexpr int delta_prepare_lds(int D) {
-  return 2 * DC * (D + 8) * 2 + DC * (D + 4) * 4 + 14 * 64 * 16 + 4 * D * 4 +
-         (3 * DC + 4) * 4;
+  return 2 * DC * (D + 8) * 2 + DC * (D + 4) * 4 + 10 * 64 * 16 + 4 * D * 4 +
+         (3 * DC + 8) * 4;
 }
 
 template <int KT>
-__global__ __launch_bounds__(256) void delta_chunk_prepare_kernel(
+__global__ __launch_bounds__(256, 2) void delta_chunk_prepare_kernel(
     float* __restrict__ scratch, const bf16* __restrict__ u, int64_t ldu,
     const float* __restrict__ decay, int64_t lda,
     const bf16* __restrict__ beta, int64_t ldb, const float* __restrict__ rate,
@@ -86,13 +90,16 @@ __global__ __launch_bounds__(256) void delta_chunk_prepare_kernel(
   bf16* k_s = reinterpret_cast<bf16*>(smem);           // [DC][LK]
   bf16* q_s = k_s + DC * LK;                           // [DC][LK]
   float* c_s = reinterpret_cast<float*>(q_s + DC * LK);  // [DC][LC]
-  float4v* l_s = reinterpret_cast<float4v*>(c_s + DC * LC);  // [10][64]
-  float4v* inv_s = l_s + 10 * 64;                      // [4][64]
-  float* tot_s = reinterpret_cast<float*>(inv_s + 4 * 64);  // [4][D]
+  // L's blocks below the diagonal, then the diagonal ones, which their
+  // inverses replace
+  float4v* l_s = reinterpret_cast<float4v*>(c_s + DC * LC);  // [6 + 4][64]
+  float4v* inv_s = l_s + 6 * 64;                       // [4][64]
+  float* tot_s = reinterpret_cast<float*>(l_s + 10 * 64);  // [4][D]
   float* rk_s = tot_s + 4 * D;                         // [DC]
   float* rq_s = rk_s + DC;                             // [DC]
   float* b_s = rq_s + DC;                              // [DC]
   float* min_s = b_s + DC;                             // [4]
+  float* pair_s = min_s + 4;                           // [4]
   const int h = blockIdx.x, chunk = blockIdx.y;
   const int t0 = cu[chunk], n = min(cu[chunk + 1] - t0, DC);
   const int I = threadIdx.x / 64, lane = threadIdx.x % 64;
@@ -101,18 +108,34 @@ __global__ __launch_bounds__(256) void delta_chunk_prepare_kernel(
   const DeltaChunk lay = delta_chunk_layout(D, V);
   float* base = scratch + ((int64_t)chunk * H + h) * lay.total;
 
-  // ---- rows of block I: raw q, k, their unit factors, log decays
+  // ---- rows of block I: raw q, k, their unit factors, log decays. Loads
+  // are of rows that exist (the last one again past the end) and are not
+  // branched around, so that they are all in flight together
+  constexpr int DL = (D + 63) / 64;  // channels per lane
+  float dec[DL][16];
+#pragma unroll
+  for (int j = 0; j < DL; ++j)
+#pragma unroll
+    for (int r = 0; r < 16; ++r)
+      dec[j][r] = decay[(int64_t)(t0 + min(16 * I + r, n - 1)) * lda +
+                        (int64_t)h * D + min(lane + 64 * j, D - 1)];
+  ushort8 qin[4], kin[4];
+  const bool live = m * 8 < D;
+#pragma unroll
+  for (int it = 0; it < 4; ++it) {  // 16 lanes per row
+    const bf16* qr = u + (int64_t)(t0 + min(16 * I + 4 * it + g, n - 1)) * ldu +
+                     (int64_t)gk * D + min(m * 8, D - 8);
+    qin[it] = *reinterpret_cast<const ushort8*>(qr);
+    kin[it] = *reinterpret_cast<const ushort8*>(qr + (int64_t)G * D);
+  }
 #pragma unroll
   for (int it = 0; it < 4; ++it) {
-    const int row = 16 * I + 4 * it + g;  // 16 lanes per row
-    ushort8 qv, kv;
+    const int row = 16 * I + 4 * it + g;
+    ushort8 qv = qin[it], kv = kin[it];
 #pragma unroll
-    for (int e = 0; e < 8; ++e) { qv[e] = 0; kv[e] = 0; }
-    const bool live = m * 8 < D;
-    if (live && row < n) {
-      const bf16* qr = u + (int64_t)(t0 + row) * ldu + (int64_t)gk * D + m * 8;
-      qv = *reinterpret_cast<const ushort8*>(qr);
-      kv = *reinterpret_cast<const ushort8*>(qr + (int64_t)G * D);
+    for (int e = 0; e < 8; ++e) {
+      qv[e] = live && row < n ? qv[e] : (uint16_t)0;
+      kv[e] = live && row < n ? kv[e] : (uint16_t)0;
     }
     float qq = 0.f, kk = 0.f;
 #pragma unroll
@@ -140,23 +163,32 @@ __global__ __launch_bounds__(256) void delta_chunk_prepare_kernel(
   }
   {
     const float rt = rate[h];
-    float lowest = 0.f;
-    for (int d = lane; d < D; d += 64) {
-      const float db = dt_bias[(int64_t)h * D + d];
-      float c = 0.f;
+    float lowest = 0.f, pair = 0.f;
+#pragma unroll
+    for (int j = 0; j < DL; ++j) {
+      const int d = lane + 64 * j;
+      const float db = dt_bias[(int64_t)h * D + min(d, D - 1)];
+      float c = 0.f, mid = 0.f, prev2 = 0.f;
 #pragma unroll
       for (int r = 0; r < 16; ++r) {
-        const int row = 16 * I + r;
-        if (row < n)
-          c -= rt * softplus_fast(
-                        decay[(int64_t)(t0 + row) * lda + (int64_t)h * D + d] + db);
-        c_s[row * LC + d] = c;
+        const float step = rt * softplus_fast(dec[j][r] + db);
+        c -= 16 * I + r < n ? step : 0.f;
+        if (d < D) c_s[(16 * I + r) * LC + d] = c;
+        if (r == 7) mid = c;
+        if (r % 2) {  // two rows' log decay
+          pair = fminf(pair, c - prev2);
+          prev2 = c;
+        }
       }
-      tot_s[I * D + d] = c;
-      lowest = fminf(lowest, c);
+      if (d < D) tot_s[I * D + d] = c;
+      lowest = fminf(lowest, fminf(mid, c - mid));
     }
     lowest = -wave_reduce_max(-lowest);
-    if (lane == 0) min_s[I] = lowest;
+    pair = -wave_reduce_max(-pair);
+    if (lane == 0) {
+      min_s[I] = lowest;
+      pair_s[I] = pair;
+    }
   }
   __syncthreads();
 
@@ -171,44 +203,105 @@ __global__ __launch_bounds__(256) void delta_chunk_prepare_kernel(
       const ushort4v kr = *reinterpret_cast<const ushort4v*>(k_s + row * LK + d);
       const ushort4v qr = *reinterpret_cast<const ushort4v*>(q_s + row * LK + d);
       const float4v c = *reinterpret_cast<const float4v*>(c_s + row * LC + d);
-      float4v qg;
+      float4v qg, pre = {0.f, 0.f, 0.f, 0.f};
+      for (int M = 0; M < I; ++M)
+        pre += *reinterpret_cast<const float4v*>(tot_s + M * D + d);
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
         const float x = __expf(c[e]);
         kI[kt][e] = bf16_bits_to_float(kr[e]) * rk * x;
         qI[kt][e] = bf16_bits_to_float(qr[e]) * rq * x;
-        float pre = 0.f;
-        for (int M = 0; M < I; ++M) pre += tot_s[M * D + d + e];
-        qg[e] = qI[kt][e] * __expf(pre);
+        qg[e] = qI[kt][e] * __expf(pre[e]);
       }
       *reinterpret_cast<float4v*>(base + lay.Q + ((I * KT + kt) * 64 + lane) * 4) = qg;
     }
     const float bI = b_s[row];
+    const bool split = min_s[I] > MIN_HALF_LOG;
+    const bool groups = pair_s[I] > MIN_HALF_LOG;
     for (int J = 0; J <= I; ++J) {
       float4v kk = {0.f, 0.f, 0.f, 0.f}, qk = {0.f, 0.f, 0.f, 0.f};
       const int rj = 16 * J + m;
       const float rkj = rk_s[rj];
-      if (J < I || min_s[I] > MIN_BLOCK_LOG) {
+      if (J < I) {
 #pragma unroll
         for (int kt = 0; kt < KT; ++kt) {
           const int d = 16 * kt + 4 * g;
           const ushort4v kr = *reinterpret_cast<const ushort4v*>(k_s + rj * LK + d);
-          const float4v c = *reinterpret_cast<const float4v*>(c_s + rj * LC + d);
+          float4v x = -*reinterpret_cast<const float4v*>(c_s + rj * LC + d);
+          for (int M = J; M < I; ++M)
+            x += *reinterpret_cast<const float4v*>(tot_s + M * D + d);
           float4v a;
 #pragma unroll
-          for (int e = 0; e < 4; ++e) {
-            float x = -c[e];
-            if (J < I) {
-              for (int M = J; M < I; ++M) x += tot_s[M * D + d + e];
-              x = fminf(x, 0.f);
-            }
-            a[e] = bf16_bits_to_float(kr[e]) * rkj * __expf(x);
-          }
+          for (int e = 0; e < 4; ++e)
+            a[e] = bf16_bits_to_float(kr[e]) * rkj * __expf(fminf(x[e], 0.f));
           kk = mm16(kk, a, kI[kt]);
           qk = mm16(qk, a, qI[kt]);
         }
+      } else if (split) {
+#pragma unroll
+        for (int kt = 0; kt < KT; ++kt) {
+          const int d = 16 * kt + 4 * g;
+          const ushort4v kr = *reinterpret_cast<const ushort4v*>(k_s + row * LK + d);
+          const ushort4v qr = *reinterpret_cast<const ushort4v*>(q_s + row * LK + d);
+          const float4v x = *reinterpret_cast<const float4v*>(c_s + row * LC + d) -
+                            *reinterpret_cast<const float4v*>(c_s + (16 * I + 7) * LC + d);
+          float4v a, kd, qd;
+#pragma unroll
+          for (int e = 0; e < 4; ++e) {
+            const float up = __expf(x[e]);
+            a[e] = bf16_bits_to_float(kr[e]) * rk * __expf(-x[e]);
+            kd[e] = bf16_bits_to_float(kr[e]) * rk * up;
+            qd[e] = bf16_bits_to_float(qr[e]) * rq * up;
+          }
+          kk = mm16(kk, a, kd);
+          qk = mm16(qk, a, qd);
+        }
+      } else if (groups) {
+        // lane's row m as i (operand B) and as j (operand A). Pass b < 3:
+        // the border behind group b, j in group b, i in a later group; pass
+        // 3: i and j of one group about its second row, what it says about
+        // other pairs is dropped
+        float4v kk3 = {0.f, 0.f, 0.f, 0.f}, qk3 = {0.f, 0.f, 0.f, 0.f};
+        const int mg = m / 4;
+        for (int b = 0; b < 4; ++b) {
+          const int ref = 16 * I + (b < 3 ? 4 * b + 3 : 4 * mg + 1);
+          const float use_j = b == 3 || mg == b ? rk : 0.f;
+          const float use_i = b == 3 || mg > b ? 1.f : 0.f;
+          float4v k1 = {0.f, 0.f, 0.f, 0.f}, q1 = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+          for (int kt = 0; kt < KT; ++kt) {
+            const int d = 16 * kt + 4 * g;
+            const ushort4v kr = *reinterpret_cast<const ushort4v*>(k_s + row * LK + d);
+            const ushort4v qr = *reinterpret_cast<const ushort4v*>(q_s + row * LK + d);
+            const float4v x = *reinterpret_cast<const float4v*>(c_s + row * LC + d) -
+                              *reinterpret_cast<const float4v*>(c_s + ref * LC + d);
+            float4v a, kd, qd;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+              // a row that is not used keeps a finite factor
+              const float up = use_i * __expf(fminf(x[e], 80.f));
+              a[e] = bf16_bits_to_float(kr[e]) * use_j * __expf(fminf(-x[e], 80.f));
+              kd[e] = bf16_bits_to_float(kr[e]) * rk * up;
+              qd[e] = bf16_bits_to_float(qr[e]) * rq * up;
+            }
+            k1 = mm16(k1, a, kd);
+            q1 = mm16(q1, a, qd);
+          }
+          if (b < 3) {
+            kk += k1;
+            qk += q1;
+          } else {
+            kk3 = k1;
+            qk3 = q1;
+          }
+        }
+        // lane holds (i = m, j = 4 g + r): one group where g == m / 4
+        if (g == mg) {
+          kk = kk3;
+          qk = qk3;
+        }
       } else {
-        // strong decays: element (i = m, j = 4 g + r) channel by channel
+        // element (i = m, j = 4 g + r) channel by channel
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           const int j = 16 * I + 4 * g + r;
@@ -269,12 +362,24 @@ __global__ __launch_bounds__(256) void delta_chunk_prepare_kernel(
 
   // ---- columns of [K~ | V] through the substitution, 16 at a time
   const int VT = V / 16;
+  // q is not needed any more: a 16x16 tile per wave to turn -W's tiles from
+  // result layout into operand layout
+  float* turn = reinterpret_cast<float*>(q_s) + I * 16 * 20;
   for (int tile = I; tile < KT + VT; tile += 4) {
     const bool is_k = tile < KT;
     const int ct = is_k ? tile : tile - KT;
     const int d = 16 * ct + m;
-    float4v X[4];
+    float4v X[4], vin[4];
     float pre = 0.f;
+    if (!is_k) {
+      const bf16* vp = u + (int64_t)t0 * ldu + 2 * (int64_t)G * D + (int64_t)h * V + d;
+#pragma unroll
+      for (int B = 0; B < 4; ++B)
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          vin[B][r] = bf16_bits_to_float(
+              vp[(int64_t)min(16 * B + 4 * g + r, n - 1) * ldu]);
+    }
 #pragma unroll
     for (int B = 0; B < 4; ++B) {
       float4v rhs;
@@ -285,9 +390,8 @@ __global__ __launch_bounds__(256) void delta_chunk_prepare_kernel(
         if (is_k) {
           x = bf16_bits_to_float(k_s[row * LK + d]) * rk_s[row] *
               __expf(pre + c_s[row * LC + d]);
-        } else if (row < n) {
-          x = bf16_bits_to_float(
-              u[(int64_t)(t0 + row) * ldu + 2 * (int64_t)G * D + (int64_t)h * V + d]);
+        } else {
+          x = vin[B][r];  // rows past the end have b_s 0
         }
         rhs[r] = x * b_s[row];
       }
@@ -300,11 +404,13 @@ __global__ __launch_bounds__(256) void delta_chunk_prepare_kernel(
       const float4v zero = {0.f, 0.f, 0.f, 0.f};
       X[B] = mm16(zero, inv_s[B * 64 + lane], rhs);
       if (is_k) {
-        // -W as an operand A: element (row, column d) in its lane's place
-        float* dst = base + lay.W + (B * KT + ct) * 256;
+        // within one wave: LDS serves its accesses in order
 #pragma unroll
-        for (int r = 0; r < 4; ++r)
-          dst[(4 * g + r + 16 * (m / 4)) * 4 + m % 4] = -X[B][r];
+        for (int r = 0; r < 4; ++r) turn[(4 * g + r) * 20 + m] = -X[B][r];
+        __builtin_amdgcn_wave_barrier();
+        *reinterpret_cast<float4v*>(base + lay.W + ((B * KT + ct) * 64 + lane) * 4) =
+            *reinterpret_cast<const float4v*>(turn + m * 20 + 4 * g);
+        __builtin_amdgcn_wave_barrier();
       } else {
         *reinterpret_cast<float4v*>(base + lay.U + ((ct * 4 + B) * 64 + lane) * 4) = X[B];
       }
@@ -331,150 +437,192 @@ __global__ __launch_bounds__(256) void delta_chunk_prepare_kernel(
                              tot_s[3 * D + d]);
 }
 
-// One block per (sequence, head, 16 value columns). Wave w owns the state's
-// 16-row tiles w, w + 4, ... (operands B as they are), sums its part of
-// [-W; Q~] S0 and rows 16 w .. 16 w + 15 of U and O.
-template <int KT>
-__global__ __launch_bounds__(256) void delta_chunk_scan_kernel(
+// One block per (sequence, head, NC * 16 value columns); a sequence's chunks
+// are DC rows each, the last one what is left. Wave w computes rows
+// 16 w .. 16 w + 15 of -W S0, Q~ S0, U and O, and owns the state's 16-row
+// tiles w, w + 4, ...; state and U tiles pass between the waves through LDS in
+// the layout they have in registers.
+template <int KT, int NC>
+__global__ __launch_bounds__(256, 2) void delta_chunk_scan_kernel(
     float* __restrict__ o, const float* __restrict__ scratch,
     float* __restrict__ state, const int* __restrict__ chunk_off,
-    const int* __restrict__ chunk_cu, const int* __restrict__ cu,
-    const int* __restrict__ seq_lens, const int* __restrict__ slots, int H,
-    int V, int groups) {
+    const int* __restrict__ cu, const int* __restrict__ seq_lens,
+    const int* __restrict__ slots, int H, int V, int groups) {
   constexpr int D = 16 * KT;
   constexpr int RT = (KT + 3) / 4;
-  __shared__ float4v part_s[4][8][64];
-  __shared__ float4v u_s[4][64];
+  __shared__ float4v s_s[NC][KT][64];
+  __shared__ float4v u_s[NC][4][64];
   // the column blocks of one (sequence, head) sit on one XCD, whose L2
   // then reads the chunk operands once for all of them
-  const int VT = V / 16;
-  const int group = (blockIdx.x / 8 / VT) * 8 + blockIdx.x % 8;
-  const int ct = (blockIdx.x / 8) % VT;
+  const int VB = V / (16 * NC);
+  const int group = (blockIdx.x / 8 / VB) * 8 + blockIdx.x % 8;
+  const int ct = (blockIdx.x / 8) % VB * NC;  // first 16-column tile
   if (group >= groups) return;
   const int s = group / H, h = group % H;
   const int c_begin = chunk_off[s], c_end = chunk_off[s + 1];
   if (c_begin == c_end) return;
-  const int w = threadIdx.x / 64, lane = threadIdx.x % 64;
+  const int w = __builtin_amdgcn_readfirstlane(threadIdx.x / 64);
+  const int lane = threadIdx.x % 64;
   const int g = lane / 16, m = lane % 16;
-  const int start = seq_lens[s] - (cu[s + 1] - cu[s]);
+  const int row0 = cu[s], row_end = cu[s + 1];
+  const int start = seq_lens[s] - (row_end - row0);
   const int slot = slots[s];
   float* sp = state + ((int64_t)(slot < 0 ? 0 : slot) * H + h) * D * V + 16 * ct + m;
   const DeltaChunk lay = delta_chunk_layout(D, V);
   const int64_t step = (int64_t)H * lay.total;
   const float* base = scratch + ((int64_t)c_begin * H + h) * lay.total;
-  float4v S[RT];
-#pragma unroll
-  for (int i = 0; i < RT; ++i) {
-    const int rt = w + 4 * i;
-#pragma unroll
-    for (int r = 0; r < 4; ++r)
-      S[i][r] = rt < KT && start > 0 && slot >= 0
-                    ? sp[(int64_t)(16 * rt + 4 * g + r) * V] : 0.f;
-  }
+  // whether tile w + 4 i exists: known at compile time for whole rounds
+  auto mine = [&](int i) { return KT % 4 == 0 || w + 4 * i < KT; };
   const float4v zero = {0.f, 0.f, 0.f, 0.f};
-  float4v wf[RT][4], qf[RT][4];
-  auto load_wq = [&](const float* b) {
+  float4v S[NC][RT];
 #pragma unroll
-    for (int i = 0; i < RT; ++i) {
-      const int kt = w + 4 * i;
-      if (kt < KT) {
-#pragma unroll
-        for (int t = 0; t < 4; ++t) {
-          wf[i][t] = *reinterpret_cast<const float4v*>(b + lay.W + ((t * KT + kt) * 64 + lane) * 4);
-          qf[i][t] = *reinterpret_cast<const float4v*>(b + lay.Q + ((t * KT + kt) * 64 + lane) * 4);
-        }
-      }
-    }
-  };
-  load_wq(base);
-  for (int c = c_begin; c < c_end; ++c, base += step) {
-    // this chunk's remaining operands, used after the first barrier
-    float4v kf[RT][4], eg[RT], af[4], u0;
+  for (int c = 0; c < NC; ++c)
 #pragma unroll
     for (int i = 0; i < RT; ++i) {
       const int rt = w + 4 * i;
-      if (rt < KT) {
 #pragma unroll
-        for (int t = 0; t < 4; ++t)
-          kf[i][t] = *reinterpret_cast<const float4v*>(base + lay.K + ((rt * 4 + t) * 64 + lane) * 4);
-        eg[i] = *reinterpret_cast<const float4v*>(base + lay.E + 16 * rt + 4 * g);
+      for (int r = 0; r < 4; ++r)
+        S[c][i][r] = mine(i) && start > 0 && slot >= 0
+                         ? sp[(int64_t)(16 * rt + 4 * g + r) * V + 16 * c] : 0.f;
+      if (mine(i)) s_s[c][rt][lane] = S[c][i];
+    }
+  // this wave's operands of one chunk. Each is loaded for the next chunk as
+  // soon as its last product has been issued, so that a load has a whole
+  // chunk's time and the loads are spread among the products; the scheduling
+  // barriers keep them there.
+  float4v xw[KT], xq[KT], xk[RT][4], xe[RT], xa[4], xu[NC];
+  auto load_wq = [&](const float* b, int kt) {
+    xw[kt] = *reinterpret_cast<const float4v*>(b + lay.W + ((w * KT + kt) * 64 + lane) * 4);
+    xq[kt] = *reinterpret_cast<const float4v*>(b + lay.Q + ((w * KT + kt) * 64 + lane) * 4);
+  };
+  auto load_u = [&](const float* b, int c) {
+    xu[c] = *reinterpret_cast<const float4v*>(b + lay.U + (((ct + c) * 4 + w) * 64 + lane) * 4);
+  };
+  auto load_a = [&](const float* b, int J) {
+    xa[J] = *reinterpret_cast<const float4v*>(b + lay.A + ((w * 4 + min(J, w)) * 64 + lane) * 4);
+  };
+  auto load_k = [&](const float* b, int i, int t) {
+    if (mine(i))
+      xk[i][t] = *reinterpret_cast<const float4v*>(b + lay.K + (((w + 4 * i) * 4 + t) * 64 + lane) * 4);
+  };
+  auto load_e = [&](const float* b, int i) {
+    if (mine(i))
+      xe[i] = *reinterpret_cast<const float4v*>(b + lay.E + 16 * (w + 4 * i) + 4 * g);
+  };
+#pragma unroll
+  for (int kt = 0; kt < KT; ++kt) load_wq(base, kt);
+#pragma unroll
+  for (int c = 0; c < NC; ++c) load_u(base, c);
+#pragma unroll
+  for (int J = 0; J < 4; ++J) load_a(base, J);
+#pragma unroll
+  for (int i = 0; i < RT; ++i) {
+    load_e(base, i);
+#pragma unroll
+    for (int t = 0; t < 4; ++t) load_k(base, i, t);
+  }
+  const int chunks = c_end - c_begin;
+  __syncthreads();
+  for (int n = 0; n < chunks; ++n) {
+    const float* next = base + min(n + 1, chunks - 1) * step;
+    // two accumulators per product, so that no MFMA waits for the one
+    // before it
+    float4v aw[NC][2], aq[NC][2];
+#pragma unroll
+    for (int c = 0; c < NC; ++c)
+#pragma unroll
+      for (int p = 0; p < 2; ++p) { aw[c][p] = zero; aq[c][p] = zero; }
+#pragma unroll
+    for (int kt = 0; kt < KT; kt += 2) {
+      float4v b[NC][2];
+#pragma unroll
+      for (int c = 0; c < NC; ++c)
+#pragma unroll
+        for (int p = 0; p < 2; ++p) b[c][p] = s_s[c][kt + p][lane];
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+#pragma unroll
+        for (int p = 0; p < 2; ++p)
+#pragma unroll
+          for (int c = 0; c < NC; ++c) {
+            aw[c][p] = __builtin_amdgcn_mfma_f32_16x16x4f32(xw[kt + p][e], b[c][p][e], aw[c][p], 0, 0, 0);
+            aq[c][p] = __builtin_amdgcn_mfma_f32_16x16x4f32(xq[kt + p][e], b[c][p][e], aq[c][p], 0, 0, 0);
+          }
+      load_wq(next, kt);
+      load_wq(next, kt + 1);
+      __builtin_amdgcn_sched_barrier(0);
+    }
+    float4v ow[NC];
+#pragma unroll
+    for (int c = 0; c < NC; ++c) {
+      u_s[c][w][lane] = xu[c] + aw[c][0] + aw[c][1];
+      ow[c] = aq[c][0] + aq[c][1];
+      load_u(next, c);
+    }
+    __syncthreads();
+    float4v ub[NC][4];
+#pragma unroll
+    for (int c = 0; c < NC; ++c)
+#pragma unroll
+      for (int t = 0; t < 4; ++t) ub[c][t] = u_s[c][t][lane];
+#pragma unroll
+    for (int i = 0; i < RT; ++i)
+      if (mine(i)) {
+#pragma unroll
+        for (int c = 0; c < NC; ++c) S[c][i] *= xe[i];
+        load_e(next, i);
       }
+#pragma unroll
+    for (int t = 0; t < 4; ++t) {
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+#pragma unroll
+        for (int i = 0; i < RT; ++i)
+          if (mine(i)) {
+#pragma unroll
+            for (int c = 0; c < NC; ++c)
+              S[c][i] = __builtin_amdgcn_mfma_f32_16x16x4f32(xk[i][t][e], ub[c][t][e], S[c][i], 0, 0, 0);
+          }
+#pragma unroll
+      for (int i = 0; i < RT; ++i) load_k(next, i, t);
+      __builtin_amdgcn_sched_barrier(0);
     }
 #pragma unroll
-    for (int J = 0; J < 4; ++J)
-      af[J] = J <= w ? *reinterpret_cast<const float4v*>(base + lay.A + ((w * 4 + J) * 64 + lane) * 4)
-                     : zero;
-    u0 = *reinterpret_cast<const float4v*>(base + lay.U + ((ct * 4 + w) * 64 + lane) * 4);
-    const int t0 = chunk_cu[c];
-    const int n = chunk_cu[c + 1] - t0;
-
-    float4v aw[4], aq[4];
+    for (int c = 0; c < NC; ++c)
 #pragma unroll
-    for (int t = 0; t < 4; ++t) { aw[t] = zero; aq[t] = zero; }
+      for (int i = 0; i < RT; ++i)
+        if (mine(i)) s_s[c][w + 4 * i][lane] = S[c][i];
+    // the rows' own part of O: nobody waits for it
 #pragma unroll
-    for (int i = 0; i < RT; ++i) {
-      if (w + 4 * i < KT) {
-        // independent accumulators take turns, so that no MFMA waits for
-        // the one before it
+    for (int t = 0; t < 4; ++t)
+      if (t <= w) {
 #pragma unroll
         for (int e = 0; e < 4; ++e)
 #pragma unroll
-          for (int t = 0; t < 4; ++t) {
-            aw[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(wf[i][t][e], S[i][e], aw[t], 0, 0, 0);
-            aq[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(qf[i][t][e], S[i][e], aq[t], 0, 0, 0);
-          }
+          for (int c = 0; c < NC; ++c)
+            ow[c] = __builtin_amdgcn_mfma_f32_16x16x4f32(xa[t][e], ub[c][t][e], ow[c], 0, 0, 0);
       }
-    }
 #pragma unroll
-    for (int t = 0; t < 4; ++t) {
-      part_s[w][t][lane] = aw[t];
-      part_s[w][4 + t][lane] = aq[t];
-    }
-    if (c + 1 < c_end) load_wq(base + step);
+    for (int J = 0; J < 4; ++J) load_a(next, J);
+    const int t0 = row0 + n * DC + 16 * w + 4 * g;
+#pragma unroll
+    for (int c = 0; c < NC; ++c)
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+        if (t0 + r < row_end)
+          o[((int64_t)(t0 + r) * H + h) * V + 16 * (ct + c) + m] = ow[c][r];
     __syncthreads();
-    float4v uw = u0, ow = zero;
-#pragma unroll
-    for (int p = 0; p < 4; ++p) {
-      uw += part_s[p][w][lane];
-      ow += part_s[p][4 + w][lane];
-    }
-    u_s[w][lane] = uw;
-    __syncthreads();
-    float4v ub[4];
-#pragma unroll
-    for (int t = 0; t < 4; ++t) ub[t] = u_s[t][lane];
-#pragma unroll
-    for (int i = 0; i < RT; ++i)
-      if (w + 4 * i < KT) S[i] *= eg[i];
-#pragma unroll
-    for (int t = 0; t < 4; ++t) {
-#pragma unroll
-      for (int e = 0; e < 4; ++e) {
-#pragma unroll
-        for (int i = 0; i < RT; ++i)
-          if (w + 4 * i < KT)
-            S[i] = __builtin_amdgcn_mfma_f32_16x16x4f32(kf[i][t][e], ub[t][e], S[i], 0, 0, 0);
-        if (t <= w)
-          ow = __builtin_amdgcn_mfma_f32_16x16x4f32(af[t][e], ub[t][e], ow, 0, 0, 0);
-      }
-    }
-#pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int row = 16 * w + 4 * g + r;
-      if (row < n)
-        o[((int64_t)(t0 + row) * H + h) * V + 16 * ct + m] = ow[r];
-    }
   }
   if (slot >= 0) {
 #pragma unroll
-    for (int i = 0; i < RT; ++i) {
-      const int rt = w + 4 * i;
-      if (rt < KT) {
+    for (int c = 0; c < NC; ++c)
 #pragma unroll
-        for (int r = 0; r < 4; ++r)
-          sp[(int64_t)(16 * rt + 4 * g + r) * V] = S[i][r];
-      }
-    }
+      for (int i = 0; i < RT; ++i)
+        if (mine(i)) {
+#pragma unroll
+          for (int r = 0; r < 4; ++r)
+            sp[(int64_t)(16 * (w + 4 * i) + 4 * g + r) * V + 16 * c] = S[c][i][r];
+        }
   }
 }
 
@@ -555,10 +703,17 @@ static void launch_delta_chunks(float* o, float* scratch, const void* u,
                      (const float*)rate, (const float*)dt_bias, chunk_cu, H, G,
                      V, unit_eps);
   const int groups = S * H;
-  hipLaunchKernelGGL((delta_chunk_scan_kernel<KT>),
-                     dim3((groups + 7) / 8 * 8 * (V / 16)), dim3(256), 0,
-                     stream, o, scratch, (float*)state, chunk_off, chunk_cu, cu,
-                     seq_lens, slots, H, V, groups);
+  // 32 columns a block (half the operand traffic per column) once that
+  // still gives every CU a block
+  const int nc = V % 32 == 0 && (int64_t)groups * (V / 32) >= DELTA_CUS ? 2 : 1;
+  const dim3 grid((groups + 7) / 8 * 8 * (V / (16 * nc)));
+#define SC(NC)                                                               \
+  hipLaunchKernelGGL((delta_chunk_scan_kernel<KT, NC>), grid, dim3(256), 0,  \
+                     stream, o, scratch, (float*)state, chunk_off, cu,       \
+                     seq_lens, slots, H, V, groups)
+  if (nc == 2) SC(2);
+  else SC(1);
+#undef SC
 }
 
 }  // namespace arks

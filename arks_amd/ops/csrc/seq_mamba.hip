@@ -82,8 +82,35 @@ __global__ __launch_bounds__(256) void causal_conv_silu_vec8_kernel(
       for (int e = 0; e < 4; ++e) { wv[j][e] = w0[e]; wv[j][4 + e] = w1[e]; }
     }
   }
-  const int t_end = min(T, (int)(blockIdx.x + 1) * rpt);
-  for (int t = blockIdx.x * rpt; t < t_end; ++t) {
+  const int t_begin = blockIdx.x * rpt;
+  const int t_end = min(T, t_begin + rpt);
+  if (taps == 4 && rpt == CONV_RPT && t_end - t_begin == CONV_RPT) {
+    // rows of one sequence with all their inputs in this step (uniform over
+    // the block): every row is loaded once, all loads in flight together
+    const SeqRow r = seq_row(t_begin, token_seq, cu, seq_lens, slots);
+    if (t_begin - 3 >= r.first_row && t_end <= r.first_row + r.rows) {
+      ushort8 in[CONV_RPT + 3];
+#pragma unroll
+      for (int i = 0; i < CONV_RPT + 3; ++i)
+        in[i] = *reinterpret_cast<const ushort8*>(
+            x + (int64_t)(t_begin - 3 + i) * ldx + c);
+#pragma unroll
+      for (int i = 0; i < CONV_RPT; ++i) {
+        ushort8 o;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+          float acc = bv[e];
+#pragma unroll
+          for (int j = 0; j < 4; ++j)
+            acc += wv[j][e] * bf16_bits_to_float(in[i + j][e]);
+          o[e] = float_to_bf16_bits(acc / (1.f + __expf(-acc)));
+        }
+        *reinterpret_cast<ushort8*>(out + (int64_t)(t_begin + i) * C + c) = o;
+      }
+      return;
+    }
+  }
+  for (int t = t_begin; t < t_end; ++t) {
     const SeqRow r = seq_row(t, token_seq, cu, seq_lens, slots);
     const int i = t - r.first_row;
     const bool has_state = r.start > 0 && r.slot >= 0;

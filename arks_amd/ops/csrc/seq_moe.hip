@@ -10,6 +10,8 @@
 //       renorm is off. Ties go to the lower index (groups and experts).
 //       matrix (optional, [T, E]): the row's weights at the experts it uses,
 //       0 elsewhere.
+//   moe_sort_pairs  (row, expert) pairs in expert order, stable: the row of
+//       every sorted place, every pair's place, the pairs per expert
 //   moe_mix_rows  out[t] = sum_j w[t][j] * y[row(t, j)], row given, or
 //       ids[t][j] * T + t for dense per-expert outputs y [E, T, H].
 #include "seq_common.h"
@@ -118,6 +120,78 @@ __global__ __launch_bounds__(64) void moe_route_grouped_kernel(
   }
 }
 
+// Stable counting sort in one block. Wave w owns the w-th run of pairs; its
+// pairs of expert e go to a run of places of their own, in order: a lane's
+// place inside a group of 64 pairs is the number of lower lanes with the same
+// expert, found by intersecting ballots of the expert's bits.
+constexpr int SORT_WAVES = 16;
+constexpr int SORT_MAX_E = 512;
+
+__global__ __launch_bounds__(64 * SORT_WAVES) void moe_sort_pairs_kernel(
+    int* __restrict__ row_of_place, int* __restrict__ place,
+    int* __restrict__ counts, const int* __restrict__ ids, int n, int k, int E,
+    int pad) {
+  extern __shared__ int at_s[];  // [SORT_WAVES][E]: next free place
+  __shared__ int first_s[SORT_MAX_E];
+  const int w = threadIdx.x / 64, lane = threadIdx.x % 64;
+  const int per = (n + SORT_WAVES * 64 - 1) / (SORT_WAVES * 64) * 64;
+  const int lo = min(w * per, n), hi = min(lo + per, n);
+  for (int i = threadIdx.x; i < SORT_WAVES * E; i += blockDim.x) at_s[i] = 0;
+  for (int i = threadIdx.x; i < pad; i += blockDim.x) row_of_place[n + i] = 0;
+  __syncthreads();
+  for (int i = lo + lane; i < hi; i += 64) atomicAdd(&at_s[w * E + ids[i]], 1);
+  __syncthreads();
+  for (int e = threadIdx.x; e < E; e += blockDim.x) {
+    int sum = 0;
+    for (int v = 0; v < SORT_WAVES; ++v) {
+      const int c = at_s[v * E + e];
+      at_s[v * E + e] = sum;
+      sum += c;
+    }
+    counts[e] = sum;
+    first_s[e] = sum;
+  }
+  __syncthreads();
+  if (w == 0) {  // exclusive sum over the experts, 64 at a time
+    int before = 0;
+    for (int e0 = 0; e0 < E; e0 += 64) {
+      const int c = e0 + lane < E ? first_s[e0 + lane] : 0;
+      int sum = c;
+#pragma unroll
+      for (int off = 1; off < 64; off <<= 1) {
+        const int v = __shfl_up(sum, off, 64);
+        if (lane >= off) sum += v;
+      }
+      if (e0 + lane < E) first_s[e0 + lane] = before + sum - c;
+      before += __shfl(sum, 63, 64);
+    }
+  }
+  __syncthreads();
+  const int bits = 32 - __clz(max(E - 1, 1));
+  volatile int* next_s = at_s + w * E;  // written by other lanes of the wave
+  for (int i0 = lo; i0 < hi; i0 += 64) {
+    const int i = i0 + lane;
+    const bool live = i < hi;
+    const int e = live ? ids[i] : 0;
+    unsigned long long same = __ballot(live);
+    for (int b = 0; b < bits; ++b) {
+      const unsigned long long set = __ballot(live && ((e >> b) & 1));
+      same &= (e >> b) & 1 ? set : ~set;
+    }
+    if (live) {
+      const int rank = __popcll(same & ((1ull << lane) - 1));
+      const int used = next_s[e];
+      const int p = first_s[e] + used + rank;
+      row_of_place[p] = i / k;
+      place[i] = p;
+      // the group's last lane moves the run on; lanes of one wave, so all of
+      // them have read the old value
+      if ((same >> lane) == 1ull) next_s[e] = used + rank + 1;
+    }
+    __builtin_amdgcn_wave_barrier();
+  }
+}
+
 template <typename AT>
 __global__ __launch_bounds__(256) void moe_mix_rows_kernel(
     AT* __restrict__ out, const AT* __restrict__ y,
@@ -184,6 +258,18 @@ extern "C" int arks_seq_moe_route_grouped(void* weights, void* ids,
                      (float*)weights, (int*)ids, (const float*)logits, E, top,
                      groups, keep, sigmoid, renorm, (float*)matrix,
                      (const float*)bias);
+  return 0;
+}
+
+// ids are trusted to be in [0, E): they come from the routing kernel.
+extern "C" int arks_seq_moe_sort_pairs(void* row_of_place, void* place,
+                                       void* counts, const void* ids, int n,
+                                       int k, int E, int pad,
+                                       hipStream_t stream) {
+  if (E > SORT_MAX_E || E < 1 || k < 1) return 1;
+  hipLaunchKernelGGL(moe_sort_pairs_kernel, dim3(1), dim3(64 * SORT_WAVES),
+                     SORT_WAVES * E * sizeof(int), stream, (int*)row_of_place,
+                     (int*)place, (int*)counts, (const int*)ids, n, k, E, pad);
   return 0;
 }
 

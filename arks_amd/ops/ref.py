@@ -1019,6 +1019,21 @@ def moe_glu_scaled(gu, scale, experts, ff, shared_ff, scale_input=True):
     return torch.cat(parts, -1).to(gu.dtype)
 
 
+def moe_sort_pairs(ids, experts, pad=0):
+    """Pairs (row t, expert ids[t, j]) in expert order, stable: (the row of
+    every sorted place followed by `pad` zeros [T*k + pad] int32, every
+    pair's place [T, k] int32, pairs per expert [experts] int32)."""
+    T, k = ids.shape
+    flat = ids.reshape(-1).long()
+    order = torch.argsort(flat, stable=True)
+    place = torch.empty_like(order)
+    place[order] = torch.arange(T * k, device=ids.device)
+    rows = torch.zeros(T * k + pad, dtype=torch.int32, device=ids.device)
+    rows[:T * k] = torch.div(order, k, rounding_mode="floor")
+    return (rows, place.view(T, k).to(torch.int32),
+            torch.bincount(flat, minlength=experts).to(torch.int32))
+
+
 def route_scale_matrix(weights, ids, experts):
     """[T, experts] fp32: a row's weight at each expert it uses, 0 elsewhere."""
     out = torch.zeros(weights.shape[0], experts, dtype=torch.float32)

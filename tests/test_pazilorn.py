@@ -928,6 +928,29 @@ def test_router_bias_decides_and_outputs_are_weighed(device, dtype):
                     assert float(got.abs().max()) == 0.0
 
 
+@pytest.mark.parametrize("device", ["cpu", pytest.param("cuda", marks=pytest.mark.gpu)])
+@pytest.mark.parametrize("T,k,E", [(1, 1, 1), (7, 2, 3), (300, 4, 16),
+                                   (1111, 3, 70), (5000, 1, 2), (2050, 8, 300)])
+def test_pairs_sorted_by_expert(device, T, k, E):
+    """Stable order, places and counts, with an expert nobody chose and rows
+    of one expert only."""
+    from arks_amd import ops
+
+    g = torch.Generator().manual_seed(T)
+    ids = torch.randint(0, E, (T, k), generator=g, dtype=torch.int32)
+    if E > 2:
+        ids[ids == 1] = 2
+        ids[T // 2:T // 2 + 70] = 0
+    rows, place, counts = (t.cpu().long() for t in
+                           ops.moe_sort_pairs(ids.to(device), E, 5))
+    flat = ids.reshape(-1).long()
+    order = torch.argsort(flat, stable=True)
+    assert torch.equal(counts, torch.bincount(flat, minlength=E))
+    assert torch.equal(rows[:T * k], order // k)
+    assert torch.equal(rows[T * k:], torch.zeros(5, dtype=torch.long))
+    assert torch.equal(place.reshape(-1)[order], torch.arange(T * k))
+
+
 @pytest.mark.gpu
 def test_captured_decode_steps_equal_eager_ones(tmp_path):
     """The captured decode step, replayed many times with eager prompt steps
