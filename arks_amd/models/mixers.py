@@ -390,7 +390,7 @@ class Mamba1Mixer(nn.Module):
         u = ops.causal_conv_silu(
             xz[:, :C], self.conv_w, self.conv_b, cache.get("conv"),
             batch.cu_seqlens, batch.seq_lens, batch.state_slots,
-            batch.token_seq, self.conv_w_t)
+            batch.token_seq, self.conv_w_t, batch.max_q_len)
         dbc = linear(u, self.w_x)
         dt_pre = None
         if xs.is_cuda and self.R >= 8:
@@ -717,7 +717,6 @@ class LatentAttention(SplitMixer):
 
     def _expanded(self, q, batch: ForwardBatch, ckv, gate, out,
                   out_scale) -> None:
-        T = q.shape[0]
         H, D, R, V, rank = self.H, self.D, self.R, self.V, self.rank
         bs = ckv.shape[2]
         idx, table, lens = self._reachable_pages(batch, bs)
@@ -729,9 +728,8 @@ class LatentAttention(SplitMixer):
         kt[..., D:] = lat[..., rank:]
         vt = torch.empty((NB, H, bs, V), dtype=q.dtype, device=q.device)
         vt.copy_(linear(c, self.uv).view(NB, bs, H, V).transpose(1, 2))
-        qf = torch.empty((T, H, D + R), dtype=q.dtype, device=q.device)
-        ops.latent_query(q, None, batch.positions, self.inv_freq, qf,
-                         self.interleaved, self.rot_mag)
+        qf = ops.latent_query(q, None, batch.positions, self.inv_freq, q,
+                              self.interleaved, self.rot_mag)  # in place
         heads = out.unflatten(-1, (H, V))
         # only distances between rows and keys enter: lens without the
         # skipped pages on both sides keeps them
@@ -801,7 +799,7 @@ class Mamba2Mixer(SplitMixer):
         xbc = ops.causal_conv_silu(
             p[:, inner:inner + ch], self.conv_w, self.conv_b, cache.get("conv"),
             batch.cu_seqlens, batch.seq_lens, batch.state_slots,
-            batch.token_seq, self.conv_w_t)
+            batch.token_seq, self.conv_w_t, batch.max_q_len)
         y = ops.mamba2_scan(
             xbc, p[:, inner + ch:inner + ch + self.P], self.dt_bias, self.rate,
             self.D, cache["ssm"], batch.cu_seqlens, batch.seq_lens,

@@ -149,14 +149,97 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(
     turn_pair<AT>(dst + Rk, kr + Rk, i, P, pos * freq[i], half_split, mag);
 }
 
+// bf16 rows, 16-byte accesses (Rq, Rk, strides multiples of 8, half-split
+// pairs with P a multiple of 8, Rq + Rk <= 8 * 256 * LP_IT): the row's pieces
+// stay in registers between the sums of squares and the scaling.
+constexpr int LP_IT = 2;
+
+__global__ __launch_bounds__(256) void latent_prepare_vec8_kernel(
+    bf16* __restrict__ cqn, const bf16* __restrict__ cq, int64_t ldq,
+    const bf16* __restrict__ ckv, int64_t ldk, const float* __restrict__ qw,
+    const float* __restrict__ kw, float eps,
+    const int64_t* __restrict__ positions, const float* __restrict__ freq,
+    bf16* __restrict__ cache, const int64_t* __restrict__ slot_mapping, int Rq,
+    int Rk, int P, float mag) {
+  __shared__ float red[4][2];
+  const int t = blockIdx.x;
+  const int nq = Rq / 8, n = nq + Rk / 8;
+  const int64_t slot = slot_mapping[t];
+  bf16* dst = cache + (slot < 0 ? 0 : slot) * (int64_t)(Rk + 2 * P);
+  const bf16* kr = ckv + (int64_t)t * ldk;
+  ushort8 in[LP_IT];
+  float sq = 0.f, sk = 0.f;
+#pragma unroll
+  for (int it = 0; it < LP_IT; ++it) {
+    const int i = it * 256 + threadIdx.x;
+    if (i < n) {
+      in[it] = *reinterpret_cast<const ushort8*>(
+          i < nq ? cq + (int64_t)t * ldq + i * 8 : kr + (i - nq) * 8);
+      float s = 0.f;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        const float a = bf16_bits_to_float(in[it][e]);
+        s += a * a;
+      }
+      (i < nq ? sq : sk) += s;
+    }
+  }
+  // the rotated part: the last threads, 8 pairs each
+  const int rot = 255 - (int)threadIdx.x;
+  if (rot < P / 8 && slot >= 0) {
+    const float pos = (float)positions[t];
+    const ushort8 a = *reinterpret_cast<const ushort8*>(kr + Rk + rot * 8);
+    const ushort8 b = *reinterpret_cast<const ushort8*>(kr + Rk + P + rot * 8);
+    ushort8 x, y;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      float sn, cs;
+      sincosf(pos * freq[rot * 8 + e], &sn, &cs);
+      const float u = bf16_bits_to_float(a[e]), v = bf16_bits_to_float(b[e]);
+      x[e] = float_to_bf16_bits((u * cs - v * sn) * mag);
+      y[e] = float_to_bf16_bits((v * cs + u * sn) * mag);
+    }
+    *reinterpret_cast<ushort8*>(dst + Rk + rot * 8) = x;
+    *reinterpret_cast<ushort8*>(dst + Rk + P + rot * 8) = y;
+  }
+  sq = wave_reduce_sum(sq);
+  sk = wave_reduce_sum(sk);
+  if (threadIdx.x % 64 == 0) {
+    red[threadIdx.x / 64][0] = sq;
+    red[threadIdx.x / 64][1] = sk;
+  }
+  __syncthreads();
+  sq = red[0][0] + red[1][0] + red[2][0] + red[3][0];
+  sk = red[0][1] + red[1][1] + red[2][1] + red[3][1];
+  const float rq = 1.f / sqrtf(sq / (float)Rq + eps);
+  const float rk = 1.f / sqrtf(sk / (float)Rk + eps);
+#pragma unroll
+  for (int it = 0; it < LP_IT; ++it) {
+    const int i = it * 256 + threadIdx.x;
+    if (i < n) {
+      const bool is_q = i < nq;
+      const float* w = is_q ? qw + i * 8 : kw + (i - nq) * 8;
+      const float r = is_q ? rq : rk;
+      ushort8 o;
+#pragma unroll
+      for (int e = 0; e < 8; ++e)
+        o[e] = float_to_bf16_bits(bf16_bits_to_float(in[it][e]) * r * w[e]);
+      if (is_q)
+        *reinterpret_cast<ushort8*>(cqn + (int64_t)t * Rq + i * 8) = o;
+      else if (slot >= 0)
+        *reinterpret_cast<ushort8*>(dst + (i - nq) * 8) = o;
+    }
+  }
+}
+
 // out [T, H, Rk + 2P] = [q_abs[h, t, :] | rotated q[t, h, D:]]; one block
-// per row, waves over heads. q_abs null: the first part is q[t, h, :D].
+// per row, waves over heads. q_abs null: the first part is q[t, h, :D], and
+// out may be q itself.
 template <typename AT>
 __global__ __launch_bounds__(256) void latent_query_kernel(
-    AT* __restrict__ out, const AT* __restrict__ q,
-    const AT* __restrict__ q_abs, const int64_t* __restrict__ positions,
-    const float* __restrict__ freq, int T, int H, int D, int Rk, int P,
-    int half_split, float mag) {
+    AT* out, const AT* q, const AT* __restrict__ q_abs,
+    const int64_t* __restrict__ positions, const float* __restrict__ freq,
+    int T, int H, int D, int Rk, int P, int half_split, float mag) {
   const int t = blockIdx.x;
   const int wave = threadIdx.x / 64, lane = threadIdx.x % 64;
   const float pos = (float)positions[t];
@@ -165,10 +248,59 @@ __global__ __launch_bounds__(256) void latent_query_kernel(
     // without q_abs the plain part is q's own (Rk == D)
     const AT* src = q_abs ? q_abs + ((int64_t)hh * T + t) * Rk
                           : q + ((int64_t)t * H + hh) * (D + 2 * P);
-    for (int i = lane; i < Rk; i += 64) dst[i] = src[i];
+    if (dst != src)
+      for (int i = lane; i < Rk; i += 64) dst[i] = src[i];
     const AT* qr = q + ((int64_t)t * H + hh) * (D + 2 * P) + D;
     for (int i = lane; i < P; i += 64)
       turn_pair<AT>(dst + Rk, qr, i, P, pos * freq[i], half_split, mag);
+  }
+}
+
+// bf16, 16-byte accesses (D, Rk multiples of 8, half-split pairs with P a
+// multiple of 8): the row's sines and cosines are evaluated once into LDS.
+constexpr int LQ_MAX_P = 128;
+
+__global__ __launch_bounds__(256) void latent_query_vec8_kernel(
+    bf16* out, const bf16* q, const bf16* __restrict__ q_abs,
+    const int64_t* __restrict__ positions, const float* __restrict__ freq,
+    int T, int H, int D, int Rk, int P, float mag) {
+  __shared__ float sn_s[LQ_MAX_P], cs_s[LQ_MAX_P];
+  const int64_t t = blockIdx.x;
+  const float pos = (float)positions[t];
+  for (int i = threadIdx.x; i < P; i += 256) {
+    float sn, cs;
+    sincosf(pos * freq[i], &sn, &cs);
+    sn_s[i] = sn * mag;
+    cs_s[i] = cs * mag;
+  }
+  __syncthreads();
+  // without q_abs the plain part is q's own (Rk == D), already there if out
+  // is q
+  const int np = !q_abs && out == q ? 0 : Rk / 8;
+  const int per = np + P / 8;  // pieces of a head: plain ones, pairs
+  for (int i = threadIdx.x; i < H * per; i += 256) {
+    const int hh = i / per, j = i % per;
+    const bf16* qr = q + (t * H + hh) * (D + 2 * P);
+    bf16* dst = out + (t * H + hh) * (Rk + 2 * P);
+    if (j < np) {
+      const bf16* src = q_abs ? q_abs + ((int64_t)hh * T + t) * Rk : qr;
+      *reinterpret_cast<ushort8*>(dst + j * 8) =
+          *reinterpret_cast<const ushort8*>(src + j * 8);
+      continue;
+    }
+    const int p0 = (j - np) * 8;
+    const ushort8 a = *reinterpret_cast<const ushort8*>(qr + D + p0);
+    const ushort8 b = *reinterpret_cast<const ushort8*>(qr + D + P + p0);
+    ushort8 x, y;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      const float u = bf16_bits_to_float(a[e]), v = bf16_bits_to_float(b[e]);
+      const float sn = sn_s[p0 + e], cs = cs_s[p0 + e];
+      x[e] = float_to_bf16_bits(u * cs - v * sn);
+      y[e] = float_to_bf16_bits(v * cs + u * sn);
+    }
+    *reinterpret_cast<ushort8*>(dst + Rk + p0) = x;
+    *reinterpret_cast<ushort8*>(dst + Rk + P + p0) = y;
   }
 }
 
@@ -205,6 +337,18 @@ extern "C" void arks_seq_latent_prepare(
     int Rk, int P, int half_split, float mag, int act_f32,
     hipStream_t stream) {
   if (T == 0) return;
+  if (!act_f32 && half_split && Rq % 8 == 0 && Rk % 8 == 0 && P % 8 == 0 &&
+      P <= 1024 && Rq + Rk <= 8 * 256 * LP_IT && ldq % 8 == 0 && ldk % 8 == 0 &&
+      (((uintptr_t)cqn | (uintptr_t)cq | (uintptr_t)ckv | (uintptr_t)cache) &
+       15) == 0) {
+    hipLaunchKernelGGL(latent_prepare_vec8_kernel, dim3(T), dim3(256), 0,
+                       stream, (bf16*)cqn, (const bf16*)cq, ldq,
+                       (const bf16*)ckv, ldk, (const float*)qw,
+                       (const float*)kw, eps, (const int64_t*)positions,
+                       (const float*)freq, (bf16*)cache,
+                       (const int64_t*)slot_mapping, Rq, Rk, P, mag);
+    return;
+  }
   SEQ_DISPATCH_ACT(act_f32, hipLaunchKernelGGL(
       (latent_prepare_kernel<AT>), dim3(T), dim3(256), 0, stream, (AT*)cqn,
       (const AT*)cq, ldq, (const AT*)ckv, ldk, (const float*)qw,
@@ -218,6 +362,15 @@ extern "C" void arks_seq_latent_query(void* out, const void* q,
                                       int Rk, int P, int half_split, float mag,
                                       int act_f32, hipStream_t stream) {
   if (T == 0) return;
+  if (!act_f32 && half_split && D % 8 == 0 && Rk % 8 == 0 && P % 8 == 0 &&
+      P <= LQ_MAX_P &&
+      (((uintptr_t)out | (uintptr_t)q | (uintptr_t)q_abs) & 15) == 0) {
+    hipLaunchKernelGGL(latent_query_vec8_kernel, dim3(T), dim3(256), 0, stream,
+                       (bf16*)out, (const bf16*)q, (const bf16*)q_abs,
+                       (const int64_t*)positions, (const float*)freq, T, H, D,
+                       Rk, P, mag);
+    return;
+  }
   SEQ_DISPATCH_ACT(act_f32, hipLaunchKernelGGL(
       (latent_query_kernel<AT>), dim3(T), dim3(256), 0, stream, (AT*)out,
       (const AT*)q, (const AT*)q_abs, (const int64_t*)positions,

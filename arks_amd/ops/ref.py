@@ -853,14 +853,15 @@ def latent_prepare(cq, ckv, q_norm_w, kv_norm_w, eps, positions, inv_freq,
 def latent_query(q, q_abs, positions, inv_freq, out, interleaved=True,
                  rot_mag=1.0):
     """out [T, H, Rk + 2P] = [q_abs (given as [H, T, Rk]) | the last 2P
-    dims of q [T, H, D + 2P] turned by the row's position as latent_prepare].
+    dims of q [T, H, D + 2P] turned by the row's position as latent_prepare];
+    without q_abs out may be q itself.
     q_abs None: the first part is q's own first D dims."""
     D = q.shape[2] - 2 * inv_freq.numel()
     rank = q_abs.shape[2] if q_abs is not None else D
     ang = positions.float()[:, None, None] * inv_freq.float()[None, None, :]
     out[..., :rank] = q_abs.transpose(0, 1) if q_abs is not None else q[..., :D]
     out[..., rank:] = (_rotate_pairs(q[..., D:].float(), ang, interleaved)
-                       * rot_mag).to(out.dtype)
+                       * rot_mag).to(out.dtype)  # read before it is written
     return out
 
 

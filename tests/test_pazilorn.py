@@ -768,7 +768,9 @@ def test_window_edges_over_latents(device, dtype, decode, rank, R):
 
 @pytest.mark.parametrize("device,dtype", CASES)
 @pytest.mark.parametrize("interleaved", [False, True])
-def test_latent_rows_norm_turn_and_pages(device, dtype, interleaved):
+@pytest.mark.parametrize("sizes", [(6, 10, 14, 8), (8, 24, 40, 16), (64, 1536, 512, 64)],
+                         ids=["odd", "vector", "large"])
+def test_latent_rows_norm_turn_and_pages(device, dtype, interleaved, sizes):
     """The latent is normed and not turned, the shared key part turned (with
     the scaling's magnitude) and not normed; only the row's own place in the
     pages changes; the query's plain part passes unchanged."""
@@ -776,51 +778,63 @@ def test_latent_rows_norm_turn_and_pages(device, dtype, interleaved):
     from arks_amd.models.mixers import ramp_scaled_inv_freq
 
     dev, dt = _dev(device), TDT[dtype]
-    rot = {"base": 100.0, "dims": 8,
+    D, Rq, Rk, R = sizes
+    rot = {"base": 100.0, "dims": R,
            "scaling": {"factor": 4.0, "original": 16, "fast": 4.0, "slow": 0.5}}
     f, mag = ramp_scaled_inv_freq(rot["base"], rot["dims"], rot["scaling"])
     of, omag = O.ramped_freqs(rot)
     assert torch.allclose(f.double(), of, rtol=1e-6) and math.isclose(mag, omag)
     assert mag > 1.1
-    T, H, D, Rq, Rk = 45, 3, 6, 10, 14
+    T, H, W = 45, 3, Rk + R
     g = torch.Generator().manual_seed(9)
-    p = _rounded(torch.randn(T, Rq + Rk + 8 + 3, generator=g, dtype=F64), dtype)
+    p = _rounded(torch.randn(T, Rq + W + 3 if D == 6 else Rq + W + 8, generator=g,
+                             dtype=F64), dtype)
     qw, kw = (torch.randn(k, generator=g, dtype=F64).float().double()
               for k in (Rq, Rk))
-    q = _rounded(torch.randn(T, H, D + 8, generator=g, dtype=F64), dtype)
+    q = _rounded(torch.randn(T, H, D + R, generator=g, dtype=F64), dtype)
+    q_abs = _rounded(torch.randn(H, T, Rk, generator=g, dtype=F64), dtype)
 
     def turn(x):  # rows are positions 0 .. T-1
         if interleaved:
             x = torch.cat([x[..., 0::2], x[..., 1::2]], -1)
         y = O.rotate_half(x, rot)
         if interleaved:
-            y = torch.stack([y[..., :4], y[..., 4:]], -1).flatten(-2)
+            y = torch.stack([y[..., :R // 2], y[..., R // 2:]], -1).flatten(-2)
         return y
 
-    cache = torch.full((4, 1, 16, Rk + 8), 3.0, dtype=dt, device=dev)
+    cache = torch.full((4, 1, 16, W), 3.0, dtype=dt, device=dev)
     pos = torch.arange(T)
-    pd = p.to(dt).to(dev)
-    cq = ops.latent_prepare(pd[:, :Rq], pd[:, Rq:Rq + Rk + 8],
+    slots = (pos + 16).to(dev)
+    slots[7] = -1  # a padding row writes no page
+    pd, fd = p.to(dt).to(dev), f.to(dev)
+    cq = ops.latent_prepare(pd[:, :Rq], pd[:, Rq:Rq + W],
                             qw.float().to(dev), kw.float().to(dev), 1e-5,
-                            pos.to(dev), f.to(dev), cache, (pos + 16).to(dev),
-                            interleaved, mag)
+                            pos.to(dev), fd, cache, slots, interleaved, mag)
     tol = 1e-5 if dtype == "float32" else 2e-2
     assert torch.allclose(cq.double().cpu(), O.rms_norm(p[:, :Rq], qw, 1e-5),
                           atol=tol, rtol=tol)
-    got = cache.double().cpu().reshape(-1, Rk + 8)
+    got = cache.double().cpu().reshape(-1, W)
     assert float((got[:16] - 3.0).abs().max()) == 0.0
     assert float((got[16 + T:] - 3.0).abs().max()) == 0.0
-    got = got[16:16 + T]
-    assert torch.allclose(got[:, :Rk], O.rms_norm(p[:, Rq:Rq + Rk], kw, 1e-5),
+    assert float((got[16 + 7] - 3.0).abs().max()) == 0.0
+    keep = pos != 7
+    got = got[16:16 + T][keep]
+    assert torch.allclose(got[:, :Rk], O.rms_norm(p[:, Rq:Rq + Rk], kw, 1e-5)[keep],
                           atol=tol, rtol=tol)
-    want = turn(p[:, None, Rq + Rk:Rq + Rk + 8])[:, 0]
-    assert torch.allclose(got[:, Rk:], want, atol=tol, rtol=tol)
-    out = torch.zeros(T, H, D + 8, dtype=dt, device=dev)
-    ops.latent_query(q.to(dt).to(dev), None, pos.to(dev), f.to(dev), out,
-                     interleaved, mag)
-    res = out.double().cpu()
-    assert torch.equal(res[..., :D], q[..., :D])
-    assert torch.allclose(res[..., D:], turn(q[..., D:]), atol=tol, rtol=tol)
+    want = turn(p[:, None, Rq + Rk:Rq + W])[:, 0]
+    assert torch.allclose(got[:, Rk:], want[keep], atol=tol, rtol=tol)
+    for absorbed in (True, False):
+        plain = q_abs.transpose(0, 1) if absorbed else q[..., :D]
+        qd = q.to(dt).to(dev)
+        out = (torch.zeros(T, H, W, dtype=dt, device=dev) if absorbed
+               else torch.zeros_like(qd))
+        for o in (out, qd)[:1 if absorbed else 2]:  # a new tensor, then in place
+            ops.latent_query(qd, q_abs.to(dt).to(dev) if absorbed else None,
+                             pos.to(dev), fd, o, interleaved, mag)
+            res = o.double().cpu()
+            n = plain.shape[-1]
+            assert torch.equal(res[..., :n], plain)
+            assert torch.allclose(res[..., n:], turn(q[..., D:]), atol=tol, rtol=tol)
 
 
 @pytest.mark.parametrize("device,dtype", CASES)
