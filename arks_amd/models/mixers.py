@@ -717,17 +717,13 @@ class LatentAttention(SplitMixer):
 
     def _expanded(self, q, batch: ForwardBatch, ckv, gate, out,
                   out_scale) -> None:
-        H, D, R, V, rank = self.H, self.D, self.R, self.V, self.rank
+        H, R, V, rank = self.H, self.R, self.V, self.rank
         bs = ckv.shape[2]
         idx, table, lens = self._reachable_pages(batch, bs)
-        NB = idx.shape[0]
-        lat = ckv[idx]  # [NB, 1, bs, rank + R]
-        c = lat[..., :rank].reshape(NB * bs, rank)
-        kt = torch.empty((NB, H, bs, D + R), dtype=q.dtype, device=q.device)
-        kt[..., :D] = linear(c, self.uk).view(NB, bs, H, D).transpose(1, 2)
-        kt[..., D:] = lat[..., rank:]
-        vt = torch.empty((NB, H, bs, V), dtype=q.dtype, device=q.device)
-        vt.copy_(linear(c, self.uv).view(NB, bs, H, V).transpose(1, 2))
+        lat = ckv[idx].view(-1, rank + R)
+        c = lat[:, :rank].contiguous()  # the tuned products take dense rows
+        kt, vt = ops.latent_pages(linear(c, self.uk), linear(c, self.uv), lat,
+                                  H, R, bs)
         qf = ops.latent_query(q, None, batch.positions, self.inv_freq, q,
                               self.interleaved, self.rot_mag)  # in place
         heads = out.unflatten(-1, (H, V))

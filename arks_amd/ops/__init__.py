@@ -1149,6 +1149,18 @@ def latent_query(q, q_abs, positions, inv_freq, out, interleaved=True,
                             rot_mag)
 
 
+def latent_pages(k_up, v_up, lat, heads, rot_dim, block_size):
+    """Per-head key and value pages from up-projected context rows and the
+    shared key part (ref.latent_pages)."""
+    if lat.is_cuda:
+        pages = (lat.shape[0] // block_size, heads, block_size)
+        kt = lat.new_empty(pages + (k_up.shape[1] // heads + rot_dim,))
+        vt = lat.new_empty(pages + (v_up.shape[1] // heads,))
+        _native_seq().latent_pages(kt, vt, k_up, v_up, lat)
+        return kt, vt
+    return ref.latent_pages(k_up, v_up, lat, heads, rot_dim, block_size)
+
+
 # rows per chunk of mamba2's chunk-parallel prefill: a chunk's state
 # (heads x state x vdim floats) is written and read four times, so chunks
 # are long; the scan itself is sequential inside a chunk either way

@@ -134,6 +134,10 @@ void arks_seq_latent_query(void* out, const void* q, const void* q_abs,
                            const void* positions, const void* freq, int T,
                            int H, int D, int Rk, int P, int half_split,
                            float mag, int act_f32, hipStream_t stream);
+void arks_seq_latent_pages(void* kt, void* vt, const void* k_up,
+                           const void* v_up, const void* lat, int64_t ld_lat,
+                           int NB, int bs, int H, int D, int R, int V,
+                           int rank, int elem_bytes, hipStream_t stream);
 int arks_seq_mamba2_scan(void* out, const void* xbc, int64_t ldx,
                          const void* dt_raw, int64_t ldd, const void* dt_bias,
                          const void* rate, const void* Dp, void* state,
@@ -1272,6 +1276,30 @@ void latent_query(Tensor out, Tensor q, OptTensor q_abs, Tensor positions,
                         current_stream());
 }
 
+void latent_pages(Tensor kt, Tensor vt, Tensor k_up, Tensor v_up, Tensor lat) {
+  const int f32 = act_flag(kt, "kt");
+  TORCH_CHECK(kt.dim() == 4 && vt.dim() == 4 && kt.is_contiguous() &&
+              vt.is_contiguous() && k_up.is_contiguous() &&
+              v_up.is_contiguous());
+  const int64_t NB = kt.size(0), H = kt.size(1), bs = kt.size(2);
+  const int64_t V = vt.size(3), n = NB * bs;
+  TORCH_CHECK(vt.size(0) == NB && vt.size(1) == H && vt.size(2) == bs);
+  TORCH_CHECK(k_up.dim() == 2 && k_up.size(0) == n && k_up.size(1) % H == 0 &&
+              v_up.dim() == 2 && v_up.size(0) == n && v_up.size(1) == H * V);
+  const int64_t D = k_up.size(1) / H, R = kt.size(3) - D;
+  TORCH_CHECK(lat.dim() == 2 && lat.size(0) == n && R >= 0 &&
+              lat.size(1) >= R && H <= 65535);
+  TORCH_CHECK(vt.scalar_type() == kt.scalar_type() &&
+              k_up.scalar_type() == kt.scalar_type() &&
+              v_up.scalar_type() == kt.scalar_type() &&
+              lat.scalar_type() == kt.scalar_type());
+  arks_seq_latent_pages(kt.data_ptr(), vt.data_ptr(), k_up.data_ptr(),
+                        v_up.data_ptr(), lat.data_ptr(),
+                        row_stride(lat, "lat"), (int)NB, (int)bs, (int)H,
+                        (int)D, (int)R, (int)V, (int)(lat.size(1) - R),
+                        f32 ? 4 : 2, current_stream());
+}
+
 void mamba2_scan(OptTensor out, Tensor xbc, Tensor dt_raw, Tensor dt_bias,
                  Tensor rate, Tensor Dp, Tensor state, Tensor cu,
                  Tensor seq_lens, Tensor slots, int64_t P, int64_t V,
@@ -1570,6 +1598,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("channel_delta_chunks", &channel_delta_chunks);
   m.def("latent_prepare", &latent_prepare);
   m.def("latent_query", &latent_query);
+  m.def("latent_pages", &latent_pages);
   m.def("mamba2_scan", &mamba2_scan);
   m.def("mamba2_combine", &mamba2_combine);
   m.def("gate_group_norm", &gate_group_norm);

@@ -5,7 +5,9 @@
 //   latent_prepare: RMS norm of the query latent; RMS norm of the key/value
 //       latent and rotation of the shared key part, written to the row's
 //       place in the paged latent cache;
-//   latent_query: [absorbed query | rotated part] per head.
+//   latent_query: [absorbed query | rotated part] per head;
+//   latent_pages: per-head key and value pages from up-projected rows and
+//       the shared key part.
 #include "seq_common.h"
 
 namespace arks {
@@ -304,6 +306,28 @@ __global__ __launch_bounds__(256) void latent_query_vec8_kernel(
   }
 }
 
+// One block per (page, head). All sizes and row strides count pieces PT.
+template <typename PT>
+__global__ __launch_bounds__(256) void latent_pages_kernel(
+    PT* __restrict__ kt, PT* __restrict__ vt, const PT* __restrict__ k_up,
+    const PT* __restrict__ v_up, const PT* __restrict__ lat, int64_t ld_lat,
+    int bs, int H, int D, int R, int V, int rank) {
+  const int64_t page = blockIdx.x, head = blockIdx.y;
+  const int64_t row0 = page * bs, to = (page * H + head) * bs;
+  const int DR = D + R, nk = bs * DR, n = nk + bs * V;
+  for (int i = threadIdx.x; i < n; i += 256) {
+    if (i < nk) {
+      const int t = i / DR, c = i % DR;
+      const int64_t row = row0 + t;
+      kt[(to + t) * DR + c] = c < D ? k_up[(row * H + head) * D + c]
+                                    : lat[row * ld_lat + rank + c - D];
+    } else {
+      const int t = (i - nk) / V, c = (i - nk) % V;
+      vt[(to + t) * V + c] = v_up[((row0 + t) * H + head) * V + c];
+    }
+  }
+}
+
 }  // namespace arks
 
 using namespace arks;
@@ -375,4 +399,33 @@ extern "C" void arks_seq_latent_query(void* out, const void* q,
       (latent_query_kernel<AT>), dim3(T), dim3(256), 0, stream, (AT*)out,
       (const AT*)q, (const AT*)q_abs, (const int64_t*)positions,
       (const float*)freq, T, H, D, Rk, P, half_split, mag));
+}
+
+extern "C" void arks_seq_latent_pages(void* kt, void* vt, const void* k_up,
+                                      const void* v_up, const void* lat,
+                                      int64_t ld_lat, int NB, int bs, int H,
+                                      int D, int R, int V, int rank,
+                                      int elem_bytes, hipStream_t stream) {
+  if (NB == 0) return;
+  const int per = 16 / elem_bytes;  // elements of a 16-byte piece
+  const dim3 grid(NB, H);
+  if (D % per == 0 && R % per == 0 && V % per == 0 && rank % per == 0 &&
+      ld_lat % per == 0 &&
+      (((uintptr_t)kt | (uintptr_t)vt | (uintptr_t)k_up | (uintptr_t)v_up |
+        (uintptr_t)lat) & 15) == 0) {
+    hipLaunchKernelGGL((latent_pages_kernel<uint4>), grid, dim3(256), 0, stream,
+                       (uint4*)kt, (uint4*)vt, (const uint4*)k_up,
+                       (const uint4*)v_up, (const uint4*)lat, ld_lat / per, bs,
+                       H, D / per, R / per, V / per, rank / per);
+  } else if (elem_bytes == 4) {
+    hipLaunchKernelGGL((latent_pages_kernel<uint32_t>), grid, dim3(256), 0,
+                       stream, (uint32_t*)kt, (uint32_t*)vt,
+                       (const uint32_t*)k_up, (const uint32_t*)v_up,
+                       (const uint32_t*)lat, ld_lat, bs, H, D, R, V, rank);
+  } else {
+    hipLaunchKernelGGL((latent_pages_kernel<uint16_t>), grid, dim3(256), 0,
+                       stream, (uint16_t*)kt, (uint16_t*)vt,
+                       (const uint16_t*)k_up, (const uint16_t*)v_up,
+                       (const uint16_t*)lat, ld_lat, bs, H, D, R, V, rank);
+  }
 }

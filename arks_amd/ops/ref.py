@@ -865,6 +865,17 @@ def latent_query(q, q_abs, positions, inv_freq, out, interleaved=True,
     return out
 
 
+def latent_pages(k_up, v_up, lat, heads, rot_dim, block_size):
+    """k_up [n, H*D], v_up [n, H*V], lat [n, rank + R] (R = rot_dim), n whole
+    pages of rows: pages (keys [n / bs, H, bs, D + R], each row's key with
+    the row's last R columns of lat behind it, values [n / bs, H, bs, V])."""
+    NB, bs, H = lat.shape[0] // block_size, block_size, heads
+    k = k_up.view(NB, bs, H, -1).transpose(1, 2)
+    kr = lat[:, lat.shape[1] - rot_dim:].reshape(NB, 1, bs, rot_dim)
+    return (torch.cat([k, kr.expand(NB, H, bs, rot_dim)], -1),
+            v_up.view(NB, bs, H, -1).transpose(1, 2).contiguous())
+
+
 def mamba2_scan(xbc, dt_raw, dt_bias, rate, Dp, state, cu_seqlens, seq_lens,
                 state_slots, heads, vdim, nstate, groups):
     """Scalar-decay state-space recurrence per head: xbc [T, P*V + 2*G*N] =

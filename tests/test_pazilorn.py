@@ -838,6 +838,26 @@ def test_latent_rows_norm_turn_and_pages(device, dtype, interleaved, sizes):
 
 
 @pytest.mark.parametrize("device,dtype", CASES)
+@pytest.mark.parametrize("sizes", [(3, 6, 4, 5, 10), (4, 24, 8, 16, 32), (1, 1, 2, 1, 1)])
+def test_latent_pages_of_single_heads(device, dtype, sizes):
+    from arks_amd import ops
+
+    H, D, R, V, rank = sizes
+    NB, bs = 5, 16
+    g = torch.Generator().manual_seed(3)
+    k, v, lat = (torch.randn(NB * bs, n, generator=g).to(TDT[dtype]).to(device)
+                 for n in (H * D, H * V, rank + R))
+    kt, vt = (x.cpu() for x in ops.latent_pages(k, v, lat, H, R, bs))
+    assert kt.shape == (NB, H, bs, D + R) and vt.shape == (NB, H, bs, V)
+    for n in range(NB * bs):
+        for h in range(H):
+            at = (n // bs, h, n % bs)
+            assert torch.equal(kt[at][:D], k[n, h * D:(h + 1) * D].cpu())
+            assert torch.equal(kt[at][D:], lat[n, rank:].cpu())
+            assert torch.equal(vt[at], v[n, h * V:(h + 1) * V].cpu())
+
+
+@pytest.mark.parametrize("device,dtype", CASES)
 @pytest.mark.parametrize("V", [10, 64])
 def test_head_gate(device, dtype, V):
     """Each head by its own number; heads-first inputs, strided rows, in
