@@ -185,12 +185,16 @@ class HybridModelConfig:
     loop: dict = None
     # cap c on the logits, c tanh(z / c) (0: none)
     logit_softcap: float = 0.0
+    # second embedding table, row (previous token * mul_prev + token *
+    # mul_cur) mod buckets ({"buckets", "mul_prev", "mul_cur"} or None)
+    bigram: dict = None
 
     # what the engine asks of any model config
     sliding_window = None
 
-    ARCHITECTURES = ("Gagorax", "Fusolix", "Legalix", "Rivolix", "Pazilorn")
-    MOE_ARCHITECTURES = ("Fusolix", "Rivolix", "Pazilorn")
+    ARCHITECTURES = ("Gagorax", "Fusolix", "Legalix", "Rivolix", "Pazilorn",
+                     "Fuzelorn")
+    MOE_ARCHITECTURES = ("Fusolix", "Rivolix", "Pazilorn", "Fuzelorn")
     # the logits are taken with the embedding table (no "head" tensor)
     TIED_HEAD_ARCHITECTURES = ("Rivolix", "Pazilorn")
     # mixer type -> {size: tensor whose row count it is}
@@ -253,7 +257,17 @@ class HybridModelConfig:
             residual_mult=float(cfg.get("residual_mult", 1.0)),
             loop=cls._read_loop(cfg.get("loop"), len(layers)),
             logit_softcap=float(cfg.get("logit_softcap") or 0.0),
+            bigram=cls._read_bigram((cfg.get("embedding") or {}).get("bigram")),
         )
+
+    @staticmethod
+    def _read_bigram(spec):
+        if not spec:
+            return None
+        out = {k: int(spec[k]) for k in ("buckets", "mul_prev", "mul_cur")}
+        if out["buckets"] < 1 or min(out.values()) < 0:
+            raise ValueError(f"bigram {spec!r}: no buckets or negative factors")
+        return out
 
     @staticmethod
     def _check_weight_owners(layers: list) -> None:
@@ -339,6 +353,14 @@ class HybridModelConfig:
             out.update({"embedding": {"scale": self.embed_scale},
                         "residual_mult": self.residual_mult,
                         "logit_softcap": self.logit_softcap})
+        if self.architecture == "Fuzelorn":
+            out.pop("logit_scale")
+            out.update({"embedding": {"scale": self.embed_scale},
+                        "logit_softcap": self.logit_softcap})
+            if self.bigram:
+                out["embedding"]["bigram"] = dict(self.bigram)
+            if self.loop:
+                out["loop"] = dict(self.loop)
         return out
 
     @property
@@ -499,6 +521,35 @@ def _pazilorn_preset(width, vocab, pattern, heads, kv_heads, dim, vdim, taps,
         architecture="Pazilorn", vocab_size=vocab, hidden_size=width,
         layers=layers, rms_norm_eps=1e-6, embed_scale=1.0,
         residual_mult=0.5, logit_softcap=30.0)
+
+
+def _fuzelorn_preset(width, vocab, pattern, heads, kv_heads, dim, vdim, window,
+                     d_heads, d_kv_heads, d_dim, d_vdim, taps, ff, experts,
+                     top, groups, keep, expert_ff, shared_ff, buckets,
+                     loop=None) -> HybridModelConfig:
+    """pattern: one letter per layer for its feed-forward, d (dense), m
+    (experts) or n (none); every layer has the two-sided mixer."""
+    layers = []
+    for ch in pattern:
+        mixer = {
+            "left": {"heads": heads, "kv_heads": kv_heads, "dim": dim,
+                     "vdim": vdim, "scale": dim ** -0.5,
+                     "mask": {"size": window},
+                     "q_temp": {"coef": 0.1, "every": 1024}},
+            "right": {"heads": d_heads, "kv_heads": d_kv_heads, "dim": d_dim,
+                      "vdim": d_vdim, "conv": taps}}
+        mlp = ({"kind": "dense", "ff": ff} if ch == "d" else
+               {"kind": "moe", "expert": {"ff": expert_ff, "limit": 7.0},
+                "router": {"experts": experts, "top": top,
+                           "groups": {"count": groups, "keep": keep}},
+                "shared": {"ff": shared_ff, "limit": 7.0}}
+               if ch == "m" else None)
+        layers.append({"type": "parallel", "mixer": mixer, "mlp": mlp})
+    return HybridModelConfig(
+        architecture="Fuzelorn", vocab_size=vocab, hidden_size=width,
+        layers=layers, rms_norm_eps=1e-6, embed_scale=1.0, logit_softcap=30.0,
+        bigram={"buckets": buckets, "mul_prev": 1009, "mul_cur": 13},
+        loop=loop)
 
 
 # Named synthetic configs for benchmarks / tests (random-init weights; no
@@ -815,6 +866,16 @@ PRESET_CONFIGS: dict[str, ModelConfig] = {
     "tiny-pazilorn": _pazilorn_preset(
         128, 512, "clcl", 4, 2, 16, 24, 4, 12, 4, 16, 8, 24, 32, 40, 24, 8, 2,
         48, shared={2: 0, 3: 1}),
+    # Fuzelorn at the layer sizes of an ~8B model: 32/8 heads x 128 over a
+    # 1024-token window beside a delta rule with 16 heads x 128/128 (4 taps);
+    # 16 experts of ff 3584, 4 per row from 2 of 4 groups, beside a shared
+    # expert of ff 3584; one dense layer of ff 14336
+    "fuzelorn-8b-slice": _fuzelorn_preset(
+        4096, 32000, "dmmmmmmm", 32, 8, 128, 128, 1024, 16, 16, 128, 128, 4,
+        14336, 16, 4, 4, 2, 3584, 3584, 65536),
+    "tiny-fuzelorn": _fuzelorn_preset(
+        128, 512, "dmnm", 4, 2, 32, 24, 24, 4, 2, 16, 24, 4, 192, 8, 2, 4, 2,
+        48, 80, 301, loop={"start": 1, "stop": 3, "times": 2}),
     "tiny-gpu": ModelConfig(  # GPU-test-sized (head_dim 128 kernels)
         architecture="Qwen2ForCausalLM",
         vocab_size=2048,

@@ -42,6 +42,12 @@ _REGISTRY = {
     # in every layer, layers on other layers' weights; capped logits through
     # the embedding table (models/hybrid.py SandwichBlock)
     "Pazilorn": HybridForCausalLM,
+    # layer-list decoder: an RMS norm before every sublayer; windowed
+    # attention with a distance bias beside a delta rule with one decay per
+    # head, squared-relu or group-routed clamped experts with a gated shared
+    # one, a looped run of layers, a hashed embedding of token pairs, capped
+    # logits (models/hybrid.py PreNormBlock)
+    "Fuzelorn": HybridForCausalLM,
 }
 
 

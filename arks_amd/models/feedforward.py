@@ -36,7 +36,13 @@ constants as constructor parameters:
   projections, an activation whose factor is 0 for the experts a row does
   not use (so their columns are exactly 0), and ONE down GEMM over all
   columns, which sums the chosen experts and the shared one. Above it the
-  (row, expert) pairs are sorted by expert as in GroupedMoE.
+  (row, expert) pairs are sorted by expert as in GroupedMoE. Experts may also
+  be chosen in groups, by scores with a correction per expert that the
+  weights do not see, and a group ranked by its best or its two best;
+  the activation may be ClampedGLU's (limit, and shared_limit for the shared
+  expert); and the shared expert may be weighed by sigmoid(W_sg h), a row of
+  the router's matrix.
+- SquaredReLU: W_down max(W_up x + b_up, 0)^2 + b_down.
 """
 
 from __future__ import annotations
@@ -125,6 +131,25 @@ class ClampedGLU(GLU):
                          alpha=alpha)
 
 
+class SquaredReLU(nn.Module):
+    """W_down max(W_up x + b_up, 0)^2 + b_down."""
+
+    def __init__(self, width: int, ff: int, dtype):
+        super().__init__()
+        self.up = _param(ff, width, dtype=dtype)
+        self.up_b = _param(ff, dtype=dtype)
+        self.down = _param(width, ff, dtype=dtype)
+        self.down_b = _param(width, dtype=dtype)
+
+    def weight_map(self) -> dict:
+        return {"up": (self.up, 0), "up.b": (self.up_b, 0),
+                "down": (self.down, 0), "down.b": (self.down_b, 0)}
+
+    def forward(self, h, batch=None, cache=None) -> torch.Tensor:
+        return linear(ops.relu_square(linear(h, self.up, self.up_b)),
+                      self.down, self.down_b)
+
+
 class GroupedMoE(nn.Module):
     DENSE_TOKENS = 256  # see models/llama_family.py MoEMLP.DENSE_TOKENS
 
@@ -173,24 +198,43 @@ class RoutedMoE(nn.Module):
     def __init__(self, width: int, experts: int, ff: int, top: int, dtype,
                  shared_ff: int = 0, score: str = "sigmoid",
                  renorm: bool = False, weigh: str = "input",
-                 router_bias: bool = False):
+                 router_bias: bool = False, groups: int = 1, keep: int = 1,
+                 group_top: int = 1, correction: bool = False,
+                 act: str = "swiglu", limit: float = 0.0,
+                 shared_limit: float = 0.0, alpha: float = 1.0,
+                 shared_gate: bool = False):
         super().__init__()
+        assert experts % groups == 0 and keep <= groups
+        assert top <= keep * (experts // groups)
+        assert act == "swiglu" or weigh == "output"
+        assert not shared_gate or (shared_ff and weigh == "output")
+        self.groups, self.keep, self.group_top = groups, keep, group_top
+        self.act, self.alpha = act, float(alpha)
+        self.limit, self.shared_limit = float(limit), float(shared_limit)
+        self.shared_gate = shared_gate
+        self.correction = (_param(experts, dtype=torch.float32) if correction
+                           else None)
         assert 1 <= top <= experts and score in ("sigmoid", "softmax")
         assert weigh in ("input", "output")
         self.weigh_input = weigh == "input"
         self.E, self.ff, self.top, self.sff = experts, ff, top, int(shared_ff)
         self.width, self.score, self.renorm = width, score, renorm
-        self.router = _param(experts, width, dtype=dtype)
+        # the shared expert's gate is one row more
+        self.router = _param(experts + bool(shared_gate), width, dtype=dtype)
         self.router_b = (_param(experts, dtype=torch.float32) if router_bias
                          else None)
         self.w_gu = _param(experts * 2 * ff + 2 * self.sff, width, dtype=dtype)
         self.w_down = _param(width, experts * ff + self.sff, dtype=dtype)
 
     def weight_map(self) -> dict:
-        m = {"router": (self.router, 0)}
+        W, ff, E, sff = self.width, self.ff, self.E, self.sff
+        m = {"router": (self.router, 0, 0, (E, W))}
         if self.router_b is not None:
             m["router.b"] = (self.router_b, 0)
-        W, ff, E, sff = self.width, self.ff, self.E, self.sff
+        if self.correction is not None:
+            m["correction"] = (self.correction, 0)
+        if self.shared_gate:
+            m["shared.sg"] = (self.router, E, 0, (1, W))
         for e in range(E):
             m[f"e{e}.gate"] = (self.w_gu, e * 2 * ff)
             m[f"e{e}.up"] = (self.w_gu, e * 2 * ff + ff)
@@ -205,15 +249,18 @@ class RoutedMoE(nn.Module):
         T = h.shape[0]
         E, ff, sff, k = self.E, self.ff, self.sff, self.top
         z = linear_f32(h, self.router)  # fp32 logits
+        route = dict(score=self.score, renorm=self.renorm, bias=self.router_b,
+                     correction=self.correction, group_top=self.group_top,
+                     shared_gate=self.shared_gate)
         if T <= self.DENSE_TOKENS:
             _, _, scale = ops.moe_route_grouped(
-                z, k, 1, 1, self.score, self.renorm, matrix=True,
-                bias=self.router_b)
+                z, k, self.groups, self.keep, matrix=True, **route)
             gu = linear(h, self.w_gu)
-            return linear(ops.moe_glu_scaled(gu, scale, E, ff, sff,
-                                             self.weigh_input), self.w_down)
-        weights, ids = ops.moe_route_grouped(z, k, 1, 1, self.score,
-                                             self.renorm, bias=self.router_b)
+            return linear(ops.moe_glu_scaled(
+                gu, scale, E, ff, sff, self.weigh_input, self.act, self.limit,
+                self.shared_limit, self.alpha, self.shared_gate), self.w_down)
+        weights, ids = ops.moe_route_grouped(z, k, self.groups, self.keep,
+                                             **route)
         xs, place, counts = sort_by_expert(h, ids, E)
         gu = expert_products(
             xs, counts, lambda e: self.w_gu[e * 2 * ff:(e + 1) * 2 * ff].t())
@@ -222,12 +269,19 @@ class RoutedMoE(nn.Module):
             row_scale = torch.zeros(gu.shape[0], dtype=torch.float32,
                                     device=h.device)
             row_scale[place.reshape(-1).long()] = weights.reshape(-1)
-        a = ops.glu_act(gu, "swiglu", row_scale=row_scale)
+        a = ops.glu_act(gu, self.act, self.limit, self.alpha,
+                        row_scale=row_scale)
         y = expert_products(
             a, counts, lambda e: self.w_down[:, e * ff:(e + 1) * ff].t())
         shared = None
         if sff:
-            sa = ops.glu_act(linear(h, self.w_gu[E * 2 * ff:]), "swiglu")
+            su = linear(h, self.w_gu[E * 2 * ff:])
+            if self.shared_gate:  # one expert that every row uses
+                sa = ops.moe_glu_scaled(
+                    su, torch.sigmoid(z[:, E:]), 1, sff, 0, False, self.act,
+                    self.shared_limit, 0.0, self.alpha)
+            else:
+                sa = ops.glu_act(su, self.act, self.shared_limit, self.alpha)
             shared = linear(sa, self.w_down[:, E * ff:])
         return ops.moe_mix_rows_seq(y, torch.ones_like(weights)
                                     if self.weigh_input else weights,
@@ -250,6 +304,21 @@ def build_feedforward(mlp: dict, width: int, dtype, arch: str = "") -> nn.Module
         return RoutedMoE(width, r["experts"], mlp["expert"]["ff"], r["top"],
                          dtype, score="softmax", renorm=True, weigh="output",
                          router_bias=True)
+    if arch == "Fuzelorn":
+        if kind == "dense":
+            return SquaredReLU(width, mlp["ff"], dtype)
+        if kind != "moe":
+            raise ValueError(f"unknown feed-forward kind {kind!r}")
+        r, shared = mlp["router"], mlp.get("shared") or {}
+        groups = r.get("groups") or {}
+        return RoutedMoE(
+            width, r["experts"], mlp["expert"]["ff"], r["top"], dtype,
+            shared_ff=shared.get("ff", 0), score="sigmoid", renorm=True,
+            weigh="output", groups=groups.get("count", 1),
+            keep=groups.get("keep", 1), group_top=2, correction=True,
+            act="clamped", limit=mlp["expert"]["limit"],
+            shared_limit=shared.get("limit", 0.0), alpha=1.702,
+            shared_gate=bool(shared))
     if kind == "dense":
         return ClampedGLU(width, mlp["ff"], mlp["limit"], dtype)
     if kind == "moe":

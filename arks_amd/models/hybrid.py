@@ -77,6 +77,24 @@ Pazilorn's is:
   sublayer's result, adds it to the fp32 residual and norms the new row for
   the next sublayer, one pass) -> sublayer.
 
+Fuzelorn's is:
+  - an RMS norm in FRONT of every sublayer, one sublayer after the other
+    (PreNormBlock): x += mixer(norm1(x)), x += ff(norm2(x)); the mixer is two
+    mixers on the same rows, whose results are normed over the model width,
+    each with a weight of its own, and half their sum joins the residual
+  - x starts as the scaled embedding plus a row of a second table, picked by
+    a hash of (previous token, token); the previous token is per-sequence
+    state of the model, beside the layers'
+  - mixer "parallel": windowed attention with a distance bias, sink and
+    whole-row q/k norms beside the delta rule with one decay per head;
+    feed-forward SquaredReLU or RoutedMoE (grouped choice by corrected
+    scores, clamped activation, gated shared expert); a run of layers may
+    loop; capped logits through a head of their own
+  Kernel plan per layer: residual_sandwich_norm (adds what the previous
+  sublayer left, one or two results, normed or not, and norms the new row,
+  one pass) -> ONE GEMM for both mixers' in-projections -> their kernels ->
+  an out GEMM per side -> residual_sandwich_norm -> feed-forward.
+
 The per-layer cache is a dict of tensors (paged KV for attention, slot
 state for the recurrent mixers and the token shift), allocated by
 allocate_cache() from each mixer's cache_layout(). A sequence that starts at
@@ -86,6 +104,7 @@ without clearing. Tensor parallelism is not implemented for these models.
 
 from __future__ import annotations
 
+import math
 import zlib
 from dataclasses import dataclass
 
@@ -113,7 +132,9 @@ class BlockArrangement:
     # sublayers side by side, a per-channel scale on each result
     # (DualNormBlock);
     # "sandwich": an RMS norm in front of and one behind each sublayer
-    # (SandwichBlock)
+    # (SandwichBlock);
+    # "pre": an RMS norm in front of each sublayer, and one behind each side
+    # of a two-sided mixer (PreNormBlock)
     norm_place: str = "output"
 
 
@@ -127,6 +148,8 @@ ARRANGEMENTS = {
                                 norm_place="dual"),
     "Pazilorn": BlockArrangement(token_shift=False, gated_residual=False,
                                  norm_place="sandwich"),
+    "Fuzelorn": BlockArrangement(token_shift=False, gated_residual=False,
+                                 norm_place="pre"),
 }
 
 
@@ -372,11 +395,45 @@ class SandwichBlock(nn.Module):
     def cache_layout(self, block_size: int, dtype) -> dict:
         return dict(self.mixer.cache_layout(block_size, dtype))
 
-    def sublayers(self):
-        """(norm in front, sublayer, norm behind) in order."""
-        yield self.norm1, self.mixer, self.norm1b
+    def sublayers(self, mult: float):
+        """(norm in front, sublayer, norms behind its results, factor on
+        their sum) in order."""
+        yield self.norm1, self.mixer, (self.norm1b,), mult
         if self.ffn is not None:
-            yield self.norm2, self.ffn, self.norm2b
+            yield self.norm2, self.ffn, (self.norm2b,), mult
+
+
+class PreNormBlock(nn.Module):
+    """x += (l(norm1(x)) + r(norm1(x))) / 2 for the two normed sides of the
+    mixer, then x += ff(norm2(x)); RMS norms with a plain weight. The norms
+    and the sums are the kernels between the sublayers, as in
+    SandwichBlock."""
+
+    def __init__(self, width: int, spec: dict, eps: float, dtype, arch: str):
+        super().__init__()
+        f32 = torch.float32
+        self.mixer = build_mixer(spec["type"], spec["mixer"], width, eps, dtype,
+                                 arch=arch)
+        self.ffn = (build_feedforward(spec["mlp"], width, dtype, arch)
+                    if spec.get("mlp") is not None else None)
+        self.norm1 = _param(width, dtype=f32)
+        self.norm2 = _param(width, dtype=f32) if self.ffn is not None else None
+
+    def weight_map(self) -> dict:
+        m = {"mix." + k: v for k, v in self.mixer.weight_map().items()}
+        m["norm1"] = (self.norm1, 0)
+        if self.ffn is not None:
+            m.update({"mlp." + k: v for k, v in self.ffn.weight_map().items()})
+            m["norm2"] = (self.norm2, 0)
+        return m
+
+    def cache_layout(self, block_size: int, dtype) -> dict:
+        return dict(self.mixer.cache_layout(block_size, dtype))
+
+    def sublayers(self, mult: float):
+        yield self.norm1, self.mixer, self.mixer.out_norms, 0.5 * mult
+        if self.ffn is not None:
+            yield self.norm2, self.ffn, (None,), mult
 
 
 class HybridForCausalLM(nn.Module):
@@ -415,6 +472,11 @@ class HybridForCausalLM(nn.Module):
                    if cfg.weight_owner(i) == i}
             self.layers = nn.ModuleList(own[cfg.weight_owner(i)]
                                         for i in range(len(cfg.layers)))
+        elif arr.norm_place == "pre":
+            self.layers = nn.ModuleList(
+                PreNormBlock(W, spec, cfg.rms_norm_eps, dtype,
+                             cfg.architecture)
+                for spec in cfg.layers)
         else:
             self.layers = nn.ModuleList(
                 HybridBlock(W, spec, cfg.rms_norm_eps, dtype, arr)
@@ -434,6 +496,12 @@ class HybridForCausalLM(nn.Module):
         else:
             self.head = _param(cfg.vocab_size, W, dtype=dtype)
             self._wmap["head"] = (self.head, 0)
+        # hashed table of token pairs beside the embedding, and a row for
+        # the first token of a sequence
+        self.bigram = None
+        if getattr(cfg, "bigram", None):
+            self.bigram = _param(cfg.bigram["buckets"] + 1, W, dtype=dtype)
+            self._wmap["bigram"] = (self.bigram, 0)
         if arr.norm_place == "input":
             self.final_norm_b = _param(W, dtype=torch.float32)
             self._wmap["final.norm.b"] = (self.final_norm_b, 0)
@@ -458,9 +526,12 @@ class HybridForCausalLM(nn.Module):
     # ------------------------------------------------------------ cache
     def cache_layout(self, block_size: int) -> list:
         """One dict per layer RUN: every pass of a looped layer has pages
-        and state of its own."""
-        return [self.layers[i].cache_layout(block_size, self.dtype)
-                for i in self.run_order]
+        and state of its own; behind them the model's own state, if any."""
+        out = [self.layers[i].cache_layout(block_size, self.dtype)
+               for i in self.run_order]
+        if self.bigram is not None:
+            out.append({"prev_token": ("slot", (), torch.int32)})
+        return out
 
     def kv_block_bytes(self, block_size: int) -> int:
         total = 0
@@ -475,7 +546,7 @@ class HybridForCausalLM(nn.Module):
         for layout in self.cache_layout(16):
             for kind, shape, dt in layout.values():
                 if kind == "slot":
-                    total += int(torch.tensor(shape).prod()) * dt.itemsize
+                    total += math.prod(shape) * dt.itemsize
         return total
 
     def allocate_cache(self, num_blocks: int, block_size: int, num_slots: int,
@@ -498,7 +569,7 @@ class HybridForCausalLM(nn.Module):
             return self._forward_shared(batch, caches)
         if self.arr.norm_place == "dual":
             return self._forward_dual(batch, caches)
-        if self.arr.norm_place == "sandwich":
+        if self.arr.norm_place in ("sandwich", "pre"):
             return self._forward_sandwich(batch, caches)
         x = self.embed[batch.input_ids].float()
         for i, layer in enumerate(self.layers):
@@ -616,30 +687,53 @@ class HybridForCausalLM(nn.Module):
                                       dtype)
         return linear_f32(n, self.head) * cfg.logit_scale
 
-    def _forward_sandwich(self, batch: ForwardBatch, caches: list) -> torch.Tensor:
-        """Sandwich-norm arrangement: a sublayer's result waits until the
-        kernel that norms the next sublayer's input; that kernel norms the
-        result, adds it to the residual and norms the new row, so each
-        sublayer costs one pass over the fp32 rows."""
-        cfg, dtype = self.cfg, self.dtype
-        eps, mult = cfg.rms_norm_eps, cfg.residual_mult
+    def _embed_rows(self, batch: ForwardBatch, caches: list) -> torch.Tensor:
+        """The residual's first rows: the scaled embedding, plus the hashed
+        table's rows where the design has one."""
+        cfg = self.cfg
+        if self.bigram is not None:
+            return ops.hashed_embed(
+                batch.input_ids, self.embed, self.bigram,
+                caches[-1]["prev_token"], batch.cu_seqlens, batch.seq_lens,
+                batch.state_slots, batch.token_seq, cfg.embed_scale,
+                cfg.bigram["mul_prev"], cfg.bigram["mul_cur"],
+                batch.max_q_len)
         x = self.embed[batch.input_ids].float()
         if cfg.embed_scale != 1.0:
             x *= cfg.embed_scale
-        y = post = None
-        for i, layer in enumerate(self.layers):
-            for pre, sub, after in layer.sublayers():
-                h = ops.residual_sandwich_norm(x, y, post, mult, pre, eps, dtype)
-                y, post = sub(h, batch, caches[i]), after
+        return x
+
+    def _forward_sandwich(self, batch: ForwardBatch, caches: list) -> torch.Tensor:
+        """Sandwich- and pre-norm arrangements: a sublayer's result (or two
+        of them) waits until the kernel that norms the next sublayer's input;
+        that kernel norms the result where the design does, adds it to the
+        residual and norms the new row, so each sublayer costs one pass over
+        the fp32 rows."""
+        cfg, dtype = self.cfg, self.dtype
+        eps = cfg.rms_norm_eps
+        x = self._embed_rows(batch, caches)
+        pend, posts, mult = (), (), 1.0
+
+        def settle(w_pre):
+            res = list(pend) + [None] * (2 - len(pend))
+            w = list(posts) + [None] * (2 - len(posts))
+            return ops.residual_sandwich_norm(x, res[0], w[0], mult, w_pre,
+                                              eps, dtype, res[1], w[1])
+
+        for run, i in enumerate(self.run_order):
+            for pre, sub, after, factor in self.layers[i].sublayers(
+                    cfg.residual_mult):
+                y = sub(settle(pre), batch, caches[run])
+                pend = y if isinstance(y, tuple) else (y,)
+                posts, mult = after, factor
             if self.residual_tap is not None:
-                ops.residual_sandwich_norm(x, y, post, mult, None, eps, dtype)
-                y = None
-                self.residual_tap(i, x)
+                settle(None)
+                pend, posts = (), ()
+                self.residual_tap(run, x)
         if batch.logits_indices is not None:
             x = x[batch.logits_indices]
-            y = y[batch.logits_indices] if y is not None else None
-        n = ops.residual_sandwich_norm(x, y, post, mult, self.final_norm, eps,
-                                       dtype)
+            pend = tuple(y[batch.logits_indices] for y in pend)
+        n = settle(self.final_norm)
         logits = linear_f32(n, self.head)
         if cfg.logit_scale != 1.0:
             logits = logits * cfg.logit_scale
@@ -724,16 +818,24 @@ class HybridForCausalLM(nn.Module):
                 w = 0.5 + rn(0.1)
             elif leaf in ("mix.lq1", "mix.lk1", "mix.lq2", "mix.lk2"):
                 w = rn(0.3)
-            elif leaf in ("mix.q.conv", "mix.k.conv", "mix.v.conv"):
+            elif leaf.endswith((".q.conv", ".k.conv", ".v.conv")):
+                w = rn(0.5)
+            elif leaf in ("mix.right.b", "mix.right.a"):
+                w = rn(shape[-1] ** -0.5)
+            elif leaf in ("mix.left.out", "mix.right.out"):
+                w = 1.0 + rn(0.1)
+            elif leaf == "mlp.correction":
+                w = rn(0.1)
+            elif leaf == "bigram":
                 w = rn(0.5)
             elif leaf.endswith("norm") or leaf in ("norm1", "norm2", "norm1b",
                                                    "norm2b"):
                 w = 1.0 + rn(0.1)
-            elif leaf == "mix.dt_bias":
-                # delta-rule channels remember for tens to hundreds of tokens
-                w = (rn(1.0) - 4.0 if self.arr.norm_place == "sandwich"
+            elif leaf in ("mix.dt_bias", "mix.right.dt_bias"):
+                # delta rules remember for tens to hundreds of tokens
+                w = (rn(1.0) - 4.0 if self.arr.norm_place in ("sandwich", "pre")
                      else rn(0.5) - 1.0)
-            elif leaf == "mix.sink":
+            elif leaf in ("mix.sink", "mix.left.sink"):
                 w = rn(1.0)
             elif leaf.startswith("canon"):
                 w = rn(0.3)
@@ -747,7 +849,7 @@ class HybridForCausalLM(nn.Module):
                 w = rn(2.0 * shape[-1] ** -0.5)
             elif leaf == "shift":
                 w = torch.rand(shape, generator=g, device=dev)
-            elif leaf == "mix.A_log":
+            elif leaf in ("mix.A_log", "mix.right.A_log"):
                 w = torch.log(1.0 + 7.0 * torch.rand(shape, generator=g, device=dev))
             elif leaf == "mix.dt.b":
                 w = rn(0.5) - 3.0

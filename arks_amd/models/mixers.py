@@ -48,8 +48,17 @@ constructor parameters so that more than one design can use it:
   projection, unit queries and keys behind short convolutions, a
   [dim x vdim] fp32 state per head and sequence, gated unit-RMS read-out.
 
+- HeadDeltaMixer: the same rule with one decay per head and a silu gate.
+- BiasedWindowAttention: grouped-query softmax attention over a sliding
+  window, positions only as a distance bias per head on the scores and a
+  query factor that grows with the logarithm of the position; q and k normed
+  over all their heads at once, a learned per-head sink.
+- ParallelMixer can also norm each side's result over the model width where
+  the two join the residual (out_norm), with an out-projection per side.
+
 WindowPoolAttention, RetentionMixer, LatentAttention, Mamba2Mixer,
-DiffAttention and ChannelDeltaMixer are "split" mixers: they name the rows of their
+DiffAttention, ChannelDeltaMixer, HeadDeltaMixer and BiasedWindowAttention
+are "split" mixers: they name the rows of their
 in-projection (in_spans) and the columns of their out-projection
 (out_cols) and do everything between in core(), so that a parent can fuse
 the projections of several of them; alone, SplitMixer.forward runs the
@@ -1017,17 +1026,163 @@ class ChannelDeltaMixer(SplitMixer):
             step_chunks(batch, p.device, ops.DELTA_CHUNK))
 
 
+class HeadDeltaMixer(SplitMixer):
+    """Delta rule with one decay per head. In-projection rows [q: G*D |
+    k: G*D | v: H*V | g: H*V | b: H | a: H]; head h uses q/k head h // (H/G).
+    Everything as in ChannelDeltaMixer but the decay, exp(-exp(A_log)
+    softplus(a + dt_bias)), one number per head and row, and the output's
+    gate, silu(g): the same kernels run it."""
+
+    pad_rows = 64
+
+    def __init__(self, width: int, heads: int, kv_heads: int, dim: int,
+                 vdim: int, conv: int, eps: float, dtype,
+                 own_projections: bool = True):
+        super().__init__()
+        assert heads % kv_heads == 0 and conv >= 1
+        self.H, self.G, self.D, self.V = heads, kv_heads, dim, vdim
+        self.taps, self.eps = int(conv), eps
+        self.n_qk = kv_heads * dim
+        self.ch = 2 * self.n_qk + heads * vdim  # convolved channels
+        self.out_cols = heads * vdim
+        f32 = torch.float32
+        self.conv_w = _param(self.ch, self.taps, dtype=f32)
+        self.dt_bias = _param(heads, dtype=f32)
+        self.A_log = _param(heads, dtype=f32)
+        self.norm = _param(vdim, dtype=f32)
+        self.register_buffer("rate", torch.zeros(heads, dtype=f32),
+                             persistent=False)
+        self.register_buffer("conv_w_t", torch.zeros(self.taps, self.ch, dtype=f32),
+                             persistent=False)
+        if own_projections:
+            self._make_projections(width, dtype)
+
+    def in_spans(self) -> list:
+        HV = self.H * self.V
+        return [("q", self.n_qk, False), ("k", self.n_qk, False),
+                ("v", HV, False), ("g", HV, False), ("b", self.H, False),
+                ("a", self.H, False)]
+
+    def extra_weights(self) -> dict:
+        HV = self.H * self.V
+        return {"q.conv": (self.conv_w, 0, 0, (self.n_qk, self.taps)),
+                "k.conv": (self.conv_w, self.n_qk, 0, (self.n_qk, self.taps)),
+                "v.conv": (self.conv_w, 2 * self.n_qk, 0, (HV, self.taps)),
+                "dt_bias": (self.dt_bias, 0), "A_log": (self.A_log, 0),
+                "norm": (self.norm, 0)}
+
+    def finish_loading(self) -> None:
+        self.rate.copy_(torch.exp(self.A_log.data.float()))
+        self.conv_w_t.copy_(self.conv_w.data.t())
+
+    def cache_layout(self, block_size: int, dtype) -> dict:
+        out = {"S": ("slot", (self.H, self.D, self.V), torch.float32)}
+        if self.taps > 1:
+            out["conv"] = ("slot", (self.taps - 1, self.ch), torch.float32)
+        return out
+
+    def core(self, p, batch: ForwardBatch, cache: dict, out, out_scale) -> None:
+        assert out_scale == 1.0
+        H, ch = self.H, self.ch
+        u = ops.causal_conv_silu(
+            p[:, :ch], self.conv_w, None, cache.get("conv"), batch.cu_seqlens,
+            batch.seq_lens, batch.state_slots, batch.token_seq, self.conv_w_t,
+            batch.max_q_len)
+        at = ch + H * self.V
+        ops.channel_delta(
+            u, p[:, at + H:at + 2 * H], p[:, at:at + H], p[:, ch:at],
+            self.rate, self.dt_bias, self.norm, self.eps, cache["S"],
+            batch.cu_seqlens, batch.seq_lens, batch.state_slots, H, self.G,
+            self.D, self.V, out, batch.max_q_len,
+            step_chunks(batch, p.device, ops.DELTA_CHUNK), head_decay=True,
+            silu_gate=True)
+
+
+def distance_slopes(heads: int) -> torch.Tensor:
+    """2^(-8 (h + 1) / heads) for head h, rounded once from float64."""
+    h = torch.arange(1, heads + 1, dtype=torch.float64)
+    return torch.pow(torch.tensor(2.0, dtype=torch.float64),
+                     -8.0 * h / heads).float()
+
+
+class BiasedWindowAttention(SplitMixer):
+    """Softmax attention, query head h on key/value head h // (H/G), without
+    rotation. In-projection rows [q: H*D | k: G*D | v: G*V]. q and k are
+    divided by the root mean square over all their heads at once, times a
+    weight per element; q is multiplied by 1 + temp_coef ln(floor((p + 1) /
+    temp_every) + 1) at position p (temp_every 0: no factor). Row i sees key j
+    with 0 <= i - j < window (0: every j <= i) at score q.k scale -
+    slope_h (i - j), slope_h = 2^(-8 (h+1) / H); with `sink` the denominator
+    also holds exp(sink_h)."""
+
+    def __init__(self, width: int, heads: int, kv_heads: int, dim: int,
+                 vdim: int, scale: float, window: int, temp_coef: float,
+                 temp_every: int, eps: float, dtype, sink: bool = True,
+                 own_projections: bool = True):
+        super().__init__()
+        assert heads % kv_heads == 0
+        self.H, self.G, self.D, self.V = heads, kv_heads, dim, vdim
+        self.scale, self.window, self.eps = float(scale), int(window), eps
+        self.temp_coef, self.temp_every = float(temp_coef), int(temp_every)
+        self.out_cols = heads * vdim
+        f32 = torch.float32
+        self.q_norm = _param(heads * dim, dtype=f32)
+        self.k_norm = _param(kv_heads * dim, dtype=f32)
+        self.sink = _param(heads, dtype=f32) if sink else None
+        self.register_buffer("slopes", distance_slopes(heads),
+                             persistent=False)
+        if own_projections:
+            self._make_projections(width, dtype)
+
+    def in_spans(self) -> list:
+        return [("q", self.H * self.D, False), ("k", self.G * self.D, False),
+                ("v", self.G * self.V, False)]
+
+    def extra_weights(self) -> dict:
+        m = {"q.norm": (self.q_norm, 0), "k.norm": (self.k_norm, 0)}
+        if self.sink is not None:
+            m["sink"] = (self.sink, 0)
+        return m
+
+    def cache_layout(self, block_size: int, dtype) -> dict:
+        return {"k": ("paged", (self.G, block_size, self.D), dtype),
+                "v": ("paged", (self.G, block_size, self.V), dtype)}
+
+    def core(self, p, batch: ForwardBatch, cache: dict, out, out_scale) -> None:
+        H, G, D, V = self.H, self.G, self.D, self.V
+        nq, nk, nv = H * D, G * D, G * V
+        q = ops.row_norm_qk_cache(
+            p[:, :nq], p[:, nq:nq + nk], p[:, nq + nk:nq + nk + nv],
+            self.q_norm, self.k_norm, self.eps, batch.positions,
+            self.temp_coef, self.temp_every, cache["k"], cache["v"],
+            batch.slot_mapping)
+        ops.attention_sink_paged(
+            q.view(-1, H, D), cache["k"], cache["v"], batch.block_tables,
+            batch.seq_lens, batch.cu_seqlens, batch.token_seq, self.scale,
+            False, None, False, batch.max_q_len, batch.positions,
+            sink_w=self.sink, window=self.window, slopes=self.slopes,
+            out=out.unflatten(-1, (H, V)), out_scale=out_scale)
+
+
 class ParallelMixer(nn.Module):
     """left_scale * left(h) + right_scale * right(h) for two split mixers:
     one GEMM projects h for both, each core() writes its head outputs,
     already multiplied by its scale, into its columns of one buffer, and
     one GEMM over [W_o,left | W_o,right] sums the two results. The left
     out-projection's bias (times its scale) is handed to the caller as
-    out_bias (fp32), to be added where the result meets the residual."""
+    out_bias (fp32), to be added where the result meets the residual.
+
+    out_norm: each side has an out-projection of its own, and forward()
+    returns both results, which the block norms with the weights `out_norms`
+    where it adds them to the residual (left_scale and right_scale are the
+    block's to apply). pad_rows: the in-projection's rows are padded with
+    zero rows to a multiple of it."""
 
     def __init__(self, width: int, left: SplitMixer, right: SplitMixer,
-                 left_scale: float, right_scale: float, dtype):
+                 left_scale: float, right_scale: float, dtype,
+                 out_norm: bool = False, pad_rows: int = 1):
         super().__init__()
+        assert not out_norm or not (left.out_has_bias or right.out_has_bias)
         self.left, self.right = left, right
         self.scales = (float(left_scale), float(right_scale))
         self._spans = [("left." + n, r, b) for n, r, b in left.in_spans()] + \
@@ -1035,10 +1190,20 @@ class ParallelMixer(nn.Module):
         self.rows = (sum(r for _, r, _ in left.in_spans()),
                      sum(r for _, r, _ in right.in_spans()))
         self.cols = (left.out_cols, right.out_cols)
-        self.w_in = _param(sum(self.rows), width, dtype=dtype)
-        self.b_in = (_param(sum(self.rows), dtype=dtype)
+        rows = sum(self.rows)
+        rows += -rows % pad_rows
+        self.w_in = _param(rows, width, dtype=dtype)
+        self.b_in = (_param(rows, dtype=dtype)
                      if any(b for _, _, b in self._spans) else None)
-        self.w_out = _param(width, sum(self.cols), dtype=dtype)
+        self.out_norms = None
+        if out_norm:
+            self.w_left = _param(width, self.cols[0], dtype=dtype)
+            self.w_right = _param(width, self.cols[1], dtype=dtype)
+            self.norm_left = _param(width, dtype=torch.float32)
+            self.norm_right = _param(width, dtype=torch.float32)
+            self.out_norms = (self.norm_left, self.norm_right)
+        else:
+            self.w_out = _param(width, sum(self.cols), dtype=dtype)
         self.o_b = {side: _param(width, dtype=torch.float32)
                     for side, m in (("left", left), ("right", right))
                     if m.out_has_bias}
@@ -1049,12 +1214,19 @@ class ParallelMixer(nn.Module):
 
     def weight_map(self) -> dict:
         m, row = {}, 0
+        width = self.w_in.shape[1]
         for name, n, has_b in self._spans:
-            m[name] = (self.w_in, row)
+            m[name] = (self.w_in, row, 0, (n, width))
             if has_b:
                 m[name + ".b"] = (self.b_in, row)
             row += n
-        width = self.w_out.shape[0]
+        for side, mixer in (("left.", self.left), ("right.", self.right)):
+            m.update({side + k: v for k, v in mixer.extra_weights().items()})
+        if self.out_norms is not None:
+            m["left.o"], m["right.o"] = (self.w_left, 0), (self.w_right, 0)
+            m["left.out"] = (self.norm_left, 0)
+            m["right.out"] = (self.norm_right, 0)
+            return m
         m["left.o"] = (self.w_out, 0, 0, (width, self.cols[0]))
         m["right.o"] = (self.w_out, 0, self.cols[0], (width, self.cols[1]))
         for side in self.o_b:
@@ -1062,6 +1234,9 @@ class ParallelMixer(nn.Module):
         return m
 
     def finish_loading(self) -> None:
+        for mixer in (self.left, self.right):
+            if hasattr(mixer, "finish_loading"):
+                mixer.finish_loading()
         if self.out_bias is not None:
             total = torch.zeros_like(self.out_bias.data)
             for side, scale in zip(("left", "right"), self.scales):
@@ -1076,12 +1251,22 @@ class ParallelMixer(nn.Module):
                     self.right.cache_layout(block_size, dtype).items()})
         return out
 
-    def forward(self, xs, batch: ForwardBatch, cache: dict) -> torch.Tensor:
+    def forward(self, xs, batch: ForwardBatch, cache: dict):
         p = linear(xs, self.w_in, self.b_in)
-        out = torch.empty((xs.shape[0], sum(self.cols)), dtype=xs.dtype,
-                          device=xs.device)
         lc = {k[5:]: v for k, v in cache.items() if k.startswith("left.")}
         rc = {k[6:]: v for k, v in cache.items() if k.startswith("right.")}
+        if self.out_norms is not None:
+            res = []
+            for mixer, c, w, cols, at in (
+                    (self.left, lc, self.w_left, self.cols[0], 0),
+                    (self.right, rc, self.w_right, self.cols[1], self.rows[0])):
+                out = torch.empty((xs.shape[0], cols), dtype=xs.dtype,
+                                  device=xs.device)
+                mixer.core(p[:, at:], batch, c, out, 1.0)
+                res.append(linear(out, w))
+            return tuple(res)
+        out = torch.empty((xs.shape[0], sum(self.cols)), dtype=xs.dtype,
+                          device=xs.device)
         self.left.core(p[:, :self.rows[0]], batch, lc, out[:, :self.cols[0]],
                        self.scales[0])
         self.right.core(p[:, self.rows[0]:], batch, rc, out[:, self.cols[0]:],
@@ -1150,6 +1335,21 @@ def build_mixer(kind: str, m: dict, width: int, eps: float, dtype,
                 own_projections=own_projections, sink=False,
                 interleaved=False, rot_scaling=rot.get("scaling"),
                 window=(m.get("mask") or {}).get("size") or 0, head_gate=True)
+        raise ValueError(f"unknown mixer type {kind!r}")
+    if arch == "Fuzelorn":
+        if kind == "parallel":
+            L, R = m["left"], m["right"]
+            temp = L.get("q_temp") or {}
+            left = BiasedWindowAttention(
+                width, L["heads"], L["kv_heads"], L["dim"], L["vdim"],
+                L["scale"], (L.get("mask") or {}).get("size") or 0,
+                temp.get("coef", 0.0), temp.get("every", 0), eps, dtype,
+                own_projections=False)
+            right = HeadDeltaMixer(
+                width, R["heads"], R["kv_heads"], R["dim"], R["vdim"],
+                R["conv"], eps, dtype, own_projections=False)
+            return ParallelMixer(width, left, right, 1.0, 1.0, dtype,
+                                 out_norm=True, pad_rows=64)
         raise ValueError(f"unknown mixer type {kind!r}")
     if kind == "attention":
         return SinkRotaryAttention(

@@ -680,9 +680,10 @@ def attention_sink_paged(q, k_cache, v_cache, block_tables, seq_lens,
                          inv_freq_v=None, interleaved=True, max_q_len=0,
                          positions=None, tiles=None, sink_w=None,
                          softcap=0.0, window=0, keep_first=0, out=None,
-                         out_scale=1.0, maps=1):
+                         out_scale=1.0, maps=1, slopes=None):
     """Causal attention of packed rows over paged keys with an optional
-    sink (score 0, or sink_w per head), tanh-capped scores, a sliding
+    sink (score 0, or sink_w per head), tanh-capped scores, a distance bias
+    (slopes [H]: slope[h] (i - j) off the scores), a sliding
     window that keeps the first keep_first keys, and position-turned values
     (see ref.attention_sink_paged). bf16 rows with equal q/k and value head
     sizes the MFMA kernels are built for run those (then a pass that turns
@@ -693,6 +694,7 @@ def attention_sink_paged(q, k_cache, v_cache, block_tables, seq_lens,
     row holds M keys side by side that share the row's value, and query
     head group g * M + m reads key m of key/value head g."""
     masked = (sink_w is not None or softcap > 0 or window > 0
+              or slopes is not None
               or out is not None or maps > 1
               or k_cache.untyped_storage().data_ptr()
               == v_cache.untyped_storage().data_ptr())
@@ -706,11 +708,11 @@ def attention_sink_paged(q, k_cache, v_cache, block_tables, seq_lens,
                 and S.attention_masked_mfma(
                     out, q, k_cache, v_cache, block_tables, seq_lens,
                     cu_seqlens, token_seq, scale, sink_w, softcap, window,
-                    keep_first, out_scale, max_q_len == 1, maps)):
+                    keep_first, out_scale, max_q_len == 1, maps, slopes)):
             S.attention_sink_paged(
                 out, q, k_cache, v_cache, block_tables, seq_lens, cu_seqlens,
                 token_seq, scale, sink, None, interleaved, max_q_len, sink_w,
-                softcap, window, keep_first, out_scale, maps)
+                softcap, window, keep_first, out_scale, maps, slopes)
         return out
     if q.is_cuda:
         T, H, D = q.shape
@@ -740,12 +742,12 @@ def attention_sink_paged(q, k_cache, v_cache, block_tables, seq_lens,
         _native_seq().attention_sink_paged(
             out, q, k_cache, v_cache, block_tables, seq_lens, cu_seqlens,
             token_seq, scale, sink, inv_freq_v, interleaved, max_q_len, None,
-            0.0, 0, 0, 1.0, 1)
+            0.0, 0, 0, 1.0, 1, None)
         return out
     res = ref.attention_sink_paged(q, k_cache, v_cache, block_tables,
                                    seq_lens, cu_seqlens, scale, sink,
                                    inv_freq_v, interleaved, sink_w, softcap,
-                                   window, keep_first, maps)
+                                   window, keep_first, maps, slopes)
     if out is None:
         return res
     out.copy_((res.float() * out_scale).to(out.dtype))
@@ -1048,25 +1050,35 @@ def glu_act(gu, kind, limit=0.0, alpha=1.0, out=None, row_scale=None):
 
 
 def moe_route_grouped(logits, top, groups=1, keep=1, score="softmax",
-                      renorm=True, matrix=False, bias=None):
+                      renorm=True, matrix=False, bias=None, correction=None,
+                      group_top=1, shared_gate=False):
     """Group-limited routing: (weights [T, top] fp32, ids [T, top] int32);
     score "softmax" or "sigmoid" of the logits (+ bias [E] fp32), renorm: the
-    chosen scores divided by their sum. matrix: also a [T, E] fp32 tensor holding each row's weights at
-    the experts it uses and 0 elsewhere."""
+    chosen scores divided by their sum. correction [E]: added to the scores
+    where experts and groups are chosen, not to the weights; group_top: how
+    many of a group's largest choice scores make its own (1 or 2). matrix:
+    also a [T, E] fp32 tensor holding each row's weights at the experts it
+    uses and 0 elsewhere. shared_gate: the logits' last column is the shared
+    expert's, and its sigmoid the matrix's."""
     if logits.is_cuda:
         T, E = logits.shape
         w = torch.empty((T, top), dtype=torch.float32, device=logits.device)
         ids = torch.empty((T, top), dtype=torch.int32, device=logits.device)
         mat = (torch.empty((T, E), dtype=torch.float32, device=logits.device)
                if matrix else None)
-        _native_seq().moe_route_grouped(w, ids, logits.contiguous(), top,
-                                        groups, keep, score == "sigmoid",
-                                        bool(renorm), mat, bias)
+        _native_seq().moe_route_grouped(w, ids, logits, top, groups, keep,
+                                        score == "sigmoid", bool(renorm), mat,
+                                        bias, correction, group_top,
+                                        bool(shared_gate))
         return (w, ids, mat) if matrix else (w, ids)
-    w, ids = ref.moe_route_grouped(logits, top, groups, keep, score, renorm,
-                                   bias)
+    experts = logits[:, :logits.shape[1] - bool(shared_gate)]
+    w, ids = ref.moe_route_grouped(experts, top, groups, keep, score, renorm,
+                                   bias, correction, group_top)
     if matrix:
-        return w, ids, ref.route_scale_matrix(w, ids, logits.shape[1])
+        mat = ref.route_scale_matrix(w, ids, experts.shape[1])
+        if shared_gate:
+            mat = torch.cat([mat, torch.sigmoid(logits[:, -1:].float())], 1)
+        return w, ids, mat
     return w, ids
 
 
@@ -1267,35 +1279,44 @@ def diff_head_norm_gate(a, gate, lam, eps, mult, heads, kv_heads, out):
                                    out)
 
 
-def moe_glu_scaled(gu, scale, experts, ff, shared_ff, scale_input=True):
+def moe_glu_scaled(gu, scale, experts, ff, shared_ff, scale_input=True,
+                   act="swiglu", limit=0.0, shared_limit=0.0, alpha=1.0,
+                   shared_scale=False):
     """Activated rows of all experts side by side, each expert's gate and
     up (or, without scale_input, their activated product) scaled by the
-    row's weight for it, plus the shared expert's (ref.moe_glu_scaled)."""
+    row's weight for it, plus the shared expert's, scaled by the last column
+    of scale with shared_scale (ref.moe_glu_scaled)."""
     if gu.is_cuda:
         out = torch.empty((gu.shape[0], experts * ff + shared_ff),
                           dtype=gu.dtype, device=gu.device)
         _native_seq().moe_glu_scaled(out, gu, scale, experts, ff, shared_ff,
-                                     bool(scale_input))
+                                     bool(scale_input), act == "clamped",
+                                     bool(shared_scale), float(limit),
+                                     float(shared_limit), float(alpha))
         return out
-    return ref.moe_glu_scaled(gu, scale, experts, ff, shared_ff, scale_input)
+    return ref.moe_glu_scaled(gu, scale, experts, ff, shared_ff, scale_input,
+                              act, limit, shared_limit, alpha, shared_scale)
 
 
 # ----------------------------------------------------------------------
 # Sandwich-norm blocks, per-head output gate, capped logits, channel-decay
 # delta rule (same extension, same rule).
 # ----------------------------------------------------------------------
-def residual_sandwich_norm(x, y, w_post, mult, w_pre, eps, out_dtype):
-    """x (fp32 residual, in place) += mult * rms_norm(y) * w_post when y is
-    given; returns rms_norm(x) * w_pre in out_dtype (None without w_pre):
-    the norm behind one sublayer, the sum and the norm in front of the next
-    from one pass."""
+def residual_sandwich_norm(x, y, w_post, mult, w_pre, eps, out_dtype,
+                           y2=None, w_post2=None):
+    """x (fp32 residual, in place) += mult * (rms_norm(y) * w_post +
+    rms_norm(y2) * w_post2) for the results given (one without a weight is
+    added as it is); returns rms_norm(x) * w_pre in out_dtype (None without
+    w_pre): the norms behind one sublayer, the sum and the norm in front of
+    the next from one pass."""
     if x.is_cuda:
         h = (torch.empty(x.shape, dtype=out_dtype, device=x.device)
              if w_pre is not None else None)
         _native_seq().residual_sandwich_norm(x, h, y, w_post, float(mult),
-                                             w_pre, float(eps))
+                                             w_pre, float(eps), y2, w_post2)
         return h
-    return ref.residual_sandwich_norm(x, y, w_post, mult, w_pre, eps, out_dtype)
+    return ref.residual_sandwich_norm(x, y, w_post, mult, w_pre, eps,
+                                      out_dtype, y2, w_post2)
 
 
 def softcap_(x, cap):
@@ -1321,9 +1342,11 @@ use_delta_mfma = True  # tests switch it off to compare both paths
 
 def channel_delta(u, decay, beta, gate, rate, dt_bias, norm_w, eps, state,
                   cu_seqlens, seq_lens, state_slots, heads, kv_heads, dim,
-                  vdim, out, max_q_len=0, chunks=None):
-    """Delta rule with a decay per key channel and its gated unit-RMS
-    read-out (ref.channel_delta) into out [T, H*V] (rows may be strided).
+                  vdim, out, max_q_len=0, chunks=None, head_decay=False,
+                  silu_gate=False):
+    """Delta rule with a decay per key channel (head_decay: one per head) and
+    its gated unit-RMS read-out (ref.channel_delta; silu_gate: silu instead
+    of sigmoid) into out [T, H*V] (rows may be strided).
     chunks (scan_chunks of this step, DELTA_CHUNK rows each): bf16 rows with
     head sizes the matrix-core kernels are built for run those; anything
     else runs row by row."""
@@ -1333,13 +1356,60 @@ def channel_delta(u, decay, beta, gate, rate, dt_bias, norm_w, eps, state,
                     out, u, decay, beta, gate, rate, dt_bias, norm_w,
                     float(eps), ref.DELTA_UNIT_EPS, state, chunks["off"],
                     chunks["cu"], cu_seqlens, seq_lens, state_slots, heads,
-                    kv_heads, dim, vdim)):
+                    kv_heads, dim, vdim, bool(head_decay), bool(silu_gate))):
             return out
         _native_seq().channel_delta_scan(
             out, u, decay, beta, gate, rate, dt_bias, norm_w, float(eps),
             ref.DELTA_UNIT_EPS, state, cu_seqlens, seq_lens, state_slots,
-            heads, kv_heads, dim, vdim, max_q_len)
+            heads, kv_heads, dim, vdim, max_q_len, bool(head_decay),
+            bool(silu_gate))
         return out
     return ref.channel_delta(u, decay, beta, gate, rate, dt_bias, norm_w, eps,
                              state, cu_seqlens, seq_lens, state_slots, heads,
-                             kv_heads, dim, vdim, out)
+                             kv_heads, dim, vdim, out, head_decay, silu_gate)
+
+
+# ----------------------------------------------------------------------
+# Pre-norm two-mixer blocks: hashed embedding of token pairs, q/k norm over
+# all heads at once, squared relu (same extension, same rule).
+# ----------------------------------------------------------------------
+def hashed_embed(ids, embed, table, prev, cu_seqlens, seq_lens, state_slots,
+                 token_seq, scale, mul_prev, mul_cur, max_q_len=0):
+    """fp32 rows embed[token] * scale + table[hash of (previous token,
+    token)] (ref.hashed_embed). prev [slots] int32: every sequence's last
+    token, replaced. max_q_len 1 (one row per sequence): one launch."""
+    if embed.is_cuda:
+        x = torch.empty((ids.shape[0], embed.shape[1]), dtype=torch.float32,
+                        device=embed.device)
+        _native_seq().hashed_embed(x, ids, embed, table, prev, cu_seqlens,
+                                   seq_lens, state_slots, token_seq,
+                                   float(scale), int(mul_prev), int(mul_cur),
+                                   max_q_len == 1)
+        return x
+    return ref.hashed_embed(ids, embed, table, prev, cu_seqlens, seq_lens,
+                            state_slots, scale, mul_prev, mul_cur)
+
+
+def row_norm_qk_cache(q, k, v, q_norm_w, k_norm_w, eps, positions, temp_coef,
+                      temp_every, k_cache, v_cache, slot_mapping):
+    """q [T, H*D] and k [T, G*D] normed over all their heads at once, q times
+    the position's factor, k and v to their pages (ref.row_norm_qk_cache).
+    Returns q [T, H*D]."""
+    if q.is_cuda:
+        qo = torch.empty(q.shape, dtype=q.dtype, device=q.device)
+        _native_seq().row_norm_qk_cache(
+            qo, q, k, v, q_norm_w, k_norm_w, float(eps), positions,
+            float(temp_coef), int(temp_every), k_cache, v_cache, slot_mapping)
+        return qo
+    return ref.row_norm_qk_cache(q, k, v, q_norm_w, k_norm_w, eps, positions,
+                                 temp_coef, temp_every, k_cache, v_cache,
+                                 slot_mapping)
+
+
+def relu_square(x):
+    """max(x, 0)^2."""
+    if x.is_cuda:
+        out = torch.empty(x.shape, dtype=x.dtype, device=x.device)
+        _native_seq().relu_square(out, x)
+        return out
+    return ref.relu_square(x)

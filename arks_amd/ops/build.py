@@ -57,6 +57,7 @@ SEQ_SOURCES = [
     os.path.join(CSRC, "seq_masked_mfma.hip"),
     os.path.join(CSRC, "seq_dual.hip"),
     os.path.join(CSRC, "seq_sandwich.hip"),
+    os.path.join(CSRC, "seq_prenorm.hip"),
     os.path.join(CSRC, "seq_delta.hip"),
     os.path.join(CSRC, "seq_delta_mfma.hip"),
 ]

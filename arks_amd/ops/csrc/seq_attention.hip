@@ -10,8 +10,9 @@
 // key of score 0 without a value, i.e. the running state starts at
 // (max 0, sum 1) instead of (-inf, 0); with sink_w the sink's score is a
 // number per head, (max sink_w[h], sum 1). softcap c > 0 turns a score s
-// into c tanh(s / c). window w > 0: the row at position i sees key j <= i
-// only if i - j < w or j < keep_first; tiles with no visible key are
+// into c tanh(s / c); slopes [H] takes slope[h] (i - j) off the score of the
+// row at position i for key j (not off the sink). window w > 0: the row at
+// position i sees key j <= i only if i - j < w or j < keep_first; tiles with no visible key are
 // skipped. Key and value rows have their own strides (ldk, ldv), so the
 // value may be a leading part of the key's row (latent attention keeps one
 // row per token for both). The output is a row-strided view (ldo), scaled
@@ -37,7 +38,7 @@ __global__ __launch_bounds__(64) void attn_sink_generic_kernel(
     int H, int G, int D, int V, int block_size, int max_blocks,
     const float* __restrict__ sink_w, float softcap, int window,
     int keep_first, int64_t ldk, int64_t ldv, int64_t ldo, float out_scale,
-    int maps) {
+    int maps, const float* __restrict__ slopes) {
   __shared__ float q_s[ATT_MAX_D];
   __shared__ float p_s[64];
   __shared__ int64_t voff_s[64];
@@ -60,6 +61,7 @@ __global__ __launch_bounds__(64) void attn_sink_generic_kernel(
   float acc[ATT_VPT];
 #pragma unroll
   for (int i = 0; i < ATT_VPT; ++i) acc[i] = 0.f;
+  const float slope = slopes ? slopes[h] : 0.f;
   // first key of the window; keys in [keep_first, lo) are hidden
   const int lo = window > 0 ? max(0, pos - window + 1) : 0;
   for (int j0 = 0; j0 < nkeys; j0 += 64) {
@@ -76,6 +78,7 @@ __global__ __launch_bounds__(64) void attn_sink_generic_kernel(
       for (int d = 0; d < D; ++d) dot += q_s[d] * Act<AT>::ld(kr + d);
       sc = dot * scale;
       if (softcap > 0.f) sc = softcap * tanhf(sc / softcap);
+      if (slopes) sc -= slope * (float)(pos - j);
     }
     const float m_new = fmaxf(m, wave_reduce_max(sc));
     const float p = valid ? expf(sc - m_new) : 0.f;
@@ -140,7 +143,7 @@ extern "C" int arks_seq_attn_sink_generic(
     int interleaved, int T, int H, int G, int D, int V, int block_size,
     int max_blocks, int act_f32, const void* sink_w, float softcap,
     int window, int keep_first, int64_t ldk, int64_t ldv, int64_t ldo,
-    float out_scale, int maps, hipStream_t stream) {
+    float out_scale, int maps, const void* slopes, hipStream_t stream) {
   if (D > ATT_MAX_D || V > 64 * ATT_VPT) return 1;
   if (T == 0) return 0;
   SEQ_DISPATCH_ACT(act_f32, hipLaunchKernelGGL(
@@ -149,6 +152,6 @@ extern "C" int arks_seq_attn_sink_generic(
       (const int*)block_tables, (const int*)seq_lens, (const int*)cu,
       (const int*)token_seq, scale, sink, (const float*)freq_v, interleaved, H,
       G, D, V, block_size, max_blocks, (const float*)sink_w, softcap, window,
-      keep_first, ldk, ldv, ldo, out_scale, maps));
+      keep_first, ldk, ldv, ldo, out_scale, maps, (const float*)slopes));
   return 0;
 }

@@ -38,7 +38,7 @@ int arks_seq_attn_sink_generic(
     int interleaved, int T, int H, int G, int D, int V, int block_size,
     int max_blocks, int act_f32, const void* sink_w, float softcap,
     int window, int keep_first, int64_t ldk, int64_t ldv, int64_t ldo,
-    float out_scale, int maps, hipStream_t stream);
+    float out_scale, int maps, const void* slopes, hipStream_t stream);
 int arks_seq_lightning_scan(void* out, const void* q, const void* k,
                             const void* v, int64_t ldq, int64_t ldk,
                             int64_t ldv, const void* decay, void* state,
@@ -164,12 +164,14 @@ int arks_seq_attn_masked_mfma(void* out, int64_t ldo, const void* q,
                               int T, int H, int G, int D, int V, int bs,
                               int max_blocks, int num_seqs, int single_rows,
                               void* ws, int ksplit, int maps,
-                              hipStream_t stream);
+                              const void* slopes, hipStream_t stream);
 int arks_seq_attn_masked_ksplit(int T, int H, int G, int max_blocks);
 int arks_seq_moe_route_grouped(void* weights, void* ids, const void* logits,
-                               int T, int E, int top, int groups, int keep,
-                               int sigmoid, int renorm, void* matrix,
-                               const void* bias, hipStream_t stream);
+                               int64_t ldl, int T, int E, int top, int groups,
+                               int keep, int sigmoid, int renorm, void* matrix,
+                               const void* bias, const void* correction,
+                               int group_top, int shared_gate,
+                               hipStream_t stream);
 int arks_seq_moe_sort_pairs(void* row_of_place, void* place, void* counts,
                             const void* ids, int n, int k, int E, int pad,
                             hipStream_t stream);
@@ -196,13 +198,30 @@ int arks_seq_diff_head_norm_gate(void* out, int64_t ldo, const void* a,
                                  float eps, float mult, int T, int H, int G,
                                  int V, int act_f32, hipStream_t stream);
 void arks_seq_moe_glu_scaled(void* out, const void* gu, int64_t ldg,
-                             const void* scale, int64_t T, int E, int ff,
-                             int sff, int scale_in, int act_f32,
-                             hipStream_t stream);
+                             const void* scale, int64_t lds, int64_t T, int E,
+                             int ff, int sff, int scale_in, int clamped,
+                             int shared_scale, float limit, float shared_limit,
+                             float alpha, int act_f32, hipStream_t stream);
 void arks_seq_residual_sandwich_norm(void* x, void* h, const void* y,
-                                     const void* w_post, float mult,
+                                     const void* w_post, const void* y2,
+                                     const void* w_post2, float mult,
                                      const void* w_pre, float eps, int64_t T,
                                      int C, int act_f32, hipStream_t stream);
+void arks_seq_hashed_embed(void* x, const void* ids, const void* embed,
+                           const void* table, void* prev, const void* cu,
+                           const void* seq_lens, const void* slots,
+                           const void* token_seq, float scale,
+                           int64_t mul_prev, int64_t mul_cur, int64_t buckets,
+                           int T, int S, int W, int single, int act_f32,
+                           hipStream_t stream);
+void arks_seq_row_norm_qk_cache(
+    void* qo, const void* q, const void* k, const void* v, int64_t ldq,
+    int64_t ldk, int64_t ldv, const void* qw, const void* kw, float eps,
+    const void* positions, float temp_coef, int temp_every, void* k_cache,
+    void* v_cache, const void* slot_mapping, int T, int H, int G, int D, int V,
+    int bs, int act_f32, hipStream_t stream);
+void arks_seq_relu_square(void* out, const void* x, int64_t n, int act_f32,
+                          hipStream_t stream);
 void arks_seq_softcap(void* x, int64_t n, float cap, hipStream_t stream);
 void arks_seq_head_gate(void* out, int64_t lot, int64_t loh, const void* o,
                         int64_t lit, int64_t lih, const void* gate,
@@ -214,7 +233,8 @@ int arks_seq_channel_delta_scan(
     int gate_f32, const void* rate, const void* dt_bias, const void* norm_w,
     float eps, float unit_eps, void* state, const void* cu,
     const void* seq_lens, const void* slots, int S, int H, int G, int D, int V,
-    int max_rows, int one_row, int act_f32, hipStream_t stream);
+    int max_rows, int one_row, int head_decay, int silu_gate, int act_f32,
+    hipStream_t stream);
 int64_t arks_seq_delta_chunk_floats(int D, int V);
 int arks_seq_delta_chunks_fit(int64_t ldo, int64_t ldu, int64_t ldg,
                               const void* out, const void* u, const void* gate,
@@ -226,7 +246,8 @@ int arks_seq_delta_chunks(
     const void* dt_bias, const void* norm_w, float eps, float unit_eps,
     void* state, const void* chunk_off, const void* chunk_cu, const void* cu,
     const void* seq_lens, const void* slots, int64_t T, int chunks, int S,
-    int H, int G, int D, int V, hipStream_t stream);
+    int H, int G, int D, int V, int head_decay, int silu_gate,
+    hipStream_t stream);
 void arks_seq_lightning_combine(void* part, const void* decay, void* state,
                                 const void* chunk_off, const void* chunk_rows,
                                 const void* cu, const void* seq_lens,
@@ -459,13 +480,21 @@ void qk_norm_rope_cache(Tensor qo, Tensor q, Tensor k, Tensor v, OptTensor qw,
   TORCH_CHECK(rc == 0, "more rotary pairs than the kernel's table holds");
 }
 
+// Slopes of a distance bias, one per query head (or none).
+const void* slopes_ptr(const OptTensor& slopes, int H) {
+  if (!slopes.has_value()) return nullptr;
+  check_f32(*slopes, "slopes");
+  TORCH_CHECK(slopes->numel() == H);
+  return slopes->data_ptr();
+}
+
 void attention_sink_paged(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache,
                           Tensor block_tables, Tensor seq_lens, Tensor cu,
                           Tensor token_seq, double scale, bool sink,
                           OptTensor freq_v, bool interleaved,
                           int64_t max_q_len, OptTensor sink_w, double softcap,
                           int64_t window, int64_t keep_first,
-                          double out_scale, int64_t maps) {
+                          double out_scale, int64_t maps, OptTensor slopes) {
   const int f32 = act_flag(q, "q");
   TORCH_CHECK(q.is_contiguous() && q.dim() == 3 && maps >= 1);
   const int T = q.size(0), H = q.size(1), D = q.size(2);
@@ -506,7 +535,7 @@ void attention_sink_paged(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache,
       token_seq.data_ptr(), (float)scale, sink ? 1 : 0, fv_p,
       interleaved ? 1 : 0, T, H, G, D, V, bs, (int)block_tables.size(1), f32,
       sw_p, (float)softcap, (int)window, (int)keep_first, ldk, ldv, ldo,
-      (float)out_scale, (int)maps, current_stream());
+      (float)out_scale, (int)maps, slopes_ptr(slopes, H), current_stream());
   TORCH_CHECK(rc == 0, "attention head sizes beyond the kernel's limits (",
               D, ", ", V, ")");
 }
@@ -964,28 +993,39 @@ bool attention_window_pool_mfma(Tensor out, Tensor q, Tensor k_cache,
 
 void moe_route_grouped(Tensor weights, Tensor ids, Tensor logits, int64_t top,
                        int64_t groups, int64_t keep, bool sigmoid, bool renorm,
-                       OptTensor matrix, OptTensor bias) {
-  check_f32(logits, "router logits");
+                       OptTensor matrix, OptTensor bias, OptTensor correction,
+                       int64_t group_top, bool shared_gate) {
+  TORCH_CHECK(logits.is_cuda() && logits.scalar_type() == torch::kFloat32 &&
+              logits.dim() == 2, "router logits must be float [T, E]");
   check_f32(weights, "weights");
   check_i32(ids, "ids");
-  const int T = logits.size(0), E = logits.size(1);
+  // shared_gate: one logit more per row, the shared expert's
+  const int T = logits.size(0), E = logits.size(1) - (shared_gate ? 1 : 0);
+  TORCH_CHECK(group_top == 1 || group_top == 2);
   TORCH_CHECK(weights.size(0) == T && weights.size(1) == top &&
               ids.size(0) == T && ids.size(1) == top);
   void* mat_p = nullptr;
   if (matrix.has_value()) {
     check_f32(*matrix, "scale matrix");
     TORCH_CHECK(matrix->dim() == 2 && matrix->size(0) == T &&
-                matrix->size(1) == E);
+                matrix->size(1) == logits.size(1));
     mat_p = matrix->data_ptr();
   }
   if (bias.has_value()) {
     check_f32(*bias, "router bias");
     TORCH_CHECK(bias->numel() == E);
   }
+  if (correction.has_value()) {
+    check_f32(*correction, "choice correction");
+    TORCH_CHECK(correction->numel() == E);
+  }
   const int rc = arks_seq_moe_route_grouped(
-      weights.data_ptr(), ids.data_ptr(), logits.data_ptr(), T, E, (int)top,
+      weights.data_ptr(), ids.data_ptr(), logits.data_ptr(),
+      row_stride(logits, "logits"), T, E, (int)top,
       (int)groups, (int)keep, sigmoid ? 1 : 0, renorm ? 1 : 0, mat_p,
-      bias.has_value() ? bias->data_ptr() : nullptr, current_stream());
+      bias.has_value() ? bias->data_ptr() : nullptr,
+      correction.has_value() ? correction->data_ptr() : nullptr,
+      (int)group_top, shared_gate ? 1 : 0, current_stream());
   TORCH_CHECK(rc == 0, "routing sizes the kernel does not hold");
 }
 
@@ -1158,21 +1198,26 @@ void diff_head_norm_gate(Tensor out, Tensor a, Tensor gate, double lam,
 }
 
 void moe_glu_scaled(Tensor out, Tensor gu, Tensor scale, int64_t experts,
-                    int64_t ff, int64_t shared_ff, bool scale_input) {
+                    int64_t ff, int64_t shared_ff, bool scale_input,
+                    bool clamped, bool shared_scale, double limit,
+                    double shared_limit, double alpha) {
   const int f32 = act_flag(gu, "gate|up");
-  check_f32(scale, "scale");
+  TORCH_CHECK(scale.is_cuda() && scale.scalar_type() == torch::kFloat32);
   const int64_t T = gu.size(0);
   TORCH_CHECK(gu.dim() == 2 &&
               gu.size(1) == experts * 2 * ff + 2 * shared_ff &&
               scale.dim() == 2 && scale.size(0) == T &&
-              scale.size(1) == experts);
+              scale.size(1) == experts + (shared_scale ? 1 : 0));
   TORCH_CHECK(out.scalar_type() == gu.scalar_type() && out.is_contiguous() &&
               out.dim() == 2 && out.size(0) == T &&
               out.size(1) == experts * ff + shared_ff);
   arks_seq_moe_glu_scaled(out.data_ptr(), gu.data_ptr(),
-                          row_stride(gu, "gate|up"), scale.data_ptr(), T,
-                          (int)experts, (int)ff, (int)shared_ff,
-                          scale_input ? 1 : 0, f32, current_stream());
+                          row_stride(gu, "gate|up"), scale.data_ptr(),
+                          row_stride(scale, "scale"), T, (int)experts, (int)ff,
+                          (int)shared_ff, scale_input ? 1 : 0, clamped ? 1 : 0,
+                          shared_scale ? 1 : 0, (float)limit,
+                          (float)shared_limit, (float)alpha, f32,
+                          current_stream());
 }
 
 }  // namespace
@@ -1384,7 +1429,8 @@ bool attention_masked_mfma(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache,
                            Tensor block_tables, Tensor seq_lens, Tensor cu,
                            Tensor token_seq, double scale, OptTensor sink_w,
                            double softcap, int64_t window, int64_t keep_first,
-                           double out_scale, bool single_rows, int64_t maps) {
+                           double out_scale, bool single_rows, int64_t maps,
+                           OptTensor slopes) {
   TORCH_CHECK(q.is_cuda() && q.scalar_type() == torch::kBFloat16 &&
               q.is_contiguous() && q.dim() == 3 && maps >= 1);
   const int T = q.size(0), H = q.size(1), D = q.size(2);
@@ -1429,12 +1475,12 @@ bool attention_masked_mfma(Tensor out, Tensor q, Tensor k_cache, Tensor v_cache,
              (float)scale, sw_p, (float)softcap, (int)window, (int)keep_first,
              (float)out_scale, T, H, G, D, V, bs, (int)block_tables.size(1),
              m.S, single_rows ? 1 : 0, ksplit > 1 ? ws.data_ptr() : nullptr,
-             ksplit, (int)maps, current_stream()) == 0;
+             ksplit, (int)maps, slopes_ptr(slopes, H), current_stream()) == 0;
 }
 
 void residual_sandwich_norm(Tensor x, OptTensor h, OptTensor y,
                             OptTensor w_post, double mult, OptTensor w_pre,
-                            double eps) {
+                            double eps, OptTensor y2, OptTensor w_post2) {
   check_f32(x, "x");
   TORCH_CHECK(x.dim() == 2);
   const int64_t T = x.size(0);
@@ -1459,11 +1505,85 @@ void residual_sandwich_norm(Tensor x, OptTensor h, OptTensor y,
   const void* y_p = row_tensor(y, "y");
   const void* wpo = weight(w_post, "w_post");
   const void* wpr = weight(w_pre, "w_pre");
-  TORCH_CHECK((y_p != nullptr) <= (wpo != nullptr) &&
+  const void* y2_p = row_tensor(y2, "y2");
+  const void* wpo2 = weight(w_post2, "w_post2");
+  TORCH_CHECK((wpo != nullptr) <= (y_p != nullptr) &&
+              (y2_p != nullptr) <= (y_p != nullptr) &&
+              (wpo2 != nullptr) <= (y2_p != nullptr) &&
               (h_p != nullptr) == (wpr != nullptr));
-  arks_seq_residual_sandwich_norm(x.data_ptr(), h_p, y_p, wpo, (float)mult,
-                                  wpr, (float)eps, T, C, f32 == 1 ? 1 : 0,
-                                  current_stream());
+  arks_seq_residual_sandwich_norm(x.data_ptr(), h_p, y_p, wpo, y2_p, wpo2,
+                                  (float)mult, wpr, (float)eps, T, C,
+                                  f32 == 1 ? 1 : 0, current_stream());
+}
+
+// prev [slots] int32: every sequence's last token of the steps before.
+void hashed_embed(Tensor x, Tensor ids, Tensor embed, Tensor table,
+                  Tensor prev, Tensor cu, Tensor seq_lens, Tensor slots,
+                  Tensor token_seq, double scale, int64_t mul_prev,
+                  int64_t mul_cur, bool single) {
+  check_f32(x, "x");
+  check_i64(ids, "input_ids");
+  check_i32(prev, "previous tokens");
+  const int f32 = act_flag(embed, "embed");
+  const int64_t T = ids.numel();
+  TORCH_CHECK(x.dim() == 2 && x.size(0) == T && embed.dim() == 2 &&
+              table.dim() == 2 && embed.size(1) == x.size(1) &&
+              table.size(1) == x.size(1) && table.size(0) >= 2 &&
+              embed.is_contiguous() && table.is_contiguous() &&
+              table.scalar_type() == embed.scalar_type());
+  TORCH_CHECK(mul_prev >= 0 && mul_cur >= 0);
+  const SeqMeta m = check_meta(cu, seq_lens, &slots, &token_seq, T);
+  arks_seq_hashed_embed(x.data_ptr(), ids.data_ptr(), embed.data_ptr(),
+                        table.data_ptr(), prev.data_ptr(), cu.data_ptr(),
+                        seq_lens.data_ptr(), slots.data_ptr(),
+                        token_seq.data_ptr(), (float)scale, mul_prev, mul_cur,
+                        table.size(0) - 1, (int)T, m.S, (int)x.size(1),
+                        single && T == m.S ? 1 : 0, f32, current_stream());
+}
+
+// q [T, H * D], k [T, G * D], v [T, G * V]: row-strided views.
+void row_norm_qk_cache(Tensor qo, Tensor q, Tensor k, Tensor v, Tensor qw,
+                       Tensor kw, double eps, Tensor positions,
+                       double temp_coef, int64_t temp_every, Tensor k_cache,
+                       Tensor v_cache, Tensor slot_mapping) {
+  const int f32 = act_flag(q, "q");
+  TORCH_CHECK(q.dim() == 2 && k.dim() == 2 && v.dim() == 2 &&
+              k_cache.dim() == 4 && v_cache.dim() == 4);
+  const int64_t T = q.size(0);
+  const int64_t G = k_cache.size(1), bs = k_cache.size(2), D = k_cache.size(3),
+                V = v_cache.size(3);
+  TORCH_CHECK(k.scalar_type() == q.scalar_type() &&
+              v.scalar_type() == q.scalar_type() &&
+              qo.scalar_type() == q.scalar_type() &&
+              k_cache.scalar_type() == q.scalar_type() &&
+              v_cache.scalar_type() == q.scalar_type());
+  TORCH_CHECK(k_cache.is_contiguous() && v_cache.is_contiguous() &&
+              v_cache.size(0) == k_cache.size(0) && v_cache.size(1) == G &&
+              v_cache.size(2) == bs);
+  TORCH_CHECK(q.size(1) % (G * D) == 0 && k.size(0) == T && v.size(0) == T &&
+              k.size(1) == G * D && v.size(1) == G * V);
+  TORCH_CHECK(qo.is_contiguous() && qo.sizes() == q.sizes());
+  check_f32(qw, "q norm weight");
+  check_f32(kw, "k norm weight");
+  TORCH_CHECK(qw.numel() == q.size(1) && kw.numel() == G * D);
+  check_i64(positions, "positions");
+  check_i64(slot_mapping, "slot_mapping");
+  TORCH_CHECK(positions.numel() == T && slot_mapping.numel() == T);
+  arks_seq_row_norm_qk_cache(
+      qo.data_ptr(), q.data_ptr(), k.data_ptr(), v.data_ptr(),
+      row_stride(q, "q"), row_stride(k, "k"), row_stride(v, "v"), qw.data_ptr(),
+      kw.data_ptr(), (float)eps, positions.data_ptr(), (float)temp_coef,
+      (int)temp_every, k_cache.data_ptr(), v_cache.data_ptr(),
+      slot_mapping.data_ptr(), (int)T, (int)(q.size(1) / D), (int)G, (int)D,
+      (int)V, (int)bs, f32, current_stream());
+}
+
+void relu_square(Tensor out, Tensor x) {
+  const int f32 = act_flag(x, "x");
+  TORCH_CHECK(x.is_contiguous() && out.is_contiguous() &&
+              out.scalar_type() == x.scalar_type() && out.sizes() == x.sizes());
+  arks_seq_relu_square(out.data_ptr(), x.data_ptr(), x.numel(), f32,
+                       current_stream());
 }
 
 void softcap(Tensor x, double cap) {
@@ -1503,14 +1623,19 @@ DeltaArgs check_delta(const Tensor& out, const Tensor& u, const Tensor& decay,
                       const Tensor& beta, const Tensor& gate,
                       const Tensor& rate, const Tensor& dt_bias,
                       const Tensor& norm_w, const Tensor& state, int64_t H,
-                      int64_t G, int64_t D, int64_t V) {
+                      int64_t G, int64_t D, int64_t V, bool head_decay) {
   DeltaArgs a;
   a.f32 = act_flag(u, "u");
   const int64_t T = u.size(0);
   TORCH_CHECK(G >= 1 && H % G == 0 && D >= 1 && V >= 1);
   TORCH_CHECK(u.dim() == 2 && u.size(1) == 2 * G * D + H * V);
-  TORCH_CHECK(decay.is_cuda() && decay.scalar_type() == torch::kFloat32 &&
-              decay.dim() == 2 && decay.size(0) == T && decay.size(1) == H * D);
+  // one decay per head comes in the rows' type, one per channel in fp32
+  const int64_t decays = head_decay ? H : H * D;
+  TORCH_CHECK(decay.is_cuda() &&
+              decay.scalar_type() ==
+                  (head_decay ? u.scalar_type() : torch::kFloat32) &&
+              decay.dim() == 2 && decay.size(0) == T &&
+              decay.size(1) == decays);
   TORCH_CHECK(beta.scalar_type() == u.scalar_type() && beta.dim() == 2 &&
               beta.size(0) == T && beta.size(1) == H);
   a.gate_f32 = act_flag(gate, "gate");
@@ -1522,7 +1647,7 @@ DeltaArgs check_delta(const Tensor& out, const Tensor& u, const Tensor& decay,
   check_f32(dt_bias, "dt_bias");
   check_f32(norm_w, "norm weight");
   check_f32(state, "state");
-  TORCH_CHECK(rate.numel() == H && dt_bias.numel() == H * D &&
+  TORCH_CHECK(rate.numel() == H && dt_bias.numel() == decays &&
               norm_w.numel() == V);
   TORCH_CHECK(state.dim() == 4 && state.size(1) == H && state.size(2) == D &&
               state.size(3) == V);
@@ -1539,9 +1664,9 @@ void channel_delta_scan(Tensor out, Tensor u, Tensor decay, Tensor beta,
                         Tensor norm_w, double eps, double unit_eps,
                         Tensor state, Tensor cu, Tensor seq_lens, Tensor slots,
                         int64_t H, int64_t G, int64_t D, int64_t V,
-                        int64_t max_rows) {
+                        int64_t max_rows, bool head_decay, bool silu_gate) {
   const DeltaArgs a = check_delta(out, u, decay, beta, gate, rate, dt_bias,
-                                  norm_w, state, H, G, D, V);
+                                  norm_w, state, H, G, D, V, head_decay);
   const SeqMeta m = check_meta(cu, seq_lens, &slots, nullptr, 0);
   const int rc = arks_seq_channel_delta_scan(
       out.data_ptr(), a.ldo, u.data_ptr(), a.ldu, decay.data_ptr(), a.lda,
@@ -1549,7 +1674,8 @@ void channel_delta_scan(Tensor out, Tensor u, Tensor decay, Tensor beta,
       rate.data_ptr(), dt_bias.data_ptr(), norm_w.data_ptr(), (float)eps,
       (float)unit_eps, state.data_ptr(), cu.data_ptr(), seq_lens.data_ptr(),
       slots.data_ptr(), m.S, (int)H, (int)G, (int)D, (int)V, (int)max_rows,
-      u.size(0) == m.S ? 1 : 0, a.f32, current_stream());
+      u.size(0) == m.S ? 1 : 0, head_decay ? 1 : 0, silu_gate ? 1 : 0, a.f32,
+      current_stream());
   TORCH_CHECK(rc == 0, "delta-rule head sizes the kernel does not hold (", D,
               ", ", V, ")");
 }
@@ -1562,9 +1688,10 @@ bool channel_delta_chunks(Tensor out, Tensor u, Tensor decay, Tensor beta,
                           Tensor norm_w, double eps, double unit_eps,
                           Tensor state, Tensor chunk_off, Tensor chunk_cu,
                           Tensor cu, Tensor seq_lens, Tensor slots, int64_t H,
-                          int64_t G, int64_t D, int64_t V) {
+                          int64_t G, int64_t D, int64_t V, bool head_decay,
+                          bool silu_gate) {
   const DeltaArgs a = check_delta(out, u, decay, beta, gate, rate, dt_bias,
-                                  norm_w, state, H, G, D, V);
+                                  norm_w, state, H, G, D, V, head_decay);
   const SeqMeta m = check_meta(cu, seq_lens, &slots, nullptr, 0);
   check_i32(chunk_off, "chunk_off");
   check_i32(chunk_cu, "chunk_cu");
@@ -1586,12 +1713,16 @@ bool channel_delta_chunks(Tensor out, Tensor u, Tensor decay, Tensor beta,
              (float)unit_eps, state.data_ptr(), chunk_off.data_ptr(),
              chunk_cu.data_ptr(), cu.data_ptr(), seq_lens.data_ptr(),
              slots.data_ptr(), T, (int)chunks, m.S, (int)H, (int)G, (int)D,
-             (int)V, current_stream()) == 0;
+             (int)V, head_decay ? 1 : 0, silu_gate ? 1 : 0,
+             current_stream()) == 0;
 }
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("residual_tanh_norm", &residual_tanh_norm);
   m.def("residual_sandwich_norm", &residual_sandwich_norm);
+  m.def("hashed_embed", &hashed_embed);
+  m.def("row_norm_qk_cache", &row_norm_qk_cache);
+  m.def("relu_square", &relu_square);
   m.def("softcap", &softcap);
   m.def("head_gate", &head_gate);
   m.def("channel_delta_scan", &channel_delta_scan);

@@ -41,6 +41,12 @@ __device__ __forceinline__ float softplus_f(float x) {
   return x > 20.f ? x : log1pf(expf(x));
 }
 
+__device__ __forceinline__ float query_factor(int64_t pos, float coef,
+                                              int every) {
+  if (every <= 0) return 1.f;
+  return 1.f + coef * logf((float)((pos + 1) / every) + 1.f);
+}
+
 struct SeqRow {
   int seq, first_row, rows, start, slot;
 };

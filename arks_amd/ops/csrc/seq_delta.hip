@@ -1,12 +1,14 @@
-// Delta rule with a decay per head and key channel
-// (arks_amd/models/mixers.py ChannelDeltaMixer), row by row, any head sizes,
-// bf16 or float rows, fp32 arithmetic: per head, with unit-length q and k
-// (q times D^-1/2), g = exp(-rate softplus(decay + dt_bias)) per key channel
-// and b = sigmoid(beta),
+// Delta rule with a decay per head and key channel, or one per head
+// (arks_amd/models/mixers.py ChannelDeltaMixer, HeadDeltaMixer), row by row,
+// any head sizes, bf16 or float rows, fp32 arithmetic: per head, with
+// unit-length q and k (q times D^-1/2), g = exp(-rate softplus(decay +
+// dt_bias)) per key channel (or the same for all of them) and b =
+// sigmoid(beta),
 //   S <- g S,  w = b (v - S^T k),  S <- S + k w^T,  o = S^T q,
 // then o at unit RMS over the head, times the norm weight, times
-// sigmoid(gate). With s = g S from the same pass, S^T q after the update is
-// s^T q + (k . q) w, so one pass over the state serves both products.
+// sigmoid(gate) or silu(gate). With s = g S from the same pass, S^T q after
+// the update is s^T q + (k . q) w, so one pass over the state serves both
+// products.
 //
 // One block per (sequence, head). A wave owns CPW = 64 / NRG value columns;
 // its lanes are NRG groups of state rows x CPW columns, RPT rows of one
@@ -24,12 +26,35 @@ struct DeltaDims {
   int64_t ldo, ldu, lda, ldb, ldg;
   int gate_f32;
   float eps, unit_eps;
+  // head_decay: decay [T, H] in the rows' type and dt_bias [H] instead of
+  // float [T, H * D] and [H * D]
+  int head_decay, silu_gate;
 };
+
+template <typename AT>
+__device__ __forceinline__ float delta_decay(const void* decay,
+                                             const float* dt_bias, int64_t t,
+                                             int h, int d, float rate,
+                                             const DeltaDims& a) {
+  const float z =
+      a.head_decay
+          ? Act<AT>::ld(reinterpret_cast<const AT*>(decay) + t * a.lda + h) +
+                dt_bias[h]
+          : reinterpret_cast<const float*>(decay)[t * a.lda +
+                                                  (int64_t)h * a.D + d] +
+                dt_bias[(int64_t)h * a.D + d];
+  return expf(-rate * softplus_f(z));
+}
+
+__device__ __forceinline__ float delta_gate(float z, const DeltaDims& a) {
+  const float s = sigmoid_f(z);
+  return a.silu_gate ? z * s : s;
+}
 
 template <typename AT, int RPT, int NRG>
 __global__ __launch_bounds__(512) void channel_delta_scan_kernel(
     AT* __restrict__ out, const AT* __restrict__ u,
-    const float* __restrict__ decay, const AT* __restrict__ beta,
+    const void* __restrict__ decay, const AT* __restrict__ beta,
     const void* __restrict__ gate, const float* __restrict__ rate,
     const float* __restrict__ dt_bias, const float* __restrict__ norm_w,
     float* __restrict__ state, const int* __restrict__ cu,
@@ -100,8 +125,7 @@ __global__ __launch_bounds__(512) void channel_delta_scan_kernel(
         if (d < D) {
           qv = Act<AT>::ld(qr + d) * rq;
           kv = Act<AT>::ld(kr + d) * rk;
-          gv = expf(-rt * softplus_f(decay[t * a.lda + (int64_t)h * D + d] +
-                                     dt_bias[(int64_t)h * D + d]));
+          gv = delta_decay<AT>(decay, dt_bias, t, h, d, rt, a);
         }
         q_s[at] = qv;
         k_s[at] = kv;
@@ -172,7 +196,7 @@ __global__ __launch_bounds__(512) void channel_delta_scan_kernel(
         const float gv = a.gate_f32
                              ? reinterpret_cast<const float*>(gate)[gat + v]
                              : Act<AT>::ld(reinterpret_cast<const AT*>(gate) + gat + v);
-        Act<AT>::st(orow + v, o_s[r * V + v] * ro * norm_w[v] * sigmoid_f(gv));
+        Act<AT>::st(orow + v, o_s[r * V + v] * ro * norm_w[v] * delta_gate(gv, a));
       }
     }
   }
@@ -185,7 +209,7 @@ __global__ __launch_bounds__(512) void channel_delta_scan_kernel(
 template <typename AT, int NI>
 __global__ __launch_bounds__(512) void channel_delta_step_kernel(
     AT* __restrict__ out, const AT* __restrict__ u,
-    const float* __restrict__ decay, const AT* __restrict__ beta,
+    const void* __restrict__ decay, const AT* __restrict__ beta,
     const void* __restrict__ gate, const float* __restrict__ rate,
     const float* __restrict__ dt_bias, const float* __restrict__ norm_w,
     float* __restrict__ state, const int* __restrict__ cu,
@@ -220,8 +244,7 @@ __global__ __launch_bounds__(512) void channel_delta_step_kernel(
     if (d < D) {
       qv = Act<AT>::ld(qr + d);
       kv = Act<AT>::ld(kr + d);
-      gv = expf(-rate[h] * softplus_f(decay[t * a.lda + (int64_t)h * D + d] +
-                                      dt_bias[(int64_t)h * D + d]));
+      gv = delta_decay<AT>(decay, dt_bias, t, h, d, rate[h], a);
     }
     q_s[d] = qv;
     k_s[d] = kv;
@@ -296,7 +319,7 @@ __global__ __launch_bounds__(512) void channel_delta_step_kernel(
                            ? reinterpret_cast<const float*>(gate)[gat + e]
                            : Act<AT>::ld(reinterpret_cast<const AT*>(gate) + gat + e);
       Act<AT>::st(out + t * a.ldo + (int64_t)h * V + v + e,
-                  o[e] * ro * norm_w[v + e] * sigmoid_f(gv));
+                  o[e] * ro * norm_w[v + e] * delta_gate(gv, a));
     }
   }
 }
@@ -319,7 +342,7 @@ static int launch_delta_scan(void* out, const void* u, const void* decay,
   const size_t lds = (size_t)a.BR * row_floats * 4;
   hipLaunchKernelGGL((channel_delta_scan_kernel<AT, RPT, NRG>), dim3(a.H, S),
                      dim3(nw * 64), lds, stream, (AT*)out, (const AT*)u,
-                     (const float*)decay, (const AT*)beta, gate,
+                     decay, (const AT*)beta, gate,
                      (const float*)rate, (const float*)dt_bias,
                      (const float*)norm_w, (float*)state, (const int*)cu,
                      (const int*)seq_lens, (const int*)slots, a);
@@ -336,16 +359,17 @@ extern "C" int arks_seq_channel_delta_scan(
     int gate_f32, const void* rate, const void* dt_bias, const void* norm_w,
     float eps, float unit_eps, void* state, const void* cu,
     const void* seq_lens, const void* slots, int S, int H, int G, int D, int V,
-    int max_rows, int one_row, int act_f32, hipStream_t stream) {
+    int max_rows, int one_row, int head_decay, int silu_gate, int act_f32,
+    hipStream_t stream) {
   if (S == 0 || H == 0) return 0;
   const DeltaDims a{H, G, D, V, 0, ldo, ldu, lda, ldb, ldg, gate_f32, eps,
-                    unit_eps};
+                    unit_eps, head_decay, silu_gate};
   if (max_rows == 1 && one_row && V % 4 == 0 && V <= 256 && D <= 128) {
 #define DT(NI)                                                                \
   SEQ_DISPATCH_ACT(act_f32, {                                                 \
     hipLaunchKernelGGL((channel_delta_step_kernel<AT, NI>), dim3(H, S),       \
                        dim3((V + 31) / 32 * 64), 0, stream, (AT*)out,         \
-                       (const AT*)u, (const float*)decay, (const AT*)beta,    \
+                       (const AT*)u, decay, (const AT*)beta,                  \
                        gate, (const float*)rate, (const float*)dt_bias,       \
                        (const float*)norm_w, (float*)state, (const int*)cu,   \
                        (const int*)seq_lens, (const int*)slots, a);           \

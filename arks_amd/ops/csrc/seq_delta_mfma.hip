@@ -1,7 +1,8 @@
-// Channel-decay delta rule of long portions on the fp32 matrix cores
+// Delta rule of long portions on the fp32 matrix cores
 // (v_mfma_f32_16x16x4_f32): the recurrence of seq_delta.hip over chunks of
 // up to 64 rows. With G_i the running sum of log decays inside a chunk
-// (per key channel), S0 the state in front of it, and unit rows q_i, k_i:
+// (per key channel, or one number per row where the decay is one per head),
+// S0 the state in front of it, and unit rows q_i, k_i:
 //
 //   (I + L) U = beta V - (beta K~) S0,   K~_i = k_i exp(G_i),
 //   L_ij = beta_i sum_d k_id k_jd exp(G_id - G_jd)   (j < i)
@@ -24,6 +25,9 @@
 // at the last row of j's group (exponents <= 0 again, one pass per group),
 // pairs inside a group about its second row; and where even two rows decay
 // past MIN_HALF_LOG, exp(c_i - c_j) is taken per channel, element by element.
+// One decay per head needs none of this: exp(G_i - G_j) is a factor of the
+// finished product, which is exact in fp32 from the raw bf16 rows
+// (v_mfma_f32_16x16x32_bf16); it is summed from the block border on as above.
 //
 // Fragments: with k = 4 g + e (g = lane / 16) the operand A of four
 // consecutive MFMAs is row lane % 16, columns 4 g .. 4 g + 3 of a 16x16 tile
@@ -71,21 +75,26 @@ __host__ __device__ inline DeltaChunk delta_chunk_layout(int D, int V) {
   return c;
 }
 
+// HEAD: one decay per head (a float per row in LDS, not one per channel)
+template <bool HEAD>
 __host__ __device__ constexpr int delta_prepare_lds(int D) {
-  return 2 * DC * (D + 8) * 2 + DC * (D + 4) * 4 + 10 * 64 * 16 + 4 * D * 4 +
-         (3 * DC + 8) * 4;
+  return 2 * DC * (D + 8) * 2 + DC * (HEAD ? 1 : D + 4) * 4 + 10 * 64 * 16 +
+         4 * (HEAD ? 1 : D) * 4 + (3 * DC + 8) * 4;
 }
 
-template <int KT>
-__global__ __launch_bounds__(256, 2) void delta_chunk_prepare_kernel(
+typedef __attribute__((ext_vector_type(8))) __bf16 delta_bf16x8;
+
+template <int KT, bool HEAD>
+__global__ __launch_bounds__(256, HEAD ? 3 : 2) void delta_chunk_prepare_kernel(
     float* __restrict__ scratch, const bf16* __restrict__ u, int64_t ldu,
-    const float* __restrict__ decay, int64_t lda,
+    const void* __restrict__ decay_p, int64_t lda,
     const bf16* __restrict__ beta, int64_t ldb, const float* __restrict__ rate,
     const float* __restrict__ dt_bias, const int* __restrict__ cu, int H,
     int G, int V, float unit_eps) {
   constexpr int D = 16 * KT;
   constexpr int LK = D + 8;  // bf16 row stride
-  constexpr int LC = D + 4;  // float row stride
+  constexpr int LC = HEAD ? 1 : D + 4;  // float row stride
+  constexpr int TC = HEAD ? 1 : D;      // decays of a block's totals
   extern __shared__ __align__(16) char smem[];
   bf16* k_s = reinterpret_cast<bf16*>(smem);           // [DC][LK]
   bf16* q_s = k_s + DC * LK;                           // [DC][LK]
@@ -94,8 +103,8 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_prepare_kernel(
   // inverses replace
   float4v* l_s = reinterpret_cast<float4v*>(c_s + DC * LC);  // [6 + 4][64]
   float4v* inv_s = l_s + 6 * 64;                       // [4][64]
-  float* tot_s = reinterpret_cast<float*>(l_s + 10 * 64);  // [4][D]
-  float* rk_s = tot_s + 4 * D;                         // [DC]
+  float* tot_s = reinterpret_cast<float*>(l_s + 10 * 64);  // [4][TC]
+  float* rk_s = tot_s + 4 * TC;                        // [DC]
   float* rq_s = rk_s + DC;                             // [DC]
   float* b_s = rq_s + DC;                              // [DC]
   float* min_s = b_s + DC;                             // [4]
@@ -107,18 +116,27 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_prepare_kernel(
   const int gk = h / (H / G);
   const DeltaChunk lay = delta_chunk_layout(D, V);
   float* base = scratch + ((int64_t)chunk * H + h) * lay.total;
+  // log decays up to a row of its block, and of a whole block
+  auto row_log = [&](int row, int d) { return c_s[row * LC + (HEAD ? 0 : d)]; };
+  auto block_log = [&](int M, int d) { return tot_s[M * TC + (HEAD ? 0 : d)]; };
 
   // ---- rows of block I: raw q, k, their unit factors, log decays. Loads
   // are of rows that exist (the last one again past the end) and are not
   // branched around, so that they are all in flight together
   constexpr int DL = (D + 63) / 64;  // channels per lane
-  float dec[DL][16];
+  float dec[HEAD ? 1 : DL][HEAD ? 1 : 16];
+  if constexpr (HEAD) {
+    dec[0][0] = bf16_bits_to_float(reinterpret_cast<const bf16*>(
+        decay_p)[(int64_t)(t0 + min(16 * I + m, n - 1)) * lda + h]);
+  } else {
+    const float* decay = reinterpret_cast<const float*>(decay_p);
 #pragma unroll
-  for (int j = 0; j < DL; ++j)
+    for (int j = 0; j < DL; ++j)
 #pragma unroll
-    for (int r = 0; r < 16; ++r)
-      dec[j][r] = decay[(int64_t)(t0 + min(16 * I + r, n - 1)) * lda +
-                        (int64_t)h * D + min(lane + 64 * j, D - 1)];
+      for (int r = 0; r < 16; ++r)
+        dec[j][r] = decay[(int64_t)(t0 + min(16 * I + r, n - 1)) * lda +
+                          (int64_t)h * D + min(lane + 64 * j, D - 1)];
+  }
   ushort8 qin[4], kin[4];
   const bool live = m * 8 < D;
 #pragma unroll
@@ -161,7 +179,20 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_prepare_kernel(
                    ? sigmoid_f(bf16_bits_to_float(beta[(int64_t)(t0 + row) * ldb + h]))
                    : 0.f;
   }
-  {
+  if constexpr (HEAD) {
+    // running sum over the block's rows, lane m of every 16 lanes has row m
+    float c = 16 * I + m < n
+                  ? -rate[h] * softplus_fast(dec[0][0] + dt_bias[h]) : 0.f;
+#pragma unroll
+    for (int off = 1; off < 16; off <<= 1) {
+      const float before = __shfl_up(c, off, 16);
+      if (m >= off) c += before;
+    }
+    if (g == 0) {
+      c_s[16 * I + m] = c;
+      if (m == 15) tot_s[I] = c;
+    }
+  } else {
     const float rt = rate[h];
     float lowest = 0.f, pair = 0.f;
 #pragma unroll
@@ -193,7 +224,54 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_prepare_kernel(
   __syncthreads();
 
   // ---- scores of block row I against every block J <= I
-  {
+  if constexpr (HEAD) {
+    const int row = 16 * I + m;
+    const float rk = rk_s[row], rq = rq_s[row], bI = b_s[row];
+    const float ci = c_s[row];
+    float pre = 0.f;
+    for (int M = 0; M < I; ++M) pre += tot_s[M];
+    const float fq = rq * __expf(pre + ci);
+#pragma unroll
+    for (int kt = 0; kt < KT; ++kt) {
+      const ushort4v qr =
+          *reinterpret_cast<const ushort4v*>(q_s + row * LK + 16 * kt + 4 * g);
+      float4v qg;
+#pragma unroll
+      for (int e = 0; e < 4; ++e) qg[e] = bf16_bits_to_float(qr[e]) * fq;
+      *reinterpret_cast<float4v*>(base + lay.Q + ((I * KT + kt) * 64 + lane) * 4) = qg;
+    }
+    constexpr int STEPS = D / 32;
+    delta_bf16x8 kI[STEPS], qI[STEPS];
+#pragma unroll
+    for (int st = 0; st < STEPS; ++st) {
+      kI[st] = *reinterpret_cast<const delta_bf16x8*>(k_s + row * LK + st * 32 + 8 * g);
+      qI[st] = *reinterpret_cast<const delta_bf16x8*>(q_s + row * LK + st * 32 + 8 * g);
+    }
+    float between = 0.f;  // whole blocks between J and I
+    for (int J = I; J >= 0; --J) {
+      float4v kk = {0.f, 0.f, 0.f, 0.f}, qk = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int st = 0; st < STEPS; ++st) {
+        const delta_bf16x8 a = *reinterpret_cast<const delta_bf16x8*>(
+            k_s + (16 * J + m) * LK + st * 32 + 8 * g);
+        kk = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, kI[st], kk, 0, 0, 0);
+        qk = __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, qI[st], qk, 0, 0, 0);
+      }
+      // lane holds (row i = m of block I, columns j = 4 g + r of block J)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int j = 4 * g + r;
+        const float cj = c_s[16 * J + j];
+        const float x = J == I ? ci - cj : (tot_s[J] - cj) + between + ci;
+        const float f = __expf(fminf(x, 0.f)) * rk_s[16 * J + j];
+        kk[r] = J == I && j >= m ? 0.f : kk[r] * f * rk * bI;
+        qk[r] = J == I && j > m ? 0.f : qk[r] * f * rq;
+      }
+      if (J < I) between += tot_s[J];
+      l_s[(J == I ? 6 + I : I * (I - 1) / 2 + J) * 64 + lane] = kk;
+      *reinterpret_cast<float4v*>(base + lay.A + ((I * 4 + J) * 64 + lane) * 4) = qk;
+    }
+  } else {
     float4v kI[KT], qI[KT];  // k_i exp(c_i), q_i exp(c_i): row m, 4 channels
     const int row = 16 * I + m;
     const float rk = rk_s[row], rq = rq_s[row];
@@ -389,13 +467,13 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_prepare_kernel(
         float x = 0.f;
         if (is_k) {
           x = bf16_bits_to_float(k_s[row * LK + d]) * rk_s[row] *
-              __expf(pre + c_s[row * LC + d]);
+              __expf(pre + row_log(row, d));
         } else {
           x = vin[B][r];  // rows past the end have b_s 0
         }
         rhs[r] = x * b_s[row];
       }
-      if (is_k) pre += tot_s[B * D + d];
+      if (is_k) pre += block_log(B, d);
       float4v acc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int J = 0; J < 4; ++J)
@@ -422,19 +500,19 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_prepare_kernel(
     const int rt = tile / 4, kt = tile % 4;
     const int d = 16 * rt + m;
     float post = 0.f;
-    for (int M = kt; M < 4; ++M) post += tot_s[M * D + d];
+    for (int M = kt; M < 4; ++M) post += block_log(M, d);
     float4v o;
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
       const int j = 16 * kt + 4 * g + e;
       o[e] = bf16_bits_to_float(k_s[j * LK + d]) * rk_s[j] *
-             __expf(fminf(post - c_s[j * LC + d], 0.f));
+             __expf(fminf(post - row_log(j, d), 0.f));
     }
     *reinterpret_cast<float4v*>(base + lay.K + ((rt * 4 + kt) * 64 + lane) * 4) = o;
   }
   for (int d = threadIdx.x; d < D; d += 256)
-    base[lay.E + d] = __expf(tot_s[d] + tot_s[D + d] + tot_s[2 * D + d] +
-                             tot_s[3 * D + d]);
+    base[lay.E + d] = __expf(block_log(0, d) + block_log(1, d) +
+                             block_log(2, d) + block_log(3, d));
 }
 
 // One block per (sequence, head, NC * 16 value columns); a sequence's chunks
@@ -626,14 +704,14 @@ __global__ __launch_bounds__(256, 2) void delta_chunk_scan_kernel(
   }
 }
 
-// out = o / rms(o) * w * sigmoid(gate) per head: 16 lanes per (row, head),
+// out = o / rms(o) * w * sigmoid(gate), or silu(gate), per head: 16 lanes per (row, head),
 // VPL consecutive values per lane and turn (V a multiple of 16 * VPL).
 template <int VPL>
 __global__ __launch_bounds__(256) void delta_read_out_kernel(
     bf16* __restrict__ out, int64_t ldo, const float* __restrict__ o,
     const void* __restrict__ gate, int64_t ldg, int gate_f32,
     const float* __restrict__ norm_w, float eps, int64_t heads_total, int H,
-    int V) {
+    int V, int silu_gate) {
   const int64_t i = (int64_t)blockIdx.x * 16 + threadIdx.x / 16;
   const int m = threadIdx.x % 16;
   const bool live = i < heads_total;
@@ -673,13 +751,14 @@ __global__ __launch_bounds__(256) void delta_read_out_kernel(
       ushort4v z;
 #pragma unroll
       for (int j = 0; j < 4; ++j)
-        z[j] = float_to_bf16_bits(x[j] * r * w[j] / (1.f + __expf(-gv[j])));
+        z[j] = float_to_bf16_bits(x[j] * r * w[j] * (silu_gate ? gv[j] : 1.f) /
+                                  (1.f + __expf(-gv[j])));
       *reinterpret_cast<ushort4v*>(dst + v) = z;
     }
   }
 }
 
-template <int KT>
+template <int KT, bool HEAD>
 static void launch_delta_chunks(float* o, float* scratch, const void* u,
                                 int64_t ldu, const void* decay, int64_t lda,
                                 const void* beta, int64_t ldb, const void* rate,
@@ -689,17 +768,17 @@ static void launch_delta_chunks(float* o, float* scratch, const void* u,
                                 const int* seq_lens, const int* slots,
                                 int chunks, int S, int H, int G, int V,
                                 hipStream_t stream) {
-  constexpr int lds = delta_prepare_lds(16 * KT);
+  constexpr int lds = delta_prepare_lds<HEAD>(16 * KT);
   static bool set = false;
   if (!set) {
     (void)hipFuncSetAttribute(
-        reinterpret_cast<const void*>(delta_chunk_prepare_kernel<KT>),
+        reinterpret_cast<const void*>(delta_chunk_prepare_kernel<KT, HEAD>),
         hipFuncAttributeMaxDynamicSharedMemorySize, lds);
     set = true;
   }
-  hipLaunchKernelGGL((delta_chunk_prepare_kernel<KT>), dim3(H, chunks),
+  hipLaunchKernelGGL((delta_chunk_prepare_kernel<KT, HEAD>), dim3(H, chunks),
                      dim3(256), lds, stream, scratch, (const bf16*)u, ldu,
-                     (const float*)decay, lda, (const bf16*)beta, ldb,
+                     decay, lda, (const bf16*)beta, ldb,
                      (const float*)rate, (const float*)dt_bias, chunk_cu, H, G,
                      V, unit_eps);
   const int groups = S * H;
@@ -732,26 +811,33 @@ extern "C" int arks_seq_delta_chunks(
     const void* dt_bias, const void* norm_w, float eps, float unit_eps,
     void* state, const void* chunk_off, const void* chunk_cu, const void* cu,
     const void* seq_lens, const void* slots, int64_t T, int chunks, int S,
-    int H, int G, int D, int V, hipStream_t stream) {
+    int H, int G, int D, int V, int head_decay, int silu_gate,
+    hipStream_t stream) {
   if (T == 0 || chunks == 0) return 0;
+#define DKH(KT, HEAD)                                                        \
+  launch_delta_chunks<KT, HEAD>(                                             \
+      (float*)o, (float*)scratch, u, ldu, decay, lda, beta, ldb, rate,       \
+      dt_bias, unit_eps, state, (const int*)chunk_off, (const int*)chunk_cu, \
+      (const int*)cu, (const int*)seq_lens, (const int*)slots, chunks, S, H, \
+      G, V, stream)
 #define DK(KT)                                                               \
-  launch_delta_chunks<KT>((float*)o, (float*)scratch, u, ldu, decay, lda,    \
-                          beta, ldb, rate, dt_bias, unit_eps, state,         \
-                          (const int*)chunk_off, (const int*)chunk_cu,       \
-                          (const int*)cu, (const int*)seq_lens,              \
-                          (const int*)slots, chunks, S, H, G, V, stream)
+  do {                                                                       \
+    if (head_decay) DKH(KT, true);                                           \
+    else DKH(KT, false);                                                     \
+  } while (0)
   if (D == 32) DK(2);
   else if (D == 64) DK(4);
   else if (D == 96) DK(6);
   else if (D == 128) DK(8);
   else return 1;
 #undef DK
+#undef DKH
   const int64_t heads = T * H;
   const unsigned blocks = (unsigned)((heads + 15) / 16);
 #define RO(VPL)                                                              \
   hipLaunchKernelGGL((delta_read_out_kernel<VPL>), dim3(blocks), dim3(256),  \
                      0, stream, (bf16*)out, ldo, (const float*)o, gate, ldg, \
-                     gate_f32, (const float*)norm_w, eps, heads, H, V)
+                     gate_f32, (const float*)norm_w, eps, heads, H, V, silu_gate)
   if (V % 128 == 0) RO(8);
   else RO(4);
 #undef RO

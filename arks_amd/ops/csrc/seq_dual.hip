@@ -16,9 +16,10 @@
 //       reader of the first sees the old ones)
 //   diff_head_norm_gate  (a1 - lambda a2) / rms * mult * sigmoid(gate) per
 //       head from the two maps' attention outputs
-//   moe_glu_scaled       silu(s g) * (s u), or s * silu(g) * u, for every
-//       expert's [gate | up] columns with the row's factor for that expert,
-//       silu(g) * u for the shared expert's
+//   moe_glu_scaled       silu(s g) * (s u), or s * silu(g) * u, or s times
+//       the clamped activation, for every expert's [gate | up] columns with
+//       the row's factor for that expert; the shared expert's with factor 1
+//       or one of its own
 #include "seq_common.h"
 
 namespace arks {
@@ -151,12 +152,6 @@ struct QkvConvArgs {
   float temp_coef;
   int temp_every;
 };
-
-__device__ __forceinline__ float query_factor(int64_t pos, float coef,
-                                              int every) {
-  if (every <= 0) return 1.f;
-  return 1.f + coef * logf((float)((pos + 1) / every) + 1.f);
-}
 
 // channel c of a query row [head, map, dim] -> [kv head, map, head of the
 // group, dim]
@@ -438,41 +433,57 @@ __global__ __launch_bounds__(256) void diff_head_norm_gate_vec8_kernel(
 }
 
 // ------------------------------------------------------- expert activation
+struct ExpertAct {
+  int64_t lds;       // row stride of the scales
+  int scale_in;      // silu: the scale on gate and up, not on the product
+  int clamped;       // min(g, l) sigmoid(alpha g) (clamp(u, -l, l) + 1)
+  int shared_scale;  // column E of the scales: the shared expert's
+  float limit, shared_limit, alpha;
+};
+
 template <typename AT>
 __global__ __launch_bounds__(256) void moe_glu_scaled_kernel(
     AT* __restrict__ out, const AT* __restrict__ gu, int64_t ldg,
     const float* __restrict__ scale, int64_t total, int E, int ff, int sff,
-    int scale_in) {
+    ExpertAct a) {
   const int64_t idx = (int64_t)blockIdx.x * 256 + threadIdx.x;
   if (idx >= total) return;
   const int F = E * ff + sff;
   const int64_t t = idx / F;
   const int c = (int)(idx % F);
   const AT* row = gu + t * ldg;
-  float g, u;
+  float g, u, s = 1.f;
   if (c < E * ff) {
     const int e = c / ff, i = c % ff;
-    const float s = scale[t * E + e];
+    s = scale[t * a.lds + e];
     if (s == 0.f) {  // an expert the row does not use: exactly nothing
       Act<AT>::st(out + idx, 0.f);
       return;
     }
     g = Act<AT>::ld(row + (int64_t)e * 2 * ff + i);
-    if (scale_in) g *= s;
-    u = s * Act<AT>::ld(row + (int64_t)e * 2 * ff + ff + i);
+    u = Act<AT>::ld(row + (int64_t)e * 2 * ff + ff + i);
   } else {
     const int i = c - E * ff;
+    if (a.shared_scale) s = scale[t * a.lds + E];
     g = Act<AT>::ld(row + (int64_t)E * 2 * ff + i);
     u = Act<AT>::ld(row + (int64_t)E * 2 * ff + sff + i);
   }
-  Act<AT>::st(out + idx, silu_f(g) * u);
+  if (a.clamped) {
+    const float l = c < E * ff ? a.limit : a.shared_limit;
+    g = fminf(g, l);
+    u = fminf(fmaxf(u, -l), l) + 1.f;
+    Act<AT>::st(out + idx, s * (g * sigmoid_f(a.alpha * g) * u));
+    return;
+  }
+  if (a.scale_in) g *= s;
+  Act<AT>::st(out + idx, silu_f(g) * (s * u));
 }
 
 // bf16, 8 columns per thread (ff and sff multiples of 8)
 __global__ __launch_bounds__(256) void moe_glu_scaled_vec8_kernel(
     bf16* __restrict__ out, const bf16* __restrict__ gu, int64_t ldg,
     const float* __restrict__ scale, int64_t total8, int E, int ff, int sff,
-    int scale_in) {
+    ExpertAct a) {
   const int64_t idx = (int64_t)blockIdx.x * 256 + threadIdx.x;
   if (idx >= total8) return;
   const int F = E * ff + sff;
@@ -484,11 +495,12 @@ __global__ __launch_bounds__(256) void moe_glu_scaled_vec8_kernel(
   const bf16 *gp, *up;
   if (c < E * ff) {
     const int e = c / ff, i = c % ff;
-    s = scale[t * E + e];
+    s = scale[t * a.lds + e];
     gp = row + (int64_t)e * 2 * ff + i;
     up = gp + ff;
   } else {
     const int i = c - E * ff;
+    if (a.shared_scale) s = scale[t * a.lds + E];
     gp = row + (int64_t)E * 2 * ff + i;
     up = gp + sff;
   }
@@ -499,9 +511,17 @@ __global__ __launch_bounds__(256) void moe_glu_scaled_vec8_kernel(
   } else {
     const ushort8 gv = *reinterpret_cast<const ushort8*>(gp);
     const ushort8 uv = *reinterpret_cast<const ushort8*>(up);
-    const float sg = scale_in ? s : 1.f;
+    const float sg = a.scale_in ? s : 1.f;
+    const float l = c < E * ff ? a.limit : a.shared_limit;
 #pragma unroll
     for (int e = 0; e < 8; ++e) {
+      if (a.clamped) {
+        const float g = fminf(bf16_bits_to_float(gv[e]), l);
+        const float u =
+            fminf(fmaxf(bf16_bits_to_float(uv[e]), -l), l) + 1.f;
+        o[e] = float_to_bf16_bits(s * (g / (1.f + __expf(-a.alpha * g)) * u));
+        continue;
+      }
       const float g = sg * bf16_bits_to_float(gv[e]);
       const float u = s * bf16_bits_to_float(uv[e]);
       o[e] = float_to_bf16_bits(g / (1.f + __expf(-g)) * u);
@@ -614,10 +634,15 @@ extern "C" int arks_seq_diff_head_norm_gate(
 }
 
 extern "C" void arks_seq_moe_glu_scaled(void* out, const void* gu, int64_t ldg,
-                                        const void* scale, int64_t T, int E,
-                                        int ff, int sff, int scale_in,
+                                        const void* scale, int64_t lds,
+                                        int64_t T, int E, int ff, int sff,
+                                        int scale_in, int clamped,
+                                        int shared_scale, float limit,
+                                        float shared_limit, float alpha,
                                         int act_f32, hipStream_t stream) {
   if (T == 0) return;
+  const ExpertAct a{lds,   scale_in,     clamped, shared_scale,
+                    limit, shared_limit, alpha};
   const int64_t total = T * ((int64_t)E * ff + sff);
   if (!act_f32 && ff % 8 == 0 && sff % 8 == 0 && ldg % 8 == 0 &&
       ((uintptr_t)gu % 16) == 0) {
@@ -625,11 +650,11 @@ extern "C" void arks_seq_moe_glu_scaled(void* out, const void* gu, int64_t ldg,
     hipLaunchKernelGGL(moe_glu_scaled_vec8_kernel,
                        dim3((unsigned)((total8 + 255) / 256)), dim3(256), 0,
                        stream, (bf16*)out, (const bf16*)gu, ldg,
-                       (const float*)scale, total8, E, ff, sff, scale_in);
+                       (const float*)scale, total8, E, ff, sff, a);
     return;
   }
   SEQ_DISPATCH_ACT(act_f32, hipLaunchKernelGGL(
       (moe_glu_scaled_kernel<AT>), dim3((unsigned)((total + 255) / 256)),
       dim3(256), 0, stream, (AT*)out, (const AT*)gu, ldg, (const float*)scale,
-      total, E, ff, sff, scale_in));
+      total, E, ff, sff, a));
 }

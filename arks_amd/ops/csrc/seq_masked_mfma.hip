@@ -17,8 +17,9 @@
 //   * masks per (column, key): key j for the column at position i iff
 //     j <= i and (i - j < window or j < keep_first); a tile walks the key
 //     tiles that hold kept keys, then those from its oldest row's window on;
-//   * scores may be capped, s <- c tanh(s / c), and the running softmax may
-//     start from a sink (max sink[h], sum 1);
+//   * scores may be capped, s <- c tanh(s / c), a distance bias slope[h] (i - j)
+//     may be taken off them, and the running softmax may start from a sink
+//     (max sink[h], sum 1);
 //   * key and value rows have strides of their own (ldk, ldv);
 //   * no host work list: a workgroup finds its (sequence, first position)
 //     by walking cu_seqlens, or — steps of single rows — from token_seq;
@@ -52,6 +53,7 @@ struct MaskArgs {
   // that share the row's value; the kernels' G counts (key/value head, map)
   // groups, group g reads key g % maps of the rows of head g / maps
   int maps;
+  const float* slopes;  // [H], or null: no distance bias
 };
 
 template <int D, int V>  // V: the value columns one workgroup holds
@@ -149,6 +151,7 @@ void attn_masked_tile_kernel(
     }
   }
   const float inv_cap = a.softcap > 0.f ? 1.f / a.softcap : 0.f;
+  const float slope = a.slopes ? a.slopes[h] : 0.f;
   const bool sunk = sink_w != nullptr && kz == 0;
   float m_run = sunk ? sink_w[h] : -FLT_MAX;
   float l_run = sunk ? 1.f : 0.f;
@@ -284,6 +287,7 @@ void attn_masked_tile_kernel(
                    (kg > my_pos - a.window || kg < a.keep_first);
           float s = sc[sub][r] * a.scale;
           if (a.softcap > 0.f) s = mk_cap(s, a.softcap, inv_cap);
+          if (a.slopes) s -= slope * (float)(my_pos - kg);
           p[i] = msk[i] ? s : -FLT_MAX;
           tile_max = fmaxf(tile_max, p[i]);
         }
@@ -464,6 +468,7 @@ __global__ __launch_bounds__(256, 2) void attn_masked_dec_kernel(
     }
   }
   const float inv_cap = a.softcap > 0.f ? 1.f / a.softcap : 0.f;
+  const float slope = a.slopes && head_valid ? a.slopes[kvh * GQ + lq] : 0.f;
   const bool sunk = sink_w != nullptr && wave == 0 && head_valid;
   float m_run = sunk ? sink_w[kvh * GQ + lq] : -FLT_MAX;
   float l_run = sunk ? 1.f : 0.f;
@@ -557,6 +562,7 @@ __global__ __launch_bounds__(256, 2) void attn_masked_dec_kernel(
             kg <= pos && (kg > pos - a.window || kg < a.keep_first);
         float s = sc[sub][r] * a.scale;
         if (a.softcap > 0.f) s = mk_cap(s, a.softcap, inv_cap);
+        if (a.slopes) s -= slope * (float)(pos - kg);
         p[i] = vis ? s : -FLT_MAX;
         tile_max = fmaxf(tile_max, p[i]);
       }
@@ -736,7 +742,7 @@ extern "C" int arks_seq_attn_masked_mfma(
     const void* sink_w, float softcap, int window, int keep_first,
     float out_scale, int T, int H, int G, int D, int V, int bs, int max_blocks,
     int num_seqs, int single_rows, void* ws, int ksplit, int maps,
-    hipStream_t stream) {
+    const void* slopes, hipStream_t stream) {
   // G: key groups, maps of them per key/value head of the cache
   if (maps < 1 || G % maps || (maps > 1 && v_cache == k_cache)) return 1;
   if (bs != MK_PAGE || H % G || ldk % 8 || ldv % 8 || ldo % 8 ||
@@ -752,6 +758,7 @@ extern "C" int arks_seq_attn_masked_mfma(
   a.window = window > 0 ? window : (1 << 30);
   a.keep_first = window > 0 ? keep_first : 0;
   a.maps = maps;
+  a.slopes = (const float*)slopes;
   const bool shared_rows = v_cache == k_cache && ldv == ldk;
   const int hpt_shift = masked_hpt_shift(GQ);
   const int ppt = MK_QTILE >> hpt_shift;

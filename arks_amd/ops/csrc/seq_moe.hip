@@ -4,12 +4,16 @@
 //
 //   moe_route_grouped  scores over all E experts (logits + bias) in fp32, their softmax or
 //       (sigmoid) each logit's own sigmoid; experts are cut into
-//       `groups` contiguous runs of E/groups, a run's score is its highest
-//       expert score and only the `keep` highest-scoring runs stay eligible; the `top`
-//       largest scores among those, divided by their sum (+1e-20) unless
-//       renorm is off. Ties go to the lower index (groups and experts).
+//       `groups` contiguous runs of E/groups. Choices are made by the score
+//       plus (optional) a correction per expert: a run's choice score is its
+//       highest, or the sum of its two highest (group_top), and only the
+//       `keep` best runs stay eligible; the `top` experts with the largest
+//       choice scores among those get their scores, without the correction,
+//       divided by their sum (+1e-20) unless renorm is off. Ties go to the
+//       lower index (groups and experts).
 //       matrix (optional, [T, E]): the row's weights at the experts it uses,
-//       0 elsewhere.
+//       0 elsewhere; with shared_gate the logits have a column E more, whose
+//       sigmoid is the matrix's column E.
 //   moe_sort_pairs  (row, expert) pairs in expert order, stable: the row of
 //       every sorted place, every pair's place, the pairs per expert
 //   moe_mix_rows  out[t] = sum_j w[t][j] * y[row(t, j)], row given, or
@@ -26,13 +30,15 @@ constexpr int ROUTE_MAX_K = 32;
 // One wave per row.
 __global__ __launch_bounds__(64) void moe_route_grouped_kernel(
     float* __restrict__ weights, int* __restrict__ ids,
-    const float* __restrict__ logits, int E, int top, int groups, int keep,
-    int sigmoid, int renorm, float* __restrict__ matrix,
-    const float* __restrict__ bias) {
-  __shared__ float s_s[ROUTE_MAX_E];
+    const float* __restrict__ logits, int64_t ldl, int E, int top, int groups,
+    int keep, int sigmoid, int renorm, float* __restrict__ matrix,
+    const float* __restrict__ bias, const float* __restrict__ correction,
+    int group_top, int shared_gate) {
+  __shared__ float s_s[ROUTE_MAX_E];  // choice scores
   __shared__ float g_s[ROUTE_MAX_E];  // group scores (groups <= E)
   const int t = blockIdx.x, lane = threadIdx.x;
-  const float* row = logits + (int64_t)t * E;
+  const float* row = logits + (int64_t)t * ldl;
+  const int64_t ldm = E + shared_gate;
   if (sigmoid) {
     for (int e = lane; e < E; e += 64)
       s_s[e] = sigmoid_f(row[e] + (bias ? bias[e] : 0.f));
@@ -52,24 +58,34 @@ __global__ __launch_bounds__(64) void moe_route_grouped_kernel(
     const float inv = 1.f / sum;
     for (int e = lane; e < E; e += 64) s_s[e] *= inv;
   }
-  if (matrix)
-    for (int e = lane; e < E; e += 64) matrix[(int64_t)t * E + e] = 0.f;
+  if (correction)  // own entries
+    for (int e = lane; e < E; e += 64) s_s[e] += correction[e];
+  if (matrix) {
+    for (int e = lane; e < E; e += 64) matrix[(int64_t)t * ldm + e] = 0.f;
+    if (shared_gate && lane == 0)
+      matrix[(int64_t)t * ldm + E] = sigmoid_f(row[E]);
+  }
   __syncthreads();
   const int per = E / groups;
   for (int gI = lane; gI < groups; gI += 64) {
-    float best = -1.f;
-    for (int i = 0; i < per; ++i) best = fmaxf(best, s_s[gI * per + i]);
-    g_s[gI] = best;
+    float best = -INFINITY, second = -INFINITY;
+    for (int i = 0; i < per; ++i) {
+      const float v = s_s[gI * per + i];
+      second = fmaxf(second, fminf(best, v));
+      best = fmaxf(best, v);
+    }
+    g_s[gI] = group_top > 1 && per > 1 ? best + second : best;
   }
   __syncthreads();
   // the eligible runs: `keep` argmax passes, the others' experts are
-  // marked unavailable (score -1)
+  // marked unavailable. +inf marks a chosen run, -inf an expert that cannot
+  // be chosen (any more)
   if (keep < groups) {
     for (int r = 0; r < keep; ++r) {
-      float best = -2.f;
+      float best = -INFINITY;
       int bi = groups;
       for (int gI = lane; gI < groups; gI += 64) {
-        const float v = g_s[gI];
+        const float v = g_s[gI] == INFINITY ? -INFINITY : g_s[gI];
         if (v > best || (v == best && gI < bi)) { best = v; bi = gI; }
       }
 #pragma unroll
@@ -79,18 +95,18 @@ __global__ __launch_bounds__(64) void moe_route_grouped_kernel(
         if (ob > best || (ob == best && oi < bi)) { best = ob; bi = oi; }
       }
       __syncthreads();
-      if (lane == 0) g_s[bi] = -3.f;  // chosen
+      if (lane == 0) g_s[min(bi, groups - 1)] = INFINITY;
       __syncthreads();
     }
     for (int e = lane; e < E; e += 64)
-      if (g_s[e / per] != -3.f) s_s[e] = -1.f;
+      if (g_s[e / per] != INFINITY) s_s[e] = -INFINITY;
     __syncthreads();
   }
   float wsum = 0.f;
   float wk[ROUTE_MAX_K];
   int ik[ROUTE_MAX_K];
   for (int r = 0; r < top; ++r) {
-    float best = -2.f;
+    float best = -INFINITY;
     int bi = E;
     for (int e = lane; e < E; e += 64) {
       const float v = s_s[e];
@@ -102,11 +118,16 @@ __global__ __launch_bounds__(64) void moe_route_grouped_kernel(
       const int oi = __shfl_xor(bi, off, 64);
       if (ob > best || (ob == best && oi < bi)) { best = ob; bi = oi; }
     }
-    wk[r] = best;
+    bi = min(bi, E - 1);  // rows of NaNs stay in bounds
+    // the score itself: the choice score where there is no correction
+    const float sc = !correction ? best
+                     : sigmoid   ? sigmoid_f(row[bi] + (bias ? bias[bi] : 0.f))
+                                 : best - correction[bi];
+    wk[r] = sc;
     ik[r] = bi;
-    wsum += best;
+    wsum += sc;
     __syncthreads();
-    if (lane == 0) s_s[bi] = -2.f;
+    if (lane == 0) s_s[bi] = -INFINITY;
     __syncthreads();
   }
   if (lane == 0) {
@@ -115,7 +136,7 @@ __global__ __launch_bounds__(64) void moe_route_grouped_kernel(
       const float w = renorm ? wk[r] / d : wk[r];
       weights[(int64_t)t * top + r] = w;
       ids[(int64_t)t * top + r] = ik[r];
-      if (matrix) matrix[(int64_t)t * E + ik[r]] = w;
+      if (matrix) matrix[(int64_t)t * ldm + ik[r]] = w;
     }
   }
 }
@@ -245,19 +266,22 @@ __global__ __launch_bounds__(256) void moe_mix_rows_vec8_kernel(
 using namespace arks;
 
 extern "C" int arks_seq_moe_route_grouped(void* weights, void* ids,
-                                          const void* logits, int T, int E,
-                                          int top, int groups, int keep,
-                                          int sigmoid, int renorm,
+                                          const void* logits, int64_t ldl,
+                                          int T, int E, int top, int groups,
+                                          int keep, int sigmoid, int renorm,
                                           void* matrix, const void* bias,
+                                          const void* correction,
+                                          int group_top, int shared_gate,
                                           hipStream_t stream) {
   if (E > ROUTE_MAX_E || top > ROUTE_MAX_K || groups < 1 || E % groups ||
       keep > groups || top > keep * (E / groups))
     return 1;
   if (T == 0) return 0;
   hipLaunchKernelGGL(moe_route_grouped_kernel, dim3(T), dim3(64), 0, stream,
-                     (float*)weights, (int*)ids, (const float*)logits, E, top,
-                     groups, keep, sigmoid, renorm, (float*)matrix,
-                     (const float*)bias);
+                     (float*)weights, (int*)ids, (const float*)logits, ldl, E,
+                     top, groups, keep, sigmoid, renorm, (float*)matrix,
+                     (const float*)bias, (const float*)correction, group_top,
+                     shared_gate);
   return 0;
 }
 

@@ -1,8 +1,9 @@
 // Row kernels of the sandwich-norm blocks (arks_amd/models/hybrid.py
 // SandwichBlock), bf16 or float rows, fp32 arithmetic:
 //
-//   residual_sandwich_norm  x += mult * rms_norm(y) * w_post on the fp32
-//       residual (y, the previous sublayer's result, optional), then
+//   residual_sandwich_norm  x += mult * (rms_norm(y) * w_post + rms_norm(y2)
+//       * w_post2) on the fp32 residual (y and y2, the previous sublayer's
+//       results, optional; without a weight a result is added as it is), then
 //       h = rms_norm(x) * w_pre (optional), the next sublayer's input
 //   head_gate  out[t, h] = o[t, h] * sigmoid(gate[t, h]) * out_scale
 //   softcap    x = cap * tanh(x / cap) in place
@@ -14,26 +15,34 @@ namespace arks {
 template <typename AT>
 __global__ __launch_bounds__(256) void residual_sandwich_norm_kernel(
     float* __restrict__ x, AT* __restrict__ h, const AT* __restrict__ y,
-    const float* __restrict__ w_post, float mult,
+    const float* __restrict__ w_post, const AT* __restrict__ y2,
+    const float* __restrict__ w_post2, float mult,
     const float* __restrict__ w_pre, float eps, int C) {
-  __shared__ float red[4], red2[4];
+  __shared__ float red[4], red2[4], red3[4];
   const int64_t t = blockIdx.x;
   float* xr = x + t * C;
-  float ry = 0.f;
-  if (y) {
+  auto row_scale = [&](const AT* r, float* scratch) {
     float ss = 0.f;
     for (int c = threadIdx.x; c < C; c += 256) {
-      const float v = Act<AT>::ld(y + t * C + c);
+      const float v = Act<AT>::ld(r + t * C + c);
       ss += v * v;
     }
-    ss = block_reduce_sum<256>(ss, red);
-    ry = 1.f / sqrtf(ss / (float)C + eps);
-  }
+    ss = block_reduce_sum<256>(ss, scratch);
+    return 1.f / sqrtf(ss / (float)C + eps);
+  };
+  const float ry = y && w_post ? row_scale(y, red) : 1.f;
+  const float ry2 = y2 && w_post2 ? row_scale(y2, red3) : 1.f;
   float ss = 0.f;
   for (int c = threadIdx.x; c < C; c += 256) {
     float v = xr[c];
     if (y) {
-      v += mult * (Act<AT>::ld(y + t * C + c) * ry * w_post[c]);
+      float z = Act<AT>::ld(y + t * C + c);
+      if (w_post) z *= ry * w_post[c];
+      if (y2) {
+        const float z2 = Act<AT>::ld(y2 + t * C + c);
+        z += w_post2 ? z2 * ry2 * w_post2[c] : z2;
+      }
+      v += mult * z;
       xr[c] = v;
     }
     ss += v * v;
@@ -46,13 +55,14 @@ __global__ __launch_bounds__(256) void residual_sandwich_norm_kernel(
 }
 
 // bf16 rows, C % 8 == 0, C <= 2048 * IT: every thread keeps its pieces of
-// both rows in registers through the two reductions.
-template <int IT>
+// the rows in registers through the reductions. TWO: y2 is given.
+template <int IT, bool TWO>
 __global__ __launch_bounds__(256) void residual_sandwich_norm_vec8_kernel(
     float* __restrict__ x, bf16* __restrict__ h, const bf16* __restrict__ y,
-    const float* __restrict__ w_post, float mult,
+    const float* __restrict__ w_post, const bf16* __restrict__ y2,
+    const float* __restrict__ w_post2, float mult,
     const float* __restrict__ w_pre, float eps, int C) {
-  __shared__ float red[4], red2[4];
+  __shared__ float red[4], red2[4], red3[4];
   const int64_t t = blockIdx.x;
   float* xr = x + t * C;
   float v[IT][8];
@@ -70,36 +80,51 @@ __global__ __launch_bounds__(256) void residual_sandwich_norm_vec8_kernel(
     }
   }
   if (y) {
-    float yv[IT][8];
-    float ss = 0.f;
+    ushort8 yv[IT], zv[IT];
+    float ss = 0.f, ss2 = 0.f;
 #pragma unroll
     for (int it = 0; it < IT; ++it) {
       const int c = (it * 256 + threadIdx.x) * 8;
+      yv[it] = ushort8{};
+      zv[it] = ushort8{};
       if (c < C) {
-        const ushort8 u = *reinterpret_cast<const ushort8*>(y + t * C + c);
+        yv[it] = *reinterpret_cast<const ushort8*>(y + t * C + c);
+        if (TWO) zv[it] = *reinterpret_cast<const ushort8*>(y2 + t * C + c);
+      }
 #pragma unroll
-        for (int e = 0; e < 8; ++e) {
-          yv[it][e] = bf16_bits_to_float(u[e]);
-          ss += yv[it][e] * yv[it][e];
-        }
-      } else {
-#pragma unroll
-        for (int e = 0; e < 8; ++e) yv[it][e] = 0.f;
+      for (int e = 0; e < 8; ++e) {
+        const float a = bf16_bits_to_float(yv[it][e]);
+        const float b = bf16_bits_to_float(zv[it][e]);
+        ss += a * a;
+        if (TWO) ss2 += b * b;
       }
     }
-    ss = block_reduce_sum<256>(ss, red);
-    const float ry = mult / sqrtf(ss / (float)C + eps);
+    float ry = mult, ry2 = mult;
+    if (w_post) ry /= sqrtf(block_reduce_sum<256>(ss, red) / (float)C + eps);
+    if (TWO && w_post2)
+      ry2 /= sqrtf(block_reduce_sum<256>(ss2, red3) / (float)C + eps);
+    auto add_row = [&](int it, int c, const ushort8& r, const float* w,
+                       float f) {
+      float4v wa = {1.f, 1.f, 1.f, 1.f}, wb = {1.f, 1.f, 1.f, 1.f};
+      if (w) {
+        wa = *reinterpret_cast<const float4v*>(w + c);
+        wb = *reinterpret_cast<const float4v*>(w + c + 4);
+      }
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        v[it][e] += bf16_bits_to_float(r[e]) * f * wa[e];
+        v[it][4 + e] += bf16_bits_to_float(r[4 + e]) * f * wb[e];
+      }
+    };
 #pragma unroll
     for (int it = 0; it < IT; ++it) {
       const int c = (it * 256 + threadIdx.x) * 8;
       if (c < C) {
-        const float4v wa = *reinterpret_cast<const float4v*>(w_post + c);
-        const float4v wb = *reinterpret_cast<const float4v*>(w_post + c + 4);
+        add_row(it, c, yv[it], w_post, ry);
+        if (TWO) add_row(it, c, zv[it], w_post2, ry2);
         float4v a, b;
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
-          v[it][e] += yv[it][e] * ry * wa[e];
-          v[it][4 + e] += yv[it][4 + e] * ry * wb[e];
           a[e] = v[it][e];
           b[e] = v[it][4 + e];
         }
@@ -190,28 +215,35 @@ __global__ __launch_bounds__(256) void softcap_kernel(float* __restrict__ x,
 using namespace arks;
 
 extern "C" void arks_seq_residual_sandwich_norm(
-    void* x, void* h, const void* y, const void* w_post, float mult,
-    const void* w_pre, float eps, int64_t T, int C, int act_f32,
-    hipStream_t stream) {
+    void* x, void* h, const void* y, const void* w_post, const void* y2,
+    const void* w_post2, float mult, const void* w_pre, float eps, int64_t T,
+    int C, int act_f32, hipStream_t stream) {
   if (T == 0) return;
   const bool aligned = (((uintptr_t)x | (uintptr_t)h | (uintptr_t)y |
-                         (uintptr_t)w_post | (uintptr_t)w_pre) & 15) == 0;
+                         (uintptr_t)w_post | (uintptr_t)y2 |
+                         (uintptr_t)w_post2 | (uintptr_t)w_pre) & 15) == 0;
   if (!act_f32 && C % 8 == 0 && C <= 8192 && aligned) {
-#define SN(IT)                                                                \
-  hipLaunchKernelGGL((residual_sandwich_norm_vec8_kernel<IT>), dim3(T),       \
+#define SN(IT, TWO)                                                           \
+  hipLaunchKernelGGL((residual_sandwich_norm_vec8_kernel<IT, TWO>), dim3(T),  \
                      dim3(256), 0, stream, (float*)x, (bf16*)h,               \
-                     (const bf16*)y, (const float*)w_post, mult,              \
-                     (const float*)w_pre, eps, C)
-    if (C <= 2048) SN(1);
-    else if (C <= 4096) SN(2);
-    else SN(4);
+                     (const bf16*)y, (const float*)w_post, (const bf16*)y2,   \
+                     (const float*)w_post2, mult, (const float*)w_pre, eps, C)
+#define SN2(IT)        \
+  do {                 \
+    if (y2) SN(IT, true); \
+    else SN(IT, false);   \
+  } while (0)
+    if (C <= 2048) SN2(1);
+    else if (C <= 4096) SN2(2);
+    else SN2(4);
+#undef SN2
 #undef SN
     return;
   }
   SEQ_DISPATCH_ACT(act_f32, hipLaunchKernelGGL(
       (residual_sandwich_norm_kernel<AT>), dim3(T), dim3(256), 0, stream,
-      (float*)x, (AT*)h, (const AT*)y, (const float*)w_post, mult,
-      (const float*)w_pre, eps, C));
+      (float*)x, (AT*)h, (const AT*)y, (const float*)w_post, (const AT*)y2,
+      (const float*)w_post2, mult, (const float*)w_pre, eps, C));
 }
 
 extern "C" void arks_seq_softcap(void* x, int64_t n, float cap,

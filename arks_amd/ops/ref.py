@@ -442,7 +442,7 @@ def qk_norm_rope_cache(q, k, v, q_norm_w, k_norm_w, eps, positions,
 def attention_sink_paged(q, k_cache, v_cache, block_tables, seq_lens,
                          cu_seqlens, scale, sink=True, inv_freq_v=None,
                          interleaved=True, sink_w=None, softcap=0.0,
-                         window=0, keep_first=0, maps=1):
+                         window=0, keep_first=0, maps=1, slopes=None):
     """Causal attention of packed new rows over each sequence's paged keys.
     maps M > 1: a key row holds M keys of D dims side by side (k_cache
     [pages, G, bs, M*D]) that share the row's value; q has G*M groups of
@@ -450,7 +450,8 @@ def attention_sink_paged(q, k_cache, v_cache, block_tables, seq_lens,
     sink=True adds a value-less key of score 0 to every softmax (one more
     in the denominator); sink_w [H] gives that key a score per head
     instead (taken as it is: neither scaled nor capped). softcap c > 0:
-    scores become c tanh(score / c). window w > 0: the row at position i
+    scores become c tanh(score / c). slopes [H]: slope[h] (i - j) is taken
+    off the score of row i and key j (not off the sink's). window w > 0: the row at position i
     sees key j only if i - j < w or j < keep_first. inv_freq_v: each row's
     output is turned back by its own position over the value dims. v_cache
     may be a view into k_cache's rows. q [T,H,D] -> [T,H,V] in q.dtype."""
@@ -479,6 +480,9 @@ def attention_sink_paged(q, k_cache, v_cache, block_tables, seq_lens,
         if softcap > 0:
             sc = softcap * torch.tanh(sc / softcap)
         kpos = torch.arange(L)[None, :]
+        if slopes is not None:
+            sc = sc - slopes.float()[:, None, None] * (
+                qpos[:, None] - kpos).float()[None]
         mask = kpos > qpos[:, None]
         if window > 0:
             mask = mask | ((qpos[:, None] - kpos >= window)
@@ -783,26 +787,30 @@ def glu_act(gu, kind, limit=0.0, alpha=1.0, row_scale=None):
 
 
 def moe_route_grouped(logits, top, groups, keep, score="softmax",
-                      renorm=True, bias=None):
-    """Scores of logits (+ bias [E]) over all experts: their softmax, or (score="sigmoid") each
-    logit's own sigmoid; without renorm the chosen scores are the weights as
-    they are. Experts are cut into `groups`
-    contiguous runs of E/groups, a run's score is its highest expert score
-    and only the `keep` highest-scoring runs stay eligible; the `top` largest scores among those, their
-    scores divided by their sum (+1e-20). Ties go to the lower index.
-    logits [T, E] fp32 -> (weights [T, top] fp32, ids [T, top] int32)."""
+                      renorm=True, bias=None, correction=None, group_top=1):
+    """Scores of logits (+ bias [E]) over all experts: their softmax, or
+    (score="sigmoid") each logit's own sigmoid; without renorm the chosen
+    scores are the weights as they are. Choices go by the score plus the
+    correction [E], if there is one. Experts are cut into `groups`
+    contiguous runs of E/groups, a run's choice score is its highest
+    (group_top 2: the sum of its two highest) and only the `keep` best runs
+    stay eligible; the `top` experts with the largest choice scores among
+    those, their scores divided by their sum (+1e-20). Ties go to the lower
+    index. logits [T, E] fp32 -> (weights [T, top] fp32, ids [T, top] int32)."""
     if bias is not None:
         logits = logits.float() + bias.float()
     s = (torch.sigmoid(logits.float()) if score == "sigmoid"
          else torch.softmax(logits.float(), -1))
     T, E = s.shape
     per = E // groups
-    gs = s.view(T, groups, per).amax(-1)
+    choice = s if correction is None else s + correction.float()
+    gs = torch.topk(choice.view(T, groups, per), min(group_top, per),
+                    dim=-1).values.sum(-1)
     kept = torch.topk(gs, keep, dim=-1).indices  # [T, keep]
     allow = torch.zeros(T, groups, dtype=torch.bool)
     allow.scatter_(1, kept, True)
     masked = torch.where(allow[:, :, None].expand(T, groups, per).reshape(T, E),
-                         s, torch.full_like(s, -1.0))
+                         choice, torch.full_like(s, float("-inf")))
     ids = torch.topk(masked, top, dim=-1).indices
     w = s.gather(1, ids)
     if renorm:
@@ -1011,15 +1019,29 @@ def diff_head_norm_gate(a, gate, lam, eps, mult, heads, kv_heads, out):
     return out
 
 
-def moe_glu_scaled(gu, scale, experts, ff, shared_ff, scale_input=True):
+def moe_glu_scaled(gu, scale, experts, ff, shared_ff, scale_input=True,
+                   act="swiglu", limit=0.0, shared_limit=0.0, alpha=1.0,
+                   shared_scale=False):
     """gu [T, experts * 2 ff + 2 shared_ff]: per expert [gate | up], then
     the shared expert's [gate | up]. Column c of expert e becomes
     silu(s g) * (s u) with s = scale[t, e] (fp32; 0 for an expert the row
     does not use), or s * silu(g) * u without scale_input; the shared columns
-    silu(g) * u. -> [T, experts * ff + shared_ff]."""
+    silu(g) * u. act "clamped": s times glu_act's clamped form instead, with
+    a limit of its own for the shared expert. shared_scale: the shared
+    columns' activated product is multiplied by scale[t, experts].
+    -> [T, experts * ff + shared_ff]."""
     T = gu.shape[0]
     ex = gu[:, :experts * 2 * ff].float().view(T, experts, 2, ff)
-    s = scale.float()[:, :, None]
+    s = scale.float()[:, :experts, None]
+    if act == "clamped" or shared_scale:
+        assert not scale_input
+        parts = [(glu_act(ex.flatten(2), act, limit, alpha) * s)
+                 .reshape(T, experts * ff)]
+        if shared_ff:
+            sh = glu_act(gu[:, experts * 2 * ff:].float(), act, shared_limit,
+                         alpha)
+            parts.append(sh * scale.float()[:, experts:] if shared_scale else sh)
+        return torch.cat(parts, -1).to(gu.dtype)
     g, u = ex[:, :, 0], ex[:, :, 1] * s
     if scale_input:
         g = g * s
@@ -1056,14 +1078,18 @@ def route_scale_matrix(weights, ids, experts):
 # ----------------------------------------------------------------------
 # Sandwich-norm blocks, per-head output gate, channel-decay delta rule.
 # ----------------------------------------------------------------------
-def residual_sandwich_norm(x, y, w_post, mult, w_pre, eps, out_dtype):
-    """x (fp32, in place) += mult * rms_norm(y) * w_post when y is given;
-    returns rms_norm(x) * w_pre in out_dtype (None without w_pre)."""
+def residual_sandwich_norm(x, y, w_post, mult, w_pre, eps, out_dtype,
+                           y2=None, w_post2=None):
+    """x (fp32, in place) += mult * (rms_norm(y) * w_post + rms_norm(y2) *
+    w_post2) for the results given, one without a weight as it is; returns
+    rms_norm(x) * w_pre in out_dtype (None without w_pre)."""
     def unit(t):
         return t * torch.rsqrt(t.pow(2).mean(-1, keepdim=True) + eps)
 
-    if y is not None:
-        x += mult * (unit(y.float()) * w_post.float())
+    for r, w in ((y, w_post), (y2, w_post2)):
+        if r is not None:
+            x += mult * (r.float() if w is None
+                         else unit(r.float()) * w.float())
     if w_pre is None:
         return None
     return (unit(x) * w_pre.float()).to(out_dtype)
@@ -1089,13 +1115,14 @@ DELTA_UNIT_EPS = 1e-6  # under the root of q's and k's unit length
 
 def channel_delta(u, decay, beta, gate, rate, dt_bias, norm_w, eps, state,
                   cu_seqlens, seq_lens, state_slots, heads, kv_heads, dim,
-                  vdim, out):
-    """Delta rule with a decay per head and key channel. u [T, 2*G*D + H*V] =
+                  vdim, out, head_decay=False, silu_gate=False):
+    """Delta rule with a decay per head and key channel (head_decay: one per
+    head, decay [T, H], dt_bias [H]). u [T, 2*G*D + H*V] =
     [q | k | v] (after conv and silu), decay [T, H*D] and beta [T, H] raw
     projections, gate [T, H*V] raw. Per head h with q/k head h // (H/G):
     q, k to unit length, q times D^-1/2; g = exp(-rate_h softplus(decay +
     dt_bias)); S <- g S, w = sigmoid(beta) (v - S^T k), S <- S + k w^T,
-    o = S^T q; out = rms_norm(o) norm_w sigmoid(gate). state [slots, H, D, V]
+    o = S^T q; out = rms_norm(o) norm_w sigmoid(gate), or silu(gate). state [slots, H, D, V]
     fp32 (updated)."""
     T, H, G, D, V = u.shape[0], heads, kv_heads, dim, vdim
     f = u.float()
@@ -1108,7 +1135,8 @@ def channel_delta(u, decay, beta, gate, rate, dt_bias, norm_w, eps, state,
     q, k = (t.repeat_interleave(H // G, 1) for t in (q, k))
     v = f[:, 2 * G * D:].reshape(T, H, V)
     g = torch.exp(-rate.float()[None, :, None] * torch.nn.functional.softplus(
-        decay.float() + dt_bias.float(), threshold=20.0).reshape(T, H, D))
+        decay.float() + dt_bias.float(), threshold=20.0).reshape(
+            T, H, 1 if head_decay else D))
     b = torch.sigmoid(beta.float())
     o = torch.empty(T, H, V, dtype=torch.float32)
     for lo, hi, start, slot in _seq_spans(cu_seqlens, seq_lens, state_slots):
@@ -1122,6 +1150,56 @@ def channel_delta(u, decay, beta, gate, rate, dt_bias, norm_w, eps, state,
         if slot >= 0:
             state[slot] = S
     o = o * torch.rsqrt(o.pow(2).mean(-1, keepdim=True) + eps) * norm_w.float()
-    o = o * torch.sigmoid(gate.float()).reshape(T, H, V)
+    z = gate.float().reshape(T, H, V)
+    o = o * torch.sigmoid(z) * (z if silu_gate else 1.0)
     out.copy_(o.reshape(T, H * V).to(out.dtype))
     return out
+
+
+# ----------------------------------------------------------------------
+# Pre-norm two-mixer blocks: hashed embedding of token pairs, q/k norm over
+# all heads at once, squared relu.
+# ----------------------------------------------------------------------
+def hashed_embed(ids, embed, table, prev, cu_seqlens, seq_lens, state_slots,
+                 scale, mul_prev, mul_cur):
+    """fp32 rows embed[token] * scale + table[row], row = (previous token *
+    mul_prev + token * mul_cur) mod buckets with buckets = len(table) - 1,
+    and row `buckets` at a sequence's first position. prev [slots] int32: the
+    token in front of a later portion (updated)."""
+    buckets = table.shape[0] - 1
+    rows = torch.full_like(ids, buckets)
+    for a, b, start, slot in _seq_spans(cu_seqlens, seq_lens, state_slots):
+        rows[a + 1:b] = (ids[a:b - 1] * mul_prev + ids[a + 1:b] * mul_cur) % buckets
+        if start > 0 and slot >= 0:
+            rows[a] = (int(prev[slot]) * mul_prev + int(ids[a]) * mul_cur) % buckets
+        if slot >= 0:
+            prev[slot] = ids[b - 1].to(prev.dtype)
+    return embed[ids].float() * scale + table[rows].float()
+
+
+def row_norm_qk_cache(q, k, v, q_norm_w, k_norm_w, eps, positions, temp_coef,
+                      temp_every, k_cache, v_cache, slot_mapping):
+    """q [T, H*D] and k [T, G*D] divided by the root mean square of the whole
+    row and times a weight per element; q times 1 + temp_coef ln(floor((p + 1)
+    / temp_every) + 1) at position p (temp_every 0: no factor); k and v
+    [T, G*V] to their pages (slot -1: nowhere). Returns q in its dtype."""
+    def unit(t):
+        return t * torch.rsqrt(t.pow(2).mean(-1, keepdim=True) + eps)
+
+    qf = unit(q.float()) * q_norm_w.float()
+    kf = unit(k.float()) * k_norm_w.float()
+    if temp_every > 0:
+        turns = torch.div(positions + 1, temp_every, rounding_mode="floor")
+        qf = qf * (1.0 + temp_coef * torch.log(turns.float() + 1.0))[:, None]
+    G, bs = k_cache.shape[1], k_cache.shape[2]
+    ok = slot_mapping >= 0
+    blk = (slot_mapping[ok] // bs).long()
+    off = (slot_mapping[ok] % bs).long()
+    k_cache[blk, :, off] = kf[ok].unflatten(-1, (G, -1)).to(k_cache.dtype)
+    v_cache[blk, :, off] = v[ok].unflatten(-1, (G, -1)).to(v_cache.dtype)
+    return qf.to(q.dtype)
+
+
+def relu_square(x):
+    """max(x, 0)^2."""
+    return x.float().clamp(min=0.0).square().to(x.dtype)
