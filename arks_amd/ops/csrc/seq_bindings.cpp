@@ -1726,7 +1726,14 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("softcap", &softcap);
   m.def("head_gate", &head_gate);
   m.def("channel_delta_scan", &channel_delta_scan);
-  m.def("channel_delta_chunks", &channel_delta_chunks);
+  m.def("channel_delta_chunks", &channel_delta_chunks,
+        py::arg("out"), py::arg("u"), py::arg("decay"), py::arg("beta"),
+        py::arg("gate"), py::arg("rate"), py::arg("dt_bias"),
+        py::arg("norm_w"), py::arg("eps"), py::arg("unit_eps"),
+        py::arg("state"), py::arg("chunk_off"), py::arg("chunk_cu"),
+        py::arg("cu"), py::arg("seq_lens"), py::arg("slots"), py::arg("H"),
+        py::arg("G"), py::arg("D"), py::arg("V"), py::arg("head_decay") =
+        false, py::arg("silu_gate") = false);
   m.def("latent_prepare", &latent_prepare);
   m.def("latent_query", &latent_query);
   m.def("latent_pages", &latent_pages);
@@ -1737,7 +1744,13 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("conv_qkv_cache", &conv_qkv_cache);
   m.def("diff_head_norm_gate", &diff_head_norm_gate);
   m.def("moe_glu_scaled", &moe_glu_scaled);
-  m.def("attention_masked_mfma", &attention_masked_mfma);
+  m.def("attention_masked_mfma", &attention_masked_mfma,
+        py::arg("out"), py::arg("q"), py::arg("k_cache"),
+        py::arg("v_cache"), py::arg("block_tables"), py::arg("seq_lens"),
+        py::arg("cu"), py::arg("token_seq"), py::arg("scale"),
+        py::arg("sink_w"), py::arg("softcap"), py::arg("window"),
+        py::arg("keep_first"), py::arg("out_scale"), py::arg("single_rows"),
+        py::arg("maps"), py::arg("slopes") = py::none());
   m.def("stream_mix_norm", &stream_mix_norm);
   m.def("short_conv_residual", &short_conv_residual);
   m.def("head_norm_gate", &head_norm_gate);

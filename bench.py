@@ -60,12 +60,12 @@ def parse_args():
     p.add_argument("--design-bench", action="store_true")
     p.add_argument("--design-only",
                    choices=["gagorax", "fusolix", "legalix", "rivolix",
-                            "pazilorn", "llama", "moe", "mixtral"],
+                            "pazilorn", "fuzelorn", "llama", "moe", "mixtral"],
                    default=None)
     # which layer-list design --design-bench measures beside llama
     p.add_argument("--design",
                    choices=["gagorax", "fusolix", "legalix", "rivolix",
-                            "pazilorn"],
+                            "pazilorn", "fuzelorn"],
                    default="gagorax")
     p.add_argument("--cold-start", action="store_true")
     p.add_argument("--ckpt-dir", default="/tmp/arks_ckpt")
@@ -137,10 +137,11 @@ def run_cold_start(args):
 
 
 def run_design_bench(args):
-    """A layer-list design (--design: Gagorax, Fusolix, Legalix, Rivolix or
-    Pazilorn, 8 blocks at the sizes of an 8B model) against llama-3-8b cut to
-    8 layers (Rivolix: against a Qwen2-MoE-shaped, Pazilorn: against a
-    Mixtral-shaped model of equal sizes): prefill
+    """A layer-list design (--design: Gagorax, Fusolix, Legalix, Rivolix,
+    Pazilorn or Fuzelorn, 8 blocks at the sizes of an 8B model) against
+    llama-3-8b cut to 8 layers (Rivolix and Fuzelorn: against a
+    Qwen2-MoE-shaped, Pazilorn: against a Mixtral-shaped model of equal
+    sizes; Fuzelorn also against Pazilorn): prefill
     tokens/s for one long prompt and for a batch of prompts, decode tokens/s
     for a batch at a fixed context. Random weights, synthetic tokens, one
     GPU."""
@@ -153,7 +154,7 @@ def run_design_bench(args):
         PRESET_CONFIGS["llama-3-8b"], num_hidden_layers=8)
     use_gpu = torch.cuda.is_available()
     models = {args.design: args.design + "-8b-slice", "llama": "llama-3-8b-8l"}
-    if args.design == "rivolix":
+    if args.design in ("rivolix", "fuzelorn"):
         # the same expert layout in the llama family: 16 experts of ff 3584,
         # 4 per row, a shared expert of ff 3584, 32/8 heads x 128
         PRESET_CONFIGS["qwen2moe-8b-8l"] = dataclasses.replace(
@@ -162,7 +163,12 @@ def run_design_bench(args):
             num_experts_per_tok=4, moe_intermediate_size=3584,
             shared_expert_intermediate_size=3584, norm_topk_prob=False,
             attention_bias=True, tie_word_embeddings=True)
-        models = {"rivolix": "rivolix-8b-slice", "moe": "qwen2moe-8b-8l"}
+        models = {args.design: args.design + "-8b-slice",
+                  "moe": "qwen2moe-8b-8l"}
+    if args.design == "fuzelorn":
+        # the layer-list design with the same kinds of layers: a delta rule,
+        # windowed attention, 16 experts of ff 3584, 4 per row
+        models["pazilorn"] = "pazilorn-8b-slice"
     if args.design == "pazilorn":
         # the same routed experts: 16 of ff 3584, 4 per row, 32/8 heads x 128
         PRESET_CONFIGS["mixtral-8b-8l"] = dataclasses.replace(

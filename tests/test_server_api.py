@@ -501,7 +501,7 @@ def test_cli_flags_map_to_engine_config():
 
 @pytest.mark.parametrize("preset", ["tiny-gagorax", "tiny-fusolix",
                                     "tiny-legalix", "tiny-rivolix",
-                                    "tiny-pazilorn"])
+                                    "tiny-pazilorn", "tiny-fuzelorn"])
 def test_layer_list_preset_serves_completions(preset):
     """A layer-list model (recurrent state slots, no prefix reuse) behind
     the same HTTP front: a completion and a streamed chat, twice, so slots
