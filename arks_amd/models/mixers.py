@@ -1148,6 +1148,24 @@ class BiasedWindowAttention(SplitMixer):
         return {"k": ("paged", (self.G, block_size, self.D), dtype),
                 "v": ("paged", (self.G, block_size, self.V), dtype)}
 
+    def _prompt_tiles(self, batch: ForwardBatch, q, out, cache_k):
+        """Work list of the 256-row prefill kernel for a step whose longest
+        portion fills a tile (host-built once per step and head layout; every
+        sequence of the step is in it); None where the masked or general
+        kernels run."""
+        if (not q.is_cuda or q.dtype != torch.bfloat16 or self.D != self.V
+                or self.D not in ops.PREFILL_MAP_DIMS or not ops.use_ladder_bias
+                or batch.kv_lens_list is None or self.scale <= 0
+                or batch.max_q_len < ops.EXTEND2_QTILE
+                or not out.is_contiguous() or cache_k.shape[2] != 16):
+            return None
+        key = ("biased", self.H, self.D)
+        if key not in batch.tile_cache:
+            batch.tile_cache[key] = ops.build_extend_tiles(
+                batch.seq_lens_list, batch.kv_lens_list, False, q.device,
+                num_q_heads=self.H, flash_decode=False, min_ladder=1)
+        return batch.tile_cache[key]
+
     def core(self, p, batch: ForwardBatch, cache: dict, out, out_scale) -> None:
         H, G, D, V = self.H, self.G, self.D, self.V
         nq, nk, nv = H * D, G * D, G * V
@@ -1156,6 +1174,15 @@ class BiasedWindowAttention(SplitMixer):
             self.q_norm, self.k_norm, self.eps, batch.positions,
             self.temp_coef, self.temp_every, cache["k"], cache["v"],
             batch.slot_mapping)
+        tiles = (self._prompt_tiles(batch, q, out, cache["k"])
+                 if out_scale == 1.0 else None)
+        if tiles is not None:
+            ops.attention_extend_paged(
+                q.view(-1, H, D), cache["k"], cache["v"], batch.block_tables,
+                batch.seq_lens, batch.cu_seqlens, None, self.scale,
+                window=self.window, tiles=tiles, native=ops.seq_extension(),
+                sink_w=self.sink, slopes=self.slopes, out=out.view(-1, H, V))
+            return
         ops.attention_sink_paged(
             q.view(-1, H, D), cache["k"], cache["v"], batch.block_tables,
             batch.seq_lens, batch.cu_seqlens, batch.token_seq, self.scale,

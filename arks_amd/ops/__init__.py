@@ -146,7 +146,8 @@ EXTEND2_MIN_QLEN = 97
 
 def build_extend_tiles(q_lens: list[int], kv_lens: list[int] | None,
                        kv_fp8: bool, device, num_q_heads: int = 32,
-                       ladder: bool = True, flash_decode: bool = True):
+                       ladder: bool = True, flash_decode: bool = True,
+                       min_ladder: int = EXTEND2_MIN_QLEN):
     """Per-seq routing for the extend dispatcher:
     (tiles64, tiles256 [n,4], decode_rows, combine_table, ws_rows).
 
@@ -160,15 +161,16 @@ def build_extend_tiles(q_lens: list[int], kv_lens: list[int] | None,
     the batch is too small to fill the chip, deep 256-row tiles are
     additionally SPLIT over their KV range flash-decode-style (part rows
     + a combine pass over f32 partials); split parts sort first so the
-    partial workspace only covers them. Build once per batch and reuse
-    across all layers."""
+    partial workspace only covers them. min_ladder: the shortest portion
+    that goes to the 256-row kernel. Build once per batch and reuse across
+    all layers."""
     t64, t256, dec = [], [], []
     kvl = kv_lens if kv_lens is not None else q_lens
     for i, n in enumerate(q_lens):
         off = kvl[i] - n
         if n == 1 and flash_decode:
             dec.append(i)
-        elif kv_fp8 or n < EXTEND2_MIN_QLEN or not ladder:
+        elif kv_fp8 or n < min_ladder or not ladder:
             for q0 in range(0, n, PREFILL_QTILE):
                 t64.append((i, q0, min(kvl[i], off + q0 + PREFILL_QTILE)))
         else:
@@ -232,7 +234,8 @@ def build_extend_tiles(q_lens: list[int], kv_lens: list[int] | None,
 def attention_extend_paged(
     q, k_cache, v_cache, block_tables, kv_lens, cu_seqlens_q,
     q_lens: list[int], scale: float, window: int = 0, tiles=None,
-    sink: bool = False, native=None, maps: int = 1,
+    sink: bool = False, native=None, maps: int = 1, sink_w=None, slopes=None,
+    out=None,
 ):
     """Causal attention of packed NEW tokens over each sequence's full paged
     KV history (cached prefix + new tokens already written by
@@ -244,7 +247,10 @@ def attention_extend_paged(
     kernels runs (default: arks_amd_C). maps M > 1: a key row of the cache
     holds M keys side by side that share the row's value (k_cache [pages, G,
     16, M*D]); q has G*M groups of heads, group g*M + m reads key m of head
-    g (tiles built without the flash-decode rows).
+    g (tiles built without the flash-decode rows). sink_w, slopes [Hq] fp32:
+    a sink's score per head, a distance bias slope[h] (i - j) off the scores
+    (256-row tiles only: build_extend_tiles(min_ladder=1)). out: a contiguous
+    [Tq, Hq, D] tensor to write.
 
     Dispatch: big chunks run the 8-wave 32x32-MFMA ladder kernel
     (attn_extend2.hip, 256-row q tiles); small chunks and fp8-KV runs use
@@ -252,9 +258,10 @@ def attention_extend_paged(
     if q.is_cuda:
         C = native if native is not None else _native()
         sink = 1 if sink else 0
-        out = torch.empty(
-            (q.shape[0], q.shape[1], q.shape[2]), dtype=q.dtype, device=q.device
-        )
+        if out is None:
+            out = torch.empty(
+                (q.shape[0], q.shape[1], q.shape[2]), dtype=q.dtype,
+                device=q.device)
         kv_fp8 = k_cache.dtype != torch.bfloat16
         t64, t256, (drows, dseqs), ctab, ws_rows = (
             tiles if tiles is not None
@@ -271,13 +278,14 @@ def attention_extend_paged(
                 ws = q.new_empty(0, dtype=torch.float32)
             C.attention_extend_paged2(
                 out, q, k_cache, v_cache, block_tables, kv_lens, cu_seqlens_q,
-                t256, ws, scale, window, sink, maps,
+                t256, ws, scale, window, sink, maps, sink_w, slopes,
             )
             if ctab.numel():
                 C.attention_extend2_combine(
                     out, ws, ctab, cu_seqlens_q, scale,
                 )
         if t64.numel():
+            assert sink_w is None and slopes is None
             C.attention_extend_paged(
                 out, q, k_cache, v_cache, block_tables, kv_lens, cu_seqlens_q,
                 t64, scale, window, sink, maps,
@@ -759,6 +767,8 @@ use_masked_mfma = True  # tests switch it off to compare both paths
 # (head sizes of the 256-row ladder kernel) instead of the masked tiles
 use_ladder_maps = True
 PREFILL_MAP_DIMS = (64, 128)
+# prompt portions under a distance bias or per-head sinks: the same kernel
+use_ladder_bias = True
 
 
 def seq_extension():

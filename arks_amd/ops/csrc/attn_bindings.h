@@ -33,6 +33,7 @@ void arks_attn_extend_paged2(void* out, const void* q, const void* k_cache,
                              float scale, int num_q_heads, int num_kv_heads,
                              int head_dim, int max_blocks, int64_t q_stride,
                              int window, int sink, int maps,
+                             const void* sink_w, const void* slopes,
                              hipStream_t stream);
 void arks_attn_extend2_combine(void* out, const void* part_ws,
                                const void* combine_table,
@@ -150,7 +151,8 @@ inline void attention_extend_paged2(torch::Tensor out, torch::Tensor q,
                              torch::Tensor cu_seqlens_q,
                              torch::Tensor tile_info, torch::Tensor part_ws,
                              double scale, int64_t window, int64_t sink,
-                             int64_t maps) {
+                             int64_t maps, c10::optional<torch::Tensor> sink_w,
+                             c10::optional<torch::Tensor> slopes) {
   check_bf16_contig(out, "out");
   check_bf16_rowstrided(q, "q");
   check_bf16_contig(k_cache, "k_cache");
@@ -171,6 +173,13 @@ inline void attention_extend_paged2(torch::Tensor out, torch::Tensor q,
               "cache rows do not fit the heads and key maps");
   TORCH_CHECK(k_cache.size(2) == 16, "KV block size must be 16");
   TORCH_CHECK(head_dim == 64 || head_dim == 128, "head_dim must be 64 or 128");
+  // a sink's score and a distance bias' slope per query head
+  auto per_head = [&](const c10::optional<torch::Tensor>& t) -> const void* {
+    if (!t.has_value()) return nullptr;
+    TORCH_CHECK(t->is_cuda() && t->scalar_type() == torch::kFloat32 &&
+                t->is_contiguous() && t->numel() == num_q_heads && scale > 0);
+    return t->data_ptr();
+  };
   const int ntiles = tile_info.size(0);
   const int max_blocks = block_tables.size(1);
   void* ws = nullptr;
@@ -185,6 +194,7 @@ inline void attention_extend_paged2(torch::Tensor out, torch::Tensor q,
                           tile_info.data_ptr(), ws, ntiles, (float)scale,
                           num_q_heads, num_kv_heads, head_dim, max_blocks,
                           q.stride(0), (int)window, (int)sink, (int)maps,
+                          per_head(sink_w), per_head(slopes),
                           attn_current_stream());
 }
 inline void attention_extend2_combine(torch::Tensor out, torch::Tensor part_ws,
@@ -205,7 +215,12 @@ inline void attention_extend2_combine(torch::Tensor out, torch::Tensor part_ws,
 inline void def_paged_attention(pybind11::module_& m) {
   m.def("attention_decode_paged", &attention_decode_paged);
   m.def("attention_extend_paged", &attention_extend_paged);
-  m.def("attention_extend_paged2", &attention_extend_paged2);
+  using pybind11::arg;
+  m.def("attention_extend_paged2", &attention_extend_paged2, arg("out"),
+        arg("q"), arg("k_cache"), arg("v_cache"), arg("block_tables"),
+        arg("kv_lens"), arg("cu_seqlens_q"), arg("tile_info"), arg("part_ws"),
+        arg("scale"), arg("window"), arg("sink"), arg("maps"),
+        arg("sink_w") = pybind11::none(), arg("slopes") = pybind11::none());
   m.def("attention_extend2_combine", &attention_extend2_combine);
 }
 

@@ -21,6 +21,12 @@
 // `window` key positions per query (Mistral-style); the KV loop starts at
 // the first tile any of this workgroup's rows can see.
 //
+// BIASED: a distance bias slopes[h] * (i - j) off the scaled scores (the
+// score accumulators start from it) and a sink of a score per head
+// (sink_w[h]: the running softmax starts from it). These launches also walk
+// sequences of a few rows beside long ones, so a wave skips the tiles none of
+// its rows can see.
+//
 // This is the prefix-caching / chunked-prefill attention of the runtime
 // slot (the reference delegates it to vLLM/SGLang images
 // at arksapplication_controller.go:941-1002).
@@ -58,7 +64,7 @@ __device__ __forceinline__ uint32_t cvt_pk_bf16(float lo, float hi) {
 // conflicted) while the tr16 read pairs overlap by only 8 of 64 banks.
 constexpr int VBLK_ELEMS = 80;
 
-template <int HEAD_DIM>
+template <int HEAD_DIM, bool BIASED>
 __global__ __launch_bounds__(512) void attn_extend2_kernel(
     bf16* __restrict__ out,            // [Tq, Hq, D]
     const bf16* __restrict__ q,        // [Tq, Hq, D] (packed new tokens)
@@ -80,7 +86,9 @@ __global__ __launch_bounds__(512) void attn_extend2_kernel(
     // side that share the row's value (k_cache [nblocks, Hkv / maps, 16,
     // maps * D], v_cache [nblocks, Hkv / maps, 16, D]); key group g reads
     // key g % maps of the rows of head g / maps
-    const int maps) {
+    const int maps,
+    // BIASED: [Hq] each, or null
+    const float* __restrict__ sink_w, const float* __restrict__ slopes) {
   constexpr int STEPS = HEAD_DIM / 16;   // QK^T K-contraction steps
   constexpr int DTILES = HEAD_DIM / 32;  // 32-dim output tiles
   constexpr int CB = HEAD_DIM / 16;      // 16-col blocks per key row
@@ -98,7 +106,8 @@ __global__ __launch_bounds__(512) void attn_extend2_kernel(
   const int* __restrict__ bt = block_tables + (int64_t)seq_idx * max_blocks;
 
   const int tid = threadIdx.x;
-  const int wave = tid / WAVE_SIZE;
+  const int wave = BIASED ? __builtin_amdgcn_readfirstlane(tid / WAVE_SIZE)
+                          : tid / WAVE_SIZE;
   const int lane = tid % WAVE_SIZE;
   const int col = lane & 31;   // q-row within wave (QK^T) / dim col (PV)
   const int half = lane >> 5;  // lane half
@@ -140,6 +149,12 @@ __global__ __launch_bounds__(512) void attn_extend2_kernel(
   // then carries it like any other key
   float m_run = (sink && part == 0) ? 0.f : -1e30f;
   float l_run = (sink && part == 0) ? 1.f : 0.f;
+  // in raw score units, like the running max
+  const float slope = BIASED && slopes ? slopes[h] / scale : 0.f;
+  if (BIASED && sink_w && part == 0) {
+    m_run = sink_w[h] / scale;
+    l_run = 1.f;
+  }
   f32x16 oacc[DTILES];
 #pragma unroll
   for (int n = 0; n < DTILES; ++n) oacc[n] = {};
@@ -239,157 +254,173 @@ __global__ __launch_bounds__(512) void attn_extend2_kernel(
     ushort8 krn[VPT], vrn[VPT];
     if (j + 1 < ntiles) load_tile(j + 1, krn, vrn);
 
-    // ---- QK^T (swapped): A = K rows (32 keys), B = Q. C[key][qrow=col].
-    // The two subtiles interleave so consecutive MFMAs hit independent
-    // accumulators (the 32x32 dependent-accumulator latency exceeds the
-    // 32-cycle issue interval).
-    f32x16 sc[2];
-    sc[0] = {};
-    sc[1] = {};
-    const char* krow0 = reinterpret_cast<const char*>(
-        k_lds + buf * KBUF + col * HEAD_DIM);
-    const char* krow1 = krow0 + 32 * HEAD_DIM * 2;
-    const int swz_mask = (col & 7) << 4;
+    const int wrow0 = q0 + wave * 32;  // this wave's first row
+    const bool busy =
+        !BIASED || (wrow0 < q_len && key_base <= kv_off + wrow0 + 31 &&
+                    (window <= 0 ||
+                     key_base + E2_KVBLK > kv_off + wrow0 - window + 1));
+    if (busy) {
+      // ---- QK^T (swapped): A = K rows (32 keys), B = Q. C[key][qrow=col].
+      // The two subtiles interleave so consecutive MFMAs hit independent
+      // accumulators (the 32x32 dependent-accumulator latency exceeds the
+      // 32-cycle issue interval).
+      f32x16 sc[2];
+      sc[0] = {};
+      sc[1] = {};
+      if constexpr (BIASED) {
+        const float b0 = -slope * (float)(my_pos - key_base - 4 * half);
 #pragma unroll
-    for (int s = 0; s < STEPS; ++s) {
-      const int off = ((s * 16 + 8 * half) * 2) ^ swz_mask;
-      ushort8 u0 = *reinterpret_cast<const ushort8*>(krow0 + off);
-      ushort8 u1 = *reinterpret_cast<const ushort8*>(krow1 + off);
-      sc[0] = e2_mfma32(*reinterpret_cast<e2_bf16x8*>(&u0), qfrag[s], sc[0]);
-      sc[1] = e2_mfma32(*reinterpret_cast<e2_bf16x8*>(&u1), qfrag[s], sc[1]);
-    }
+        for (int sub = 0; sub < 2; ++sub)
+#pragma unroll
+          for (int r16 = 0; r16 < 16; ++r16)
+            sc[sub][r16] = __builtin_fmaf(
+                slope, (float)(32 * sub + 8 * (r16 >> 2) + (r16 & 3)), b0);
+      }
+      const char* krow0 = reinterpret_cast<const char*>(
+          k_lds + buf * KBUF + col * HEAD_DIM);
+      const char* krow1 = krow0 + 32 * HEAD_DIM * 2;
+      const int swz_mask = (col & 7) << 4;
+#pragma unroll
+      for (int s = 0; s < STEPS; ++s) {
+        const int off = ((s * 16 + 8 * half) * 2) ^ swz_mask;
+        ushort8 u0 = *reinterpret_cast<const ushort8*>(krow0 + off);
+        ushort8 u1 = *reinterpret_cast<const ushort8*>(krow1 + off);
+        sc[0] = e2_mfma32(*reinterpret_cast<e2_bf16x8*>(&u0), qfrag[s], sc[0]);
+        sc[1] = e2_mfma32(*reinterpret_cast<e2_bf16x8*>(&u1), qfrag[s], sc[1]);
+      }
 
-    // ---- Masked softmax, fully in-register (exp2 domain). Lane's 32
-    // scores are all for q-row `my_qrow`; C reg 4g+r of subtile `sub` is
-    // key key_base + 32*sub + 8g + 4*half + r. Tiles fully visible to
-    // every row of this wave (the bulk of the causal region) skip the 32
-    // per-key compares; the reductions are trees, not 31-deep chains.
-    float p[32];
-    const bool full_vis =
-        (q0 + wave * 32 + 31 < q_len) &&
-        (key_base + E2_KVBLK - 1 <= kv_off + q0 + wave * 32) &&
-        (key_base + E2_KVBLK <= kmax) &&
-        (window <= 0 || key_base > kv_off + q0 + wave * 32 + 31 - window);
-    if (full_vis) {
+      // ---- Masked softmax, fully in-register (exp2 domain). Lane's 32
+      // scores are all for q-row `my_qrow`; C reg 4g+r of subtile `sub` is
+      // key key_base + 32*sub + 8g + 4*half + r. Tiles fully visible to
+      // every row of this wave (the bulk of the causal region) skip the 32
+      // per-key compares; the reductions are trees, not 31-deep chains.
+      float p[32];
+      const bool full_vis =
+          (q0 + wave * 32 + 31 < q_len) &&
+          (key_base + E2_KVBLK - 1 <= kv_off + q0 + wave * 32) &&
+          (key_base + E2_KVBLK <= kmax) &&
+          (window <= 0 || key_base > kv_off + q0 + wave * 32 + 31 - window);
+      if (full_vis) {
 #pragma unroll
-      for (int sub = 0; sub < 2; ++sub)
+        for (int sub = 0; sub < 2; ++sub)
 #pragma unroll
-        for (int r16 = 0; r16 < 16; ++r16)
-          p[sub * 16 + r16] = sc[sub][r16];
-    } else {
+          for (int r16 = 0; r16 < 16; ++r16)
+            p[sub * 16 + r16] = sc[sub][r16];
+      } else {
 #pragma unroll
-      for (int sub = 0; sub < 2; ++sub) {
-        const int kb_s = key_base + 32 * sub + 4 * half;
+        for (int sub = 0; sub < 2; ++sub) {
+          const int kb_s = key_base + 32 * sub + 4 * half;
+#pragma unroll
+          for (int r16 = 0; r16 < 16; ++r16) {
+            const int kg = kb_s + 8 * (r16 >> 2) + (r16 & 3);
+            bool ok = qrow_valid && kg <= my_pos && kg < kmax;
+            if (window > 0) ok = ok && (kg > my_pos - window);
+            p[sub * 16 + r16] = ok ? sc[sub][r16] : MASKED;
+          }
+        }
+      }
+      float mt[16];
+#pragma unroll
+      for (int i = 0; i < 16; ++i) mt[i] = fmaxf(p[i], p[i + 16]);
+#pragma unroll
+      for (int w = 8; w > 0; w >>= 1)
+#pragma unroll
+        for (int i = 0; i < w; ++i) mt[i] = fmaxf(mt[i], mt[i + w]);
+      const float tmax = fmaxf(mt[0], __shfl_xor(mt[0], 32, WAVE_SIZE));
+
+      // Defer-max (T13): only rescale O when the tile max meaningfully
+      // exceeds the running max (threshold in raw units; exp2(THR)=256
+      // stays comfortably finite).
+      const float thr_raw = RESCALE_THR / scale2;
+      if (!__all(tmax - m_run <= thr_raw)) {
+        const float m_new = fmaxf(m_run, tmax);
+        const float alpha = __builtin_amdgcn_exp2f((m_run - m_new) * scale2);
+        l_run *= alpha;
+        m_run = m_new;
+        // O rows live across regs (C layout): fetch each row's alpha from
+        // the lane that owns that q-row.
 #pragma unroll
         for (int r16 = 0; r16 < 16; ++r16) {
-          const int kg = kb_s + 8 * (r16 >> 2) + (r16 & 3);
-          bool ok = qrow_valid && kg <= my_pos && kg < kmax;
-          if (window > 0) ok = ok && (kg > my_pos - window);
-          p[sub * 16 + r16] = ok ? sc[sub][r16] : MASKED;
+          const int row = 8 * (r16 >> 2) + 4 * half + (r16 & 3);
+          const float a_r = __shfl(alpha, 32 * (lane >> 5) + row, WAVE_SIZE);
+#pragma unroll
+          for (int n = 0; n < DTILES; ++n) oacc[n][r16] *= a_r;
         }
       }
-    }
-    float mt[16];
-#pragma unroll
-    for (int i = 0; i < 16; ++i) mt[i] = fmaxf(p[i], p[i + 16]);
-#pragma unroll
-    for (int w = 8; w > 0; w >>= 1)
-#pragma unroll
-      for (int i = 0; i < w; ++i) mt[i] = fmaxf(mt[i], mt[i + w]);
-    const float tmax = fmaxf(mt[0], __shfl_xor(mt[0], 32, WAVE_SIZE));
 
-    // Defer-max (T13): only rescale O when the tile max meaningfully
-    // exceeds the running max (threshold in raw units; exp2(THR)=256
-    // stays comfortably finite).
-    const float thr_raw = RESCALE_THR / scale2;
-    if (!__all(tmax - m_run <= thr_raw)) {
-      const float m_new = fmaxf(m_run, tmax);
-      const float alpha = __builtin_amdgcn_exp2f((m_run - m_new) * scale2);
-      l_run *= alpha;
-      m_run = m_new;
-      // O rows live across regs (C layout): fetch each row's alpha from
-      // the lane that owns that q-row.
+      // p = exp2((s - m) * scale2) as one fma + exp2; MASKED entries
+      // underflow to exactly 0 (|MASKED*scale2| >> |m*scale2|).
+      const float nms = -m_run * scale2;
 #pragma unroll
-      for (int r16 = 0; r16 < 16; ++r16) {
-        const int row = 8 * (r16 >> 2) + 4 * half + (r16 & 3);
-        const float a_r = __shfl(alpha, 32 * (lane >> 5) + row, WAVE_SIZE);
+      for (int i = 0; i < 32; ++i)
+        p[i] = __builtin_amdgcn_exp2f(__builtin_fmaf(p[i], scale2, nms));
+      float st[16];
 #pragma unroll
-        for (int n = 0; n < DTILES; ++n) oacc[n][r16] *= a_r;
-      }
-    }
+      for (int i = 0; i < 16; ++i) st[i] = p[i] + p[i + 16];
+#pragma unroll
+      for (int w = 8; w > 0; w >>= 1)
+#pragma unroll
+        for (int i = 0; i < w; ++i) st[i] += st[i + w];
+      l_run += st[0] + __shfl_xor(st[0], 32, WAVE_SIZE);
 
-    // p = exp2((s - m) * scale2) as one fma + exp2; MASKED entries
-    // underflow to exactly 0 (|MASKED*scale2| >> |m*scale2|).
-    const float nms = -m_run * scale2;
+      // ---- P -> bf16 PV A-fragments: per subtile, 8 cvt_pk words
+      // W[g][0] = pk(p[4g], p[4g+1]), W[g][1] = pk(p[4g+2], p[4g+3]); the
+      // permlane32_swap pairs (W[2t][*], W[2t+1][*]) then give each half its
+      // step-t fragment from both halves' key sets.
+      uint32_t afrag[4][4];  // [k-step t][4 dwords = 8 bf16]
 #pragma unroll
-    for (int i = 0; i < 32; ++i)
-      p[i] = __builtin_amdgcn_exp2f(__builtin_fmaf(p[i], scale2, nms));
-    float st[16];
+      for (int sub = 0; sub < 2; ++sub) {
+        uint32_t w0[4], w1[4];
 #pragma unroll
-    for (int i = 0; i < 16; ++i) st[i] = p[i] + p[i + 16];
-#pragma unroll
-    for (int w = 8; w > 0; w >>= 1)
-#pragma unroll
-      for (int i = 0; i < w; ++i) st[i] += st[i + w];
-    l_run += st[0] + __shfl_xor(st[0], 32, WAVE_SIZE);
-
-    // ---- P -> bf16 PV A-fragments: per subtile, 8 cvt_pk words
-    // W[g][0] = pk(p[4g], p[4g+1]), W[g][1] = pk(p[4g+2], p[4g+3]); the
-    // permlane32_swap pairs (W[2t][*], W[2t+1][*]) then give each half its
-    // step-t fragment from both halves' key sets.
-    uint32_t afrag[4][4];  // [k-step t][4 dwords = 8 bf16]
-#pragma unroll
-    for (int sub = 0; sub < 2; ++sub) {
-      uint32_t w0[4], w1[4];
-#pragma unroll
-      for (int g = 0; g < 4; ++g) {
-        const int b = sub * 16 + 4 * g;
-        w0[g] = cvt_pk_bf16(p[b + 0], p[b + 1]);
-        w1[g] = cvt_pk_bf16(p[b + 2], p[b + 3]);
-      }
-#pragma unroll
-      for (int tau = 0; tau < 2; ++tau) {
-        auto r0 = __builtin_amdgcn_permlane32_swap(w0[2 * tau], w0[2 * tau + 1],
-                                                   false, false);
-        auto r1 = __builtin_amdgcn_permlane32_swap(w1[2 * tau], w1[2 * tau + 1],
-                                                   false, false);
-        const int t = sub * 2 + tau;
-        afrag[t][0] = r0[0];
-        afrag[t][1] = r1[0];
-        afrag[t][2] = r0[1];
-        afrag[t][3] = r1[1];
-      }
-    }
-
-    // ---- PV: O[qrow][dim] += P[qrow][key] V[key][dim]; B fragments via
-    // tr16 reads of the V image (per step t: keys 16t+8*half+0..7 at
-    // column 16*(colhalf)+l&15 -> blocks kb = 4t+2*half (+1), cb per group).
-    const int g4 = lane >> 4;  // 16-lane tr16 group
-    bf16* vbase = v_img + buf * VBUF;
-    // t outer / n inner: consecutive MFMAs accumulate into the DTILES
-    // independent oacc registers instead of chaining one.
-#pragma unroll
-    for (int t = 0; t < 4; ++t) {
-      const int kb = 4 * t + 2 * (g4 >> 1);
-#pragma unroll
-      for (int n = 0; n < DTILES; ++n) {
-        const int cb = 2 * n + (g4 & 1);
-        e2_bf16x4 v1 = __builtin_amdgcn_ds_read_tr16_b64_v4bf16(
-            (__attribute__((address_space(3))) e2_bf16x4*)(
-                reinterpret_cast<char*>(vbase + (kb * CB + cb) * VBLK_ELEMS) +
-                (lane & 15) * 8));
-        e2_bf16x4 v2 = __builtin_amdgcn_ds_read_tr16_b64_v4bf16(
-            (__attribute__((address_space(3))) e2_bf16x4*)(
-                reinterpret_cast<char*>(vbase + ((kb + 1) * CB + cb) * VBLK_ELEMS) +
-                (lane & 15) * 8));
-        e2_bf16x8 vb;
-#pragma unroll
-        for (int e = 0; e < 4; ++e) {
-          vb[e] = v1[e];
-          vb[e + 4] = v2[e];
+        for (int g = 0; g < 4; ++g) {
+          const int b = sub * 16 + 4 * g;
+          w0[g] = cvt_pk_bf16(p[b + 0], p[b + 1]);
+          w1[g] = cvt_pk_bf16(p[b + 2], p[b + 3]);
         }
-        oacc[n] = e2_mfma32(*reinterpret_cast<e2_bf16x8*>(&afrag[t][0]), vb,
-                            oacc[n]);
+#pragma unroll
+        for (int tau = 0; tau < 2; ++tau) {
+          auto r0 = __builtin_amdgcn_permlane32_swap(w0[2 * tau], w0[2 * tau + 1],
+                                                     false, false);
+          auto r1 = __builtin_amdgcn_permlane32_swap(w1[2 * tau], w1[2 * tau + 1],
+                                                     false, false);
+          const int t = sub * 2 + tau;
+          afrag[t][0] = r0[0];
+          afrag[t][1] = r1[0];
+          afrag[t][2] = r0[1];
+          afrag[t][3] = r1[1];
+        }
+      }
+
+      // ---- PV: O[qrow][dim] += P[qrow][key] V[key][dim]; B fragments via
+      // tr16 reads of the V image (per step t: keys 16t+8*half+0..7 at
+      // column 16*(colhalf)+l&15 -> blocks kb = 4t+2*half (+1), cb per group).
+      const int g4 = lane >> 4;  // 16-lane tr16 group
+      bf16* vbase = v_img + buf * VBUF;
+      // t outer / n inner: consecutive MFMAs accumulate into the DTILES
+      // independent oacc registers instead of chaining one.
+#pragma unroll
+      for (int t = 0; t < 4; ++t) {
+        const int kb = 4 * t + 2 * (g4 >> 1);
+#pragma unroll
+        for (int n = 0; n < DTILES; ++n) {
+          const int cb = 2 * n + (g4 & 1);
+          e2_bf16x4 v1 = __builtin_amdgcn_ds_read_tr16_b64_v4bf16(
+              (__attribute__((address_space(3))) e2_bf16x4*)(
+                  reinterpret_cast<char*>(vbase + (kb * CB + cb) * VBLK_ELEMS) +
+                  (lane & 15) * 8));
+          e2_bf16x4 v2 = __builtin_amdgcn_ds_read_tr16_b64_v4bf16(
+              (__attribute__((address_space(3))) e2_bf16x4*)(
+                  reinterpret_cast<char*>(vbase + ((kb + 1) * CB + cb) * VBLK_ELEMS) +
+                  (lane & 15) * 8));
+          e2_bf16x8 vb;
+#pragma unroll
+          for (int e = 0; e < 4; ++e) {
+            vb[e] = v1[e];
+            vb[e + 4] = v2[e];
+          }
+          oacc[n] = e2_mfma32(*reinterpret_cast<e2_bf16x8*>(&afrag[t][0]), vb,
+                              oacc[n]);
+        }
       }
     }
 
@@ -495,9 +526,10 @@ extern "C" void arks_attn_extend_paged2(
     const void* block_tables, const void* kv_lens, const void* cu_seqlens_q,
     const void* tile_info, void* part_ws, int ntiles, float scale,
     int num_q_heads, int num_kv_heads, int head_dim, int max_blocks,
-    int64_t q_stride, int window, int sink, int maps, hipStream_t stream) {
+    int64_t q_stride, int window, int sink, int maps, const void* sink_w,
+    const void* slopes, hipStream_t stream) {
   dim3 grid(num_q_heads, ntiles), block(512);
-  static bool attr_set[2] = {false, false};
+  static bool attr_set[4] = {false, false, false, false};
   auto launch = [&](auto kern, int lds_bytes, int idx) {
     if (!attr_set[idx]) {
       (void)hipFuncSetAttribute(reinterpret_cast<const void*>(kern),
@@ -511,14 +543,17 @@ extern "C" void arks_attn_extend_paged2(
                        (const int*)kv_lens, (const int*)cu_seqlens_q,
                        (const int*)tile_info, (float*)part_ws, scale,
                        num_q_heads, num_kv_heads, max_blocks, q_stride,
-                       window, sink, maps);
+                       window, sink, maps, (const float*)sink_w,
+                       (const float*)slopes);
   };
   if (head_dim == 128) {
     constexpr int LDS = (2 * 64 * 128 + 2 * 16 * 8 * VBLK_ELEMS) * 2;
-    launch(attn_extend2_kernel<128>, LDS, 0);
+    if (sink_w || slopes) launch(attn_extend2_kernel<128, true>, LDS, 2);
+    else launch(attn_extend2_kernel<128, false>, LDS, 0);
   } else if (head_dim == 64) {
     constexpr int LDS = (2 * 64 * 64 + 2 * 16 * 4 * VBLK_ELEMS) * 2;
-    launch(attn_extend2_kernel<64>, LDS, 1);
+    if (sink_w || slopes) launch(attn_extend2_kernel<64, true>, LDS, 3);
+    else launch(attn_extend2_kernel<64, false>, LDS, 1);
   }
 }
 

@@ -1507,8 +1507,7 @@ void residual_sandwich_norm(Tensor x, OptTensor h, OptTensor y,
   const void* wpr = weight(w_pre, "w_pre");
   const void* y2_p = row_tensor(y2, "y2");
   const void* wpo2 = weight(w_post2, "w_post2");
-  TORCH_CHECK((wpo != nullptr) <= (y_p != nullptr) &&
-              (y2_p != nullptr) <= (y_p != nullptr) &&
+  TORCH_CHECK((y2_p != nullptr) <= (y_p != nullptr) &&
               (wpo2 != nullptr) <= (y2_p != nullptr) &&
               (h_p != nullptr) == (wpr != nullptr));
   arks_seq_residual_sandwich_norm(x.data_ptr(), h_p, y_p, wpo, y2_p, wpo2,

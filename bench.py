@@ -54,9 +54,10 @@ def parse_args():
     # design (--design) at real layer sizes beside the closest llama-family
     # model cut to the same width and depth (for rivolix, whose feed-forward
     # is routed experts beside a shared one: a Qwen2-MoE-shaped model of the
-    # same width, depth, head and expert sizes, "moe"; for pazilorn, routed
+    # same width, depth, head and expert sizes, "moe", as for fuzelorn, which
+    # also runs beside pazilorn; for pazilorn, routed
     # experts alone: a Mixtral-shaped one, "mixtral"), one JSON line per
-    # model and phase. --design-only NAME runs one of the two (profiling).
+    # model and phase. --design-only NAME runs one of them (profiling).
     p.add_argument("--design-bench", action="store_true")
     p.add_argument("--design-only",
                    choices=["gagorax", "fusolix", "legalix", "rivolix",

@@ -338,10 +338,11 @@ def test_fast_path_sizes(tmp_path, device, dtype):
     cfg = fast_path_config(MOE(experts=8, top=2, ff=32, groups=4, keep=2,
                                shared_ff=24))
     w = write_checkpoint(tmp_path / "m", cfg)
-    t = toks(330, seed=11)
+    t = toks(470, seed=11)
     eng = make_engine(tmp_path / "m", device, dtype, max_tokens=512)
     plan = [t[:130], t[130:131], t[131:197], t[197:198], t[198:199],
             t[199:201], t[201:]]
+    assert len(plan[-1]) > 256
     got = replay(eng, tmp_path, [[("a", p, False)] for p in plan])["a"]
     assert_logits(got, cfg, w, t, dtype)
 
@@ -351,9 +352,9 @@ def test_fast_path_sizes_in_mixed_batches(tmp_path, device, dtype):
     cfg = fast_path_config()
     w = write_checkpoint(tmp_path / "m", cfg)
     reqs = {c: toks(n, seed=s) for c, n, s in
-            [("a", 150, 1), ("b", 70, 2), ("c", 201, 3), ("d", 9, 4),
+            [("a", 350, 1), ("b", 70, 2), ("c", 201, 3), ("d", 9, 4),
              ("e", 66, 5)]}
-    steps = mixed_plan(reqs, 3, 42, [67, 1, 1, 100, 2, 1, 33, 1, 90])
+    steps = mixed_plan(reqs, 3, 42, [67, 1, 1, 270, 2, 1, 33, 1, 90])
     eng = make_engine(tmp_path / "m", device, dtype, max_tokens=672)
     got = replay(eng, tmp_path, steps)
     for c in reqs:
@@ -751,6 +752,57 @@ def test_matrix_core_attention_against_the_general_kernel(size, monkeypatch):
         slow = pg.attend(q[first:], n, *args)
         monkeypatch.setattr(ops, "use_masked_mfma", True)
         assert torch.allclose(fast, slow, atol=1e-2, rtol=1e-2), first
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("window", [1, 63, 64, 90, 300, 0])
+@pytest.mark.parametrize("H,G,D", [(8, 2, 64), (5, 1, 128), (3, 3, 64)])
+def test_prefill_kernel_with_bias_and_sinks(H, G, D, window):
+    """The 256-row kernel over sequences of 1, 2, 70, 300 and 513 rows with
+    contexts in front of them, one launch (a few heads: key ranges are split;
+    the sink is counted once): against the oracle's attention, every row."""
+    from arks_amd import ops
+
+    dev = torch.device("cuda")
+    g = torch.Generator().manual_seed(D + window)
+    rows, ctx = [1, 300, 2, 70, 513], [40, 0, 17, 130, 33]
+    total = [a + b for a, b in zip(rows, ctx)]
+    blocks = [-(-n // 16) for n in total]
+    order = torch.randperm(sum(blocks) + 2, generator=g).to(torch.int32)
+    kc = torch.full((sum(blocks) + 2, G, 16, D), 9.0, dtype=torch.bfloat16)
+    vc = kc.clone()
+    table = torch.zeros(5, max(blocks), dtype=torch.int32)
+    slopes, sinks = O.bias_slopes(H), (torch.randn(H, generator=g) + 1.0).tolist()
+    scale, of = D ** -0.5, [h // (H // G) for h in range(H)]
+    qs, want, at = [], [], 0
+    for s, n in enumerate(total):
+        table[s, :blocks[s]] = order[at:at + blocks[s]]
+        at += blocks[s]
+        q, k, v = (_rounded(torch.randn(n, x, D, generator=g, dtype=F64) * 1.5,
+                            "bfloat16") for x in (H, G, G))
+        pos = torch.arange(n)
+        page = table[s][pos // 16].long()
+        kc[page, :, pos % 16], vc[page, :, pos % 16] = k.bfloat16(), v.bfloat16()
+        qs.append(q[ctx[s]:])
+        seen = sorted({ctx[s], n - 1, *range(ctx[s], n, 37)})
+        want.append((seen, O.biased_attend(q, k[:, of], v[:, of], scale,
+                                           window or n, slopes, sinks, rows=seen)))
+    f = lambda x: torch.tensor([float(y) for y in x]).to(dev)
+    cu = [0]
+    for n in rows:
+        cu.append(cu[-1] + n)
+    tiles = ops.build_extend_tiles(rows, total, False, dev, num_q_heads=H,
+                                   flash_decode=False, min_ladder=1)
+    assert tiles[3].numel() and not tiles[0].numel()  # split, no 64-row tiles
+    out = ops.attention_extend_paged(
+        torch.cat(qs).bfloat16().to(dev), kc.to(dev), vc.to(dev), table.to(dev),
+        _i32(total, dev), _i32(cu, dev), None, scale, window=window, tiles=tiles,
+        native=ops.seq_extension(), sink_w=f(sinks), slopes=f(slopes))
+    out = out.double().cpu()
+    for s, (seen, w) in enumerate(want):
+        for i in seen:
+            assert torch.allclose(out[cu[s] + i - ctx[s]], w[i], atol=2e-2,
+                                  rtol=2e-2), (s, i)
 
 
 class DeltaRun:
