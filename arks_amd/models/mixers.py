@@ -1150,9 +1150,9 @@ class BiasedWindowAttention(SplitMixer):
 
     def _prompt_tiles(self, batch: ForwardBatch, q, out, cache_k):
         """Work list of the 256-row prefill kernel for a step whose longest
-        portion fills a tile (host-built once per step and head layout; every
-        sequence of the step is in it); None where the masked or general
-        kernels run."""
+        portion fills a tile (host-built once per step and head layout; it
+        lists the step's single rows for the decode kernel); None where the
+        masked or general kernels run."""
         if (not q.is_cuda or q.dtype != torch.bfloat16 or self.D != self.V
                 or self.D not in ops.PREFILL_MAP_DIMS or not ops.use_ladder_bias
                 or batch.kv_lens_list is None or self.scale <= 0
@@ -1163,7 +1163,7 @@ class BiasedWindowAttention(SplitMixer):
         if key not in batch.tile_cache:
             batch.tile_cache[key] = ops.build_extend_tiles(
                 batch.seq_lens_list, batch.kv_lens_list, False, q.device,
-                num_q_heads=self.H, flash_decode=False, min_ladder=1)
+                num_q_heads=self.H, min_ladder=1)
         return batch.tile_cache[key]
 
     def core(self, p, batch: ForwardBatch, cache: dict, out, out_scale) -> None:

@@ -249,7 +249,8 @@ def attention_extend_paged(
     16, M*D]); q has G*M groups of heads, group g*M + m reads key m of head
     g (tiles built without the flash-decode rows). sink_w, slopes [Hq] fp32:
     a sink's score per head, a distance bias slope[h] (i - j) off the scores
-    (256-row tiles only: build_extend_tiles(min_ladder=1)). out: a contiguous
+    (256-row tiles and single rows only: build_extend_tiles(min_ladder=1);
+    the extension must be the layer-list models'). out: a contiguous
     [Tq, Hq, D] tensor to write.
 
     Dispatch: big chunks run the 8-wave 32x32-MFMA ladder kernel
@@ -293,12 +294,20 @@ def attention_extend_paged(
         if drows is not None:
             assert maps == 1, "single rows of a two-map cache: no flash-decode"
             dq = q[drows].contiguous()
-            dout = attention_decode_paged(
-                dq, k_cache, v_cache,
-                block_tables[dseqs].contiguous(),
-                kv_lens[dseqs].contiguous(), scale, window=window,
-                sink=bool(sink), native=C,
-            )
+            dtab = block_tables[dseqs].contiguous()
+            dlens = kv_lens[dseqs].contiguous()
+            if sink_w is not None or slopes is not None:
+                each = torch.arange(dq.shape[0] + 1, dtype=torch.int32,
+                                    device=q.device)
+                dout = attention_sink_paged(
+                    dq, k_cache, v_cache, dtab, dlens, each, each[:-1], scale,
+                    bool(sink), max_q_len=1, sink_w=sink_w, window=window,
+                    slopes=slopes)
+            else:
+                dout = attention_decode_paged(
+                    dq, k_cache, v_cache, dtab, dlens, scale, window=window,
+                    sink=bool(sink), native=C,
+                )
             out[drows] = dout
         return out
     return ref.attention_extend_paged(

@@ -756,11 +756,13 @@ def test_matrix_core_attention_against_the_general_kernel(size, monkeypatch):
 
 @pytest.mark.gpu
 @pytest.mark.parametrize("window", [1, 63, 64, 90, 300, 0])
+@pytest.mark.parametrize("singles", [False, True], ids=["tiles", "single-rows"])
 @pytest.mark.parametrize("H,G,D", [(8, 2, 64), (5, 1, 128), (3, 3, 64)])
-def test_prefill_kernel_with_bias_and_sinks(H, G, D, window):
+def test_prefill_kernel_with_bias_and_sinks(H, G, D, singles, window):
     """The 256-row kernel over sequences of 1, 2, 70, 300 and 513 rows with
     contexts in front of them, one launch (a few heads: key ranges are split;
-    the sink is counted once): against the oracle's attention, every row."""
+    the sink is counted once), the single row in it or on the decode kernel:
+    against the oracle's attention, every row."""
     from arks_amd import ops
 
     dev = torch.device("cuda")
@@ -792,7 +794,8 @@ def test_prefill_kernel_with_bias_and_sinks(H, G, D, window):
     for n in rows:
         cu.append(cu[-1] + n)
     tiles = ops.build_extend_tiles(rows, total, False, dev, num_q_heads=H,
-                                   flash_decode=False, min_ladder=1)
+                                   flash_decode=singles, min_ladder=1)
+    assert (tiles[2][0] is not None) == singles
     assert tiles[3].numel() and not tiles[0].numel()  # split, no 64-row tiles
     out = ops.attention_extend_paged(
         torch.cat(qs).bfloat16().to(dev), kc.to(dev), vc.to(dev), table.to(dev),
