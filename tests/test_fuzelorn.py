@@ -348,6 +348,24 @@ def test_fast_path_sizes(tmp_path, device, dtype):
 
 
 @pytest.mark.parametrize("device,dtype", GPU_CASES)
+def test_decoded_rows_beside_long_portions(tmp_path, device, dtype):
+    """Single rows of two requests, in front of and behind a portion that
+    fills a 256-row tile."""
+    cfg = fast_path_config()
+    w = write_checkpoint(tmp_path / "m", cfg)
+    ta, tb, tc = toks(95, seed=5), toks(560, seed=6), toks(40, seed=7)
+    eng = make_engine(tmp_path / "m", device, dtype, max_tokens=768)
+    steps = [[("a", ta[:93], False), ("c", tc[:38], False)],
+             [("a", ta[93:94], False), ("b", tb[:300], False),
+              ("c", tc[38:39], False)],
+             [("b", tb[300:], False), ("c", tc[39:], False),
+              ("a", ta[94:], False)]]
+    got = replay(eng, tmp_path, steps)
+    for c, t in (("a", ta), ("b", tb), ("c", tc)):
+        assert_logits(got[c], cfg, w, t, dtype, c)
+
+
+@pytest.mark.parametrize("device,dtype", GPU_CASES)
 def test_fast_path_sizes_in_mixed_batches(tmp_path, device, dtype):
     cfg = fast_path_config()
     w = write_checkpoint(tmp_path / "m", cfg)
